@@ -17,9 +17,9 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 EXPERIMENTS = os.environ.get("MI355_BUILD_EXPERIMENTS", "0") == "1"
 SRC = [
     "csrc/mmvq.hip", "csrc/mmvq_fast.hip", "csrc/mmvq_stream.hip", "csrc/mmq.hip", "csrc/mmq_q80.hip", "csrc/act.hip", "csrc/misc.hip", "csrc/mmf.hip", "csrc/attn.hip", "csrc/attn_out.hip", "csrc/attn_prefill.hip", "csrc/clip.hip",
-    "csrc/mmb.hip", "csrc/latent_attn.hip", "csrc/mlstm.hip", "csrc/gq_attn.hip", "csrc/delta_rule.hip", "csrc/retention.hip", "csrc/routed_ff.hip",
+    "csrc/mmb.hip", "csrc/latent_attn.hip", "csrc/mlstm.hip", "csrc/gq_attn.hip", "csrc/talk_attn.hip", "csrc/delta_rule.hip", "csrc/retention.hip", "csrc/routed_ff.hip",
 ] + (["csrc/decode_engine.hip", "csrc/decode_mega.hip"] if EXPERIMENTS else ["csrc/experiments_absent.cc"]) + [
-    "host/gguf.cc", "host/runtime.cc", "host/novorax.cc", "host/fidepel.cc", "host/tuterax.cc", "host/dinilorn.cc", "host/tp_comm.cc", "host/vocab.cc", "host/sampling.cc", "host/grammar.cc", "host/json_schema.cc", "host/log.cc", "host/server_context.cc", "host/engine.cc",
+    "host/gguf.cc", "host/runtime.cc", "host/novorax.cc", "host/fidepel.cc", "host/tuterax.cc", "host/dinilorn.cc", "host/vuzazen.cc", "host/tp_comm.cc", "host/vocab.cc", "host/sampling.cc", "host/grammar.cc", "host/json_schema.cc", "host/log.cc", "host/server_context.cc", "host/engine.cc",
     "host/hip_backend.cc", "host/tp_split.cc", "host/clip.cc", "host/image_decode.cc", "csrc/c_api.cc",
 ]
 HDRS = ["csrc/dev_common.h", "csrc/kernels.h", "csrc/quant_dev.h", "csrc/mmvq_fast_dev.h", "csrc/mmvq_stream_dev.h", "csrc/attn_decode_dev.h", "host/gguf.h", "host/runtime.h", "host/tp_comm.h", "host/json.h", "host/vocab.h",
@@ -30,7 +30,9 @@ TP_WORKER = os.path.join(HERE, "bin", "mi355_tp_worker")  # a further rank of an
 SERVER = os.path.join(HERE, "bin", "mi355_server")          # the HTTP host: plain C++, dlopen()s LIB at run time (server/mi355_server.cc)
 # -ffp-contract=off: the CPU restatement this backend is checked against does not fuse mul+add
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fvisibility=hidden",
-         "-Wall", "-Wno-unused-function", "-x", "hip"]
+         "-Wall", "-Wno-unused-function", "-x", "hip",
+         # no packed-f32 instructions (v_pk_fma_f32 and its kin) anywhere: f32 arithmetic takes the scalar forms
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 # per-file flags.  Kernel-argument preload (gfx950: up to 14 dwords of the FIRST scalar arguments of a kernel arrive in SGPRs with the wave): the stream-bound
@@ -41,10 +43,6 @@ EXTRA = {
     # csrc/attn_out.hip qkv_attn_out_kernel)
     "csrc/attn_out.hip": ["-mllvm", "-amdgpu-kernarg-preload-count=5"],
 }
-# float code of these files is kept off the packed-f32 instructions (v_pk_fma_f32 and its kin): their whole arithmetic is f32 and must be the scalar forms
-NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
-for _s in ("csrc/mmb.hip", "csrc/latent_attn.hip", "csrc/mlstm.hip", "csrc/gq_attn.hip", "csrc/delta_rule.hip", "csrc/retention.hip", "csrc/routed_ff.hip"):
-    EXTRA[_s] = EXTRA.get(_s, []) + NO_PACKED_F32
 
 
 def _hipcc() -> str:
