@@ -5,10 +5,10 @@
 // optional soft cap squashes every score to cap * tanh(score / cap) first; an optional per-head sink logit joins the denominator; an optional output gate
 // multiplies head h's result by sigmoid(gate[t][h]).  Everything here is f32: positions, angles, norms, scores, weights, the running sums.
 //
-// gq_prep: per token, behind the fused q | k | v projection: an optional RMS norm of the queries and of the keys with plain weights - over the WHOLE projection
+// gq_prep: per token, behind the fused q | k | v projection: an optional short causal convolution over time on every channel; an optional RMS norm of the queries and of the keys with plain weights - over the WHOLE projection
 // (all heads at once) or over every head by itself with one weight vector shared by the heads; the rotation of the first rot_dims entries of every query and
 // key head in the rotate-half layout (entry i pairs with entry i + rot_dims / 2; the per-pair angle table comes from the host); the score multipliers (one
-// number for the layer, one per head) folded into the query; keys and values stored to the token's cache row.
+// number for the layer, one per head) folded into the query; an optional unit RMS of every value head; keys and values stored to the token's cache row.
 //
 // Optional per layer: a query multiplier that grows with the logarithm of the position (in steps of `every` positions); a learned bias per (distance bucket,
 // head) added to the score behind the soft cap (the host hands over the distance -> bucket table); cells at the first `keep_first` positions that stay seen
@@ -29,30 +29,67 @@ __device__ __forceinline__ float gq_wave_sum(float v) {
     for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
     return v;
 }
-__device__ float gq_block_sum_256(float v, float *sh) {
+template <int NT>
+__device__ float gq_block_sum(float v, float *sh) {
     v = gq_wave_sum(v);
     __syncthreads();
     if ((threadIdx.x & 63) == 0) sh[threadIdx.x >> 6] = v;
     __syncthreads();
-    return (sh[0] + sh[1]) + (sh[2] + sh[3]);
+    float s = 0.0f;
+#pragma unroll
+    for (int w = 0; w < NT / 64; w += 4) s += (sh[w] + sh[w + 1]) + (sh[w + 2] + sh[w + 3]);
+    return s;
 }
 
 constexpr int GQ_MAX_D = 512;                                   // dim and vdim the attention kernel is instantiated for (8 x 64)
 
-__global__ __launch_bounds__(256) void gq_prep_kernel(GqPrepArgs a) {
-    extern __shared__ float head_inv[];                         // norm per head: [H + G] inverse root mean squares
-    __shared__ float sh[4];
+// CONV: the token's row is the convolution of its projections with those of the tokens before it - made in LDS first (thread = channel), everything behind
+// reads it from there.  NT threads per token: a convolved row is several rows of input
+template <int NT, bool CONV>
+__global__ __launch_bounds__(NT) void gq_prep_kernel(GqPrepArgs a) {
+    extern __shared__ float gq_lds[];
+    __shared__ float sh[NT / 64];
     __shared__ float cs[2][GQ_MAX_D / 2];                       // cos / sin of the token's angle per pair: computed once, read by every head
     __shared__ float csv[2][GQ_MAX_D / 2];                      // the same for the value heads' pairs
     const int t = blockIdx.x, tid = threadIdx.x;
     const int GK = a.G * (a.maps > 1 ? a.maps : 1);             // key heads: one per (value head, map)
     const int NQ = a.H * a.dim, NK = GK * a.dim, NV = a.G * a.vdim, half = a.rot_dims >> 1;
-    const float *qr = a.p + (size_t)t * a.ld_p, *kr = qr + NQ, *vr = kr + NK;
+    float *const conv_row = gq_lds, *const head_inv = gq_lds + (CONV ? NQ + NK + NV : 0);       // norm per head: [H + GK] inverse root mean squares; v_unit: [G] behind them
+    float *const v_inv = head_inv + a.H + GK;
+    const float *qr = a.p + (size_t)t * a.ld_p;
+    if (CONV) {
+        const int C = NQ + NK + NV, back = a.conv_taps - 1, ago = a.tok_ago[t];
+        float *state = a.conv_state + (size_t)a.tok_slot[t] * back * C;
+        for (int i = tid; i < C; i += NT) {
+            float s = 0.0f;
+            for (int j = 0; j <= back; j++) {
+                const int b = back - j;                          // (tokens back: a row of the batch, or - before the segment's first row - what the slot remembers)
+                s = fmaf(a.conv_wt[(size_t)j * C + i], b <= ago ? a.p[(size_t)(t - b) * a.ld_p + i] : state[(size_t)(back - (b - ago)) * C + i], s);
+            }
+            conv_row[i] = s;
+            if (a.conv_move && back > 0) {
+                for (int j = 0; j + 1 < back; j++) state[(size_t)j * C + i] = state[(size_t)(j + 1) * C + i];
+                state[(size_t)(back - 1) * C + i] = qr[i];
+            }
+        }
+        __syncthreads();
+        qr = conv_row;
+    }
+    const float *kr = qr + NQ, *vr = kr + NK;
     float inv_q = 1.0f, inv_k = 1.0f;
+    if (a.v_unit) {                                             // sixteen lanes per value head
+        for (int g = tid >> 4; g < a.G; g += NT / 16) {
+            float ss = 0.0f;
+            for (int i = tid & 15; i < a.vdim; i += 16) { const float v = vr[(size_t)g * a.vdim + i]; ss = fmaf(v, v, ss); }
+#pragma unroll
+            for (int o = 8; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+            if ((tid & 15) == 0) v_inv[g] = 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
+        }
+    }
     const bool per_head = a.norm_per_head && a.wq_norm && a.wk_norm;
     if (per_head) {
         // sixteen lanes per head, queries then keys (q | k lie side by side in the row): every lane group's loads are on their way at once
-        for (int hh = tid >> 4; hh < a.H + GK; hh += 16) {
+        for (int hh = tid >> 4; hh < a.H + GK; hh += NT / 16) {
             const float *src = qr + (size_t)hh * a.dim;
             float ss = 0.0f;
             for (int i = tid & 15; i < a.dim; i += 16) { const float v = src[i]; ss = fmaf(v, v, ss); }
@@ -62,13 +99,13 @@ __global__ __launch_bounds__(256) void gq_prep_kernel(GqPrepArgs a) {
         }
     } else if (a.wq_norm) {
         float ss = 0.0f;
-        for (int i = tid; i < NQ; i += 256) { const float v = qr[i]; ss = fmaf(v, v, ss); }
-        inv_q = 1.0f / sqrtf(gq_block_sum_256(ss, sh) / (float)NQ + a.eps);
+        for (int i = tid; i < NQ; i += NT) { const float v = qr[i]; ss = fmaf(v, v, ss); }
+        inv_q = 1.0f / sqrtf(gq_block_sum<NT>(ss, sh) / (float)NQ + a.eps);
     }
     if (!per_head && a.wk_norm) {
         float ss = 0.0f;
-        for (int i = tid; i < NK; i += 256) { const float v = kr[i]; ss = fmaf(v, v, ss); }
-        inv_k = 1.0f / sqrtf(gq_block_sum_256(ss, sh) / (float)NK + a.eps);
+        for (int i = tid; i < NK; i += NT) { const float v = kr[i]; ss = fmaf(v, v, ss); }
+        inv_k = 1.0f / sqrtf(gq_block_sum<NT>(ss, sh) / (float)NK + a.eps);
     }
     const float p = (float)a.tok_pos[t];
     // (positions are exact in f32 up to 2^24, and so is the floor of the correctly rounded quotient for a whole-number step)
@@ -88,7 +125,7 @@ __global__ __launch_bounds__(256) void gq_prep_kernel(GqPrepArgs a) {
     float *qo = a.q + (size_t)t * a.ld_q;
     float *row = a.cache + (size_t)a.tok_cell[t] * (size_t)(NK + NV);
     // one loop over the query entries, then the key entries: element (head, d) of either
-    for (int i = tid; i < NQ + NK; i += 256) {
+    for (int i = tid; i < NQ + NK; i += NT) {
         const bool isq = i < NQ;
         const int e = isq ? i : i - NQ, d = e % a.dim, b = e - d;
         const float *src = isq ? qr : kr;
@@ -119,13 +156,13 @@ __global__ __launch_bounds__(256) void gq_prep_kernel(GqPrepArgs a) {
         } else row[e] = o;
     }
     if (!a.v_rot_freq) {
-        for (int i = tid; i < NV; i += 256) row[NK + i] = vr[i];
+        for (int i = tid; i < NV; i += NT) row[NK + i] = a.v_unit ? vr[i] * v_inv[i / a.vdim] : vr[i];
         return;
     }
-    for (int i = tid; i < NV; i += 256) {
+    for (int i = tid; i < NV; i += NT) {
         const int d = i % a.vdim, b = i - d;
         const int j = d < vhalf ? d : d - vhalf;                 // (vdim is even: every entry has a partner)
-        const float c = csv[0][j], s = csv[1][j], u = vr[b + j], w = vr[b + j + vhalf];
+        const float m = a.v_unit ? v_inv[i / a.vdim] : 1.0f, c = csv[0][j], s = csv[1][j], u = vr[b + j] * m, w = vr[b + j + vhalf] * m;
         row[NK + i] = d < vhalf ? u * c - w * s : w * c + u * s;
     }
 }
@@ -637,7 +674,45 @@ hipError_t launch_gq_prep(const GqPrepArgs &a, hipStream_t st) {
     const int n_heads = a.H + a.G * (a.maps > 1 ? a.maps : 1);
     if (a.maps > 1 && a.H % a.maps != 0) return hipErrorInvalidValue;
     if (a.norm_per_head && (size_t)n_heads * sizeof(float) > 32 * 1024) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(gq_prep_kernel, dim3((unsigned)a.T), dim3(256), a.norm_per_head ? (size_t)n_heads * sizeof(float) : 0, st, a);
+    size_t lds = (a.norm_per_head || a.v_unit ? (size_t)n_heads : 0) + (a.v_unit ? (size_t)a.G : 0);
+    if (!a.conv_wt) {
+        hipLaunchKernelGGL((gq_prep_kernel<256, false>), dim3((unsigned)a.T), dim3(256), lds * sizeof(float), st, a);
+        return hipGetLastError();
+    }
+    const size_t C = (size_t)a.H * a.dim + (size_t)a.G * (a.maps > 1 ? a.maps : 1) * a.dim + (size_t)a.G * a.vdim;
+    if (a.conv_taps < 1 || !a.tok_ago || !a.tok_slot || (a.conv_taps > 1 && !a.conv_state) || C > (size_t)GQ_CONV_MAX_CHANNELS) return hipErrorInvalidValue;
+    lds = (lds + C) * sizeof(float);
+    const auto allow = [&](const void *f) { return lds > 60 * 1024 ? hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) : hipSuccess; };
+    hipError_t e;
+    if (a.T < 64) {                                              // (a step of few rows: its time is one token's trips to memory)
+        if ((e = allow(reinterpret_cast<const void *>(&gq_prep_kernel<1024, true>))) != hipSuccess) return e;
+        hipLaunchKernelGGL((gq_prep_kernel<1024, true>), dim3((unsigned)a.T), dim3(1024), lds, st, a);
+    } else {
+        if ((e = allow(reinterpret_cast<const void *>(&gq_prep_kernel<256, true>))) != hipSuccess) return e;
+        hipLaunchKernelGGL((gq_prep_kernel<256, true>), dim3((unsigned)a.T), dim3(256), lds, st, a);
+    }
+    return hipGetLastError();
+}
+
+// the convolution state of segments of several rows: moved on behind the launch that read it.  Ascending in place: entry i + len is read before it is written
+__global__ __launch_bounds__(256) void conv_state_kernel(const float *p, int ld_p, int C, int back, float *state, const int32_t *seg_start, const int32_t *seg_len, const int32_t *seg_slot) {
+    const int seg = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
+    if (c >= C) return;
+    const int start = seg_start[seg], len = seg_len[seg];
+    float *s = state + (size_t)seg_slot[seg] * back * C + c;
+    for (int i = 0; i < back; i++) {
+        const int t = len - back + i;
+        s[(size_t)i * C] = t >= 0 ? p[(size_t)(start + t) * ld_p + c] : s[(size_t)(back + t) * C];
+    }
+}
+hipError_t launch_conv_state(const float *p, int ld_p, int C, int taps, float *state, const int32_t *seg_start, const int32_t *seg_len, const int32_t *seg_slot, int n_seg, hipStream_t st) {
+    if (n_seg <= 0 || taps <= 1 || C <= 0) return hipSuccess;
+    if (!p || !state || !seg_start || !seg_len || !seg_slot) return hipErrorInvalidValue;
+    hipLaunchKernelGGL(conv_state_kernel, dim3((unsigned)n_seg, (unsigned)((C + 255) / 256)), dim3(256), 0, st, p, ld_p, C, taps - 1, state, seg_start, seg_len, seg_slot);
+    return hipGetLastError();
+}
+hipError_t launch_gq_attn_merge(const GqAttnArgs &a, int splits, hipStream_t st) {
+    hipLaunchKernelGGL(gq_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, splits);
     return hipGetLastError();
 }
 
@@ -646,6 +721,7 @@ hipError_t launch_gq_attn(const GqAttnArgs &a, hipStream_t st) {
     const int maps = a.maps > 1 ? a.maps : 1;
     if (a.H % maps != 0 || !gq_attn_shape_ok(a.H / maps, a.G, a.dim, a.vdim) || (a.v_cs && (a.vdim & 1))) return hipErrorInvalidValue;
     if (a.rel && (!a.dist_bucket || a.n_dist < 0 || a.rel_rows < 1)) return hipErrorInvalidValue;
+    if (a.talk) return launch_talk_attn(a, st);
     // batches: the tiled pass (16-byte loads everywhere: head sizes, strides and bases must allow them); a few rows: one workgroup per (row, head)
     const auto al16 = [](const void *p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
     if (a.T >= GQ_TILE_MIN_ROWS && (a.dim & 3) == 0 && (a.vdim & 3) == 0 && (a.ld_q & 3) == 0 && (a.ld_out & 3) == 0 && al16(a.q) && al16(a.out) && al16(a.cache)) {

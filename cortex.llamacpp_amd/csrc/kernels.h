@@ -196,6 +196,9 @@ hipError_t launch_pack_q80_blocks(const ActQuant &q, int n, int T, uint8_t *bloc
 hipError_t launch_repack_rows(int type, const uint8_t *src_ggml, uint8_t *dst_dev, int64_t K, int64_t n_rows, hipStream_t st);
 // dst[i][:] = dequant(table row ids[i]) from device-layout rows
 hipError_t launch_get_rows(int type, const uint8_t *table_dev, int64_t K, const int32_t *ids, int n_ids, float *dst, hipStream_t st, float scale = 1.0f);   // dst = row * scale
+// dst[i][:] = table[ids[i]] * scale + table2[ids2[i]]: a second table's rows join the embedding rows (e.g. one indexed by a hash of neighbouring tokens)
+hipError_t launch_get_rows_pair(int type, const uint8_t *table_dev, const uint8_t *table2_dev, int64_t K, const int32_t *ids, const int32_t *ids2, int n_ids, float *dst,
+                                hipStream_t st, float scale = 1.0f);
 // scratch: cap_rows * 129 words, zero-filled once: [cap_rows ticket words | cap_rows * 64 part values | cap_rows * 64 part indices]; rows <= cap_rows
 hipError_t launch_argmax_rows(const float *x, int n, int rows, int32_t *out, float *scratch, int cap_rows, hipStream_t st);
 // ---- device-side sampling front end (reference call site common_sampler_sample, src/llama_server_context.cc:1679-1698): the k best
@@ -250,7 +253,9 @@ hipError_t launch_gather_rows_f32(const float *src, const int32_t *rows, int n_r
 // per batch instead of once per token), and the expert outputs are combined back per token in rank order.
 // Counting sort of the T*k selections by expert, stable in (token, rank) order: counts[e], offs[e] (exclusive prefix,
 // offs[n_expert] = T*k), slot_of[t*k + j] = grouped row of the pair, tok_of[row] = its token.  meta = counts | offs.
-hipError_t launch_moe_group(const int32_t *ids, int T, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, hipStream_t st);
+// w / w_of (both or neither): w_of[grouped row] = w[pair]
+hipError_t launch_moe_group(const int32_t *ids, int T, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, hipStream_t st,
+                            const float *w = nullptr, float *w_of = nullptr);
 // grouped[r] = src[tok_of[r]] for the quantised activation planes that exist in both (K codes per row)
 hipError_t launch_moe_gather_act(const ActQuant &src, const int32_t *tok_of, int n_rows, int K, const ActQuant &dst, hipStream_t st);
 // x[t][d] += sum_j y[slot_of[t*k + j]][d] * w[t][j]   (same order of operations as launch_moe_combine)
@@ -273,6 +278,9 @@ struct MMBArgs {
     float out_scale = 1.0f;                                    // multiplies every stored value (a model's logit scale)
     float epi_limit = 0.0f;                                    // MMB_CLAMP_SWIGLU: the clamp
     const float *bias = nullptr;                               // nullable, [N] f32: added to W x before the epilogue (the same vector for every outer index)
+    const float *row_scale = nullptr;                          // nullable, a factor on W x (and W2 x) of every row, by the row's place in Y in front of y_map; in front of the bias
+    const float *resid = nullptr;                              // nullable, indexed like Y (and may be Y): added behind the epilogue
+    const int32_t *x_map = nullptr, *y_map = nullptr;          // nullable, grouped batches (meta): grouped row -> row of X / of Y and resid
     int nz = 1; long long x_zs = 0, w_zs = 0, y_zs = 0;
     const int32_t *meta = nullptr;
     const int32_t *sel = nullptr; int sel_div = 1;
@@ -303,8 +311,8 @@ hipError_t launch_moe_weighted_combine(float *out, const float *y, const float *
 constexpr int MOE_COMBINE_NORM_MAX_E = 12288, MOE_COMBINE_NORM_MAX_K = 64;   // widest row and most ranks the closing launch holds in LDS
 hipError_t launch_moe_weighted_combine_norm(float *x, const float *y, const float *w, const int32_t *slot_of, const float *b, const float *sg, int ld_sg,
                                             const float *norm_w, float norm_off, float eps, int T, int E, int k, hipStream_t st);
-// x[t][:] += m * (a[t] + b[t] + sum_j w[t][j] * y[row(t, j)]): the close of a block whose mixer (a), always-on expert (b, nullable) and routed experts (y; k = 0:
-// none) all read the same normed input; row(t, j) = slot_of[t * k + j], or t * k + j without a grouping
+// x[t][:] += m * (a[t] + b[t] + sum_j w[t][j] * y[row(t, j)]): the close of a block whose mixer (a, nullable), always-on expert (b, nullable) and routed experts (y; k = 0:
+// none; w nullable: weights 1) all read the same normed input; row(t, j) = slot_of[t * k + j], or t * k + j without a grouping
 hipError_t launch_block_combine(float *x, const float *a, const float *b, const float *y, const float *w, const int32_t *slot_of, int T, int E, int k, float m, hipStream_t st);
 
 // ---------------------------------------------------------------- grouped-query attention on f32 cache rows (gq_attn.hip)
@@ -328,8 +336,18 @@ struct GqPrepArgs {
     // the attention's output is then turned back by the query's position, so that only position differences remain in the sum.  v_cs: [T][vdim] - the token's
     // cos (first vdim / 2) and sin per pair, written here for the attention launch (GqAttnArgs::v_cs)
     const float *v_rot_freq; float *v_cs;
+    int v_unit;                            // 1: every value head is divided by its root mean square (eps as above, no weight) before it is stored
+    // nullable: a short causal convolution over time on every channel of q, k and v, in front of all of the above: u_t = sum_j conv_wt[j][c] p_(t - taps + 1 + j),
+    // zeros before the sequence's start.  conv_wt: [taps][C], C = H*dim + G*dim + G*vdim in p's channel order; conv_state: [slot][taps - 1][C], the inputs before
+    // the rows of the batch, oldest first; tok_ago: rows of the token's own segment directly in front of it; tok_slot: its sequence slot.  A launch covers rows
+    // of segments no two of which share a slot.  conv_move = 1 (every segment is one row): the launch also moves the state on; longer segments: launch_conv_state
+    // behind it
+    const float *conv_wt; int conv_taps; float *conv_state; const int32_t *tok_ago, *tok_slot; int conv_move;
 };
+constexpr int GQ_CONV_MAX_CHANNELS = 36 * 1024;   // a token's convolved row is held in LDS
 hipError_t launch_gq_prep(const GqPrepArgs &a, hipStream_t st);
+// state[slot][i][c] = the segment's input taps - 1 - i tokens before its next one: the last taps - 1 inputs of every segment (rows of p, or what the slot held)
+hipError_t launch_conv_state(const float *p, int ld_p, int C, int taps, float *state, const int32_t *seg_start, const int32_t *seg_len, const int32_t *seg_slot, int n_seg, hipStream_t st);
 struct GqAttnArgs {
     const float *q; int ld_q;              // [T][H][dim] from launch_gq_prep
     float *out; int ld_out;                // [T][H][vdim]
@@ -346,6 +364,9 @@ struct GqAttnArgs {
     const float *gate; int ld_gate;        // nullable: head h's output is multiplied by sigmoid(gate[t * ld_gate + h])
     float softcap;                         // > 0: a score s becomes softcap * tanh(s / softcap) before the softmax
     const float *v_cs;                     // nullable, [T][vdim] from launch_gq_prep: the values were stored turned; a head's output turns back by minus its row's angle per pair, before the gate
+    // nullable, [H][H]: the heads' scores are mixed before the softmax - score_h becomes sum_g talk[h][g] score_g (talk_attn.hip; plain softmax layers: no maps, no
+    // rel, no softcap, no v_cs)
+    const float *talk;
     // the scanned cells cut into runs, one workgroup each, merged afterwards: `splits` runs for steps of a few rows; for prompt batches with too few tiles
     // to fill the device as many as n_kv_hint (the host's count of cells in use, 0: unknown) and the buffer allow.  part: room for part_floats floats,
     // T * H * runs * (vdim + 2) are used
@@ -358,18 +379,24 @@ constexpr int GQ_TILE_MAX_SPLITS = 16;
 constexpr int GQ_TILE_MIN_ROWS = 32;     // batches from this many rows on take the LDS-tiled pass (64 rows x 64 cells per step) instead of one workgroup per (row, head)
 bool gq_attn_shape_ok(int H, int G, int dim, int vdim);
 hipError_t launch_gq_attn(const GqAttnArgs &a, hipStream_t st);
+hipError_t launch_gq_attn_merge(const GqAttnArgs &a, int splits, hipStream_t st);   // joins the records of a cut scan: [T][H][splits][max | sum | vdim weighted values]
+// the same attention with mixed scores (talk_attn.hip); launch_gq_attn hands over when a.talk is set.  Up to TALK_ROW_RUNS records per head and step of few rows
+constexpr int TALK_ROW_SPLITS = 32, TALK_ROW_RUNS = 256, TALK_TILE_RUNS = 8;
+bool talk_attn_shape_ok(int H, int G, int dim, int vdim);
+hipError_t launch_talk_attn(const GqAttnArgs &a, hipStream_t st);
 // two score maps joined: y[t][h][:] = unit_rms(a1 - lambda * a2) * out_mult * sigmoid(gate[t * ld_gate + h * vdim + :]), a1 / a2 = att[t][2h], att[t][2h + 1]
 hipError_t launch_gq_maps_out(const float *att, int ld_att, const float *gate, int ld_gate, int T, int H, int vdim, float lambda, float out_mult, float eps,
                               float *y, int ld_y, hipStream_t st);
 
 // ---------------------------------------------------------------- latent attention (latent_attn.hip)
 // cache row of a cell: [kv_rank normed latent | rot rotated shared key part] f32.  rot_freq: [rot_dims / 2] angles per position (host-made, YaRN blend
-// included), rot_mscale multiplies cos and sin; interleaved pairs over the first rot_dims entries of the rotated part.
+// included), rot_mscale multiplies cos and sin; interleaved pairs (or halves) over the first rot_dims entries of the rotated part.
 struct LatentPrepArgs {
     const float *a; int ld_a;              // [T][q_rank | kv_rank | rot] down-projections
     int T, q_rank, kv_rank, rot, rot_dims;
     const float *wq_norm, *wkv_norm; float eps;
     const float *rot_freq; float rot_mscale;
+    int rot_halves;                        // 1: entry i turns with entry i + rot_dims / 2 instead of entry 2i with entry 2i + 1
     const int32_t *tok_pos, *tok_cell;
     float *cq;                             // [T][q_rank] normed query latent
     float *cache;                          // [n_ctx][kv_rank + rot]
@@ -385,6 +412,8 @@ struct LatentAttnArgs {
     int window;                            // cells at distance 0 .. window - 1 are seen; 0 = every earlier cell
     float scale; const float *sink;        // sink: [H] or nullptr
     const float *rot_freq; float rot_mscale;
+    int rot_halves;                        // as in LatentPrepArgs
+    const float *gate; int ld_gate;        // nullable: head h's attended latent is multiplied by sigmoid(gate[t * ld_gate + h])
     // single-token steps: the scanned cells cut into `splits` runs, one workgroup each, merged afterwards; part: T * H * splits * (kv_rank + 2) floats (nullptr / splits <= 1: one workgroup per (token, head))
     float *part; int splits;
     // nullable: per token, one past the highest cell that can hold a key of its sequence at or before its position (host-made from the cell table): the scan

@@ -5,10 +5,11 @@
 //   s = (qa . c + rope(q_rot) . r) * scale,
 // and the attended value is the weighted sum of latents, unfolded through W_uv afterwards - keys and values are never materialised, every head reads the
 // same row.  Visibility: same sequence, 0 <= pos_query - pos_cell < window (window 0: no limit).  The softmax denominator takes one extra term exp(sink_h),
-// a learned per-head logit with neither key nor value behind it.  Everything here is f32: positions, angles, scores, weights, the running sums.
+// a learned per-head logit with neither key nor value behind it.  An optional output gate multiplies head h's attended latent by sigmoid(gate[t][h]) (a factor per
+// head: it commutes with W_uv).  Everything here is f32: positions, angles, scores, weights, the running sums.
 //
 // latent_prep: per token, the two RMS norms behind the down-projections (query latent -> cq, key / value latent -> cache row) and the rotation of the
-// shared key part into the cache row.  Interleaved pairs (2i, 2i + 1); the per-pair frequency table (YaRN blend included) comes from the host.
+// shared key part into the cache row.  Interleaved pairs (2i, 2i + 1), or entry i with entry i + half the turning part; the per-pair frequency table (YaRN blend included) comes from the host.
 #include "kernels.h"
 
 namespace mi355 {
@@ -31,6 +32,20 @@ __device__ float block_sum_256(float v, float *sh) {
     if ((threadIdx.x & 63) == 0) sh[threadIdx.x >> 6] = v;
     __syncthreads();
     return sh[0] + sh[1] + sh[2] + sh[3];
+}
+
+// entry i of the turning part: its pair's index, the places of the pair's two entries, and which of them it is
+struct LatentPair { int pr, iu, iv; bool second; };
+__device__ __forceinline__ LatentPair latent_pair(int i, int dims, int halves) {
+    const int half = dims >> 1;
+    if (halves) { const int pr = i < half ? i : i - half; return {pr, pr, pr + half, i >= half}; }
+    return {i >> 1, i & ~1, i | 1, (i & 1) != 0};
+}
+// the factor of head h's attended latent: 1 over the softmax denominator, times the output gate
+__device__ __forceinline__ float latent_out_factor(const LatentAttnArgs &a, int t, int h, float den) {
+    float inv = den > 0.0f ? 1.0f / den : 0.0f;
+    if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)t * a.ld_gate + h]));
+    return inv;
 }
 
 __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepArgs a) {
@@ -56,10 +71,10 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepArgs a) {
     const float p = (float)a.tok_pos[t];
     for (int i = tid; i < a.rot; i += 256) {
         if (i < a.rot_dims) {
-            const int pr = i >> 1;
-            const float ang = p * a.rot_freq[pr], c = cosf(ang) * a.rot_mscale, s = sinf(ang) * a.rot_mscale;
-            const float u = kr[2 * pr], v = kr[2 * pr + 1];
-            dst[a.kv_rank + i] = (i & 1) ? v * c + u * s : u * c - v * s;
+            const LatentPair q = latent_pair(i, a.rot_dims, a.rot_halves);
+            const float ang = p * a.rot_freq[q.pr], c = cosf(ang) * a.rot_mscale, s = sinf(ang) * a.rot_mscale;
+            const float u = kr[q.iu], v = kr[q.iv];
+            dst[a.kv_rank + i] = q.second ? v * c + u * s : u * c - v * s;
         } else dst[a.kv_rank + i] = kr[i];
     }
 }
@@ -87,10 +102,10 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(LatentAttnArgs a) {
             const float *qr = a.q + (size_t)t * a.ld_q + (size_t)h * (a.dim + R) + a.dim;
             const int r = i - KR;
             if (r < a.rot_dims) {
-                const int pr = r >> 1;
-                const float ang = (float)tpos * a.rot_freq[pr], c = cosf(ang) * a.rot_mscale, sn = sinf(ang) * a.rot_mscale;
-                const float u = qr[2 * pr], w = qr[2 * pr + 1];
-                v = (r & 1) ? w * c + u * sn : u * c - w * sn;
+                const LatentPair q = latent_pair(r, a.rot_dims, a.rot_halves);
+                const float ang = (float)tpos * a.rot_freq[q.pr], c = cosf(ang) * a.rot_mscale, sn = sinf(ang) * a.rot_mscale;
+                const float u = qr[q.iu], w = qr[q.iv];
+                v = q.second ? w * c + u * sn : u * c - w * sn;
             } else v = qr[r];
         }
         qv[i] = v;
@@ -200,7 +215,7 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(LatentAttnArgs a) {
     for (int w = 0; w < NW; w++) MM = fmaxf(MM, wm[w]);
     float den = a.sink ? expf(a.sink[h] - MM) : 0.0f;
     for (int w = 0; w < NW; w++) den += wl[w] > 0.0f ? wl[w] * expf(wm[w] - MM) : 0.0f;
-    const float inv = den > 0.0f ? 1.0f / den : 0.0f;
+    const float inv = latent_out_factor(a, t, h, den);
     for (int i = tid; i < KR; i += blockDim.x) {
         float o = 0.0f;
         for (int w = 0; w < NW; w++) o += wl[w] > 0.0f ? wacc[w * LP + i] * expf(wm[w] - MM) : 0.0f;
@@ -215,7 +230,7 @@ __global__ __launch_bounds__(256) void latent_attn_merge_kernel(LatentAttnArgs a
     for (int s = 0; s < splits; s++) if (rec[(size_t)s * (KR + 2) + 1] > 0.0f) MM = fmaxf(MM, rec[(size_t)s * (KR + 2)]);
     float den = a.sink ? expf(a.sink[h] - MM) : 0.0f;
     for (int s = 0; s < splits; s++) { const float *r = rec + (size_t)s * (KR + 2); den += r[1] > 0.0f ? r[1] * expf(r[0] - MM) : 0.0f; }
-    const float inv = den > 0.0f ? 1.0f / den : 0.0f;
+    const float inv = latent_out_factor(a, t, h, den);
     for (int i = tid; i < KR; i += 256) {
         float o = 0.0f;
         for (int s = 0; s < splits; s++) { const float *r = rec + (size_t)s * (KR + 2); o += r[1] > 0.0f ? r[2 + i] * expf(r[0] - MM) : 0.0f; }

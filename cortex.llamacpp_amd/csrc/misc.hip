@@ -122,6 +122,20 @@ hipError_t launch_get_rows(int type, const uint8_t *table, int64_t K, const int3
     return hipGetLastError();
 }
 
+__global__ void get_rows_pair_kernel(int type, const uint8_t *table, const uint8_t *table2, int K, size_t row_bytes, const int32_t *ids, const int32_t *ids2, float *dst, float scale) {
+    const int i = blockIdx.y;
+    const uint8_t *row = table + (size_t)ids[i] * row_bytes, *row2 = table2 + (size_t)ids2[i] * row_bytes;
+    for (int e = blockIdx.x * blockDim.x + threadIdx.x; e < K; e += gridDim.x * blockDim.x)
+        dst[(size_t)i * K + e] = dequant_elem(type, row, K, e) * scale + dequant_elem(type, row2, K, e);
+}
+hipError_t launch_get_rows_pair(int type, const uint8_t *table, const uint8_t *table2, int64_t K, const int32_t *ids, const int32_t *ids2, int n_ids, float *dst, hipStream_t st, float scale) {
+    if (n_ids <= 0) return hipSuccess;
+    int bx = (int)((K + 255) / 256);
+    if (bx > 64) bx = 64;
+    hipLaunchKernelGGL(get_rows_pair_kernel, dim3(bx, n_ids), dim3(256), 0, st, type, table, table2, (int)K, dev_row_bytes(type, K), ids, ids2, dst, scale);
+    return hipGetLastError();
+}
+
 // ---------------------------------------------------------------- argmax per row (lowest index wins ties), two stages
 constexpr int ARGMAX_PARTS = 64;
 __device__ __forceinline__ void argmax_block_reduce(float &best, int &idx, float *bv, int *bi) {
@@ -436,7 +450,7 @@ hipError_t launch_moe_combine(float *x, const float *eo, const float *w, int T, 
 // One workgroup of 4 waves.  The selections are staged in LDS; wave w owns experts w, w + 4, ...: it walks the selections
 // 64 at a time in (token, rank) order, a ballot marks the ones that chose its expert and a prefix count of the ballot
 // gives each its row: stable, deterministic, no atomics.  (Runs once per layer of a prompt batch: a few microseconds.)
-__global__ __launch_bounds__(256) void moe_group_kernel(const int32_t *ids, int n_sel, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of) {
+__global__ __launch_bounds__(256) void moe_group_kernel(const int32_t *ids, int n_sel, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, const float *w, float *w_of) {
     extern __shared__ int32_t sid[];               // [n_sel]
     __shared__ int cnt[64], off[65];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -468,14 +482,16 @@ __global__ __launch_bounds__(256) void moe_group_kernel(const int32_t *ids, int 
                 const int row = r + __popcll(m & ((1ull << lane) - 1ull));
                 slot_of[b + lane] = row;
                 tok_of[row] = (b + lane) / k;
+                if (w_of) w_of[row] = w[b + lane];
             }
             r += __popcll(m);
         }
     }
 }
-hipError_t launch_moe_group(const int32_t *ids, int T, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, hipStream_t st) {
+hipError_t launch_moe_group(const int32_t *ids, int T, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, hipStream_t st, const float *w, float *w_of) {
+    if (w_of && !w) return hipErrorInvalidValue;
     if (n_expert > 64 || T * k <= 0 || (size_t)T * k * 4 > 60 * 1024) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(256), (size_t)T * k * 4, st, ids, T * k, k, n_expert, meta, slot_of, tok_of);
+    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(256), (size_t)T * k * 4, st, ids, T * k, k, n_expert, meta, slot_of, tok_of, w, w_of);
     return hipGetLastError();
 }
 // one workgroup per grouped row: 16-byte copies of the code plane(s), then the small per-block planes
@@ -620,14 +636,14 @@ __global__ void block_combine_kernel(float *x, const float *a, const float *b, c
     if (i >= (int64_t)T * E) return;
     const int t = (int)(i / E), d = (int)(i - (int64_t)t * E);
     float o = 0.0f;
-    for (int j = 0; j < k; j++) o += y[(size_t)(slot_of ? slot_of[(size_t)t * k + j] : t * k + j) * E + d] * w[(size_t)t * k + j];
+    for (int j = 0; j < k; j++) o += y[(size_t)(slot_of ? slot_of[(size_t)t * k + j] : t * k + j) * E + d] * (w ? w[(size_t)t * k + j] : 1.0f);
     if (b) o += b[i];
     if (a) o += a[i];
     x[i] = x[i] + m * o;
 }
 hipError_t launch_block_combine(float *x, const float *a, const float *b, const float *y, const float *w, const int32_t *slot_of, int T, int E, int k, float m, hipStream_t st) {
     if ((int64_t)T * E <= 0) return hipSuccess;
-    if (k > 0 && (!y || !w)) return hipErrorInvalidValue;
+    if (k > 0 && !y) return hipErrorInvalidValue;
     hipLaunchKernelGGL(block_combine_kernel, dim3((unsigned)(((int64_t)T * E + 255) / 256)), dim3(256), 0, st, x, a, b, y, w, slot_of, T, E, k, m);
     return hipGetLastError();
 }

@@ -14,7 +14,9 @@
 //   * mmb_f32   - batches in f32 mode (and every shape the other two refuse): LDS-tiled, v_fma_f32 only - products of an f32 activation and a bf16 weight
 //                 widened exactly, no reduced-precision matrix mode anywhere.
 // Epilogues: store | relu(y)^2 | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = W x capped from above and u = W2 x clamped
-// to +- the same limit (the gated ones: two weight sets, one pass over the activations).  An optional f32 bias per output column joins W x before the epilogue.
+// to +- the same limit (the gated ones: two weight sets, one pass over the activations).  Around the epilogue, each optional: a factor per row on W x (and W2 x)
+// - linear layers without a bias: the row of X itself times that number -, an f32 bias per output column in front of it, a residual row added behind it.  A
+// grouped batch may read its rows of X, and write its rows of Y, through maps (no gather in front of the launch, no scatter behind it).
 #include "kernels.h"
 
 namespace mi355 {
@@ -46,18 +48,28 @@ __device__ __forceinline__ float epi_apply(int epi, float a, float b, float lim 
 }
 
 // where the rows of outer index z live: first row and row count of X / Y, the weight set
-struct ZView { const float *x; const unsigned short *w, *w2; float *y; int rows; };
+struct ZView { const float *x; const unsigned short *w, *w2; float *y; const float *resid; int rows, x0, y0; };   // x, y, resid: bases; row t of z: x0 + t, y0 + t
 __device__ __forceinline__ ZView z_view(const MMBArgs &a, int z) {
     ZView v;
-    int wz = z, x0 = 0, y0 = 0;
+    int wz = z;
+    v.x0 = v.y0 = 0;
     v.rows = a.T;
-    if (a.sel) { wz = a.sel[z]; x0 = z / a.sel_div; y0 = z; v.rows = 1; }
-    else if (a.meta) { v.rows = a.meta[z]; x0 = y0 = a.meta[a.nz + z]; }
-    v.x = a.x + (size_t)(a.sel || a.meta ? 0 : z) * a.x_zs + (size_t)x0 * a.ldx;
-    v.y = a.y + (size_t)(a.sel || a.meta ? 0 : z) * a.y_zs + (size_t)y0 * a.ldy;
+    if (a.sel) { wz = a.sel[z]; v.x0 = z / a.sel_div; v.y0 = z; v.rows = 1; }
+    else if (a.meta) { v.rows = a.meta[z]; v.x0 = v.y0 = a.meta[a.nz + z]; }
+    v.x = a.x + (size_t)(a.sel || a.meta ? 0 : z) * a.x_zs;
+    v.y = a.y + (size_t)(a.sel || a.meta ? 0 : z) * a.y_zs;
+    v.resid = a.resid ? a.resid + (size_t)(a.sel || a.meta ? 0 : z) * a.y_zs : nullptr;
     v.w = a.w + (size_t)wz * a.w_zs;
     v.w2 = a.w2 ? a.w2 + (size_t)wz * a.w_zs : nullptr;
     return v;
+}
+
+__device__ __forceinline__ const float *x_row(const MMBArgs &a, const ZView &v, int t) { return v.x + (size_t)(a.x_map ? a.x_map[v.x0 + t] : v.x0 + t) * a.ldx; }
+__device__ __forceinline__ size_t y_row(const MMBArgs &a, const ZView &v, int t) { return (size_t)(a.y_map ? a.y_map[v.y0 + t] : v.y0 + t) * a.ldy; }
+// output (t, n) from its finished sums; yr = y_row(t), rs = the row's factor, res = the residual's entry (0: none)
+__device__ __forceinline__ void y_store(const MMBArgs &a, const ZView &v, size_t yr, int n, float s1, float s2, float rs, float res) {
+    s1 *= rs; s2 *= rs;
+    v.y[yr + n] = epi_apply(a.epi, a.bias ? s1 + a.bias[n] : s1, s2, a.epi_limit) * a.out_scale + res;
 }
 
 // ---------------------------------------------------------------- few rows: one wave per output column
@@ -86,6 +98,13 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
         for (int r = 0; r < NR; r++) { acc[r][i] = 0.0f; acc2[r][i] = 0.0f; }
     }
     const int nt = v.rows < TBR ? v.rows : TBR;
+    float res[NR][TBR], rsc[TBR];                               // (requested in front of the walk over k: nothing waits for them behind it)
+#pragma unroll
+    for (int i = 0; i < TBR; i++) {
+        rsc[i] = a.row_scale && i < nt ? a.row_scale[v.y0 + i] : 1.0f;
+#pragma unroll
+        for (int r = 0; r < NR; r++) res[r][i] = v.resid && i < nt && n0 + r < a.N ? v.resid[y_row(a, v, i) + n0 + r] : 0.0f;
+    }
     for (int k = lane * 8; k < a.K; k += 512) {
         u16x8 w8[NR], w28[NR];
 #pragma unroll
@@ -102,7 +121,7 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
 #pragma unroll
         for (int i = 0; i < TBR; i++) {
             if (i >= nt) break;
-            const float *xr = v.x + (size_t)i * a.ldx + k;
+            const float *xr = x_row(a, v, i) + k;
             const f32x4 x0 = *reinterpret_cast<const f32x4 *>(xr), x1 = *reinterpret_cast<const f32x4 *>(xr + 4);
             float xs[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
             if (pn) {
@@ -131,7 +150,7 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) { s1 += __shfl_xor(s1, o, 64); s2 += __shfl_xor(s2, o, 64); }
             if (pn) { s1 *= inv; s2 *= inv; }
-            if (lane == 0 && n0 + r < a.N) v.y[(size_t)i * a.ldy + n0 + r] = epi_apply(a.epi, a.bias ? s1 + a.bias[n0 + r] : s1, s2, a.epi_limit) * a.out_scale;
+            if (lane == 0 && n0 + r < a.N) y_store(a, v, y_row(a, v, i), n0 + r, s1, s2, rsc[i], res[r][i]);
         }
     }
 }
@@ -152,6 +171,12 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
 #pragma unroll
         for (int i = 0; i < TB; i++) { acc[i] = 0.0f; acc2[i] = 0.0f; ss[i] = 0.0f; }
         const int nt = v.rows - t0 < TB ? v.rows - t0 : TB;
+        float res[TB], rsc[TB];
+#pragma unroll
+        for (int i = 0; i < TB; i++) {
+            rsc[i] = a.row_scale && i < nt ? a.row_scale[v.y0 + t0 + i] : 1.0f;
+            res[i] = v.resid && i < nt ? v.resid[y_row(a, v, t0 + i) + n] : 0.0f;
+        }
         if (VEC) {
             for (int k = lane * 8; k < a.K; k += 512) {
                 const u16x8 w8 = *reinterpret_cast<const u16x8 *>(wr + k);
@@ -166,7 +191,7 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
 #pragma unroll
                 for (int i = 0; i < TB; i++) {
                     if (i >= nt) break;
-                    const float *xr = v.x + (size_t)(t0 + i) * a.ldx + k;
+                    const float *xr = x_row(a, v, t0 + i) + k;
                     const f32x4 x0 = *reinterpret_cast<const f32x4 *>(xr), x1 = *reinterpret_cast<const f32x4 *>(xr + 4);
                     float xs[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
                     if (pn) {
@@ -186,7 +211,7 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
 #pragma unroll
                 for (int i = 0; i < TB; i++) {
                     if (i >= nt) break;
-                    float x = v.x[(size_t)(t0 + i) * a.ldx + k];
+                    float x = x_row(a, v, t0 + i)[k];
                     if (pn) { ss[i] = fmaf(x, x, ss[i]); x = x * pw; }
                     acc[i] = fmaf(x, w, acc[i]);
                     acc2[i] = fmaf(x, w2, acc2[i]);
@@ -200,7 +225,7 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) { s += __shfl_xor(s, o, 64); s2 += __shfl_xor(s2, o, 64); q += __shfl_xor(q, o, 64); }
             if (pn) { const float inv = 1.0f / sqrtf(q / (float)a.K + a.pn_eps); s *= inv; s2 *= inv; }
-            if (lane == 0) v.y[(size_t)(t0 + i) * a.ldy + n] = epi_apply(a.epi, a.bias ? s + a.bias[n] : s, s2, a.epi_limit) * a.out_scale;
+            if (lane == 0) y_store(a, v, y_row(a, v, t0 + i), n, s, s2, rsc[i], res[i]);
         }
     }
 }
@@ -221,7 +246,7 @@ __global__ __launch_bounds__(256) void mmb_f32_kernel(MMBArgs a) {
 #pragma unroll
         for (int j = 0; j < 4; j++) { acc[i][j] = 0.0f; acc2[i][j] = 0.0f; }
     const bool xrow = t0 + lr < v.rows, wrow = n0 + lr < a.N;
-    const float *xr = v.x + (size_t)(t0 + lr) * a.ldx;
+    const float *xr = x_row(a, v, xrow ? t0 + lr : t0);
     const unsigned short *wr = v.w + (size_t)(n0 + lr) * a.ldw;
     const unsigned short *wr2 = GATED ? v.w2 + (size_t)(n0 + lr) * a.ldw : nullptr;
     for (int k0 = 0; k0 < a.K; k0 += BK) {
@@ -258,10 +283,12 @@ __global__ __launch_bounds__(256) void mmb_f32_kernel(MMBArgs a) {
     for (int i = 0; i < 4; i++) {
         const int t = t0 + ty * 4 + i;
         if (t >= v.rows) continue;
+        const size_t yr = y_row(a, v, t);
+        const float rs = a.row_scale ? a.row_scale[v.y0 + t] : 1.0f;
 #pragma unroll
         for (int j = 0; j < 4; j++) {
             const int n = n0 + tx * 4 + j;
-            if (n < a.N) v.y[(size_t)t * a.ldy + n] = epi_apply(a.epi, a.bias ? acc[i][j] + a.bias[n] : acc[i][j], acc2[i][j], a.epi_limit) * a.out_scale;
+            if (n < a.N) y_store(a, v, yr, n, acc[i][j], acc2[i][j], rs, v.resid ? v.resid[yr + n] : 0.0f);
         }
     }
 }
@@ -281,7 +308,7 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a) {
         const int n = n0 + 32 * i + m, t = t0 + 32 * i + m;     // rows past the end read the last row; their results are never stored
         wr[i] = v.w + (size_t)(n < a.N ? n : a.N - 1) * a.ldw + 8 * kg;
         wr2[i] = GATED ? v.w2 + (size_t)(n < a.N ? n : a.N - 1) * a.ldw + 8 * kg : nullptr;
-        xr[i] = v.x + (size_t)(t < v.rows ? t : v.rows - 1) * a.ldx + 8 * kg;
+        xr[i] = x_row(a, v, t < v.rows ? t : v.rows - 1) + 8 * kg;
     }
     f32x16 acc[WT][WT], acc2[GATED ? WT : 1][GATED ? WT : 1];
 #pragma unroll
@@ -343,10 +370,12 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a) {
         for (int j = 0; j < WT; j++) {
             const int t = t0 + 32 * j + m;
             if (t >= v.rows) continue;
+            const size_t yr = y_row(a, v, t);
+            const float rs = a.row_scale ? a.row_scale[v.y0 + t] : 1.0f;
 #pragma unroll
             for (int r = 0; r < 16; r++) {
                 const int n = n0 + 32 * i + (r & 3) + 8 * (r >> 2) + 4 * kg;
-                if (n < a.N) v.y[(size_t)t * a.ldy + n] = epi_apply(a.epi, a.bias ? acc[i][j][r] + a.bias[n] : acc[i][j][r], GATED ? acc2[i][j][r] : 0.0f, a.epi_limit) * a.out_scale;
+                if (n < a.N) y_store(a, v, yr, n, acc[i][j][r], GATED ? acc2[i][j][r] : 0.0f, rs, v.resid ? v.resid[yr + n] : 0.0f);
             }
         }
 }
@@ -356,7 +385,7 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a) {
 hipError_t launch_mmb(const MMBArgs &a, hipStream_t st) {
     if (a.T <= 0 || a.N <= 0 || a.nz <= 0) return hipSuccess;
     const bool gated = a.epi == MMB_SILU_MUL || a.epi == MMB_GELU_MUL || a.epi == MMB_CLAMP_SWIGLU;
-    if (a.K <= 0 || !a.x || !a.w || !a.y || (gated && !a.w2)) return hipErrorInvalidValue;
+    if (a.K <= 0 || !a.x || !a.w || !a.y || (gated && !a.w2) || (a.x_map && !a.meta) || (a.y_map && !a.meta)) return hipErrorInvalidValue;
     const auto al = [](const void *p, size_t n) { return (reinterpret_cast<uintptr_t>(p) & (n - 1)) == 0; };
     // 16-byte loads of both operands: every row start and every stride on a 16-byte boundary
     const bool vec = (a.K % 8) == 0 && (a.ldw % 8) == 0 && (a.w_zs % 8) == 0 && (a.ldx % 4) == 0 && (a.x_zs % 4) == 0 && al(a.w, 16) && al(a.x, 16) &&

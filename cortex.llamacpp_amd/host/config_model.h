@@ -1,7 +1,6 @@
 // config_model.h — what the loaders of the folder models (config.json + model.safetensors, bf16 weights) share: reading the configuration, checking every
 // tensor against it on the way to the device, and laying out the order of layer runs with its looped span.  One loader per design (novorax.cc, fidepel.cc,
-// tuterax.cc, dinilorn.cc);
-// config_model_load picks it by the configuration's "architecture".
+// tuterax.cc, dinilorn.cc, vuzazen.cc); config_model_load picks it by the configuration's "architecture".
 #pragma once
 
 #include <algorithm>
@@ -94,6 +93,20 @@ struct Bf16Loader {
         std::vector<float> h((size_t)n, widen(*(const unsigned short *)t->data));
         return (float *)dev(h.data(), h.size() * 4);
     }
+    // a [heads * D][R] bf16 tensor transposed inside every head: [heads][R][D] (a per-head product with the transpose)
+    BfMat head_transposed(const std::string &name, int heads, int D, int R) {
+        BfMat o;
+        const SafeTensor *t = need(name, "BF16", {(int64_t)heads * D, R});
+        if (!t) return o;
+        const unsigned short *s = (const unsigned short *)t->data;
+        std::vector<unsigned short> tr((size_t)heads * R * D);
+        for (int h = 0; h < heads; h++)
+            for (int d = 0; d < D; d++)
+                for (int r = 0; r < R; r++) tr[((size_t)h * R + r) * D + d] = s[((size_t)h * D + d) * R + r];
+        o.w = (unsigned short *)dev(tr.data(), tr.size() * 2);
+        o.N = R; o.K = D;
+        return o;
+    }
     // the embedding table with the row stride launch_get_rows expects
     BfMat embedding(const std::string &name, int V, int W) {
         BfMat o;
@@ -139,5 +152,6 @@ Model *novorax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
 Model *fidepel_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
 Model *tuterax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
 Model *dinilorn_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
+Model *vuzazen_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
 
 }  // namespace mi355

@@ -280,7 +280,7 @@ hipError_t Context::nvx_retention_mixer(const NvxLayer &L, const NvxRun &r, int 
         DNL_TRY(launch_retention_scan(ra, stream_));
     }
     DNL_TRY(launch_mlstm_out(nvx_o_, H * VD, nvx_a_, LD_P, L.off_g, nullptr, T, H, VD, M.eps, nvx_att_, H * VD, stream_, 0, MLSTM_GATE_SILU));
-    DNL_TRY(nvx_linear(L.o, nvx_att_, H * VD, T, nvx_y_, W));
+    DNL_TRY(nvx_close_linear(L.o, nvx_att_, H * VD, T, L.norm1b));
     prof_mark("retention");
     return hipSuccess;
 }
@@ -312,10 +312,20 @@ hipError_t Context::nvx_routed_feed_forward(const NvxLayer &L, int T, bool *clos
         stream_ = main_stream;
     }
     DNL_TRY(nvx_linear(L.route, h, W, T, nvx_a_, L.route.N, MMB_STORE, nullptr, 1.0f, pn));
-    DNL_TRY(nvx_routed_experts(L, h, pn, T, nvx_a_, L.route.N));
+    bool added = false;
+    DNL_TRY(nvx_routed_experts(L, h, pn, T, nvx_a_, L.route.N, closed ? &added : nullptr));
     if (fork) DNL_TRY(hipStreamWaitEvent(main_stream, nvx_join_ev_[0], 0));
     else if (shared) DNL_TRY(nvx_shared_expert(L, h, pn, T));
     const int32_t *slot_of = grouped ? nvx_slot_ : nullptr;
+    if (closed && !L.norm2b) {                                   // nothing behind the feed-forward: the sum goes into the stream (where the expert's own product has not put it)
+        if (shared && L.off_sg >= 0) {
+            DNL_TRY(launch_moe_weighted_combine(nvx_y_, nvx_yg_, nvx_rw_, slot_of, nvx_ys_, nvx_a_ + L.off_sg, L.route.N, T, W, L.top, stream_));
+            DNL_TRY(launch_add(x_, nvx_y_, x_, (int64_t)T * W, stream_));
+        } else if (!added) DNL_TRY(launch_block_combine(x_, nullptr, shared ? nvx_ys_ : nullptr, nvx_yg_, L.weight_in ? nullptr : nvx_rw_, slot_of, T, W, L.top, 1.0f, stream_));
+        *closed = true;
+        prof_mark("expert_sum");
+        return hipSuccess;
+    }
     const float *sb = shared ? nvx_ys_ : nullptr, *sg = shared && L.off_sg >= 0 ? nvx_a_ + L.off_sg : nullptr;
     if (closed && L.norm2b && W <= MOE_COMBINE_NORM_MAX_E && L.top <= MOE_COMBINE_NORM_MAX_K) {
         DNL_TRY(launch_moe_weighted_combine_norm(x_, nvx_yg_, nvx_rw_, slot_of, sb, sg, L.route.N, L.norm2b, M.norm_off, M.eps, T, W, L.top, stream_));

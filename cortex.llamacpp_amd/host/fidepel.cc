@@ -161,11 +161,11 @@ bool nvx_routed_as_groups(const NvxLayer &L, int T) {
     return L.ff_kind == NVX_FF_ROUTED && T * L.top > 32 && L.n_expert <= 64 && (size_t)T * L.top * 4 <= 60 * 1024;
 }
 
-// behind the block projection (nvx_a_): queries prepared, keys and values stored, attention, output projection -> nvx_y_.  With several score maps per head
+// behind the block projection (nvx_a_): queries prepared, keys and values stored, attention, output projection (nvx_close_linear).  With several score maps per head
 // every (head, map) pair runs as a query head of its own; launch_gq_maps_out joins the maps in front of the output projection.
 hipError_t Context::nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T) {
     const NovoraxModel &M = *model->nvx;
-    const int W = M.width, G = L.kv_heads, LD_P = L.proj.N, maps = L.maps > 1 ? L.maps : 1;
+    const int G = L.kv_heads, LD_P = L.proj.N, maps = L.maps > 1 ? L.maps : 1;
     const int H = L.heads * maps;                               // query heads as the kernels count them
     float *cache = nvx_cache_[(size_t)r.plane];
     GqPrepArgs pa{};
@@ -174,13 +174,33 @@ hipError_t Context::nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T) 
     pa.norm_per_head = L.qk_norm_per_head ? 1 : 0; pa.v_rot_freq = L.v_rot_freq; pa.v_cs = L.v_rot_freq ? nvx_vcs_ : nullptr;
     pa.q_scale = L.scale; pa.head_scale = L.head_scale; pa.tok_pos = d_pos_; pa.tok_cell = d_cell_;
     pa.maps = maps; pa.rot_neighbours = L.rot_neighbours ? 1 : 0; pa.q_temp_coef = L.q_temp_coef; pa.q_temp_every = L.q_temp_every;
-    pa.q = nvx_q_; pa.ld_q = H * L.dim; pa.cache = cache;
-    FDP_TRY(launch_gq_prep(pa, stream_));
+    pa.q = nvx_q_; pa.ld_q = H * L.dim; pa.cache = cache; pa.v_unit = L.v_unit ? 1 : 0;
+    if (!L.conv_wt) FDP_TRY(launch_gq_prep(pa, stream_));
+    else {
+        // the convolution reaches back over a segment's start into its slot's last inputs: a launch per set of segments that share no slot, and the slots move on
+        // with it (single rows) or behind it
+        const size_t TU = cp.n_ubatch;
+        pa.conv_wt = L.conv_wt; pa.conv_taps = L.conv_taps; pa.conv_state = r.conv_state >= 0 ? nvx_n_[(size_t)r.conv_state] : nullptr;
+        for (const auto &wv : nvx_waves_) {
+            const int *start = h_seg_ + wv.first, *len = h_seg_ + TU + wv.first;
+            const int row0 = start[0], rows = start[wv.second - 1] + len[wv.second - 1] - row0;
+            GqPrepArgs pw = pa;
+            pw.p = pa.p + (size_t)row0 * LD_P; pw.T = rows; pw.q = pa.q + (size_t)row0 * pa.ld_q; pw.tok_pos = d_pos_ + row0; pw.tok_cell = d_cell_ + row0;
+            pw.tok_ago = d_seg_ + 5 * TU + row0; pw.tok_slot = d_seq_ + row0;
+            if (pw.v_cs) pw.v_cs += (size_t)row0 * L.vdim;
+            pw.conv_move = rows == wv.second ? 1 : 0;
+            FDP_TRY(launch_gq_prep(pw, stream_));
+            if (!pw.conv_move && r.conv_state >= 0)
+                FDP_TRY(launch_conv_state(nvx_a_, LD_P, L.conv_channels(), L.conv_taps, nvx_n_[(size_t)r.conv_state], d_seg_ + wv.first, d_seg_ + TU + wv.first,
+                                          d_seg_ + 2 * TU + wv.first, wv.second, stream_));
+        }
+    }
     GqAttnArgs aa{};
     aa.q = nvx_q_; aa.ld_q = H * L.dim; aa.out = maps > 1 ? nvx_o_ : nvx_att_; aa.ld_out = H * L.vdim; aa.T = T; aa.H = H; aa.G = G; aa.dim = L.dim; aa.vdim = L.vdim;
     aa.maps = maps; aa.keep_first = L.keep_first; aa.rel = L.rel; aa.dist_bucket = L.dist_bucket; aa.n_dist = L.n_dist; aa.rel_rows = L.rel_rows;
     aa.cache = cache; aa.cell_pos = d_cell_pos_; aa.cell_seq = d_cell_seq_; aa.tok_pos = d_pos_; aa.tok_seq = d_seq_; aa.n_kv_dev = d_nkv_;
     aa.window = L.window; aa.sink = L.sink; aa.gate = L.off_gate >= 0 && !L.gate_per_entry ? nvx_a_ + L.off_gate : nullptr; aa.ld_gate = LD_P;
+    aa.talk = L.talk;
     aa.softcap = L.softcap; aa.v_cs = L.v_rot_freq ? nvx_vcs_ : nullptr;
     aa.tok_hi = d_seg_ + 3 * (size_t)cp.n_ubatch;
     aa.tok_lo = M.max_window > 0 && L.window > 0 ? d_seg_ + 4 * (size_t)cp.n_ubatch : nullptr;
@@ -191,39 +211,46 @@ hipError_t Context::nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T) 
         FDP_TRY(launch_gq_maps_out(nvx_o_, H * L.vdim, L.gate_per_entry ? nvx_a_ + L.off_gate : nullptr, LD_P, T, L.heads, L.vdim, L.map_lambda, L.map_mult, M.eps,
                                    nvx_att_, L.heads * L.vdim, stream_));
     else if (maps != 1) return hipErrorInvalidValue;
-    FDP_TRY(nvx_linear(L.o, nvx_att_, L.heads * L.vdim, T, nvx_y_, W, MMB_STORE, nullptr, 1.0f, nullptr, L.o_bias));
+    FDP_TRY(nvx_close_linear(L.o, nvx_att_, L.heads * L.vdim, T, L.norm1b, L.o_bias));
     prof_mark("gq_attention");
     return hipSuccess;
 }
 
-// the router's logits -> experts and weights; the routed experts' rows end in nvx_yg_ (row(t, j): nvx_slot_ when grouped).  Experts are relu^2 (e_up alone)
-// or the clamped gated form (e_gate set)
-hipError_t Context::nvx_routed_experts(const NvxLayer &L, const float *h, const float *pn, int T, const float *z, int ld_z) {
+// the router's logits -> experts and weights; the routed experts' rows end in nvx_yg_ (row(t, j): nvx_slot_ when grouped).  Experts are relu^2 (e_up alone),
+// silu-gated or the clamped gated form (e_gate set).  weight_in: the weight multiplies what the expert reads (a factor per row on the first products - they
+// have no bias); a single expert per token then adds into the stream itself (*closed = true)
+hipError_t Context::nvx_routed_experts(const NvxLayer &L, const float *h, const float *pn, int T, const float *z, int ld_z, bool *closed) {
     const NovoraxModel &M = *model->nvx;
     const int W = M.width, k = L.top, NE = L.n_expert, P = T * k;
-    if (L.route_kind == NVX_ROUTE_SIGMOID_BIAS) FDP_TRY(launch_moe_route_sigmoid_bias(z, ld_z, L.route_bias, T, NE, k, L.n_group, L.group_keep, nvx_ids_, nvx_rw_, stream_));
-    else FDP_TRY(launch_moe_route_groups(z, ld_z, T, NE, k, L.n_group, L.group_keep, L.router_scale, nvx_ids_, nvx_rw_, stream_));
+    if (z) {                                                     // (nullptr: nvx_ids_ / nvx_rw_ hold the choice already)
+        if (L.route_kind == NVX_ROUTE_SIGMOID_BIAS) FDP_TRY(launch_moe_route_sigmoid_bias(z, ld_z, L.route_bias, T, NE, k, L.n_group, L.group_keep, nvx_ids_, nvx_rw_, stream_));
+        else FDP_TRY(launch_moe_route_groups(z, ld_z, T, NE, k, L.n_group, L.group_keep, L.router_scale, nvx_ids_, nvx_rw_, stream_));
+    }
+    const bool direct = closed && L.weight_in && k == 1 && !L.norm2b && !M.parallel_block && L.shared_ff == 0;
     MMBArgs u;
     u.w = L.e_up.w; u.ldw = W; u.N = L.ff; u.K = W; u.epi = MMB_RELU2; u.f32 = cp.exact_f32 ? 1 : 0; u.w_zs = (long long)L.ff * W;
-    if (L.e_gate.w) { u.w = L.e_gate.w; u.w2 = L.e_up.w; u.epi = MMB_CLAMP_SWIGLU; u.epi_limit = L.expert_limit; }
+    if (L.e_gate.w) { u.w = L.e_gate.w; u.w2 = L.e_up.w; u.epi = L.ff_silu ? MMB_SILU_MUL : MMB_CLAMP_SWIGLU; u.epi_limit = L.expert_limit; }
     u.y = nvx_ff_; u.ldy = L.ff;
     MMBArgs d;
     d.w = L.e_down.w; d.ldw = L.ff; d.N = W; d.K = L.ff; d.f32 = u.f32; d.w_zs = (long long)W * L.ff;
-    d.x = nvx_ff_; d.ldx = L.ff; d.y = nvx_yg_; d.ldy = W;
+    d.x = nvx_ff_; d.ldx = L.ff; d.y = direct ? x_ : nvx_yg_; d.ldy = W; d.resid = direct ? x_ : nullptr;
     if (nvx_routed_as_groups(L, T)) {
-        // every expert sees its (token, rank) pairs as one batch of rows: counting sort by expert, gather, two grouped products
-        FDP_TRY(launch_moe_group(nvx_ids_, T, k, NE, nvx_meta_, nvx_slot_, nvx_tokof_, stream_));
-        FDP_TRY(launch_gather_rows_f32(h, nvx_tokof_, P, W, nvx_xg_, stream_));
-        u.x = nvx_xg_; u.ldx = W; u.T = P; u.nz = NE; u.meta = nvx_meta_;
+        // every expert sees its (token, rank) pairs as one batch of rows: counting sort by expert, two grouped products (the first reads its rows through the map)
+        FDP_TRY(launch_moe_group(nvx_ids_, T, k, NE, nvx_meta_, nvx_slot_, nvx_tokof_, stream_, L.weight_in ? nvx_rw_ : nullptr, L.weight_in ? nvx_rwg_ : nullptr));
+        u.x = h; u.x_map = nvx_tokof_; u.ldx = W; u.T = P; u.nz = NE; u.meta = nvx_meta_;
         d.T = P; d.nz = NE; d.meta = nvx_meta_;
+        if (L.weight_in) u.row_scale = nvx_rwg_;
+        if (direct) d.y_map = nvx_tokof_;
     } else {
         // a few tokens: one product per (token, rank) pair against the weights the pair picked
         u.x = h; u.ldx = W; u.T = 1; u.nz = P; u.sel = nvx_ids_; u.sel_div = k;
         if (pn) { u.pn_w = pn; u.pn_off = M.norm_off; u.pn_eps = M.eps; }
+        if (L.weight_in) u.row_scale = nvx_rw_;
         d.T = 1; d.nz = P; d.sel = nvx_ids_; d.sel_div = 1;
     }
     FDP_TRY(launch_mmb(u, stream_));
     FDP_TRY(launch_mmb(d, stream_));
+    if (direct) *closed = true;
     prof_mark("routed_experts");
     return hipSuccess;
 }

@@ -1,7 +1,7 @@
 // novorax.cc — the folder models (config.json + model.safetensors): the registry that picks a design's loader by "architecture", the Novorax loader, and what
 // every such design shares inside Context - buffers, cache planes and state slots, segment lists and scan bounds, the layer-run loop, the output head
 // (novorax.h describes the designs, runtime.h the context; the Fidepel loader and its block are in fidepel.cc, the Tuterax loader and the delta-rule mixer
-// in tuterax.cc, the Dinilorn loader, its retention mixer and its feed-forward in dinilorn.cc).
+// in tuterax.cc, the Dinilorn loader, its retention mixer and its feed-forward in dinilorn.cc, the Vuzazen loader in vuzazen.cc).
 //
 // The context's own machinery carries them: the cell table (find / free / sequence masks) addresses the attention layers' cache planes, the micro-batch staging
 // block brings tokens, positions, cells and sequence ids to the device, the sequence id is the slot of the recurrent state, logits / arg-max / top-k leave
@@ -50,6 +50,7 @@ Model *config_model_load(const std::string &dir, int main_gpu, std::string &err,
         {"Fidepel", fidepel_build},
         {"Tuterax", tuterax_build},
         {"Dinilorn", dinilorn_build},
+        {"Vuzazen", vuzazen_build},
     };
     status = -102;
     std::ifstream cf(dir + "/config.json");
@@ -161,15 +162,7 @@ Model *novorax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
             L.uv = ld.rows({{pm + "uv", H * L.vdim}}, L.kv_rank);
             L.o = ld.rows({{pm + "o", W}}, H * L.vdim);
             if (ld.st.find(pm + "sink")) L.sink = ld.vec(pm + "sink", H);
-            if (const SafeTensor *t = ld.need(pm + "uk", "BF16", {(int64_t)H * L.dim, L.kv_rank})) {
-                const unsigned short *s = (const unsigned short *)t->data;
-                std::vector<unsigned short> tr((size_t)H * L.kv_rank * L.dim);
-                for (int h = 0; h < H; h++)
-                    for (int d = 0; d < L.dim; d++)
-                        for (int r = 0; r < L.kv_rank; r++) tr[((size_t)h * L.kv_rank + r) * L.dim + d] = s[((size_t)h * L.dim + d) * L.kv_rank + r];
-                L.uk_t.w = (unsigned short *)ld.dev(tr.data(), tr.size() * 2);
-                L.uk_t.N = L.kv_rank; L.uk_t.K = L.dim;
-            }
+            L.uk_t = ld.head_transposed(pm + "uk", H, L.dim, L.kv_rank);
             M.max_down = std::max(M.max_down, L.q_rank + L.kv_rank + L.rot);
             M.max_q_rank = std::max(M.max_q_rank, L.q_rank);
             M.max_q = std::max(M.max_q, H * QD);
@@ -256,12 +249,14 @@ Model *novorax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
 // floats one sequence slot holds for a recurrent layer run: the state matrices; the second set (mLSTM: normalisers, delta rule: the convolutions' last
 // taps - 1 inputs); the third (mLSTM: running maxima)
 static void nvx_state_sizes(const NvxLayer &L, size_t &s_sz, size_t &n_sz, size_t &m_sz) {
+    if (L.type == NVX_GQ) { s_sz = m_sz = 0; n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.conv_channels(); return; }   // (attention: the convolution's last inputs)
     s_sz = (size_t)L.heads * L.dim * L.vdim;
     if (L.type == NVX_MLSTM) { n_sz = (size_t)L.heads * L.dim; m_sz = (size_t)L.heads; }
     else if (L.type == NVX_RETENTION) { n_sz = 0; m_sz = 0; }
     else { n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.delta_channels(); m_sz = 0; }
 }
 static bool nvx_recurrent(const NvxLayer &L) { return L.type == NVX_MLSTM || L.type == NVX_DELTA || L.type == NVX_RETENTION; }
+static int nvx_state_set(const NvxLayer &L, const NvxRun &r) { return nvx_recurrent(L) ? r.plane : r.conv_state; }   // index of a run's state set, -1: none
 
 bool Context::init_novorax(std::string &err) {
     const NovoraxModel &M = *model->nvx;
@@ -279,8 +274,8 @@ bool Context::init_novorax(std::string &err) {
     d_tok_ = (int32_t *)(d_stage_ + 16);
     d_pos_ = d_tok_ + Tp; d_seq_ = d_pos_ + Tp; d_cell_ = d_seq_ + Tp; d_outrow_ = d_cell_ + Tp;
     d_seqmask_ = (uint64_t *)(d_outrow_ + Tp);
-    d_seg_ = (int32_t *)dalloc(5 * T * 4);
-    if (!d_seg_ || hipHostMalloc((void **)&h_seg_, 5 * T * 4, hipHostMallocDefault) != hipSuccess) { err = "segment list allocation failed"; return false; }
+    d_seg_ = (int32_t *)dalloc(7 * T * 4);
+    if (!d_seg_ || hipHostMalloc((void **)&h_seg_, 7 * T * 4, hipHostMallocDefault) != hipSuccess) { err = "segment list allocation failed"; return false; }
 
     // cache planes and recurrent state
     nvx_cache_.assign((size_t)M.n_cache_runs, nullptr);
@@ -290,16 +285,18 @@ bool Context::init_novorax(std::string &err) {
         if (!nvx_recurrent(L)) {
             nvx_cache_[(size_t)r.plane] = (float *)dalloc(NC * (size_t)L.cache_row() * 4);
             if (!nvx_cache_[(size_t)r.plane]) { err = "attention cache allocation failed"; return false; }
-        } else {
+        }
+        if (const int st = nvx_state_set(L, r); st >= 0) {
             size_t s_sz, n_sz, m_sz;
             nvx_state_sizes(L, s_sz, n_sz, m_sz);
-            nvx_S_[(size_t)r.plane] = (float *)dalloc(NS * s_sz * 4);
-            nvx_n_[(size_t)r.plane] = (float *)dalloc(std::max<size_t>(NS * n_sz, 1) * 4);
-            nvx_m_[(size_t)r.plane] = (float *)dalloc(std::max<size_t>(NS * m_sz, 1) * 4);
-            if (!nvx_S_[(size_t)r.plane] || !nvx_n_[(size_t)r.plane] || !nvx_m_[(size_t)r.plane]) { err = "recurrent state allocation failed"; return false; }
+            nvx_S_[(size_t)st] = (float *)dalloc(std::max<size_t>(NS * s_sz, 1) * 4);
+            nvx_n_[(size_t)st] = (float *)dalloc(std::max<size_t>(NS * n_sz, 1) * 4);
+            nvx_m_[(size_t)st] = (float *)dalloc(std::max<size_t>(NS * m_sz, 1) * 4);
+            if (!nvx_S_[(size_t)st] || !nvx_n_[(size_t)st] || !nvx_m_[(size_t)st]) { err = "recurrent state allocation failed"; return false; }
         }
     }
     nvx_seq_len_.assign(NS, 0);
+    nvx_prev_tok_.assign(NS, -1);
     // activations
     const size_t A = (size_t)std::max(M.max_down, M.max_proj), TOP = (size_t)std::max(M.max_top, 1);
     x_ = (float *)dalloc(T * W * 4);
@@ -323,6 +320,8 @@ bool Context::init_novorax(std::string &err) {
         // grouped-query layers also cut the block chains of short prompt batches: records for up to 1024 rows x 4 runs of the widest layer
         for (const NvxLayer &L : M.layers)
             if (L.type == NVX_GQ) nvx_part_floats_ = std::max(nvx_part_floats_, std::min<size_t>(T, 1024) * (size_t)L.heads * (size_t)std::max(L.maps, 1) * 4 * (size_t)(L.vdim + 2));
+        for (const NvxLayer &L : M.layers)
+            if (L.talk) nvx_part_floats_ = std::max(nvx_part_floats_, std::max<size_t>(TALK_ROW_RUNS, std::min<size_t>(T, 1024) * TALK_TILE_RUNS) * (size_t)L.heads * (size_t)(L.vdim + 2));
         nvx_part_ = (float *)dalloc(nvx_part_floats_ * 4);
     }
     {
@@ -339,7 +338,8 @@ bool Context::init_novorax(std::string &err) {
         nvx_slot_ = (int32_t *)dalloc(T * TOP * 4);
         nvx_tokof_ = (int32_t *)dalloc(T * TOP * 4);
         nvx_rw_ = (float *)dalloc(T * TOP * 4);
-        if (!nvx_xg_ || !nvx_yg_ || !nvx_ids_ || !nvx_meta_ || !nvx_slot_ || !nvx_tokof_ || !nvx_rw_) { err = "expert batch buffers allocation failed"; return false; }
+        nvx_rwg_ = (float *)dalloc(T * TOP * 4);
+        if (!nvx_xg_ || !nvx_yg_ || !nvx_ids_ || !nvx_meta_ || !nvx_slot_ || !nvx_tokof_ || !nvx_rw_ || !nvx_rwg_) { err = "expert batch buffers allocation failed"; return false; }
     }
     if (M.max_shared_ff > 0) {
         nvx_sh_ = (float *)dalloc(T * (size_t)M.max_shared_ff * 4);
@@ -372,16 +372,17 @@ void Context::nvx_state_reset(int seq) {
     const size_t NS = cp.n_seq_max;
     for (const NvxRun &r : M.runs) {
         const NvxLayer &L = M.layers[(size_t)r.layer];
-        if (!nvx_recurrent(L)) continue;
+        const int st = nvx_state_set(L, r);
+        if (st < 0) continue;
         size_t s_sz, n_sz, m_sz;
         nvx_state_sizes(L, s_sz, n_sz, m_sz);
         const size_t first = seq < 0 ? 0 : (size_t)seq, cnt = seq < 0 ? NS : 1;
         if (first >= NS) continue;
-        (void)launch_mlstm_state_reset(nvx_S_[(size_t)r.plane] + first * s_sz, cnt * s_sz, nvx_n_[(size_t)r.plane] + first * n_sz, cnt * n_sz,
-                                       nvx_m_[(size_t)r.plane] + first * m_sz, cnt * m_sz, stream_);
+        (void)launch_mlstm_state_reset(nvx_S_[(size_t)st] + first * s_sz, cnt * s_sz, nvx_n_[(size_t)st] + first * n_sz, cnt * n_sz,
+                                       nvx_m_[(size_t)st] + first * m_sz, cnt * m_sz, stream_);
     }
-    if (seq < 0) std::fill(nvx_seq_len_.begin(), nvx_seq_len_.end(), 0);
-    else if ((size_t)seq < nvx_seq_len_.size()) nvx_seq_len_[(size_t)seq] = 0;
+    if (seq < 0) { std::fill(nvx_seq_len_.begin(), nvx_seq_len_.end(), 0); std::fill(nvx_prev_tok_.begin(), nvx_prev_tok_.end(), -1); }
+    else if ((size_t)seq < nvx_seq_len_.size()) { nvx_seq_len_[(size_t)seq] = 0; nvx_prev_tok_[(size_t)seq] = -1; }
 }
 
 void Context::nvx_state_copy(int src, int dst) {
@@ -390,17 +391,19 @@ void Context::nvx_state_copy(int src, int dst) {
     if (src < 0 || dst < 0 || (size_t)src >= NS || (size_t)dst >= NS || src == dst) return;
     for (const NvxRun &r : M.runs) {
         const NvxLayer &L = M.layers[(size_t)r.layer];
-        if (!nvx_recurrent(L)) continue;
+        const int st = nvx_state_set(L, r);
+        if (st < 0) continue;
         size_t s_sz, n_sz, m_sz;
         nvx_state_sizes(L, s_sz, n_sz, m_sz);
-        (void)hipMemcpyAsync(nvx_S_[(size_t)r.plane] + dst * s_sz, nvx_S_[(size_t)r.plane] + src * s_sz, s_sz * 4, hipMemcpyDeviceToDevice, stream_);
-        if (n_sz) (void)hipMemcpyAsync(nvx_n_[(size_t)r.plane] + dst * n_sz, nvx_n_[(size_t)r.plane] + src * n_sz, n_sz * 4, hipMemcpyDeviceToDevice, stream_);
-        if (m_sz) (void)hipMemcpyAsync(nvx_m_[(size_t)r.plane] + dst * m_sz, nvx_m_[(size_t)r.plane] + src * m_sz, m_sz * 4, hipMemcpyDeviceToDevice, stream_);
+        if (s_sz) (void)hipMemcpyAsync(nvx_S_[(size_t)st] + dst * s_sz, nvx_S_[(size_t)st] + src * s_sz, s_sz * 4, hipMemcpyDeviceToDevice, stream_);
+        if (n_sz) (void)hipMemcpyAsync(nvx_n_[(size_t)st] + dst * n_sz, nvx_n_[(size_t)st] + src * n_sz, n_sz * 4, hipMemcpyDeviceToDevice, stream_);
+        if (m_sz) (void)hipMemcpyAsync(nvx_m_[(size_t)st] + dst * m_sz, nvx_m_[(size_t)st] + src * m_sz, m_sz * 4, hipMemcpyDeviceToDevice, stream_);
     }
     nvx_seq_len_[(size_t)dst] = nvx_seq_len_[(size_t)src];
+    nvx_prev_tok_[(size_t)dst] = nvx_prev_tok_[(size_t)src];
 }
 
-bool Context::nvx_stage_segments(int n, const int32_t *seq, const int32_t *pos, const int *tcell) {
+bool Context::nvx_stage_segments(int n, const int32_t *tokens, const int32_t *seq, const int32_t *pos, const int *tcell) {
     const size_t T = cp.n_ubatch;
     {
         // per token: one past the highest cell its attention can need - the sequence's cells from earlier batches, and this batch's own cells up to the token
@@ -435,12 +438,20 @@ bool Context::nvx_stage_segments(int n, const int32_t *seq, const int32_t *pos, 
             hi[i] = base[s];
         }
     }
-    int32_t *start = h_seg_, *len = h_seg_ + T, *slot = h_seg_ + 2 * T;
+    int32_t *start = h_seg_, *len = h_seg_ + T, *slot = h_seg_ + 2 * T, *ago = h_seg_ + 5 * T, *bigram = h_seg_ + 6 * T;
     int ns = 0;
     for (int i = 0; i < n; i++) {
         if (seq[i] < 0 || seq[i] >= (int)cp.n_seq_max) { last_error = "sequence id " + std::to_string(seq[i]) + " has no state slot (n_seq_max " + std::to_string(cp.n_seq_max) + ")"; return false; }
         if (ns > 0 && slot[ns - 1] == seq[i]) len[ns - 1]++;
         else { start[ns] = i; len[ns] = 1; slot[ns] = seq[i]; ns++; }
+        ago[i] = len[ns - 1] - 1;
+        // the row of the bigram table: by the sequence's previous token - of this batch or an earlier one - and this one
+        int32_t &prev = nvx_prev_tok_[(size_t)seq[i]];
+        const NovoraxModel &M = *model->nvx;
+        if (M.bigram.w && tokens) {
+            bigram[i] = prev < 0 ? M.bigram_buckets : (int32_t)(((int64_t)prev * M.bigram_mul_prev + (int64_t)tokens[i] * M.bigram_mul_cur) % M.bigram_buckets);
+            prev = tokens[i];
+        } else bigram[i] = 0;
     }
     // segments of one launch must not share a slot: cut the list where a sequence comes back
     nvx_waves_.clear();
@@ -452,12 +463,12 @@ bool Context::nvx_stage_segments(int n, const int32_t *seq, const int32_t *pos, 
         seen |= bit;
     }
     if (ns > first) nvx_waves_.push_back({first, ns - first});
-    return hipMemcpyAsync(d_seg_, h_seg_, 5 * T * 4, hipMemcpyHostToDevice, stream_) == hipSuccess;
+    return hipMemcpyAsync(d_seg_, h_seg_, 7 * T * 4, hipMemcpyHostToDevice, stream_) == hipSuccess;
 }
 
 // pn != nullptr: the rows of x are RMS-normed with weight (norm_off + pn) on the way in (few rows: inside the launch; batches: a norm launch into xn_ first)
 hipError_t Context::nvx_linear(const BfMat &w, const float *x, int ldx, int T, float *y, int ldy, int epi, const BfMat *w2, float out_scale, const float *pn,
-                               const float *bias, float epi_limit) {
+                               const float *bias, float epi_limit, const float *resid) {
     MMBArgs a;
     if (pn && T > MMB_VEC_ROWS) {
         NVX_TRY(launch_rmsnorm_f32(x, ldx, pn, model->nvx->norm_off, nullptr, xn_, w.K, w.K, T, model->nvx->eps, stream_));
@@ -466,7 +477,14 @@ hipError_t Context::nvx_linear(const BfMat &w, const float *x, int ldx, int T, f
     a.pn_w = pn; a.pn_off = model->nvx->norm_off; a.pn_eps = model->nvx->eps;
     a.x = x; a.ldx = ldx; a.w = w.w; a.w2 = w2 ? w2->w : nullptr; a.ldw = w.K; a.y = y; a.ldy = ldy;
     a.T = T; a.N = w.N; a.K = w.K; a.epi = epi; a.f32 = cp.exact_f32 ? 1 : 0; a.out_scale = out_scale; a.bias = bias; a.epi_limit = epi_limit;
+    a.resid = resid;
     return launch_mmb(a, stream_);
+}
+
+hipError_t Context::nvx_close_linear(const BfMat &w, const float *x, int ldx, int T, const float *norm_behind, const float *bias) {
+    const int W = model->nvx->width;
+    if (norm_behind || model->nvx->parallel_block) return nvx_linear(w, x, ldx, T, nvx_y_, W, MMB_STORE, nullptr, 1.0f, nullptr, bias);
+    return nvx_linear(w, x, ldx, T, x_, W, MMB_STORE, nullptr, 1.0f, nullptr, bias, 0.0f, x_);
 }
 
 hipError_t Context::nvx_feed_forward(const NvxLayer &L, int T, bool *closed) {
@@ -474,10 +492,10 @@ hipError_t Context::nvx_feed_forward(const NvxLayer &L, int T, bool *closed) {
     const int W = M.width;
     if (L.ff_kind == NVX_FF_ROUTED) return nvx_routed_feed_forward(L, T, closed);
     if (L.ff_kind == NVX_FF_DENSE) {
-        if (L.gate.w) NVX_TRY(nvx_linear(L.gate, x_, W, T, nvx_ff_, L.ff, MMB_GELU_MUL, &L.up, 1.0f, L.norm2));
+        if (L.gate.w) NVX_TRY(nvx_linear(L.gate, x_, W, T, nvx_ff_, L.ff, L.ff_silu ? MMB_SILU_MUL : MMB_GELU_MUL, &L.up, 1.0f, L.norm2));
         else NVX_TRY(nvx_linear(L.up, x_, W, T, nvx_ff_, L.ff, MMB_RELU2, nullptr, 1.0f, L.norm2));
-        NVX_TRY(nvx_linear(L.down_ff, nvx_ff_, L.ff, T, nvx_y_, W));
-        return hipSuccess;
+        if (closed && !L.norm2b) *closed = true;                 // (nothing behind the feed-forward: its last product adds into the stream)
+        return nvx_close_linear(L.down_ff, nvx_ff_, L.ff, T, L.norm2b);
     }
     const int k = L.top, NE = L.n_expert, P = T * k;
     NVX_TRY(launch_moe_table_ids(L.table, d_tok_, T, k, nvx_ids_, stream_));
@@ -491,10 +509,9 @@ hipError_t Context::nvx_feed_forward(const NvxLayer &L, int T, bool *closed) {
     const bool fuse_norm = !grouped && T <= MMB_VEC_ROWS;         // the pair products norm their row themselves
     if (!fuse_norm) NVX_TRY(launch_rmsnorm_f32(x_, W, L.norm2, 1.0f, nullptr, xn_, W, W, T, M.eps, stream_));
     if (grouped) {
-        // every expert sees its (token, rank) pairs as one batch of rows: counting sort by expert, gather, two grouped products, combine per token
+        // every expert sees its (token, rank) pairs as one batch of rows: counting sort by expert, two grouped products (the first reads its rows through the map), combine per token
         NVX_TRY(launch_moe_group(nvx_ids_, T, k, NE, nvx_meta_, nvx_slot_, nvx_tokof_, stream_));
-        NVX_TRY(launch_gather_rows_f32(xn_, nvx_tokof_, P, W, nvx_xg_, stream_));
-        g.x = nvx_xg_; g.ldx = W; g.T = P; g.nz = NE; g.meta = nvx_meta_;
+        g.x = xn_; g.x_map = nvx_tokof_; g.ldx = W; g.T = P; g.nz = NE; g.meta = nvx_meta_;
         d.T = P; d.nz = NE; d.meta = nvx_meta_;
         NVX_TRY(launch_mmb(g, stream_));
         NVX_TRY(launch_mmb(d, stream_));
@@ -517,7 +534,9 @@ hipError_t Context::run_layers_novorax(int T) {
     const float eps = M.eps;
     cur_T_ = T;
     NVX_TRY(launch_kv_meta_set(d_cell_pos_, d_cell_seq_, d_cell_, d_pos_, d_seqmask_, T, stream_));
-    NVX_TRY(launch_get_rows(T_BF16, (const uint8_t *)M.embed.w, W, d_tok_, T, x_, stream_, M.embed_scale));
+    if (M.bigram.w)
+        NVX_TRY(launch_get_rows_pair(T_BF16, (const uint8_t *)M.embed.w, (const uint8_t *)M.bigram.w, W, d_tok_, d_seg_ + 6 * (size_t)cp.n_ubatch, T, x_, stream_, M.embed_scale));
+    else NVX_TRY(launch_get_rows(T_BF16, (const uint8_t *)M.embed.w, W, d_tok_, T, x_, stream_, M.embed_scale));
     if (M.loop_add_embed) NVX_TRY(hipMemcpyAsync(nvx_x0_, x_, (size_t)T * W * 4, hipMemcpyDeviceToDevice, stream_));
     if (M.loop_in.w) NVX_TRY(hipMemcpy2DAsync(nvx_xcat_ + W, (size_t)2 * W * 4, x_, (size_t)W * 4, (size_t)W * 4, (size_t)T, hipMemcpyDeviceToDevice, stream_));
     prof_mark("embed");
@@ -539,12 +558,12 @@ hipError_t Context::run_layers_novorax(int T) {
             continue;
         }
         if (L.type == NVX_LATENT) {
-            const int QD = L.dim + L.rot, KR = L.kv_rank, LD_A = L.q_rank + KR + L.rot;
+            const int QD = L.dim + L.rot, KR = L.kv_rank, LD_A = L.down.N;
             float *cache = nvx_cache_[(size_t)r.plane];
             NVX_TRY(nvx_linear(L.down, x_, W, T, nvx_a_, LD_A, MMB_STORE, nullptr, 1.0f, L.norm1));
             LatentPrepArgs pa{};
             pa.a = nvx_a_; pa.ld_a = LD_A; pa.T = T; pa.q_rank = L.q_rank; pa.kv_rank = KR; pa.rot = L.rot; pa.rot_dims = L.rot_dims;
-            pa.wq_norm = L.dq_norm; pa.wkv_norm = L.dkv_norm; pa.eps = eps; pa.rot_freq = L.rot_freq; pa.rot_mscale = L.rot_mscale;
+            pa.wq_norm = L.dq_norm; pa.wkv_norm = L.dkv_norm; pa.eps = eps; pa.rot_freq = L.rot_freq; pa.rot_mscale = L.rot_mscale; pa.rot_halves = L.rot_halves ? 1 : 0;
             pa.tok_pos = d_pos_; pa.tok_cell = d_cell_; pa.cq = nvx_cq_; pa.cache = cache;
             NVX_TRY(launch_latent_prep(pa, stream_));
             NVX_TRY(nvx_linear(L.uq, nvx_cq_, L.q_rank, T, nvx_q_, H * QD));
@@ -556,7 +575,8 @@ hipError_t Context::run_layers_novorax(int T) {
             aa.qa = nvx_qa_; aa.ld_qa = H * KR; aa.q = nvx_q_; aa.ld_q = H * QD; aa.out = nvx_lat_; aa.ld_out = H * KR;
             aa.T = T; aa.H = H; aa.dim = L.dim; aa.rot = L.rot; aa.kv_rank = KR; aa.rot_dims = L.rot_dims; aa.cache = cache;
             aa.cell_pos = d_cell_pos_; aa.cell_seq = d_cell_seq_; aa.tok_pos = d_pos_; aa.tok_seq = d_seq_; aa.n_kv_dev = d_nkv_;
-            aa.window = L.window; aa.scale = L.scale; aa.sink = L.sink; aa.rot_freq = L.rot_freq; aa.rot_mscale = L.rot_mscale;
+            aa.window = L.window; aa.scale = L.scale; aa.sink = L.sink; aa.rot_freq = L.rot_freq; aa.rot_mscale = L.rot_mscale; aa.rot_halves = L.rot_halves ? 1 : 0;
+            aa.gate = L.off_gate >= 0 ? nvx_a_ + L.off_gate : nullptr; aa.ld_gate = LD_A;
             aa.tok_hi = d_seg_ + 3 * (size_t)cp.n_ubatch;
             if (nvx_part_ && (long long)T * H <= LATENT_ATTN_SPLIT_MAX_PAIRS) { aa.part = nvx_part_; aa.splits = LATENT_ATTN_SPLITS; }
             NVX_TRY(launch_latent_attn(aa, stream_));
@@ -564,7 +584,7 @@ hipError_t Context::run_layers_novorax(int T) {
             ua.x = nvx_lat_; ua.ldx = H * KR; ua.x_zs = KR; ua.w = L.uv.w; ua.ldw = KR; ua.w_zs = (long long)L.vdim * KR;
             ua.y = nvx_att_; ua.ldy = H * L.vdim; ua.y_zs = L.vdim; ua.T = T; ua.N = L.vdim; ua.K = KR; ua.nz = H; ua.f32 = fa.f32;
             NVX_TRY(launch_mmb(ua, stream_));
-            NVX_TRY(nvx_linear(L.o, nvx_att_, H * L.vdim, T, nvx_y_, W));
+            NVX_TRY(nvx_close_linear(L.o, nvx_att_, H * L.vdim, T, L.norm1b));
             prof_mark("latent_attention");
         } else if (L.type == NVX_MLSTM) {
             const int LD_P = L.proj.N;
@@ -579,7 +599,7 @@ hipError_t Context::run_layers_novorax(int T) {
                 NVX_TRY(launch_mlstm_scan(ma, stream_));
             }
             NVX_TRY(launch_mlstm_out(nvx_o_, H * L.vdim, nvx_a_, LD_P, 2 * H * L.dim + H * L.vdim, L.mix_norm, T, H, L.vdim, eps, nvx_att_, H * L.vdim, stream_));
-            NVX_TRY(nvx_linear(L.o, nvx_att_, H * L.vdim, T, nvx_y_, W));
+            NVX_TRY(nvx_close_linear(L.o, nvx_att_, H * L.vdim, T, L.norm1b));
             prof_mark("mlstm");
         } else if (L.type == NVX_GQ) {
             NVX_TRY(nvx_linear(L.proj, x_, W, T, nvx_a_, L.proj.N, MMB_STORE, nullptr, 1.0f, L.norm1, L.proj_bias));
@@ -589,8 +609,9 @@ hipError_t Context::run_layers_novorax(int T) {
         } else if (L.type == NVX_RETENTION) {
             NVX_TRY(nvx_retention_mixer(L, r, T));
         } else return hipErrorInvalidValue;
-        // norm on the sublayer's output, added to the stream (norm1 / norm2 in front of a sublayer are nullptr in a design whose sublayers read the stream itself)
-        NVX_TRY(launch_rmsnorm_f32(nvx_y_, W, L.norm1b, 1.0f, x_, x_, W, W, T, eps, stream_));
+        // norm on the sublayer's output, added to the stream (norm1 / norm2 in front of a sublayer are nullptr in a design whose sublayers read the stream itself; norm1b / norm2b
+        // behind it in a design without them - its last product has added into the stream already)
+        if (L.norm1b) NVX_TRY(launch_rmsnorm_f32(nvx_y_, W, L.norm1b, 1.0f, x_, x_, W, W, T, eps, stream_));
         if (L.ff_kind != NVX_FF_NONE) {
             bool closed = false;
             NVX_TRY(nvx_feed_forward(L, T, &closed));

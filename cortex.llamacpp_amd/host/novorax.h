@@ -1,4 +1,4 @@
-// novorax.h — the layer stack of the folder models (config.json + model.safetensors, bf16 weights) as this runtime holds it.  Four designs fill it.
+// novorax.h — the layer stack of the folder models (config.json + model.safetensors, bf16 weights) as this runtime holds it.  Five designs fill it.
 //
 // Novorax: a decoder whose layers each pick a token mixer (latent attention with a sliding window and a
 // softmax sink, or the mLSTM matrix-memory recurrence) and a feed-forward (dense relu^2, or experts chosen by a token-id table), norms on both sides of every
@@ -29,6 +29,12 @@
 // experts g sigmoid(1.702 g) (u + 1) with clamped g, u; router = sigmoid scores, a selection bias that picks but does not weigh, expert groups scored by their two
 // best, un-normalised weights; a shared expert behind a one-number sigmoid gate.  A span of layers may run several times with shared weights; every pass but
 // the first opens with the embedding rows added to the stream.
+//
+// Vuzazen: norms in front of the sublayers only (x += mixer(norm(x)), x += ff(norm(x)), zero-centred weights).  The embedding row enters times a constant, plus a
+// row of a second table picked by the token and the one before it; the embedding table is the output head.  Mixers: the mLSTM; latent attention (every
+// earlier token, halves turning, a sigmoid gate per head); grouped-query attention without positions: short causal convolutions on q / k / v, whole-projection
+// q / k norms, unit values, scores mixed across the heads before the softmax, a sigmoid gate per head.  Feed-forward: silu-gated, dense or experts picked by
+// their sigmoid scores, the score multiplying what the expert reads.
 #pragma once
 
 #include <cstdint>
@@ -105,6 +111,15 @@ struct NvxLayer {
     float *rel = nullptr; int32_t *dist_bucket = nullptr; int n_dist = 0, rel_rows = 0;
     int keep_first = 0, maps = 1;
     bool rot_neighbours = false, gate_per_entry = false;
+    // ... and: a short causal convolution on every q / k / v channel (conv_wt [conv_taps][channels] f32, channels in proj's order; conv_taps above), unit value
+    // heads, scores mixed across the heads (talk [heads][heads] f32)
+    float *conv_wt = nullptr, *talk = nullptr;
+    bool v_unit = false;
+    int conv_channels() const { return heads * maps * dim + kv_heads * maps * dim + kv_heads * vdim; }
+    // latent attention: entry i of the turning part pairs with entry i + half instead of its neighbour; the gate rows of `down` start at off_gate (-1: no gate)
+    bool rot_halves = false;
+    // gated feed-forwards (dense, routed): silu; routed: the router's weight multiplies the expert's input instead of its output
+    bool ff_silu = false, weight_in = false;
     float map_lambda = 0.0f, map_mult = 1.0f;
     // retention: proj = [q: heads*dim ; k: heads*dim ; v: heads*vdim ; g: heads*vdim] rows (off_g: the gate's column), decay [heads]; rot_dims / rot_freq as above
     float *decay = nullptr;
@@ -115,6 +130,7 @@ struct NvxRun {
     int layer = 0;
     int pass = -1;                  // >= 0: first layer of loop pass `pass` (input projection + step vector come first)
     int plane = -1;                 // attention mixers: index of this run's cache plane; recurrent mixers: of its state set
+    int conv_state = -1;            // attention mixers with a convolution of several taps: index of the state set that keeps its last inputs
 };
 
 struct NovoraxModel {
@@ -124,7 +140,13 @@ struct NovoraxModel {
     float *loop_step = nullptr;     // [times][width]
     float *final_norm = nullptr;
     float logit_scale = 1.0f, eps = 1e-5f, embed_scale = 1.0f;
-    std::string design;             // "novorax" | "fidepel" | "tuterax" | "dinilorn"
+    // a second table joins the embedding rows: row (previous token * mul_prev + token * mul_cur) mod buckets, the last row for a sequence's first token
+    BfMat bigram;
+    int bigram_buckets = 0;
+    int64_t bigram_mul_prev = 0, bigram_mul_cur = 0;
+    // what a sequence keeps beside its cache cells: recurrent state, convolution inputs, the previous token - it cannot be cut back to an earlier position
+    bool has_sequence_state() const { return n_state_runs > 0 || bigram.w != nullptr; }
+    std::string design;             // "novorax" | "fidepel" | "tuterax" | "dinilorn" | "vuzazen"
     bool loop_add_embed = false;    // every pass of the looped span but the first opens with x += embedding rows
     int max_keep_first = 0;         // most first positions a windowed layer keeps seen (scan bounds)
     // norm weights: the factor is norm_off + w (1: zero-centred weights, 0: plain ones).  parallel_block: one norm per layer, mixer and feed-forward both read

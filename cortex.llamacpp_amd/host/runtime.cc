@@ -743,7 +743,7 @@ bool Context::kv_seq_rm(int seq, int p0, int p1) {
     if (seq >= 64) return false;                                   // (the cell masks are 64 bits wide)
     if (p0 < 0) p0 = 0;
     if (p1 < 0) p1 = 0x7fffffff;
-    if (model->nvx && model->nvx->n_state_runs > 0) {
+    if (model->nvx && model->nvx->has_sequence_state()) {
         // a recurrent state cannot be cut back to an earlier position: a sequence goes as a whole (its state slot starts over), or not at all
         for (int sq = 0; sq < (int)nvx_seq_len_.size(); sq++) {
             if (seq >= 0 && sq != seq) continue;
@@ -1937,7 +1937,7 @@ int Context::decode_ubatch(int n, const int32_t *tokens, const int32_t *pos, con
     static const bool profiler_safe = getenv("MI355_PROFILER_SAFE") && getenv("MI355_PROFILER_SAFE")[0] == '1';
     if (profiler_safe) (void)hipStreamSynchronize(stream_);
     if (model->nvx) {
-        if (!nvx_stage_segments(n, seq, pos, tcell.data())) { if (last_error.empty()) last_error = "segment list upload failed"; return -1; }
+        if (!nvx_stage_segments(n, tokens, seq, pos, tcell.data())) { if (last_error.empty()) last_error = "segment list upload failed"; return -1; }
         for (int i = 0; i < n; i++) nvx_seq_len_[(size_t)seq[i]] = std::max<uint64_t>(nvx_seq_len_[(size_t)seq[i]], (uint64_t)pos[i] + 1);
     }
     if (!stage_event_) (void)hipEventCreateWithFlags(&stage_event_, hipEventDisableTiming);

@@ -74,7 +74,7 @@ struct Model {
     DevTensor tok_embd, out_norm, output, rope_freqs;
     DevTensor tok_types, tok_norm, tok_norm_b;       // encoder files: token-type table (row 0 is added to every token), LayerNorm of the embeddings
     std::vector<LayerWeights> layers;
-    std::unique_ptr<NovoraxModel> nvx;  // a folder model (config.json + model.safetensors; architectures Novorax, Fidepel): its own layer stack, see novorax.h
+    std::unique_ptr<NovoraxModel> nvx;  // a folder model (config.json + model.safetensors; architectures Novorax, Fidepel, Tuterax, Dinilorn, Vuzazen): its own layer stack, see novorax.h
     uint64_t device_bytes = 0, host_bytes = 0, file_tensor_bytes = 0, bytes_per_token = 0, planes_bytes = 0;
     ~Model();
 };
@@ -182,7 +182,9 @@ class Context {
     hipError_t run_layers_novorax(int T);
     hipError_t run_output_novorax(int n_out, int out_base);
     hipError_t nvx_linear(const BfMat &w, const float *x, int ldx, int T, float *y, int ldy, int epi = MMB_STORE, const BfMat *w2 = nullptr, float out_scale = 1.0f,
-                          const float *pn = nullptr, const float *bias = nullptr, float epi_limit = 0.0f);
+                          const float *pn = nullptr, const float *bias = nullptr, float epi_limit = 0.0f, const float *resid = nullptr);
+    // the last product of a sublayer: -> nvx_y_ for the norm behind it (norm_behind set) or a block's closing sum, else added into the stream x_
+    hipError_t nvx_close_linear(const BfMat &w, const float *x, int ldx, int T, const float *norm_behind, const float *bias = nullptr);
     // -> nvx_y_; *closed = true (closed given): the norm behind the feed-forward and the residual add were part of its last launch, x_ is already updated
     hipError_t nvx_feed_forward(const NvxLayer &L, int T, bool *closed = nullptr);
     // dinilorn.cc: norm, [router ; shared gate] projection, routed experts beside the shared expert (side stream), weighted sum + closing norm + residual add
@@ -192,20 +194,21 @@ class Context {
     hipError_t nvx_parallel_block(const NvxLayer &L, const NvxRun &r, int T);
     hipError_t nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T);
     hipError_t nvx_delta_mixer(const NvxLayer &L, const NvxRun &r, int T);   // tuterax.cc: projections, convolution, recurrence, gated unit-RMS output, W_o -> nvx_y_
-    hipError_t nvx_routed_experts(const NvxLayer &L, const float *h, const float *pn, int T, const float *z, int ld_z);   // z: the router's logits [T][n_expert], row stride ld_z
+    hipError_t nvx_routed_experts(const NvxLayer &L, const float *h, const float *pn, int T, const float *z, int ld_z, bool *closed = nullptr);   // z: the router's logits [T][n_expert], row stride ld_z; closed: see nvx_feed_forward
     hipError_t nvx_shared_expert(const NvxLayer &L, const float *h, const float *pn, int T);
     float *nvx_sh_ = nullptr, *nvx_ys_ = nullptr, *nvx_rw_ = nullptr;   // shared expert's hidden rows and output; router weights [T][top]
+    float *nvx_rwg_ = nullptr;                              // the same in grouped row order
     // the three readers of a one-norm block's projection - attention, routed experts, shared expert - are independent until the block's closing sum: the two
     // feed-forward branches run on side streams forked behind the projection and joined in front of the sum (eagerly and inside the captured step alike)
     hipStream_t nvx_side_[2] = {nullptr, nullptr};
     hipEvent_t nvx_fork_ev_ = nullptr, nvx_join_ev_[2] = {nullptr, nullptr};
     bool nvx_fork_ok_ = false;
     // runs of consecutive tokens of one sequence -> segment arrays; per-token scan bounds of the attention (pinned, then device)
-    bool nvx_stage_segments(int n, const int32_t *seq, const int32_t *pos, const int *tcell);
+    bool nvx_stage_segments(int n, const int32_t *tokens, const int32_t *seq, const int32_t *pos, const int *tcell);
     void nvx_state_reset(int seq);                          // seq < 0: every slot
     void nvx_state_copy(int src, int dst);
     std::vector<float *> nvx_cache_;                        // [attention run] [n_ctx][the layer's cache_row()]
-    std::vector<float *> nvx_S_, nvx_n_, nvx_m_;            // [recurrent run] [n_seq_max][H][D][VD]; mlstm: [..][H][D], [..][H]; delta rule: [..][taps - 1][channels] in nvx_n_
+    std::vector<float *> nvx_S_, nvx_n_, nvx_m_;            // [recurrent run] [n_seq_max][H][D][VD]; mlstm: [..][H][D], [..][H]; delta rule and attention with a convolution: [..][taps - 1][channels] in nvx_n_
     std::vector<uint64_t> nvx_seq_len_;                     // tokens every sequence id has been fed (the recurrent state cannot be cut back)
     float *nvx_x0_ = nullptr, *nvx_xcat_ = nullptr, *nvx_y_ = nullptr, *nvx_a_ = nullptr, *nvx_cq_ = nullptr, *nvx_q_ = nullptr, *nvx_qa_ = nullptr, *nvx_lat_ = nullptr;
     float *nvx_vcs_ = nullptr;                              // [n_ubatch][widest turned value head]: cos | sin per pair of every token's value turn
@@ -213,7 +216,9 @@ class Context {
     size_t nvx_part_floats_ = 0;
     float *nvx_att_ = nullptr, *nvx_o_ = nullptr, *nvx_ff_ = nullptr, *nvx_xg_ = nullptr, *nvx_yg_ = nullptr;
     int32_t *nvx_ids_ = nullptr, *nvx_meta_ = nullptr, *nvx_slot_ = nullptr, *nvx_tokof_ = nullptr;
-    int32_t *h_seg_ = nullptr, *d_seg_ = nullptr;           // [5][n_ubatch]: start, length, slot of every segment; upper and lower scan bound of every token
+    // [7][n_ubatch]: start, length, slot of every segment; upper and lower scan bound of every token; rows of its segment in front of every token; its row of the bigram table
+    int32_t *h_seg_ = nullptr, *d_seg_ = nullptr;
+    std::vector<int32_t> nvx_prev_tok_;                     // last token every sequence id has been fed (-1: none)
     std::vector<std::pair<int, int>> nvx_waves_;            // segment ranges [first, count) that may share a launch (no slot twice)
     hipError_t run_output(int n_out, int out_base);
     hipError_t linear(const DevTensor &w, const ActQuant &aq, const float *x_f32, int K, int T, float *out, int ld_out,

@@ -186,7 +186,7 @@ hipError_t Context::nvx_delta_mixer(const NvxLayer &L, const NvxRun &r, int T) {
     }
     TTX_TRY(launch_mlstm_out(nvx_o_, H * VD, gate, ld_gate, off_gate, L.mix_norm, T, H, VD, M.eps, nvx_att_, H * VD, stream_, 0,
                              per_channel ? MLSTM_GATE_SIGMOID : MLSTM_GATE_SILU));
-    TTX_TRY(nvx_linear(L.o, nvx_att_, H * VD, T, nvx_y_, W));
+    TTX_TRY(nvx_close_linear(L.o, nvx_att_, H * VD, T, L.norm1b));
     prof_mark("delta_rule");
     return hipSuccess;
 }
