@@ -307,25 +307,22 @@ def novorax_section(args) -> int:
     return 0
 
 
-def fidepel_section(args) -> int:
-    """--fidepel SIZES: prefill and decode throughput of synthetic Fidepel models (bf16 weights, serving precision) beside the closest model this backend
-    already had - the Novorax folder design of the same name: equal width, depth, vocabulary and window, the same bf16 linear kernels and f32 attention
-    arithmetic - with each side's distance from its roofline: prefill as a fraction of the dense 16-bit matrix-core peak (2 FLOP per active weight and
-    token), decode as a fraction of the HBM peak (weight bytes one token reads).  One JSON line; the default workload of this script is untouched."""
+def _time_folder_pair(args, sizes, metric, pair) -> int:
+    """Two folder designs of equal size names beside each other: pair = ((name, module, writer, weight bytes of (cfg, size)), ...), the first one measured
+    against the second.  One JSON line."""
     import __graft_entry__ as ge
     pkg = ge.load_pkg()
     pkg.Backend()
-    fs, ns = pkg.fidepel_synth, pkg.novorax_synth
     rows = []
-    for size in [x for x in args.fidepel.split(",") if x]:
+    for size in [x for x in sizes.split(",") if x]:
         row = {"size": size, "prompt": args.prompt}
-        for name, mod, writer in (("fidepel", fs, fs.write_synthetic_fidepel), ("novorax", ns, ns.write_synthetic_novorax)):
+        for name, mod, writer, wbytes_of in pair(pkg):
             s = mod.SIZES[size]
             folder = os.path.join(args.model_dir, f"mi355-bench-{name}-{size}")
             if not os.path.exists(os.path.join(folder, "model.safetensors")):
                 writer(folder, size, seed=0xC0FFEE)
             cfg = mod.config_of(s)
-            wbytes = mod.weight_bytes_per_token(cfg)
+            wbytes = wbytes_of(cfg, s)
             flops_tok = wbytes - 2 * s.width                 # 2 FLOP per active weight = its bf16 bytes (the embedding row is a lookup)
             kw = dict(n_ctx=args.ctx, n_batch=N_UBATCH, n_ubatch=N_UBATCH, n_seq_max=1)
             m = pkg.Model(folder)
@@ -339,13 +336,25 @@ def fidepel_section(args) -> int:
                 for f in (os.path.join(folder, "model.safetensors"), os.path.join(folder, "config.json")):
                     if os.path.exists(f):
                         os.remove(f)
-        a, b = row["fidepel"], row["novorax"]
+        a, b = (row[name] for name, *_ in pair(pkg))
         row["roofline_ratio"] = {"prefill": round(a["prefill_frac_of_mfma_peak"] / max(b["prefill_frac_of_mfma_peak"], 1e-9), 3),
                                  "decode": round(a["decode_frac_of_hbm_peak"] / max(b["decode_frac_of_hbm_peak"], 1e-9), 3)}
         rows.append(row)
-    print(json.dumps({"metric": "fidepel_prefill_decode_tok_s_vs_novorax", "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+    print(json.dumps({"metric": metric, "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
                       "dtype": "bf16", "data": "synthetic", "higher_is_better": True, "sizes": rows}), flush=True)
     return 0
+
+
+def fidepel_section(args) -> int:
+    """--fidepel SIZES: prefill and decode throughput of synthetic Fidepel models (bf16 weights, serving precision) beside the closest model this backend
+    already had - the Novorax folder design of the same name: equal width, depth, vocabulary and window, the same bf16 linear kernels and f32 attention
+    arithmetic - with each side's distance from its roofline: prefill as a fraction of the dense 16-bit matrix-core peak (2 FLOP per active weight and
+    token), decode as a fraction of the HBM peak (weight bytes one token reads).  One JSON line; the default workload of this script is untouched."""
+    def pair(pkg):
+        m, o = pkg.fidepel_synth, pkg.novorax_synth
+        return (("fidepel", m, m.write_synthetic_fidepel, lambda cfg, s: m.weight_bytes_per_token(cfg)),
+                ("novorax", o, o.write_synthetic_novorax, lambda cfg, s: o.weight_bytes_per_token(cfg)))
+    return _time_folder_pair(args, args.fidepel, "fidepel_prefill_decode_tok_s_vs_novorax", pair)
 
 
 def tuterax_section(args) -> int:
@@ -354,40 +363,11 @@ def tuterax_section(args) -> int:
     feed-forwards, the same bf16 linear kernels, f32 attention and recurrence arithmetic, equal width, depth and vocabulary - with each side's distance
     from its roofline: prefill as a fraction of the dense 16-bit matrix-core peak (2 FLOP per active weight and token), decode as a fraction of the HBM
     peak (weight bytes one token reads).  One JSON line; the default workload of this script is untouched."""
-    import __graft_entry__ as ge
-    pkg = ge.load_pkg()
-    pkg.Backend()
-    ts, ns = pkg.tuterax_synth, pkg.novorax_synth
-    rows = []
-    for size in [x for x in args.tuterax.split(",") if x]:
-        row = {"size": size, "prompt": args.prompt}
-        for name, mod, writer in (("tuterax", ts, ts.write_synthetic_tuterax), ("novorax", ns, ns.write_synthetic_novorax)):
-            s = mod.SIZES[size]
-            folder = os.path.join(args.model_dir, f"mi355-bench-{name}-{size}")
-            if not os.path.exists(os.path.join(folder, "model.safetensors")):
-                writer(folder, size, seed=0xC0FFEE)
-            cfg = mod.config_of(s)
-            wbytes = mod.weight_bytes_per_token(cfg, s.rank_a, s.rank_g) if name == "tuterax" else mod.weight_bytes_per_token(cfg)
-            flops_tok = wbytes - 2 * s.width                 # 2 FLOP per active weight = its bf16 bytes (the embedding row is a lookup)
-            kw = dict(n_ctx=args.ctx, n_batch=N_UBATCH, n_ubatch=N_UBATCH, n_seq_max=1)
-            m = pkg.Model(folder)
-            pf, dc, ms = _time_model(pkg, m, kw, args.prompt, args.steps, args.warmup, s.vocab)
-            m.close()
-            row["width"], row["layers"] = s.width, len(cfg["layers"])
-            row[name] = {"prefill_tok_s": round(pf, 1), "decode_tok_s": round(dc, 2), "ms_per_step": round(ms, 4), "weight_bytes_per_token": wbytes,
-                         "prefill_frac_of_mfma_peak": round(pf * flops_tok / (MFMA_BF16_PEAK_TFLOPS * 1e12), 4),
-                         "decode_frac_of_hbm_peak": round(wbytes * dc / (HBM_PEAK_GBPS * 1e9), 4)}
-            if not args.keep_model:
-                for f in (os.path.join(folder, "model.safetensors"), os.path.join(folder, "config.json")):
-                    if os.path.exists(f):
-                        os.remove(f)
-        a, b = row["tuterax"], row["novorax"]
-        row["roofline_ratio"] = {"prefill": round(a["prefill_frac_of_mfma_peak"] / max(b["prefill_frac_of_mfma_peak"], 1e-9), 3),
-                                 "decode": round(a["decode_frac_of_hbm_peak"] / max(b["decode_frac_of_hbm_peak"], 1e-9), 3)}
-        rows.append(row)
-    print(json.dumps({"metric": "tuterax_prefill_decode_tok_s_vs_novorax", "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
-                      "dtype": "bf16", "data": "synthetic", "higher_is_better": True, "sizes": rows}), flush=True)
-    return 0
+    def pair(pkg):
+        m, o = pkg.tuterax_synth, pkg.novorax_synth
+        return (("tuterax", m, m.write_synthetic_tuterax, lambda cfg, s: m.weight_bytes_per_token(cfg, s.rank_a, s.rank_g)),
+                ("novorax", o, o.write_synthetic_novorax, lambda cfg, s: o.weight_bytes_per_token(cfg)))
+    return _time_folder_pair(args, args.tuterax, "tuterax_prefill_decode_tok_s_vs_novorax", pair)
 
 
 def dinilorn_section(args) -> int:
@@ -396,40 +376,24 @@ def dinilorn_section(args) -> int:
     expert, the same bf16 linear kernels, cell table and step function, equal width, depth, vocabulary, head and expert counts - with each side's distance
     from its roofline: prefill as a fraction of the dense 16-bit matrix-core peak (2 FLOP per active weight and token), decode as a fraction of the HBM
     peak (weight bytes one token reads).  One JSON line; the default workload of this script is untouched."""
-    import __graft_entry__ as ge
-    pkg = ge.load_pkg()
-    pkg.Backend()
-    ds, fs = pkg.dinilorn_synth, pkg.fidepel_synth
-    rows = []
-    for size in [x for x in args.dinilorn.split(",") if x]:
-        row = {"size": size, "prompt": args.prompt}
-        for name, mod, writer in (("dinilorn", ds, ds.write_synthetic_dinilorn), ("fidepel", fs, fs.write_synthetic_fidepel)):
-            s = mod.SIZES[size]
-            folder = os.path.join(args.model_dir, f"mi355-bench-{name}-{size}")
-            if not os.path.exists(os.path.join(folder, "model.safetensors")):
-                writer(folder, size, seed=0xC0FFEE)
-            cfg = mod.config_of(s)
-            wbytes = mod.weight_bytes_per_token(cfg)
-            flops_tok = wbytes - 2 * s.width                 # 2 FLOP per active weight = its bf16 bytes (the embedding row is a lookup)
-            kw = dict(n_ctx=args.ctx, n_batch=N_UBATCH, n_ubatch=N_UBATCH, n_seq_max=1)
-            m = pkg.Model(folder)
-            pf, dc, ms = _time_model(pkg, m, kw, args.prompt, args.steps, args.warmup, s.vocab)
-            m.close()
-            row["width"], row["layers"] = s.width, len(cfg["layers"])
-            row[name] = {"prefill_tok_s": round(pf, 1), "decode_tok_s": round(dc, 2), "ms_per_step": round(ms, 4), "weight_bytes_per_token": wbytes,
-                         "prefill_frac_of_mfma_peak": round(pf * flops_tok / (MFMA_BF16_PEAK_TFLOPS * 1e12), 4),
-                         "decode_frac_of_hbm_peak": round(wbytes * dc / (HBM_PEAK_GBPS * 1e9), 4)}
-            if not args.keep_model:
-                for f in (os.path.join(folder, "model.safetensors"), os.path.join(folder, "config.json")):
-                    if os.path.exists(f):
-                        os.remove(f)
-        a, b = row["dinilorn"], row["fidepel"]
-        row["roofline_ratio"] = {"prefill": round(a["prefill_frac_of_mfma_peak"] / max(b["prefill_frac_of_mfma_peak"], 1e-9), 3),
-                                 "decode": round(a["decode_frac_of_hbm_peak"] / max(b["decode_frac_of_hbm_peak"], 1e-9), 3)}
-        rows.append(row)
-    print(json.dumps({"metric": "dinilorn_prefill_decode_tok_s_vs_fidepel", "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
-                      "dtype": "bf16", "data": "synthetic", "higher_is_better": True, "sizes": rows}), flush=True)
-    return 0
+    def pair(pkg):
+        m, o = pkg.dinilorn_synth, pkg.fidepel_synth
+        return (("dinilorn", m, m.write_synthetic_dinilorn, lambda cfg, s: m.weight_bytes_per_token(cfg)),
+                ("fidepel", o, o.write_synthetic_fidepel, lambda cfg, s: o.weight_bytes_per_token(cfg)))
+    return _time_folder_pair(args, args.dinilorn, "dinilorn_prefill_decode_tok_s_vs_fidepel", pair)
+
+
+def vuzazen_section(args) -> int:
+    """--vuzazen SIZES: prefill and decode throughput of synthetic Vuzazen models (bf16 weights, serving precision) beside the closest model this backend
+    already had - the Novorax folder design of the same name: latent attention and the mLSTM recurrence with the same head counts and sizes, dense and expert
+    feed-forwards, the same bf16 linear kernels, cell table and step function, equal width, depth and vocabulary - with each side's distance from its
+    roofline: prefill as a fraction of the dense 16-bit matrix-core peak (2 FLOP per active weight and token), decode as a fraction of the HBM peak (weight
+    bytes one token reads).  One JSON line; the default workload of this script is untouched."""
+    def pair(pkg):
+        m, o = pkg.vuzazen_synth, pkg.novorax_synth
+        return (("vuzazen", m, m.write_synthetic_vuzazen, lambda cfg, s: m.weight_bytes_per_token(cfg)),
+                ("novorax", o, o.write_synthetic_novorax, lambda cfg, s: o.weight_bytes_per_token(cfg)))
+    return _time_folder_pair(args, args.vuzazen, "vuzazen_prefill_decode_tok_s_vs_novorax", pair)
 
 
 def main() -> int:
@@ -438,6 +402,7 @@ def main() -> int:
     ap.add_argument("--fidepel", default="", help="comma list of synthetic Fidepel sizes (w1024, w2048, w4096): time them beside the Novorax model of that size and exit")
     ap.add_argument("--tuterax", default="", help="comma list of synthetic Tuterax sizes (w1024, w2048, w4096): time them beside the Novorax model of that size and exit")
     ap.add_argument("--dinilorn", default="", help="comma list of synthetic Dinilorn sizes (w1024, w2048, w4096): time them beside the Fidepel model of that size and exit")
+    ap.add_argument("--vuzazen", default="", help="comma list of synthetic Vuzazen sizes (w1024, w2048, w4096): time them beside the Novorax model of that size and exit")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)
     ap.add_argument("--warmup", type=int, default=16)
@@ -485,6 +450,8 @@ def main() -> int:
         return tuterax_section(args)
     if args.dinilorn:
         return dinilorn_section(args)
+    if args.vuzazen:
+        return vuzazen_section(args)
 
     rank = int(os.environ.get("RANK", "0"))
     local_rank = int(os.environ.get("LOCAL_RANK", "0"))
