@@ -18,6 +18,7 @@
 // Turned values (optional): every value head is stored turned by its own position over all its entries, in the same half-and-half pairing; the weighted sum
 // of a row is turned back by the row's position - each term then carries the turn by (key position - query position), a relative position signal on the
 // value side.  The turn back happens where a row's result is finished: in the per-row kernel, in the merge of split scans, or in gq_unturn behind the tiled pass.
+#include "attn_merge_dev.h"
 #include "kernels.h"
 
 namespace mi355 {
@@ -373,36 +374,25 @@ __global__ __launch_bounds__(512) void gq_attn_kernel(GqAttnArgs a) {
 }
 
 __global__ __launch_bounds__(256) void gq_attn_merge_kernel(GqAttnArgs a, int splits) {
+    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[4 * GQ_MAX_D], sums[GQ_MAX_D];
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, VD = a.vdim;
-    const float *rec = a.part + ((size_t)t * a.H + h) * splits * (size_t)(VD + 2);
-    float MM = a.sink ? a.sink[h] : -INFINITY;
-    for (int s = 0; s < splits; s++) if (rec[(size_t)s * (VD + 2) + 1] > 0.0f) MM = fmaxf(MM, rec[(size_t)s * (VD + 2)]);
-    float den = a.sink ? expf(a.sink[h] - MM) : 0.0f;
-    for (int s = 0; s < splits; s++) { const float *r = rec + (size_t)s * (VD + 2); den += r[1] > 0.0f ? r[1] * expf(r[0] - MM) : 0.0f; }
+    const float gate = a.gate ? a.gate[(size_t)t * a.ld_gate + h] : 0.0f;
+    const float den = attn_merge_runs(a.part + ((size_t)t * a.H + h) * splits * (size_t)(VD + 2), splits, VD, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
     float inv = den > 0.0f ? 1.0f / den : 0.0f;
-    if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)t * a.ld_gate + h]));
+    if (a.gate) inv *= 1.0f / (1.0f + expf(-gate));
+    float *out = a.out + (size_t)t * a.ld_out + (size_t)h * VD;
     if (a.v_cs) {                                               // (vdim is even)
         const int vhalf = VD >> 1;
         const float *cs = a.v_cs + (size_t)t * VD;
         for (int i = tid; i < vhalf; i += 256) {
-            float o = 0.0f, o2 = 0.0f;
-            for (int s = 0; s < splits; s++) {
-                const float *r = rec + (size_t)s * (VD + 2);
-                const float f = r[1] > 0.0f ? expf(r[0] - MM) : 0.0f;
-                o += r[2 + i] * f;
-                o2 += r[2 + i + vhalf] * f;
-            }
+            float o = sums[i], o2 = sums[i + vhalf];
             gq_unturn_pair(o, o2, cs[i], cs[vhalf + i]);
-            a.out[(size_t)t * a.ld_out + (size_t)h * VD + i] = o * inv;
-            a.out[(size_t)t * a.ld_out + (size_t)h * VD + i + vhalf] = o2 * inv;
+            out[i] = o * inv;
+            out[i + vhalf] = o2 * inv;
         }
         return;
     }
-    for (int i = tid; i < VD; i += 256) {
-        float o = 0.0f;
-        for (int s = 0; s < splits; s++) { const float *r = rec + (size_t)s * (VD + 2); o += r[1] > 0.0f ? r[2 + i] * expf(r[0] - MM) : 0.0f; }
-        a.out[(size_t)t * a.ld_out + (size_t)h * VD + i] = o * inv;
-    }
+    for (int i = tid; i < VD; i += 256) out[i] = sums[i] * inv;
 }
 
 template <int NJ>

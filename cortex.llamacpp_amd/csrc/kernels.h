@@ -414,13 +414,15 @@ struct LatentAttnArgs {
     const float *rot_freq; float rot_mscale;
     int rot_halves;                        // as in LatentPrepArgs
     const float *gate; int ld_gate;        // nullable: head h's attended latent is multiplied by sigmoid(gate[t * ld_gate + h])
-    // single-token steps: the scanned cells cut into `splits` runs, one workgroup each, merged afterwards; part: T * H * splits * (kv_rank + 2) floats (nullptr / splits <= 1: one workgroup per (token, head))
-    float *part; int splits;
+    // the scanned cells cut into runs, one workgroup each, merged afterwards; part: room for part_floats floats, T * H * runs * (kv_rank + 2) are used (nullptr: one
+    // run).  n_kv_hint: the host's count of cells in use (batches; 0: unknown)
+    float *part; size_t part_floats; int n_kv_hint;
     // nullable: per token, one past the highest cell that can hold a key of its sequence at or before its position (host-made from the cell table): the scan
     // of a prompt's early tokens stops there instead of at the high-water mark
     const int32_t *tok_hi;
 };
-constexpr int LATENT_ATTN_SPLITS = 8, LATENT_ATTN_SPLIT_MAX_PAIRS = 128;   // (token, head) pairs up to which a step is split
+constexpr int LATENT_ATTN_SPLITS = 8, LATENT_ATTN_SPLIT_MAX_PAIRS = 128;   // (token, head) pairs up to which a scan by single pairs is split, into how many runs
+constexpr int LATENT_STEP_MAX_PAIRS = 512, LATENT_STEP_RUNS = 32, LATENT_TILE_RUNS = 8;   // tiles of pairs: steps (up to 512 / tiles runs), batches
 bool latent_attn_shape_ok(int kv_rank, int rot);
 hipError_t launch_latent_attn(const LatentAttnArgs &a, hipStream_t st);
 

@@ -10,6 +10,7 @@
 //
 // latent_prep: per token, the two RMS norms behind the down-projections (query latent -> cq, key / value latent -> cache row) and the rotation of the
 // shared key part into the cache row.  Interleaved pairs (2i, 2i + 1), or entry i with entry i + half the turning part; the per-pair frequency table (YaRN blend included) comes from the host.
+#include "attn_merge_dev.h"
 #include "kernels.h"
 
 namespace mi355 {
@@ -78,6 +79,8 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepArgs a) {
         } else dst[a.kv_rank + i] = kr[i];
     }
 }
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int LA_MAX_L = 1088;                                  // kv_rank + rot the attention kernel is instantiated for (17 x 64)
 
@@ -224,18 +227,11 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(LatentAttnArgs a) {
 }
 
 __global__ __launch_bounds__(256) void latent_attn_merge_kernel(LatentAttnArgs a, int splits) {
+    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[4 * LA_MAX_L], sums[LA_MAX_L];
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, KR = a.kv_rank;
-    const float *rec = a.part + ((size_t)t * a.H + h) * splits * (size_t)(KR + 2);
-    float MM = a.sink ? a.sink[h] : -INFINITY;
-    for (int s = 0; s < splits; s++) if (rec[(size_t)s * (KR + 2) + 1] > 0.0f) MM = fmaxf(MM, rec[(size_t)s * (KR + 2)]);
-    float den = a.sink ? expf(a.sink[h] - MM) : 0.0f;
-    for (int s = 0; s < splits; s++) { const float *r = rec + (size_t)s * (KR + 2); den += r[1] > 0.0f ? r[1] * expf(r[0] - MM) : 0.0f; }
+    const float den = attn_merge_runs(a.part + ((size_t)t * a.H + h) * splits * (size_t)(KR + 2), splits, KR, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
     const float inv = latent_out_factor(a, t, h, den);
-    for (int i = tid; i < KR; i += 256) {
-        float o = 0.0f;
-        for (int s = 0; s < splits; s++) { const float *r = rec + (size_t)s * (KR + 2); o += r[1] > 0.0f ? r[2 + i] * expf(r[0] - MM) : 0.0f; }
-        a.out[(size_t)t * a.ld_out + (size_t)h * KR + i] = o * inv;
-    }
+    for (int i = tid; i < KR; i += 256) a.out[(size_t)t * a.ld_out + (size_t)h * KR + i] = sums[i] * inv;
 }
 
 template <int NJ>
@@ -244,12 +240,248 @@ static hipError_t launch_latent_attn_nj(const LatentAttnArgs &a, hipStream_t st)
     const int nw = (long long)a.T * a.H <= 1024 ? 8 : 4;
     const size_t lds = (size_t)(NJ * 64 + 2 * nw + nw * NJ * 64) * sizeof(float);
     const bool vec = ((a.kv_rank + a.rot) & 3) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0;
-    const int splits = a.part && a.splits > 1 ? a.splits : 1;
+    const int splits = a.part && (long long)a.T * a.H <= LATENT_ATTN_SPLIT_MAX_PAIRS && (size_t)a.T * a.H * LATENT_ATTN_SPLITS * (a.kv_rank + 2) <= a.part_floats ? LATENT_ATTN_SPLITS : 1;
     const dim3 grid((unsigned)a.T, (unsigned)a.H, (unsigned)splits);
     if (vec) hipLaunchKernelGGL((latent_attn_kernel<NJ, true>), grid, dim3(64 * nw), lds, st, a);
     else hipLaunchKernelGGL((latent_attn_kernel<NJ, false>), grid, dim3(64 * nw), lds, st, a);
     if (splits > 1) hipLaunchKernelGGL(latent_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, splits);
     return hipGetLastError();
+}
+
+// ---- the same attention on the f32 matrix cores: every head of every row reads the same cache rows, so (row, head) pairs are the columns of one product.
+// One workgroup per (tile of 16 R pairs, run of cells), 8 waves, BC cells per block.  v_mfma_f32_16x16x4_f32 (f32 operands, f32 accumulation): lane l holds
+// A[l & 15][l >> 4], B[l >> 4][l & 15], register r of the result is D[4 (l >> 4) + r][l & 15]; the order of k is free as long as A and B agree, so a lane
+// loads 4 consecutive floats (16 bytes) and feeds them to 4 products.
+//   scores:  A = cache rows (i = cell), B = queries (j = pair; in LDS, turned on the way in): a wave takes 16 cells x 16 pairs; where a block has fewer such
+//            pieces than the workgroup waves, KS waves share one piece, each a part of the row's length, and their partial sums meet in the softmax
+//   softmax: 16 lanes per pair; weights back to LDS
+//   values:  A = cache rows (i = latent entry, k = cell), B = weights (k = cell, j = pair): a wave takes 64 entries x 16 pairs; entry i of tile jj stands for
+//            64 J + 4 i + jj, which makes every load 16 bytes and a lane's results 16 neighbouring entries of its pair
+constexpr int LT_NW = 8;
+constexpr int lt_pieces(int R, int BC) { return (BC / 16) * R; }
+constexpr int lt_ks(int R, int BC) { return lt_pieces(R, BC) >= LT_NW ? 1 : LT_NW / lt_pieces(R, BC); }
+constexpr size_t lt_lds_floats(int R, int BC, int LQ) { return (size_t)16 * R * (LQ + 4) + (size_t)lt_ks(R, BC) * 16 * R * (BC + 4) + 3 * 16 * R + 4 + 64 * R + 2 * 16 * R; }
+constexpr size_t LT_LDS_MAX = 156 * 1024;
+
+// NT: tasks (64 latent entries x 16 pairs) a wave owns at most
+template <int R, int BC, int NT>
+__global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs a, int LQ) {
+    constexpr int BQ = 16 * R, LDS_S = BC + 4, KS = lt_ks(R, BC), NS = BC / 16;
+    extern __shared__ float lds[];
+    const int KR = a.kv_rank, RT = a.rot, L = KR + RT, H = a.H, LDQ = LQ + 4;
+    float *Q = lds, *S = Q + (size_t)BQ * LDQ, *ms = S + (size_t)KS * BQ * LDS_S, *ls = ms + BQ, *al = ls + BQ;
+    int *red = reinterpret_cast<int *>(al + BQ);
+    uint64_t *vmask2 = reinterpret_cast<uint64_t *>(red + 4);    // [2][BQ], two blocks in turn
+    int *rpos = reinterpret_cast<int *>(vmask2 + 2 * BQ), *rseq = rpos + BQ;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lg = lane >> 4;
+    const int P = a.T * H, p0 = blockIdx.x * BQ;
+    const int n_kv = *a.n_kv_dev;
+    if (tid < 64) {
+        int hi = 0;
+        for (int i = tid; i < BQ; i += 64) {
+            const bool live = p0 + i < P;
+            const int t = live ? (p0 + i) / H : 0;
+            rpos[i] = live ? a.tok_pos[t] : -1;
+            rseq[i] = live ? (a.tok_seq[t] & 63) : -1;
+            ms[i] = -INFINITY; ls[i] = 0.0f;
+            if (live) { const int th = a.tok_hi ? (a.tok_hi[t] < n_kv ? a.tok_hi[t] : n_kv) : n_kv; hi = th > hi ? th : hi; }
+        }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) hi = max(hi, __shfl_xor(hi, o, 64));
+        if (tid == 0) red[0] = hi;
+    }
+    // the tile's queries: the folded part as it is, the turning part turned; zeros behind the row's length and for pairs past the end
+    for (int i = tid; i < BQ * LQ; i += 64 * LT_NW) {
+        const int r = i / LQ, d = i - r * LQ, p = p0 + r;
+        float v = 0.0f;
+        if (p < P && d < L) {
+            const int t = p / H, h = p - t * H;
+            if (d < KR) v = a.qa[(size_t)t * a.ld_qa + (size_t)h * KR + d];
+            else {
+                const float *qr = a.q + (size_t)t * a.ld_q + (size_t)h * (a.dim + RT) + a.dim;
+                const int e = d - KR;
+                if (e < a.rot_dims) {
+                    const LatentPair q = latent_pair(e, a.rot_dims, a.rot_halves);
+                    const float ang = (float)a.tok_pos[t] * a.rot_freq[q.pr], c = cosf(ang) * a.rot_mscale, sn = sinf(ang) * a.rot_mscale;
+                    const float u = qr[q.iu], w = qr[q.iv];
+                    v = q.second ? w * c + u * sn : u * c - w * sn;
+                } else v = qr[e];
+            }
+        }
+        Q[(size_t)r * LDQ + d] = v * a.scale;
+    }
+    __syncthreads();
+    int c_begin = 0, c_end = red[0];
+    if (gridDim.y > 1) {
+        const int per = ((c_end + BC - 1) / BC + (int)gridDim.y - 1) / (int)gridDim.y * BC;
+        c_begin = (int)blockIdx.y * per;
+        c_end = c_begin + per < c_end ? c_begin + per : c_end;
+    }
+    const int NJ = (KR + 63) >> 6;                              // tasks of the value pass: (J, row tile), J * R + tile
+    f32x4 o[NT][4];
+#pragma unroll
+    for (int i = 0; i < NT; i++)
+#pragma unroll
+        for (int jj = 0; jj < 4; jj++) o[i][jj] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    uint64_t *vmask = vmask2;
+    for (int c0 = c_begin; c0 < c_end; c0 += BC) {
+        vmask = vmask == vmask2 ? vmask2 + BQ : vmask2;          // (a slower wave may still be about to read the previous block's)
+        int any = 0;
+        {
+            const int cc = c0 + lane;
+            int cp = -1; uint64_t cs = 0;
+            if (lane < BC && cc < c_end) { cp = a.cell_pos[cc]; cs = a.cell_seq[cc]; }
+#pragma unroll
+            for (int i = 0; i < 2 * R; i++) {
+                const int r = wave + LT_NW * i, rp = rpos[r], rs = rseq[r];
+                const bool v = cp >= 0 && rs >= 0 && cp <= rp && ((cs >> (rs & 63)) & 1) != 0 && !(a.window > 0 && rp - cp >= a.window);
+                const uint64_t b = __ballot(v);
+                if (lane == 0) vmask[r] = b;
+                any |= b != 0;
+            }
+        }
+        if (!__syncthreads_or(any)) continue;                   // (also: the previous block's weights have been used, the masks are in place)
+        // ---- scores
+        {
+            constexpr int PIECES = lt_pieces(R, BC), PER = PIECES > LT_NW ? PIECES / LT_NW : 1;   // (PER row tiles of one cell piece per wave)
+            const int piece = wave % (PIECES < LT_NW ? PIECES : LT_NW), ks = wave / (PIECES < LT_NW ? PIECES : LT_NW), s = piece % NS, rt0 = piece / NS;
+            const int steps = LQ >> 4, per = (steps + KS - 1) / KS, u0 = ks * per, u1 = u0 + per < steps ? u0 + per : steps;
+            const int c = c0 + 16 * s + l16;
+            const float *kr = a.cache + (size_t)(c < c_end ? c : c_end - 1) * L + 4 * lg;
+            const float *qr[PER];
+            f32x4 acc[PER];
+#pragma unroll
+            for (int i = 0; i < PER; i++) { qr[i] = Q + (size_t)(16 * (rt0 + i * (LT_NW / NS)) + l16) * LDQ + 4 * lg; acc[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f}; }
+#pragma unroll 4
+            for (int u = u0; u < u1; u++) {
+                const f32x4 k4 = 16 * u + 4 * lg < L ? *reinterpret_cast<const f32x4 *>(kr + 16 * u) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+                for (int i = 0; i < PER; i++) {
+                    const f32x4 q4 = *reinterpret_cast<const f32x4 *>(qr[i] + 16 * u);
+#pragma unroll
+                    for (int e = 0; e < 4; e++) acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[e], q4[e], acc[i], 0, 0, 0);
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < PER; i++) *reinterpret_cast<f32x4 *>(S + (size_t)(ks * BQ + 16 * (rt0 + i * (LT_NW / NS)) + l16) * LDS_S + 16 * s + 4 * lg) = acc[i];
+        }
+        __syncthreads();
+        // ---- softmax: 16 lanes per pair
+        for (int r = tid >> 4; r < BQ; r += 32) {
+            const uint64_t seen = vmask[r];
+            float x[NS];
+            float bm = -INFINITY;
+#pragma unroll
+            for (int j = 0; j < NS; j++) {
+                float v = S[(size_t)r * LDS_S + 16 * j + l16];
+#pragma unroll
+                for (int k = 1; k < KS; k++) v += S[(size_t)(k * BQ + r) * LDS_S + 16 * j + l16];
+                x[j] = v;
+                if ((seen >> (16 * j + l16)) & 1) bm = fmaxf(bm, v);
+            }
+            bm = fmaxf(bm, dpp_f<DPP_QP_1032>(bm));
+            bm = fmaxf(bm, dpp_f<DPP_QP_2301>(bm));
+            bm = fmaxf(bm, dpp_f<DPP_HALF_MIRROR>(bm));
+            bm = fmaxf(bm, dpp_f<DPP_MIRROR>(bm));
+            const float m0 = ms[r], mn = fmaxf(m0, bm), alpha = m0 == -INFINITY ? 0.0f : expf(m0 - mn);
+            float ps = 0.0f;
+#pragma unroll
+            for (int j = 0; j < NS; j++) {
+                const float p = (seen >> (16 * j + l16)) & 1 ? expf(x[j] - mn) : 0.0f;
+                S[(size_t)r * LDS_S + 16 * j + l16] = p;
+                ps += p;
+            }
+            ps = row_sum16(ps);
+            if (l16 == 0) { ls[r] = ls[r] * alpha + ps; ms[r] = mn; al[r] = alpha; }
+        }
+        __syncthreads();
+        // ---- values
+#pragma unroll
+        for (int i = 0; i < NT; i++) {
+            const int task = wave + LT_NW * i;
+            if (task >= NJ * R) continue;
+            const int J = task / R, rt = task - J * R;
+            const float alpha = al[16 * rt + l16];
+#pragma unroll
+            for (int jj = 0; jj < 4; jj++) { o[i][jj].x *= alpha; o[i][jj].y *= alpha; o[i][jj].z *= alpha; o[i][jj].w *= alpha; }
+            const bool in = 64 * J + 4 * l16 < KR;
+            const float *vb = a.cache + 64 * J + 4 * l16;
+#pragma unroll
+            for (int s = 0; s < NS; s++) {
+                const f32x4 p4 = *reinterpret_cast<const f32x4 *>(S + (size_t)(16 * rt + l16) * LDS_S + 16 * s + 4 * lg);
+                f32x4 v[4];
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    const int c = c0 + 16 * s + 4 * lg + e;      // (cells past the end repeat the last one with weight 0)
+                    v[e] = in ? *reinterpret_cast<const f32x4 *>(vb + (size_t)(c < c_end ? c : c_end - 1) * L) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+                }
+#pragma unroll
+                for (int e = 0; e < 4; e++)
+#pragma unroll
+                    for (int jj = 0; jj < 4; jj++) o[i][jj] = __builtin_amdgcn_mfma_f32_16x16x4f32(v[e][jj], p4[e], o[i][jj], 0, 0, 0);
+            }
+        }
+        // (no barrier: the next block's scores are written behind the barrier that ends its visibility test)
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < NT; i++) {
+        const int task = wave + LT_NW * i;
+        if (task >= NJ * R) continue;
+        const int J = task / R, rt = task - J * R, r = 16 * rt + l16, p = p0 + r;
+        if (p >= P) continue;
+        const int t = p / H, h = p - t * H;
+        if (gridDim.y > 1) {
+            float *rec = a.part + ((size_t)p * gridDim.y + blockIdx.y) * (size_t)(KR + 2);
+            if (J == 0 && lg == 0) { rec[0] = ms[r]; rec[1] = ls[r]; }
+#pragma unroll
+            for (int rr = 0; rr < 4; rr++)
+#pragma unroll
+                for (int jj = 0; jj < 4; jj++) {
+                    const int col = 64 * J + 16 * lg + 4 * rr + jj;
+                    if (col < KR) rec[2 + col] = o[i][jj][rr];
+                }
+            continue;
+        }
+        const float MM = a.sink ? fmaxf(ms[r], a.sink[h]) : ms[r];
+        const float sc = ls[r] > 0.0f ? expf(ms[r] - MM) : 0.0f;
+        const float den = ls[r] * sc + (a.sink ? expf(a.sink[h] - MM) : 0.0f);
+        const float inv = latent_out_factor(a, t, h, den) * sc;
+#pragma unroll
+        for (int rr = 0; rr < 4; rr++)
+#pragma unroll
+            for (int jj = 0; jj < 4; jj++) {
+                const int col = 64 * J + 16 * lg + 4 * rr + jj;
+                if (col < KR) a.out[(size_t)t * a.ld_out + (size_t)h * KR + col] = o[i][jj][rr] * inv;
+            }
+    }
+}
+
+template <int R, int BC, int NT>
+static hipError_t launch_latent_tile(const LatentAttnArgs &a, hipStream_t st) {
+    const int LQ = (a.kv_rank + a.rot + 15) & ~15;
+    const size_t lds = lt_lds_floats(R, BC, LQ) * sizeof(float);
+    if (lds > 60 * 1024) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_tile_kernel<R, BC, NT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    const long long P = (long long)a.T * a.H, tiles = (P + 16 * R - 1) / (16 * R);
+    // enough runs of cells for two workgroups per CU; batches no more than there are blocks of cells (steps of few rows are launched for any number of cells)
+    long long splits = (512 + tiles - 1) / tiles;
+    if (BC == 64 && a.n_kv_hint > 0 && splits > (a.n_kv_hint + BC - 1) / BC) splits = (a.n_kv_hint + BC - 1) / BC;
+    if (splits > (BC == 64 ? LATENT_TILE_RUNS : LATENT_STEP_RUNS)) splits = BC == 64 ? LATENT_TILE_RUNS : LATENT_STEP_RUNS;
+    while (splits > 1 && (!a.part || (size_t)P * (size_t)splits * (a.kv_rank + 2) > a.part_floats)) splits--;
+    hipLaunchKernelGGL((latent_tile_kernel<R, BC, NT>), dim3((unsigned)tiles, (unsigned)splits), dim3(64 * LT_NW), lds, st, a, LQ);
+    if (splits > 1) hipLaunchKernelGGL(latent_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, (int)splits);
+    return hipGetLastError();
+}
+template <int R, int BC>
+static hipError_t launch_latent_tile_nt(const LatentAttnArgs &a, hipStream_t st) {
+    const int tasks = (a.kv_rank + 63) / 64 * R;                 // (at most 17 R)
+    if (tasks <= LT_NW) return launch_latent_tile<R, BC, 1>(a, st);
+    if (tasks <= 2 * LT_NW) return launch_latent_tile<R, BC, 2>(a, st);
+    if (tasks <= 4 * LT_NW) return launch_latent_tile<R, BC, 4>(a, st);
+    return launch_latent_tile<R, BC, 9>(a, st);
 }
 
 }  // namespace
@@ -266,7 +498,16 @@ hipError_t launch_latent_prep(const LatentPrepArgs &a, hipStream_t st) {
 hipError_t launch_latent_attn(const LatentAttnArgs &a, hipStream_t st) {
     if (a.T <= 0) return hipSuccess;
     if (!latent_attn_shape_ok(a.kv_rank, a.rot) || a.rot_dims > a.rot || (a.rot_dims & 1)) return hipErrorInvalidValue;
-    const int L = a.kv_rank + a.rot;
+    const int L = a.kv_rank + a.rot, LQ = (L + 15) & ~15;
+    // rows that allow 16-byte loads take the matrix cores: batches in tiles of 64 or 32 (row, head) pairs and blocks of 64 cells, steps of few pairs in
+    // tiles of 16 or 32 pairs and blocks of 32 cells
+    if ((L & 3) == 0 && (a.kv_rank & 3) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0) {
+        const long long P = (long long)a.T * a.H;
+        if (P <= 16) return launch_latent_tile_nt<1, 32>(a, st);
+        if (P <= LATENT_STEP_MAX_PAIRS) return launch_latent_tile_nt<2, 32>(a, st);
+        if (P >= 1024 && lt_lds_floats(4, 64, LQ) * sizeof(float) <= LT_LDS_MAX) return launch_latent_tile_nt<4, 64>(a, st);
+        return launch_latent_tile_nt<2, 64>(a, st);
+    }
     if (L <= 128) return launch_latent_attn_nj<2>(a, st);
     if (L <= 320) return launch_latent_attn_nj<5>(a, st);
     if (L <= 576) return launch_latent_attn_nj<9>(a, st);

@@ -447,17 +447,18 @@ hipError_t launch_moe_combine(float *x, const float *eo, const float *w, int T, 
     return hipGetLastError();
 }
 // ---------------------------------------------------------------- grouping by expert (ggml_mul_mat_id with a batch of tokens)
-// One workgroup of 4 waves.  The selections are staged in LDS; wave w owns experts w, w + 4, ...: it walks the selections
+// One workgroup of 16 waves.  The selections are staged in LDS; wave w owns experts w, w + 16, ...: it walks the selections
 // 64 at a time in (token, rank) order, a ballot marks the ones that chose its expert and a prefix count of the ballot
 // gives each its row: stable, deterministic, no atomics.  (Runs once per layer of a prompt batch: a few microseconds.)
-__global__ __launch_bounds__(256) void moe_group_kernel(const int32_t *ids, int n_sel, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, const float *w, float *w_of) {
+__global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *ids, int n_sel, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, const float *w, float *w_of) {
     extern __shared__ int32_t sid[];               // [n_sel]
     __shared__ int cnt[64], off[65];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    for (int i = tid; i < n_sel; i += 256) sid[i] = ids[i];
+    for (int i = tid; i < n_sel; i += 1024) sid[i] = ids[i];
     __syncthreads();
-    for (int e = wave; e < n_expert; e += 4) {
+    for (int e = wave; e < n_expert; e += 16) {
         int c = 0;
+#pragma unroll 4
         for (int b = 0; b < n_sel; b += 64) {
             const bool hit = b + lane < n_sel && sid[b + lane] == e;
             c += __popcll(__ballot(hit));
@@ -465,16 +466,20 @@ __global__ __launch_bounds__(256) void moe_group_kernel(const int32_t *ids, int 
         if (lane == 0) cnt[e] = c;
     }
     __syncthreads();
-    if (tid == 0) {
-        int run = 0;
-        for (int j = 0; j < n_expert; j++) { off[j] = run; run += cnt[j]; }
-        off[n_expert] = run;
+    if (wave == 0) {                               // exclusive prefix over the experts
+        int v = lane < n_expert ? cnt[lane] : 0;
+        const int mine = v;
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) { const int u = __shfl_up(v, o, 64); if (lane >= o) v += u; }
+        off[lane] = v - mine;
+        if (lane == 63) off[64] = v;
     }
     __syncthreads();
     if (tid < n_expert) { meta[tid] = cnt[tid]; meta[n_expert + tid] = off[tid]; }
-    if (tid == 0) meta[2 * n_expert] = off[n_expert];
-    for (int e = wave; e < n_expert; e += 4) {
+    if (tid == 0) meta[2 * n_expert] = off[64];
+    for (int e = wave; e < n_expert; e += 16) {
         int r = off[e];
+#pragma unroll 4
         for (int b = 0; b < n_sel; b += 64) {
             const bool hit = b + lane < n_sel && sid[b + lane] == e;
             const unsigned long long m = __ballot(hit);
@@ -491,7 +496,7 @@ __global__ __launch_bounds__(256) void moe_group_kernel(const int32_t *ids, int 
 hipError_t launch_moe_group(const int32_t *ids, int T, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, hipStream_t st, const float *w, float *w_of) {
     if (w_of && !w) return hipErrorInvalidValue;
     if (n_expert > 64 || T * k <= 0 || (size_t)T * k * 4 > 60 * 1024) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(256), (size_t)T * k * 4, st, ids, T * k, k, n_expert, meta, slot_of, tok_of, w, w_of);
+    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), (size_t)T * k * 4, st, ids, T * k, k, n_expert, meta, slot_of, tok_of, w, w_of);
     return hipGetLastError();
 }
 // one workgroup per grouped row: 16-byte copies of the code plane(s), then the small per-block planes

@@ -24,7 +24,17 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 // loads where the rows allow, the next key head in flight).  Mix: thread = (head, cell), a head's 32 cells are 32 neighbouring lanes, which also hold its softmax.
 // Values: thread = (head, 4 columns) - or one column -, running sums in LDS.
 constexpr int TKR_BC = 32, TKR_NT = 512;
-constexpr size_t tkr_lds_floats(int H, int dim, int vdim) { return (size_t)H * dim + (size_t)H * (TKR_BC + 1) * 2 + (size_t)H * vdim + 3 * (size_t)H + 2 * TKR_BC; }
+constexpr int TKR_TALK_LDS = 64;                                // up to this many heads the mixing matrix is held in LDS too
+constexpr size_t tkr_lds_floats(int H, int dim, int vdim) {
+    return (size_t)H * dim + (size_t)H * (TKR_BC + 1) * 2 + (size_t)H * vdim + 3 * (size_t)H + 2 * TKR_BC + (H <= TKR_TALK_LDS ? (size_t)H * H : 0);
+}
+__device__ __forceinline__ float talk_half_max(float v) {       // over the 32 lanes of a half wave
+    v = fmaxf(v, dpp_f<DPP_QP_1032>(v));
+    v = fmaxf(v, dpp_f<DPP_QP_2301>(v));
+    v = fmaxf(v, dpp_f<DPP_HALF_MIRROR>(v));
+    v = fmaxf(v, dpp_f<DPP_MIRROR>(v));
+    return fmaxf(v, __shfl_xor(v, 16, 64));
+}
 
 template <int NJ, bool VEC>
 __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
@@ -32,6 +42,8 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
     const int H = a.H, G = a.G, D = a.dim, VD = a.vdim, HG = H / G;
     float *qv = lds, *acc = qv + (size_t)H * D, *raw = acc + (size_t)H * VD, *pw = raw + (size_t)H * (TKR_BC + 1), *ms = pw + (size_t)H * (TKR_BC + 1), *ls = ms + H, *al = ls + H;
     int *vis = reinterpret_cast<int *>(al + H);                  // [TKR_BC]
+    float *tk = reinterpret_cast<float *>(vis + 2 * TKR_BC);     // [H][H]
+    const float *talk = H <= TKR_TALK_LDS ? tk : a.talk;
     const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, grp = lane >> 4, li = lane & 15;
     const size_t L = (size_t)G * (D + VD), voff = (size_t)G * D;
     const int tpos = a.tok_pos[t];
@@ -46,6 +58,7 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         c_hi = c_lo + per < c_hi ? c_lo + per : c_hi;
     }
     for (int i = tid; i < H * D; i += TKR_NT) qv[i] = a.q[(size_t)t * a.ld_q + i];
+    if (H <= TKR_TALK_LDS) for (int i = tid; i < H * H; i += TKR_NT) tk[i] = a.talk[i];
     for (int i = tid; i < H * VD; i += TKR_NT) acc[i] = 0.0f;
     for (int i = tid; i < H; i += TKR_NT) { ms[i] = -INFINITY; ls[i] = 0.0f; }
     const auto fetch = [&](int c, int kvh, float (&dst)[NJ][4]) {
@@ -76,6 +89,7 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         // ---- raw scores
         for (int kvh = 0; kvh < G; kvh++) {
             if (kvh + 1 < G) fetch(c, kvh + 1, nk);
+#pragma unroll 4
             for (int g = kvh * HG; g < (kvh + 1) * HG; g++) {
                 const float *q = qv + (size_t)g * D;
                 float dot = 0.0f;
@@ -106,18 +120,16 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         // ---- mixed scores and the running softmax: lane = cell, 32 lanes per head
         for (int idx = tid; idx < ((H * TKR_BC + 63) & ~63); idx += TKR_NT) {      // (whole waves: the shuffles below)
             const int h = idx / TKR_BC < H ? idx / TKR_BC : H - 1, cc = idx & (TKR_BC - 1);
-            const float *tr = a.talk + (size_t)h * H;
+            const float *tr = talk + (size_t)h * H;
             float s = 0.0f;
+#pragma unroll 8
             for (int g = 0; g < H; g++) s = fmaf(tr[g], raw[g * (TKR_BC + 1) + cc], s);
             const bool seen = vis[cc] != 0;
-            float bm = seen ? s : -INFINITY;
-#pragma unroll
-            for (int o = 16; o > 0; o >>= 1) bm = fmaxf(bm, __shfl_xor(bm, o, 64));
+            const float bm = talk_half_max(seen ? s : -INFINITY);
             const float m0 = ms[h], mn = fmaxf(m0, bm);
             const float p = seen ? expf(s - mn) : 0.0f;
-            float ps = p;
-#pragma unroll
-            for (int o = 16; o > 0; o >>= 1) ps += __shfl_xor(ps, o, 64);
+            float ps = row_sum16(p);
+            ps += __shfl_xor(ps, 16, 64);
             const float alpha = m0 == -INFINITY ? 0.0f : expf(m0 - mn);
             if (idx < H * TKR_BC) {
                 pw[h * (TKR_BC + 1) + cc] = p;

@@ -320,6 +320,10 @@ bool Context::init_novorax(std::string &err) {
         // grouped-query layers also cut the block chains of short prompt batches: records for up to 1024 rows x 4 runs of the widest layer
         for (const NvxLayer &L : M.layers)
             if (L.type == NVX_GQ) nvx_part_floats_ = std::max(nvx_part_floats_, std::min<size_t>(T, 1024) * (size_t)L.heads * (size_t)std::max(L.maps, 1) * 4 * (size_t)(L.vdim + 2));
+        // latent layers: steps of up to 512 (row, head) pairs hold 512 / tiles runs of 16 or 32 pairs; batches up to 8 runs of up to 1024 rows
+        for (const NvxLayer &L : M.layers)
+            if (L.type == NVX_LATENT)
+                nvx_part_floats_ = std::max(nvx_part_floats_, std::max<size_t>(512 * 32, std::min<size_t>(T, 1024) * (size_t)L.heads * LATENT_TILE_RUNS) * (size_t)(L.kv_rank + 2));
         for (const NvxLayer &L : M.layers)
             if (L.talk) nvx_part_floats_ = std::max(nvx_part_floats_, std::max<size_t>(TALK_ROW_RUNS, std::min<size_t>(T, 1024) * TALK_TILE_RUNS) * (size_t)L.heads * (size_t)(L.vdim + 2));
         nvx_part_ = (float *)dalloc(nvx_part_floats_ * 4);
@@ -578,7 +582,7 @@ hipError_t Context::run_layers_novorax(int T) {
             aa.window = L.window; aa.scale = L.scale; aa.sink = L.sink; aa.rot_freq = L.rot_freq; aa.rot_mscale = L.rot_mscale; aa.rot_halves = L.rot_halves ? 1 : 0;
             aa.gate = L.off_gate >= 0 ? nvx_a_ + L.off_gate : nullptr; aa.ld_gate = LD_A;
             aa.tok_hi = d_seg_ + 3 * (size_t)cp.n_ubatch;
-            if (nvx_part_ && (long long)T * H <= LATENT_ATTN_SPLIT_MAX_PAIRS) { aa.part = nvx_part_; aa.splits = LATENT_ATTN_SPLITS; }
+            aa.part = nvx_part_; aa.part_floats = nvx_part_floats_; aa.n_kv_hint = n_kv_;
             NVX_TRY(launch_latent_attn(aa, stream_));
             MMBArgs ua;                                         // att[t][h] = W_uv_h lat[t][h]
             ua.x = nvx_lat_; ua.ldx = H * KR; ua.x_zs = KR; ua.w = L.uv.w; ua.ldw = KR; ua.w_zs = (long long)L.vdim * KR;
