@@ -374,7 +374,7 @@ __global__ __launch_bounds__(512) void gq_attn_kernel(GqAttnArgs a) {
 }
 
 __global__ __launch_bounds__(256) void gq_attn_merge_kernel(GqAttnArgs a, int splits) {
-    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[4 * GQ_MAX_D], sums[GQ_MAX_D];
+    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[GQ_MAX_D], sums[GQ_MAX_D];
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, VD = a.vdim;
     const float gate = a.gate ? a.gate[(size_t)t * a.ld_gate + h] : 0.0f;
     const float den = attn_merge_runs(a.part + ((size_t)t * a.H + h) * splits * (size_t)(VD + 2), splits, VD, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);

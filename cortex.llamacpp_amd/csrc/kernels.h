@@ -432,18 +432,26 @@ struct MlstmArgs {
     float *o; int ld_o;                    // [T][H][VD] un-normed outputs
     int H, D, VD; float gate_cap;
     const float *i_bias, *f_bias;          // [H]
-    float *S, *n, *m;                      // state of every slot: [slot][H][D][VD], [slot][H][D], [slot][H]
+    // state of every slot: [slot][H][D][VD]; n and m in one copy per 64-column block, C = mlstm_state_copies(VD): [slot][H][C][D], [slot][H][C]
+    float *S, *n, *m;
     const int32_t *seg_start, *seg_len, *seg_slot; int n_seg;   // runs of consecutive batch rows of one sequence each; no slot twice in a launch
+    int row0, max_len;                     // first row of the first segment (the segments' rows lie side by side); rows of the longest one
+    // work buffers of long segments, by batch row (nullptr: token by token): weighted scores [T][H][64], log decay inside the chunk [T][H], running maximum [T][H],
+    // the same in front of the row's chunk [T][H], n . q [T][H]
+    float *w_A; double *w_F; float *w_m, *w_m0, *w_nq;
 };
+constexpr int MLSTM_CHUNK_MIN_ROWS = 16;  // launches whose longest segment has this many rows work on chunks of 64 tokens
 bool mlstm_shape_ok(int D, int VD);
-// the i / f columns of p become the log gates, in place (biases and the cap applied): once per batch, before the scans
-hipError_t launch_mlstm_gates(const MlstmArgs &a, int T, hipStream_t st);
-hipError_t launch_mlstm_scan(const MlstmArgs &a, hipStream_t st);
+int mlstm_state_copies(int VD);
+// gates (the i / f columns of p are overwritten) and the recurrence over the segments' T rows.  *divided: o is complete; false: o lacks its denominator, which
+// launch_mlstm_out then takes from w_nq and w_m
+hipError_t launch_mlstm(const MlstmArgs &a, int T, bool *divided, hipStream_t st);
 // y[t][h][j] = o / rms(o over the head) * w[h][j] * sigmoid(p[t][off_g + h * VD + j])
+// nq / m ([T][H], both or neither): o is divided by max(|nq|, e^-m) + 1e-6 first
 // w_stride: VD (a weight per head and entry) or 0 (one [VD] weight shared by the heads); gate: sigmoid (MLSTM_GATE_SIGMOID) or silu of the pre-activation
 enum { MLSTM_GATE_SIGMOID = 0, MLSTM_GATE_SILU = 1 };
 hipError_t launch_mlstm_out(const float *o, int ld_o, const float *p, int ld_p, int off_g, const float *w, int T, int H, int VD, float eps, float *y, int ld_y,
-                            hipStream_t st, int w_stride = -1, int gate = MLSTM_GATE_SIGMOID);
+                            hipStream_t st, int w_stride = -1, int gate = MLSTM_GATE_SIGMOID, const float *nq = nullptr, const float *m = nullptr);
 hipError_t launch_mlstm_state_reset(float *S, size_t n_s, float *n, size_t n_n, float *m, size_t n_m, hipStream_t st);   // S = 0, n = 0, m = 0
 
 // ---------------------------------------------------------------- retention (retention.hip)

@@ -227,7 +227,7 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(LatentAttnArgs a) {
 }
 
 __global__ __launch_bounds__(256) void latent_attn_merge_kernel(LatentAttnArgs a, int splits) {
-    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[4 * LA_MAX_L], sums[LA_MAX_L];
+    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[LA_MAX_L], sums[LA_MAX_L];
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, KR = a.kv_rank;
     const float den = attn_merge_runs(a.part + ((size_t)t * a.H + h) * splits * (size_t)(KR + 2), splits, KR, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
     const float inv = latent_out_factor(a, t, h, den);
@@ -290,25 +290,36 @@ __global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs 
         for (int o = 32; o > 0; o >>= 1) hi = max(hi, __shfl_xor(hi, o, 64));
         if (tid == 0) red[0] = hi;
     }
-    // the tile's queries: the folded part as it is, the turning part turned; zeros behind the row's length and for pairs past the end
-    for (int i = tid; i < BQ * LQ; i += 64 * LT_NW) {
-        const int r = i / LQ, d = i - r * LQ, p = p0 + r;
-        float v = 0.0f;
-        if (p < P && d < L) {
-            const int t = p / H, h = p - t * H;
-            if (d < KR) v = a.qa[(size_t)t * a.ld_qa + (size_t)h * KR + d];
-            else {
-                const float *qr = a.q + (size_t)t * a.ld_q + (size_t)h * (a.dim + RT) + a.dim;
-                const int e = d - KR;
-                if (e < a.rot_dims) {
-                    const LatentPair q = latent_pair(e, a.rot_dims, a.rot_halves);
-                    const float ang = (float)a.tok_pos[t] * a.rot_freq[q.pr], c = cosf(ang) * a.rot_mscale, sn = sinf(ang) * a.rot_mscale;
-                    const float u = qr[q.iu], w = qr[q.iv];
-                    v = q.second ? w * c + u * sn : u * c - w * sn;
-                } else v = qr[e];
-            }
+    // the tile's queries (rows of P consecutive pairs: ld_qa = H kv_rank, ld_q = H (dim + rot)): the folded part as it is, the turning part turned; zeros behind
+    // the row's length and for pairs past the end
+    {
+        const int K4 = KR >> 2, QD = a.dim + RT;
+#pragma unroll 8
+        for (int i = tid; i < BQ * K4; i += 64 * LT_NW) {
+            const int r = i / K4, d = (i - r * K4) * 4;
+            f32x4 v = {0.0f, 0.0f, 0.0f, 0.0f};
+            if (p0 + r < P) v = *reinterpret_cast<const f32x4 *>(a.qa + (size_t)(p0 + r) * KR + d);
+            *reinterpret_cast<f32x4 *>(Q + (size_t)r * LDQ + d) = f32x4{v.x * a.scale, v.y * a.scale, v.z * a.scale, v.w * a.scale};
         }
-        Q[(size_t)r * LDQ + d] = v * a.scale;
+        const int half = a.rot_dims >> 1, rest = LQ - KR - a.rot_dims;
+        for (int i = tid; i < BQ * half; i += 64 * LT_NW) {
+            const int r = i / half, pr = i - r * half, p = p0 + r, iu = a.rot_halves ? pr : 2 * pr, iv = a.rot_halves ? pr + half : 2 * pr + 1;
+            float x = 0.0f, y = 0.0f;
+            if (p < P) {
+                const float *qr = a.q + (size_t)p * QD + a.dim;
+                const float u = qr[iu], w = qr[iv];
+                float sn, c;
+                sincosf((float)a.tok_pos[p / H] * a.rot_freq[pr], &sn, &c);
+                sn *= a.rot_mscale * a.scale; c *= a.rot_mscale * a.scale;
+                x = u * c - w * sn; y = w * c + u * sn;
+            }
+            Q[(size_t)r * LDQ + KR + iu] = x;
+            Q[(size_t)r * LDQ + KR + iv] = y;
+        }
+        for (int i = tid; i < BQ * rest; i += 64 * LT_NW) {
+            const int r = i / rest, e = a.rot_dims + i - r * rest;
+            Q[(size_t)r * LDQ + KR + e] = p0 + r < P && e < RT ? a.q[(size_t)(p0 + r) * QD + a.dim + e] * a.scale : 0.0f;
+        }
     }
     __syncthreads();
     int c_begin = 0, c_end = red[0];
@@ -501,7 +512,7 @@ hipError_t launch_latent_attn(const LatentAttnArgs &a, hipStream_t st) {
     const int L = a.kv_rank + a.rot, LQ = (L + 15) & ~15;
     // rows that allow 16-byte loads take the matrix cores: batches in tiles of 64 or 32 (row, head) pairs and blocks of 64 cells, steps of few pairs in
     // tiles of 16 or 32 pairs and blocks of 32 cells
-    if ((L & 3) == 0 && (a.kv_rank & 3) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0) {
+    if ((L & 3) == 0 && (a.kv_rank & 3) == 0 && a.ld_qa == a.H * a.kv_rank && a.ld_q == a.H * (a.dim + a.rot) && (reinterpret_cast<uintptr_t>(a.qa) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0) {
         const long long P = (long long)a.T * a.H;
         if (P <= 16) return launch_latent_tile_nt<1, 32>(a, st);
         if (P <= LATENT_STEP_MAX_PAIRS) return launch_latent_tile_nt<2, 32>(a, st);

@@ -30,11 +30,8 @@ typedef unsigned short u16x8 __attribute__((ext_vector_type(8)));
 typedef unsigned short u16x4 __attribute__((ext_vector_type(4)));
 
 __device__ __forceinline__ float bf2f(unsigned short h) { return __uint_as_float((unsigned)h << 16); }
-__device__ __forceinline__ unsigned short f2bf(float f) {                       // round to nearest even (NaN stays NaN)
-    unsigned u = __float_as_uint(f);
-    if ((u & 0x7fffffffu) > 0x7f800000u) return (unsigned short)((u >> 16) | 0x40);
-    u += 0x7fffu + ((u >> 16) & 1u);
-    return (unsigned short)(u >> 16);
+__device__ __forceinline__ bf16x8 to_bf16(f32x4 a, f32x4 b) {                    // round to nearest even (the packed conversion instructions)
+    return bf16x8{(__bf16)a.x, (__bf16)a.y, (__bf16)a.z, (__bf16)a.w, (__bf16)b.x, (__bf16)b.y, (__bf16)b.z, (__bf16)b.w};
 }
 __device__ __forceinline__ float epi_apply(int epi, float a, float b, float lim = 0.0f) {
     if (epi == MMB_CLAMP_SWIGLU) {
@@ -157,7 +154,8 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
 
 // With the norm prologue the row's sum of squares is gathered in the same pass as the products: y = inv_rms(x) * sum_k w_k (x_k (off + g_k)) - one trip
 // through memory per wave, the scale applied to the finished sum.
-template <bool VEC>
+// TB: rows per pass - 1 for single rows (a short program: a step runs it once per launch, its first fetch is part of the time), else 8
+template <bool VEC, int TB>
 __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n = blockIdx.x * 4 + wave;
@@ -165,7 +163,6 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
     if (n >= a.N) return;
     const unsigned short *wr = v.w + (size_t)n * a.ldw, *wr2 = v.w2 ? v.w2 + (size_t)n * a.ldw : nullptr;
     const bool pn = a.pn_w != nullptr;
-    constexpr int TB = 8;
     for (int t0 = 0; t0 < v.rows; t0 += TB) {
         float acc[TB], acc2[TB], ss[TB];
 #pragma unroll
@@ -342,11 +339,7 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a) {
             if (k0 + 16 * u > klast) break;
             bf16x8 xb[WT];
 #pragma unroll
-            for (int i = 0; i < WT; i++) {
-                const f32x4 x0 = xa[buf][u][i][0], x1 = xa[buf][u][i][1];
-                u16x8 xb16 = {f2bf(x0.x), f2bf(x0.y), f2bf(x0.z), f2bf(x0.w), f2bf(x1.x), f2bf(x1.y), f2bf(x1.z), f2bf(x1.w)};
-                xb[i] = __builtin_bit_cast(bf16x8, xb16);
-            }
+            for (int i = 0; i < WT; i++) xb[i] = to_bf16(xa[buf][u][i][0], xa[buf][u][i][1]);
 #pragma unroll
             for (int i = 0; i < WT; i++)
 #pragma unroll
@@ -401,8 +394,9 @@ hipError_t launch_mmb(const MMBArgs &a, hipStream_t st) {
             else hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 4>), g4, dim3(256), 0, st, a);
             return hipGetLastError();
         }
-        if (vec) hipLaunchKernelGGL(mmb_vec_kernel<true>, grid, dim3(256), 0, st, a);
-        else hipLaunchKernelGGL(mmb_vec_kernel<false>, grid, dim3(256), 0, st, a);
+        if (vec && rows_max == 1) hipLaunchKernelGGL((mmb_vec_kernel<true, 1>), grid, dim3(256), 0, st, a);
+        else if (vec) hipLaunchKernelGGL((mmb_vec_kernel<true, 8>), grid, dim3(256), 0, st, a);
+        else hipLaunchKernelGGL((mmb_vec_kernel<false, 8>), grid, dim3(256), 0, st, a);
         return hipGetLastError();
     }
     if (!a.f32 && vec && (a.K % 16) == 0) {

@@ -204,7 +204,7 @@ constexpr size_t TKT_LDS_MAX = 156 * 1024;
 // HPW: heads a wave finishes; NV = ceil(vdim / 64); the block's heads are [blockIdx.z * 8 * HPW, + 8 * HPW)
 template <int BC, int HPW, int NV>
 __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, int wph) {
-    constexpr int LDR = BC + 4, HS = tkt_head_stride(BC), NS = BC / 16;
+    constexpr int LDR = BC + 4, HS = tkt_head_stride(BC), NS = BC / 16, CT = TKT_BQ * NS / TKT_NW, HT = BC == 64 ? 2 : 4;   // (at most 16 HT heads)
     extern __shared__ float lds[];
     const int H = a.H, G = a.G, D = a.dim, VD = a.vdim, HG = H / G;
     float *S = lds;                                             // [H][16][LDR], head stride HS
@@ -297,26 +297,41 @@ __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, in
             for (int s = 0; s < NS / 2; s++) *reinterpret_cast<f32x4 *>(S + (size_t)g * HS + l16 * LDR + 16 * (s0 + s) + 4 * lg) = acc[s];
         }
         __syncthreads();
-        // ---- mix
-        for (int ct = wave; ct < TKT_BQ * NS; ct += TKT_NW) {
-            float *col = S + (ct / NS) * LDR + (ct % NS) * 16 + l16;
-            f32x4 mx[4];                                        // (up to 64 heads)
+        // ---- mix: the wave's column pieces side by side, so that every fragment of talk is fetched once and its trip overlaps their products
+        {
+            f32x4 mx[CT][HT];
 #pragma unroll
-            for (int ht = 0; ht < 4; ht++) mx[ht] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+            for (int i = 0; i < CT; i++)
+#pragma unroll
+                for (int ht = 0; ht < HT; ht++) mx[i][ht] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+            const auto fragment = [&](int g0, float (&w)[HT]) {
+#pragma unroll
+                for (int ht = 0; ht < HT; ht++) w[ht] = g0 + lg < H && 16 * ht + l16 < H ? a.talk[(size_t)(16 * ht + l16) * H + g0 + lg] : 0.0f;
+            };
+            float w[HT], wn[HT];
+            fragment(0, w);
             for (int g0 = 0; g0 < H; g0 += 4) {
-                const int g = g0 + lg;
-                const float b = g < H ? col[(size_t)g * HS] : 0.0f;
+                fragment(g0 + 4, wn);
+                const bool in = g0 + lg < H;
 #pragma unroll
-                for (int ht = 0; ht < 4; ht++) {
-                    if (16 * ht >= H) continue;
-                    const float w = g < H && 16 * ht + l16 < H ? a.talk[(size_t)(16 * ht + l16) * H + g] : 0.0f;
-                    mx[ht] = __builtin_amdgcn_mfma_f32_16x16x4f32(w, b, mx[ht], 0, 0, 0);
+                for (int i = 0; i < CT; i++) {
+                    const int ct = wave + TKT_NW * i;
+                    const float b = in ? S[(size_t)(g0 + lg) * HS + (ct / NS) * LDR + (ct % NS) * 16 + l16] : 0.0f;
+#pragma unroll
+                    for (int ht = 0; ht < HT; ht++) if (16 * ht < H) mx[i][ht] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[ht], b, mx[i][ht], 0, 0, 0);
                 }
+#pragma unroll
+                for (int ht = 0; ht < HT; ht++) w[ht] = wn[ht];
             }
 #pragma unroll
-            for (int ht = 0; ht < 4; ht++)
+            for (int i = 0; i < CT; i++) {
+                const int ct = wave + TKT_NW * i;
+                float *col = S + (ct / NS) * LDR + (ct % NS) * 16 + l16;
 #pragma unroll
-                for (int r = 0; r < 4; r++) if (16 * ht + 4 * lg + r < H) col[(size_t)(16 * ht + 4 * lg + r) * HS] = mx[ht][r];
+                for (int ht = 0; ht < HT; ht++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) if (16 * ht + 4 * lg + r < H) col[(size_t)(16 * ht + 4 * lg + r) * HS] = mx[i][ht][r];
+            }
         }
         __syncthreads();
         // ---- softmax and values
@@ -472,7 +487,7 @@ hipError_t launch_talk_attn(const GqAttnArgs &a, hipStream_t st) {
     const auto al16 = [](const void *p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
     const bool vec = (a.dim & 3) == 0 && (a.vdim & 3) == 0 && (a.ld_q & 3) == 0 && (a.ld_out & 3) == 0 && al16(a.q) && al16(a.out) && al16(a.cache);
     if (a.T >= 16 && vec && (a.dim & 15) == 0 && a.vdim <= 256 && a.H <= 64) {
-        if (tkt_lds_floats(a.H, 64) * sizeof(float) <= TKT_LDS_MAX) return launch_talk_tile_bc<64>(a, st);
+        if (a.H <= 32 && tkt_lds_floats(a.H, 64) * sizeof(float) <= TKT_LDS_MAX) return launch_talk_tile_bc<64>(a, st);
         if (tkt_lds_floats(a.H, 32) * sizeof(float) <= TKT_LDS_MAX) return launch_talk_tile_bc<32>(a, st);
     }
     if (vec) {

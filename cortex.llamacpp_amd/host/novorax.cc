@@ -178,6 +178,7 @@ Model *novorax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
             L.f_bias = ld.vec(pm + "f.b", H);
             L.mix_norm = ld.vec(pm + "norm", H * L.vdim);
             L.o = ld.rows({{pm + "o", W}}, H * L.vdim);
+            M.max_mlstm_heads = std::max(M.max_mlstm_heads, H);
             M.max_proj = std::max(M.max_proj, L.proj.N);
             M.max_att = std::max(M.max_att, H * L.vdim);
         } else { err = "configuration: layer " + std::to_string(il) + " has unknown type '" + type + "'"; return nullptr; }
@@ -251,7 +252,7 @@ Model *novorax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
 static void nvx_state_sizes(const NvxLayer &L, size_t &s_sz, size_t &n_sz, size_t &m_sz) {
     if (L.type == NVX_GQ) { s_sz = m_sz = 0; n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.conv_channels(); return; }   // (attention: the convolution's last inputs)
     s_sz = (size_t)L.heads * L.dim * L.vdim;
-    if (L.type == NVX_MLSTM) { n_sz = (size_t)L.heads * L.dim; m_sz = (size_t)L.heads; }
+    if (L.type == NVX_MLSTM) { const size_t c = (size_t)mlstm_state_copies(L.vdim); n_sz = (size_t)L.heads * L.dim * c; m_sz = (size_t)L.heads * c; }
     else if (L.type == NVX_RETENTION) { n_sz = 0; m_sz = 0; }
     else { n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.delta_channels(); m_sz = 0; }
 }
@@ -344,6 +345,13 @@ bool Context::init_novorax(std::string &err) {
         nvx_rw_ = (float *)dalloc(T * TOP * 4);
         nvx_rwg_ = (float *)dalloc(T * TOP * 4);
         if (!nvx_xg_ || !nvx_yg_ || !nvx_ids_ || !nvx_meta_ || !nvx_slot_ || !nvx_tokof_ || !nvx_rw_ || !nvx_rwg_) { err = "expert batch buffers allocation failed"; return false; }
+    }
+    if (M.max_mlstm_heads > 0) {
+        const size_t TH = T * (size_t)M.max_mlstm_heads;
+        nvx_mw_A_ = (float *)dalloc(TH * 64 * 4);
+        nvx_mw_F_ = (double *)dalloc(TH * 8);
+        nvx_mw_v_ = (float *)dalloc(3 * TH * 4);
+        if (!nvx_mw_A_ || !nvx_mw_F_ || !nvx_mw_v_) { err = "recurrence work buffers allocation failed"; return false; }
     }
     if (M.max_shared_ff > 0) {
         nvx_sh_ = (float *)dalloc(T * (size_t)M.max_shared_ff * 4);
@@ -596,13 +604,19 @@ hipError_t Context::run_layers_novorax(int T) {
             MlstmArgs ma{};
             ma.p = nvx_a_; ma.ld_p = LD_P; ma.o = nvx_o_; ma.ld_o = H * L.vdim; ma.H = H; ma.D = L.dim; ma.VD = L.vdim; ma.gate_cap = L.gate_cap;
             ma.i_bias = L.i_bias; ma.f_bias = L.f_bias; ma.S = nvx_S_[(size_t)r.plane]; ma.n = nvx_n_[(size_t)r.plane]; ma.m = nvx_m_[(size_t)r.plane];
-            NVX_TRY(launch_mlstm_gates(ma, T, stream_));
+            ma.w_A = nvx_mw_A_; ma.w_F = nvx_mw_F_; ma.w_m = nvx_mw_v_; ma.w_m0 = nvx_mw_v_ + (size_t)cp.n_ubatch * M.max_mlstm_heads; ma.w_nq = ma.w_m0 + (size_t)cp.n_ubatch * M.max_mlstm_heads;
             const size_t TU = cp.n_ubatch;
             for (const auto &wv : nvx_waves_) {
                 ma.seg_start = d_seg_ + wv.first; ma.seg_len = d_seg_ + TU + wv.first; ma.seg_slot = d_seg_ + 2 * TU + wv.first; ma.n_seg = wv.second;
-                NVX_TRY(launch_mlstm_scan(ma, stream_));
+                const int32_t *start = h_seg_ + wv.first, *len = h_seg_ + TU + wv.first;
+                const int rows = start[wv.second - 1] + len[wv.second - 1] - start[0];
+                ma.row0 = start[0]; ma.max_len = *std::max_element(len, len + wv.second);
+                bool divided = true;
+                NVX_TRY(launch_mlstm(ma, rows, &divided, stream_));
+                const size_t r0 = (size_t)start[0], ldo = (size_t)H * L.vdim;
+                NVX_TRY(launch_mlstm_out(nvx_o_ + r0 * ldo, (int)ldo, nvx_a_ + r0 * LD_P, LD_P, 2 * H * L.dim + H * L.vdim, L.mix_norm, rows, H, L.vdim, eps, nvx_att_ + r0 * ldo, (int)ldo, stream_,
+                                         -1, MLSTM_GATE_SIGMOID, divided ? nullptr : ma.w_nq + r0 * H, divided ? nullptr : ma.w_m + r0 * H));
             }
-            NVX_TRY(launch_mlstm_out(nvx_o_, H * L.vdim, nvx_a_, LD_P, 2 * H * L.dim + H * L.vdim, L.mix_norm, T, H, L.vdim, eps, nvx_att_, H * L.vdim, stream_));
             NVX_TRY(nvx_close_linear(L.o, nvx_att_, H * L.vdim, T, L.norm1b));
             prof_mark("mlstm");
         } else if (L.type == NVX_GQ) {

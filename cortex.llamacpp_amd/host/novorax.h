@@ -158,7 +158,7 @@ struct NovoraxModel {
     int max_window = 0;             // largest window of the windowed attention layers, 0 if one of them sees every earlier cell (scan bounds)
     int max_shared_ff = 0;
     // largest sizes over the layers (activation buffers)
-    int max_down = 0, max_q_rank = 0, max_q = 0, max_qa = 0, max_att = 0, max_proj = 0, max_ff = 0, max_top = 0, max_expert = 0;
+    int max_down = 0, max_q_rank = 0, max_q = 0, max_qa = 0, max_att = 0, max_proj = 0, max_ff = 0, max_top = 0, max_expert = 0, max_mlstm_heads = 0;
 };
 
 }  // namespace mi355

@@ -208,10 +208,11 @@ class Context {
     void nvx_state_reset(int seq);                          // seq < 0: every slot
     void nvx_state_copy(int src, int dst);
     std::vector<float *> nvx_cache_;                        // [attention run] [n_ctx][the layer's cache_row()]
-    std::vector<float *> nvx_S_, nvx_n_, nvx_m_;            // [recurrent run] [n_seq_max][H][D][VD]; mlstm: [..][H][D], [..][H]; delta rule and attention with a convolution: [..][taps - 1][channels] in nvx_n_
+    std::vector<float *> nvx_S_, nvx_n_, nvx_m_;            // [recurrent run] [n_seq_max][H][D][VD]; mlstm: [..][H][copies][D], [..][H][copies]; delta rule and attention with a convolution: [..][taps - 1][channels] in nvx_n_
     std::vector<uint64_t> nvx_seq_len_;                     // tokens every sequence id has been fed (the recurrent state cannot be cut back)
     float *nvx_x0_ = nullptr, *nvx_xcat_ = nullptr, *nvx_y_ = nullptr, *nvx_a_ = nullptr, *nvx_cq_ = nullptr, *nvx_q_ = nullptr, *nvx_qa_ = nullptr, *nvx_lat_ = nullptr;
     float *nvx_vcs_ = nullptr;                              // [n_ubatch][widest turned value head]: cos | sin per pair of every token's value turn
+    float *nvx_mw_A_ = nullptr, *nvx_mw_v_ = nullptr; double *nvx_mw_F_ = nullptr;   // the mLSTM's work buffers for long segments (MlstmArgs)
     float *nvx_part_ = nullptr;                             // records of attention scans that were cut into runs (single-token steps; short prompt batches)
     size_t nvx_part_floats_ = 0;
     float *nvx_att_ = nullptr, *nvx_o_ = nullptr, *nvx_ff_ = nullptr, *nvx_xg_ = nullptr, *nvx_yg_ = nullptr;

@@ -84,6 +84,7 @@ Model *vuzazen_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
             L.i_bias = ld.vec(pm + "i.b", H);
             L.f_bias = ld.vec(pm + "f.b", H);
             L.mix_norm = ld.vec(pm + "norm", H * VD);
+            M.max_mlstm_heads = std::max(M.max_mlstm_heads, H);
             M.max_proj = std::max(M.max_proj, L.proj.N);
             active_bytes += (uint64_t)L.proj.N * W * 2;
         } else if (type == "latent_attention") {
