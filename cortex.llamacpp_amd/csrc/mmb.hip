@@ -9,14 +9,15 @@
 // Three kernels behind one launch:
 //   * mmb_vec   - up to a few dozen rows: one wave per output column walks K with 16-byte weight loads, the activations stay f32.  Weight-stream bound, the
 //                 form of every single-token step in both precisions.
-//   * mmb_mfma  - batches in bf16 mode: activations rounded to bf16 in registers, v_mfma_f32_32x32x16_bf16, one 32 x 32 (or 64 x 64) tile per wave, both operands
-//                 read K-contiguous straight into the matrix-core register layout (lane = (row, k-group of 8)).
+//   * mmb_mfma  - batches in bf16 mode: LDS-tiled, activations rounded to bf16 on the way in, v_mfma_f32_32x32x16_bf16, f32 accumulation.
 //   * mmb_f32   - batches in f32 mode (and every shape the other two refuse): LDS-tiled, v_fma_f32 only - products of an f32 activation and a bf16 weight
 //                 widened exactly, no reduced-precision matrix mode anywhere.
 // Epilogues: store | relu(y)^2 | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = W x capped from above and u = W2 x clamped
 // to +- the same limit (the gated ones: two weight sets, one pass over the activations).  Around the epilogue, each optional: a factor per row on W x (and W2 x)
 // - linear layers without a bias: the row of X itself times that number -, an f32 bias per output column in front of it, a residual row added behind it.  A
 // grouped batch may read its rows of X, and write its rows of Y, through maps (no gather in front of the launch, no scatter behind it).
+#include <type_traits>
+
 #include "kernels.h"
 
 namespace mi355 {
@@ -26,13 +27,11 @@ namespace {
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
 typedef unsigned short u16x8 __attribute__((ext_vector_type(8)));
 typedef unsigned short u16x4 __attribute__((ext_vector_type(4)));
 
 __device__ __forceinline__ float bf2f(unsigned short h) { return __uint_as_float((unsigned)h << 16); }
-__device__ __forceinline__ bf16x8 to_bf16(f32x4 a, f32x4 b) {                    // round to nearest even (the packed conversion instructions)
-    return bf16x8{(__bf16)a.x, (__bf16)a.y, (__bf16)a.z, (__bf16)a.w, (__bf16)b.x, (__bf16)b.y, (__bf16)b.z, (__bf16)b.w};
-}
 __device__ __forceinline__ float epi_apply(int epi, float a, float b, float lim = 0.0f) {
     if (epi == MMB_CLAMP_SWIGLU) {
         const float g = fminf(a, lim), u = fminf(fmaxf(b, -lim), lim);
@@ -290,87 +289,127 @@ __global__ __launch_bounds__(256) void mmb_f32_kernel(MMBArgs a) {
     }
 }
 
-// ---------------------------------------------------------------- batches, bf16 on the matrix cores: a wave owns WT x WT tiles of 32 x 32 outputs
-template <int WT, bool GATED>
-__global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a) {
+// ---------------------------------------------------------------- batches, bf16 on the matrix cores
+// 64 RN weight rows x 64 RT rows of X per workgroup, 64 of k per stage: both operands through LDS (two buffers, one barrier per stage; rows padded to an odd number
+// of 16-byte pieces), X rounded to bf16 once on its way there, the stages after next already on their way from memory in registers.  A wave owns 32 RN x 32 RT
+// outputs (v_mfma_f32_32x32x16_bf16).  The workgroups that read the same weight rows sit on the same XCD, side by side: its L2 fetches them once.
+constexpr int MMT_K = 64, MMT_LD = MMT_K + 8;                   // bf16 per LDS row
+template <int RN, int RT, bool GATED>
+__global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a, int n_tiles, int t_tiles) {
+    constexpr int TN = 64 * RN, TT = 64 * RT, NW = 2 * RN, NX = 4 * RT;   // 16-byte loads per thread and stage
+    __shared__ __attribute__((aligned(16))) unsigned short sW[2][TN][MMT_LD], sW2[GATED ? 2 : 1][GATED ? TN : 1][MMT_LD], sX[2][TT][MMT_LD];
     const ZView v = z_view(a, blockIdx.z);
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int m = lane & 31, kg = lane >> 5;
-    const int n0 = blockIdx.x * (64 * WT) + (wave & 1) * (32 * WT), t0 = blockIdx.y * (64 * WT) + (wave >> 1) * (32 * WT);
-    if (n0 >= a.N || t0 >= v.rows) return;                      // (wave-uniform, no barriers in this kernel)
-    const unsigned short *wr[WT], *wr2[WT];
-    const float *xr[WT];
+    // block -> tile: consecutive blocks go to the XCDs in turn; the t tiles of one n tile take consecutive turns of ONE of them
+    const int xcd = blockIdx.x & 7, turn = blockIdx.x >> 3, nt = xcd + 8 * (turn / t_tiles), n0 = nt * TN, t0 = (turn % t_tiles) * TT;
+    if (nt >= n_tiles || t0 >= v.rows) return;                  // (uniform: before any barrier)
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, m = lane & 31, kg = lane >> 5;
+    const int r4 = tid >> 2, q4 = tid & 3;
+    const unsigned short *wr[RN], *wr2[RN];
+    const float *xr[RT];
 #pragma unroll
-    for (int i = 0; i < WT; i++) {
-        const int n = n0 + 32 * i + m, t = t0 + 32 * i + m;     // rows past the end read the last row; their results are never stored
-        wr[i] = v.w + (size_t)(n < a.N ? n : a.N - 1) * a.ldw + 8 * kg;
-        wr2[i] = GATED ? v.w2 + (size_t)(n < a.N ? n : a.N - 1) * a.ldw + 8 * kg : nullptr;
-        xr[i] = x_row(a, v, t < v.rows ? t : v.rows - 1) + 8 * kg;
+    for (int i = 0; i < RN; i++) {
+        const int n = n0 + 64 * i + r4 < a.N ? n0 + 64 * i + r4 : a.N - 1;          // rows past the end read the last row; their results are never stored
+        wr[i] = v.w + (size_t)n * a.ldw + 8 * q4;
+        wr2[i] = GATED ? v.w2 + (size_t)n * a.ldw + 8 * q4 : nullptr;
     }
-    f32x16 acc[WT][WT], acc2[GATED ? WT : 1][GATED ? WT : 1];
 #pragma unroll
-    for (int i = 0; i < WT; i++)
+    for (int i = 0; i < RT; i++) { const int t = t0 + 64 * i + r4; xr[i] = x_row(a, v, t < v.rows ? t : v.rows - 1) + 4 * q4; }
+    f32x16 acc[RN][RT], acc2[GATED ? RN : 1][GATED ? RT : 1];
 #pragma unroll
-        for (int j = 0; j < WT; j++)
+    for (int i = 0; i < RN; i++)
+#pragma unroll
+        for (int j = 0; j < RT; j++)
 #pragma unroll
             for (int r = 0; r < 16; r++) { acc[i][j][r] = 0.0f; if (GATED) acc2[i][j][r] = 0.0f; }
-    // PD steps of k are requested together, and the next PD while these are multiplied: a request per step in the chain would wait a memory round trip
-    // for every 16 of k.  Steps past K read the row's last step again and are never multiplied.
-    constexpr int PD = WT == 1 ? 4 : 2;
-    bf16x8 wa[2][PD][WT], wb[2][PD][GATED ? WT : 1];
-    f32x4 xa[2][PD][WT][2];
-    const int klast = a.K - 16;
-    const auto request = [&](int buf, int k0) {
+    u16x8 lw[2][NW], lw2[2][GATED ? NW : 1];
+    f32x4 lx[2][NX];
+    const auto request = [&](auto set, int k0) {                // (K is a multiple of 16: a 16-byte piece is inside a row or behind its end)
+        constexpr int b = decltype(set)::value;
 #pragma unroll
-        for (int u = 0; u < PD; u++) {
-            const int k = k0 + 16 * u <= klast ? k0 + 16 * u : klast;
+        for (int i = 0; i < NW; i++) {
+            const int k = k0 + 32 * (i & 1);
+            const bool in = k + 8 * q4 < a.K;
+            lw[b][i] = in ? *reinterpret_cast<const u16x8 *>(wr[i >> 1] + k) : u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+            if (GATED) lw2[b][i] = in ? *reinterpret_cast<const u16x8 *>(wr2[i >> 1] + k) : u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+        }
 #pragma unroll
-            for (int i = 0; i < WT; i++) {
-                wa[buf][u][i] = *reinterpret_cast<const bf16x8 *>(wr[i] + k);
-                if (GATED) wb[buf][u][i] = *reinterpret_cast<const bf16x8 *>(wr2[i] + k);
-                xa[buf][u][i][0] = *reinterpret_cast<const f32x4 *>(xr[i] + k);
-                xa[buf][u][i][1] = *reinterpret_cast<const f32x4 *>(xr[i] + k + 4);
-            }
+        for (int i = 0; i < NX; i++) {
+            const int k = k0 + 16 * (i & 3);
+            lx[b][i] = k < a.K ? *reinterpret_cast<const f32x4 *>(xr[i >> 2] + k) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
         }
     };
-    const auto multiply = [&](int buf, int k0) {
+    const auto stage = [&](auto set) {
+        constexpr int b = decltype(set)::value;
 #pragma unroll
-        for (int u = 0; u < PD; u++) {
-            if (k0 + 16 * u > klast) break;
-            bf16x8 xb[WT];
+        for (int i = 0; i < NW; i++) {
+            *reinterpret_cast<u16x8 *>(&sW[b][64 * (i >> 1) + r4][32 * (i & 1) + 8 * q4]) = lw[b][i];
+            if (GATED) *reinterpret_cast<u16x8 *>(&sW2[b][64 * (i >> 1) + r4][32 * (i & 1) + 8 * q4]) = lw2[b][i];
+        }
 #pragma unroll
-            for (int i = 0; i < WT; i++) xb[i] = to_bf16(xa[buf][u][i][0], xa[buf][u][i][1]);
+        for (int i = 0; i < NX; i++) {
+            const f32x4 x = lx[b][i];
+            *reinterpret_cast<bf16x4 *>(&sX[b][64 * (i >> 2) + r4][16 * (i & 3) + 4 * q4]) = bf16x4{(__bf16)x.x, (__bf16)x.y, (__bf16)x.z, (__bf16)x.w};   // (round to nearest even)
+        }
+    };
+    const auto multiply = [&](auto set) {
+        constexpr int b = decltype(set)::value;
 #pragma unroll
-            for (int i = 0; i < WT; i++)
+        for (int u = 0; u < MMT_K / 16; u++) {
+            bf16x8 wa[RN], wb[RN], xb[RT];
 #pragma unroll
-                for (int j = 0; j < WT; j++) {
-                    acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wa[buf][u][i], xb[j], acc[i][j], 0, 0, 0);
-                    if (GATED) acc2[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wb[buf][u][i], xb[j], acc2[i][j], 0, 0, 0);
+            for (int i = 0; i < RN; i++) {
+                const int n = (wave & 1) * 32 * RN + 32 * i + m;
+                wa[i] = *reinterpret_cast<const bf16x8 *>(&sW[b][n][16 * u + 8 * kg]);
+                if (GATED) wb[i] = *reinterpret_cast<const bf16x8 *>(&sW2[b][n][16 * u + 8 * kg]);
+            }
+#pragma unroll
+            for (int j = 0; j < RT; j++) xb[j] = *reinterpret_cast<const bf16x8 *>(&sX[b][(wave >> 1) * 32 * RT + 32 * j + m][16 * u + 8 * kg]);
+#pragma unroll
+            for (int i = 0; i < RN; i++)
+#pragma unroll
+                for (int j = 0; j < RT; j++) {
+                    acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wa[i], xb[j], acc[i][j], 0, 0, 0);
+                    if (GATED) acc2[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wb[i], xb[j], acc2[i][j], 0, 0, 0);
                 }
         }
     };
-    request(0, 0);
-    for (int k0 = 0; k0 < a.K; k0 += 32 * PD) {
-        request(1, k0 + 16 * PD);
-        multiply(0, k0);
-        request(0, k0 + 32 * PD);
-        multiply(1, k0 + 16 * PD);
+    const std::integral_constant<int, 0> s0;
+    const std::integral_constant<int, 1> s1;
+    request(s0, 0);
+    request(s1, MMT_K);                                         // (a stage past K is all zeros)
+    for (int k0 = 0; k0 < a.K; k0 += 2 * MMT_K) {
+        stage(s0);
+        if (k0 + 2 * MMT_K < a.K) request(s0, k0 + 2 * MMT_K);
+        __syncthreads();
+        multiply(s0);
+        if (k0 + MMT_K >= a.K) break;
+        stage(s1);
+        if (k0 + 3 * MMT_K < a.K) request(s1, k0 + 3 * MMT_K);
+        __syncthreads();
+        multiply(s1);
     }
     // register r of a lane: weight row (r & 3) + 8 (r >> 2) + 4 kg of the tile, token = lane & 31
 #pragma unroll
-    for (int i = 0; i < WT; i++)
+    for (int j = 0; j < RT; j++) {
+        const int t = t0 + (wave >> 1) * 32 * RT + 32 * j + m;
+        if (t >= v.rows) continue;
+        const size_t yr = y_row(a, v, t);
+        const float rs = a.row_scale ? a.row_scale[v.y0 + t] : 1.0f;
 #pragma unroll
-        for (int j = 0; j < WT; j++) {
-            const int t = t0 + 32 * j + m;
-            if (t >= v.rows) continue;
-            const size_t yr = y_row(a, v, t);
-            const float rs = a.row_scale ? a.row_scale[v.y0 + t] : 1.0f;
+        for (int i = 0; i < RN; i++)
 #pragma unroll
             for (int r = 0; r < 16; r++) {
-                const int n = n0 + 32 * i + (r & 3) + 8 * (r >> 2) + 4 * kg;
+                const int n = n0 + (wave & 1) * 32 * RN + 32 * i + (r & 3) + 8 * (r >> 2) + 4 * kg;
                 if (n < a.N) y_store(a, v, yr, n, acc[i][j][r], GATED ? acc2[i][j][r] : 0.0f, rs, v.resid ? v.resid[yr + n] : 0.0f);
             }
-        }
+    }
+}
+
+template <int RN, int RT, bool GATED>
+static hipError_t launch_mmb_mfma(const MMBArgs &a, int rows_max, hipStream_t st) {
+    const int nt = (a.N + 64 * RN - 1) / (64 * RN), tt = (rows_max + 64 * RT - 1) / (64 * RT);
+    hipLaunchKernelGGL((mmb_mfma_kernel<RN, RT, GATED>), dim3((unsigned)((nt + 7) / 8 * 8 * tt), 1, (unsigned)a.nz), dim3(256), 0, st, a, nt, tt);
+    return hipGetLastError();
 }
 
 }  // namespace
@@ -400,16 +439,17 @@ hipError_t launch_mmb(const MMBArgs &a, hipStream_t st) {
         return hipGetLastError();
     }
     if (!a.f32 && vec && (a.K % 16) == 0) {
-        const dim3 big((unsigned)((a.N + 127) / 128), (unsigned)((rows_max + 127) / 128), (unsigned)a.nz);
-        // (a grouped batch sizes its grid for the most rows ONE expert could hold; what counts for filling the device is the rows an expert holds on average)
-        const unsigned rows_avg = a.meta ? (unsigned)((a.T + a.nz - 1) / a.nz) : (unsigned)rows_max;
-        if (big.x * ((rows_avg + 127) / 128) * big.z >= (a.meta ? 256u : 512u) && !gated) hipLaunchKernelGGL((mmb_mfma_kernel<2, false>), big, dim3(256), 0, st, a);
-        else {
-            const dim3 grid((unsigned)((a.N + 63) / 64), (unsigned)((rows_max + 63) / 64), (unsigned)a.nz);
-            if (gated) hipLaunchKernelGGL((mmb_mfma_kernel<1, true>), grid, dim3(256), 0, st, a);
-            else hipLaunchKernelGGL((mmb_mfma_kernel<1, false>), grid, dim3(256), 0, st, a);
-        }
-        return hipGetLastError();
+        // the tile by what a stage costs a CU in bytes fetched (KB: weights 8 RN, X 16 RT) times the rounds of workgroups the device needs; a grouped batch sizes
+        // its grid for the most rows ONE expert could hold, what counts is the rows an expert holds on average
+        const long long rows = a.meta ? (a.T + a.nz - 1) / a.nz : rows_max;
+        const auto rounds = [&](int rn, int rt, int kb) {
+            const double wg = (double)((a.N + 64 * rn - 1) / (64 * rn)) * (double)((rows + 64 * rt - 1) / (64 * rt)) * a.nz;
+            return (wg > 256.0 ? wg / 256.0 : 1.0) * kb;
+        };
+        if (gated) return rounds(1, 2, 48) < rounds(1, 1, 32) ? launch_mmb_mfma<1, 2, true>(a, rows_max, st) : launch_mmb_mfma<1, 1, true>(a, rows_max, st);
+        const double r11 = rounds(1, 1, 24), r21 = rounds(2, 1, 32), r22 = rounds(2, 2, 48);
+        if (r22 <= r11 && r22 <= r21) return launch_mmb_mfma<2, 2, false>(a, rows_max, st);
+        return r21 <= r11 ? launch_mmb_mfma<2, 1, false>(a, rows_max, st) : launch_mmb_mfma<1, 1, false>(a, rows_max, st);
     }
     const dim3 grid((unsigned)((a.N + 63) / 64), (unsigned)((rows_max + 63) / 64), (unsigned)a.nz);
     if (gated) hipLaunchKernelGGL(mmb_f32_kernel<true>, grid, dim3(256), 0, st, a);
