@@ -1,15 +1,16 @@
 // attn_merge_dev.h — joining the records of an attention scan that was cut into runs of cells: record s = [maximum | sum | n weighted values] of run s.
-// A workgroup of 256 threads per (row, head): lane s of every wave holds run s's maximum and sum (one trip to memory for all runs), then thread = value column.
+// A workgroup of NT threads per (row, head) - many threads where few rows are joined and one trip to memory is all that counts -: lane s of every wave holds run s's maximum and sum (one trip to memory for all runs), then thread = value column.
 #pragma once
 
 #include <hip/hip_runtime.h>
 
 namespace mi355 {
 
-constexpr int ATTN_MERGE_MAX_RUNS = 64;
+constexpr int ATTN_MERGE_MAX_RUNS = 64, ATTN_MERGE_FEW = 512;   // up to ATTN_MERGE_FEW (row, head) pairs are joined by 1024 threads each
 
 // sums[i] (LDS, n floats) = sum over the runs of e^(maximum_s - M) * value_s[i]; returns the softmax denominator under M = the maximum of all runs and of the
-// sink (sink = -inf: none).  part: max(n, 256) floats of LDS; the caller reads sums behind the barrier this function ends with.
+// sink (sink = -inf: none).  part: max(NT / 256 * n, NT) floats of LDS; the caller reads sums behind the barrier this function ends with.
+template <int NT>
 __device__ __forceinline__ float attn_merge_runs(const float *rec, int splits, int n, float sink, float *fac, float *part, float *sums) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const size_t stride = (size_t)n + 2;
@@ -25,8 +26,8 @@ __device__ __forceinline__ float attn_merge_runs(const float *rec, int splits, i
     if (sink > -INFINITY) den += expf(sink - M);
     if (wave == 0) fac[lane] = f;
     __syncthreads();
-    // columns side by side as far as they go; narrow records share the runs among 2 or 4 groups of threads, whose sums meet in LDS
-    const int groups = n <= 64 ? 4 : n <= 128 ? 2 : 1, width = 256 / groups, grp = tid / width;
+    // columns side by side; groups of threads share the runs, their sums meet in LDS
+    const int width = n <= 64 ? 64 : n <= 128 ? 128 : 256, groups = NT / width, grp = tid / width;
     for (int i = tid - grp * width; i < n; i += width) {
         float o = 0.0f;
 #pragma unroll 8
@@ -34,7 +35,11 @@ __device__ __forceinline__ float attn_merge_runs(const float *rec, int splits, i
         part[grp * n + i] = o;
     }
     __syncthreads();
-    for (int i = tid; i < n; i += 256) sums[i] = groups == 1 ? part[i] : groups == 2 ? part[i] + part[n + i] : (part[i] + part[n + i]) + (part[2 * n + i] + part[3 * n + i]);
+    for (int i = tid; i < n; i += NT) {
+        float o = part[i];
+        for (int g = 1; g < groups; g++) o += part[g * n + i];
+        sums[i] = o;
+    }
     __syncthreads();
     return den;
 }

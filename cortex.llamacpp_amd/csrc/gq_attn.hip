@@ -61,7 +61,25 @@ __global__ __launch_bounds__(NT) void gq_prep_kernel(GqPrepArgs a) {
     if (CONV) {
         const int C = NQ + NK + NV, back = a.conv_taps - 1, ago = a.tok_ago[t];
         float *state = a.conv_state + (size_t)a.tok_slot[t] * back * C;
-        for (int i = tid; i < C; i += NT) {
+        const bool vec = ((C | a.ld_p) & 3) == 0 && ((reinterpret_cast<uintptr_t>(a.p) | reinterpret_cast<uintptr_t>(a.conv_wt) | reinterpret_cast<uintptr_t>(a.conv_state)) & 15) == 0;
+        if (vec) {                                              // four channels per thread
+            for (int i = 4 * tid; i < C; i += 4 * NT) {
+                float4 s = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+                const auto input = [&](int b) {
+                    return *reinterpret_cast<const float4 *>(b <= ago ? a.p + (size_t)(t - b) * a.ld_p + i : state + (size_t)(back - (b - ago)) * C + i);
+                };
+#pragma unroll 4
+                for (int j = 0; j <= back; j++) {
+                    const float4 w = *reinterpret_cast<const float4 *>(a.conv_wt + (size_t)j * C + i), u = input(back - j);
+                    s.x = fmaf(w.x, u.x, s.x); s.y = fmaf(w.y, u.y, s.y); s.z = fmaf(w.z, u.z, s.z); s.w = fmaf(w.w, u.w, s.w);
+                }
+                *reinterpret_cast<float4 *>(conv_row + i) = s;
+                if (a.conv_move && back > 0) {
+                    for (int j = 0; j + 1 < back; j++) *reinterpret_cast<float4 *>(state + (size_t)j * C + i) = *reinterpret_cast<const float4 *>(state + (size_t)(j + 1) * C + i);
+                    *reinterpret_cast<float4 *>(state + (size_t)(back - 1) * C + i) = *reinterpret_cast<const float4 *>(qr + i);
+                }
+            }
+        } else for (int i = tid; i < C; i += NT) {
             float s = 0.0f;
             for (int j = 0; j <= back; j++) {
                 const int b = back - j;                          // (tokens back: a row of the batch, or - before the segment's first row - what the slot remembers)
@@ -373,18 +391,19 @@ __global__ __launch_bounds__(512) void gq_attn_kernel(GqAttnArgs a) {
     }
 }
 
-__global__ __launch_bounds__(256) void gq_attn_merge_kernel(GqAttnArgs a, int splits) {
-    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[GQ_MAX_D], sums[GQ_MAX_D];
+template <int NT>
+__global__ __launch_bounds__(NT) void gq_attn_merge_kernel(GqAttnArgs a, int splits) {
+    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[NT / 256 * GQ_MAX_D], sums[GQ_MAX_D];
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, VD = a.vdim;
     const float gate = a.gate ? a.gate[(size_t)t * a.ld_gate + h] : 0.0f;
-    const float den = attn_merge_runs(a.part + ((size_t)t * a.H + h) * splits * (size_t)(VD + 2), splits, VD, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
+    const float den = attn_merge_runs<NT>(a.part + ((size_t)t * a.H + h) * splits * (size_t)(VD + 2), splits, VD, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
     float inv = den > 0.0f ? 1.0f / den : 0.0f;
     if (a.gate) inv *= 1.0f / (1.0f + expf(-gate));
     float *out = a.out + (size_t)t * a.ld_out + (size_t)h * VD;
     if (a.v_cs) {                                               // (vdim is even)
         const int vhalf = VD >> 1;
         const float *cs = a.v_cs + (size_t)t * VD;
-        for (int i = tid; i < vhalf; i += 256) {
+        for (int i = tid; i < vhalf; i += NT) {
             float o = sums[i], o2 = sums[i + vhalf];
             gq_unturn_pair(o, o2, cs[i], cs[vhalf + i]);
             out[i] = o * inv;
@@ -392,7 +411,13 @@ __global__ __launch_bounds__(256) void gq_attn_merge_kernel(GqAttnArgs a, int sp
         }
         return;
     }
-    for (int i = tid; i < VD; i += 256) out[i] = sums[i] * inv;
+    for (int i = tid; i < VD; i += NT) out[i] = sums[i] * inv;
+}
+
+static hipError_t gq_attn_merge(const GqAttnArgs &a, int splits, hipStream_t st) {
+    if ((long long)a.T * a.H <= ATTN_MERGE_FEW) hipLaunchKernelGGL(gq_attn_merge_kernel<1024>, dim3((unsigned)a.T, (unsigned)a.H), dim3(1024), 0, st, a, splits);
+    else hipLaunchKernelGGL(gq_attn_merge_kernel<256>, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, splits);
+    return hipGetLastError();
 }
 
 template <int NJ>
@@ -405,8 +430,7 @@ static hipError_t launch_gq_attn_nj(const GqAttnArgs &a, hipStream_t st) {
     const dim3 grid((unsigned)a.T, (unsigned)a.H, (unsigned)splits);
     if (vec) hipLaunchKernelGGL((gq_attn_kernel<NJ, true>), grid, dim3(64 * nw), lds, st, a);
     else hipLaunchKernelGGL((gq_attn_kernel<NJ, false>), grid, dim3(64 * nw), lds, st, a);
-    if (splits > 1) hipLaunchKernelGGL(gq_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, splits);
-    return hipGetLastError();
+    return splits > 1 ? gq_attn_merge(a, splits, st) : hipGetLastError();
 }
 
 
@@ -640,8 +664,8 @@ static hipError_t launch_gq_attn_tile(const GqAttnArgs &a, hipStream_t st) {
     if (splits < 1) splits = 1;
     const dim3 grid((unsigned)((a.T + 31) / 32), (unsigned)a.H, (unsigned)splits);
     hipLaunchKernelGGL((gq_attn_tile_kernel<NVC, 2>), grid, dim3(256), gqt_lds_floats(32) * sizeof(float), st, a);
-    if (splits > 1) hipLaunchKernelGGL(gq_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, (int)splits);
-    else if (a.v_cs) hipLaunchKernelGGL(gq_unturn_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a);
+    if (splits > 1) return gq_attn_merge(a, (int)splits, st);
+    if (a.v_cs) hipLaunchKernelGGL(gq_unturn_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a);
     return hipGetLastError();
 }
 
@@ -701,10 +725,7 @@ hipError_t launch_conv_state(const float *p, int ld_p, int C, int taps, float *s
     hipLaunchKernelGGL(conv_state_kernel, dim3((unsigned)n_seg, (unsigned)((C + 255) / 256)), dim3(256), 0, st, p, ld_p, C, taps - 1, state, seg_start, seg_len, seg_slot);
     return hipGetLastError();
 }
-hipError_t launch_gq_attn_merge(const GqAttnArgs &a, int splits, hipStream_t st) {
-    hipLaunchKernelGGL(gq_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, splits);
-    return hipGetLastError();
-}
+hipError_t launch_gq_attn_merge(const GqAttnArgs &a, int splits, hipStream_t st) { return gq_attn_merge(a, splits, st); }
 
 hipError_t launch_gq_attn(const GqAttnArgs &a, hipStream_t st) {
     if (a.T <= 0) return hipSuccess;

@@ -304,6 +304,11 @@ hipError_t launch_moe_route_groups(const float *z, int ld_z, int T, int E, int k
 // form n_group equal groups of neighbours, a group scores as the sum of its two largest c (its only one if it holds one expert), only experts of the `keep`
 // best groups can be taken; the k open experts with the largest c, lowest index first on a tie; weights = their s as it is.  ids / w: [T][k], best first.
 hipError_t launch_moe_route_sigmoid_bias(const float *z, int ld_z, const float *bias, int T, int E, int k, int n_group, int keep, int32_t *ids, float *w, hipStream_t st);
+// the same choice (one group) for steps of few rows, with the norm in front of the router and its logits in the launch: rows x / sqrt(mean(x^2) + pn_eps) *
+// (pn_off + pn_w), logits against bf16 rows w [E][K]
+bool moe_router_rows_ok(int K, int E);
+hipError_t launch_moe_router_rows(const float *x, int ld_x, const float *pn_w, float pn_off, float pn_eps, const unsigned short *w, int K, const float *bias, int T, int E, int k,
+                                  int32_t *ids, float *wt, hipStream_t st);
 // out[t][:] = sum_j w[t][j] * y[row(t, j)] [+ sigmoid(sg[t * ld_sg]) * b[t]]: the routed experts' weighted sum (rank order) and an always-on expert b (nullable)
 // behind its one-number gate; row(t, j) = slot_of[t * k + j], or t * k + j without a grouping
 hipError_t launch_moe_weighted_combine(float *out, const float *y, const float *w, const int32_t *slot_of, const float *b, const float *sg, int ld_sg, int T, int E, int k, hipStream_t st);

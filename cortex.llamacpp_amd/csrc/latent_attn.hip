@@ -226,12 +226,19 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(LatentAttnArgs a) {
     }
 }
 
-__global__ __launch_bounds__(256) void latent_attn_merge_kernel(LatentAttnArgs a, int splits) {
-    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[LA_MAX_L], sums[LA_MAX_L];
+template <int NT>
+__global__ __launch_bounds__(NT) void latent_attn_merge_kernel(LatentAttnArgs a, int splits) {
+    __shared__ float fac[ATTN_MERGE_MAX_RUNS], part[NT / 256 * LA_MAX_L], sums[LA_MAX_L];
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, KR = a.kv_rank;
-    const float den = attn_merge_runs(a.part + ((size_t)t * a.H + h) * splits * (size_t)(KR + 2), splits, KR, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
+    const float den = attn_merge_runs<NT>(a.part + ((size_t)t * a.H + h) * splits * (size_t)(KR + 2), splits, KR, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
     const float inv = latent_out_factor(a, t, h, den);
-    for (int i = tid; i < KR; i += 256) a.out[(size_t)t * a.ld_out + (size_t)h * KR + i] = sums[i] * inv;
+    for (int i = tid; i < KR; i += NT) a.out[(size_t)t * a.ld_out + (size_t)h * KR + i] = sums[i] * inv;
+}
+
+static hipError_t latent_attn_merge(const LatentAttnArgs &a, int splits, hipStream_t st) {
+    if ((long long)a.T * a.H <= ATTN_MERGE_FEW) hipLaunchKernelGGL(latent_attn_merge_kernel<1024>, dim3((unsigned)a.T, (unsigned)a.H), dim3(1024), 0, st, a, splits);
+    else hipLaunchKernelGGL(latent_attn_merge_kernel<256>, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, splits);
+    return hipGetLastError();
 }
 
 template <int NJ>
@@ -244,8 +251,7 @@ static hipError_t launch_latent_attn_nj(const LatentAttnArgs &a, hipStream_t st)
     const dim3 grid((unsigned)a.T, (unsigned)a.H, (unsigned)splits);
     if (vec) hipLaunchKernelGGL((latent_attn_kernel<NJ, true>), grid, dim3(64 * nw), lds, st, a);
     else hipLaunchKernelGGL((latent_attn_kernel<NJ, false>), grid, dim3(64 * nw), lds, st, a);
-    if (splits > 1) hipLaunchKernelGGL(latent_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, splits);
-    return hipGetLastError();
+    return splits > 1 ? latent_attn_merge(a, splits, st) : hipGetLastError();
 }
 
 // ---- the same attention on the f32 matrix cores: every head of every row reads the same cache rows, so (row, head) pairs are the columns of one product.
@@ -483,8 +489,7 @@ static hipError_t launch_latent_tile(const LatentAttnArgs &a, hipStream_t st) {
     if (splits > (BC == 64 ? LATENT_TILE_RUNS : LATENT_STEP_RUNS)) splits = BC == 64 ? LATENT_TILE_RUNS : LATENT_STEP_RUNS;
     while (splits > 1 && (!a.part || (size_t)P * (size_t)splits * (a.kv_rank + 2) > a.part_floats)) splits--;
     hipLaunchKernelGGL((latent_tile_kernel<R, BC, NT>), dim3((unsigned)tiles, (unsigned)splits), dim3(64 * LT_NW), lds, st, a, LQ);
-    if (splits > 1) hipLaunchKernelGGL(latent_attn_merge_kernel, dim3((unsigned)a.T, (unsigned)a.H), dim3(256), 0, st, a, (int)splits);
-    return hipGetLastError();
+    return splits > 1 ? latent_attn_merge(a, (int)splits, st) : hipGetLastError();
 }
 template <int R, int BC>
 static hipError_t launch_latent_tile_nt(const LatentAttnArgs &a, hipStream_t st) {

@@ -114,7 +114,7 @@ __global__ __launch_bounds__(64 * MLS_NW) void mlstm_step_kernel(MlstmArgs a) {
     __shared__ float red[MLS_NW][64];
     const int seg = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int col = blockIdx.z * 64 + lane, NZ = gridDim.z;
-    const int H = a.H, D = a.D, VD = a.VD, row = a.seg_start[seg], slot = a.seg_slot[seg];
+    const int H = a.H, D = a.D, VD = a.VD, row = a.row0 + seg, slot = a.seg_slot[seg];   // (single rows side by side)
     const float *p = a.p + (size_t)row * a.ld_p, *q = p + h * D, *k = p + (H + h) * D;
     float *Sg = a.S + ((size_t)slot * H + h) * (size_t)D * VD + col;
     float *ng = a.n + (((size_t)slot * H + h) * NZ + blockIdx.z) * D, *mg = a.m + ((size_t)slot * H + h) * NZ + blockIdx.z;

@@ -61,6 +61,68 @@ hipError_t launch_moe_route_sigmoid_bias(const float *z, int ld_z, const float *
     return hipGetLastError();
 }
 
+// The router of a step of few rows in one launch: norm, logits and choice.  One workgroup per token: the row's inverse RMS, then a wave per expert at a time
+// (16-byte weight loads, f32 products), logits to LDS; wave 0 picks as above (one group: the scores and the bias alone).
+__global__ __launch_bounds__(1024) void moe_router_rows_kernel(const float *x, int ld_x, const float *pn_w, float pn_off, float pn_eps, const unsigned short *w, int K, const float *bias,
+                                                               int E, int k, int32_t *ids, float *wt) {
+    extern __shared__ float rr[];
+    float *h = rr, *c = h + K, *z = c + E;                       // [K] normed row, [E] choice scores, [E] logits
+    __shared__ float part[16];
+    const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const float *xr = x + (size_t)t * ld_x;
+    float ss = 0.0f;
+    for (int i = 4 * tid; i < K; i += 4096) {
+        const float4 v = *reinterpret_cast<const float4 *>(xr + i), g = *reinterpret_cast<const float4 *>(pn_w + i);
+        ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
+        *reinterpret_cast<float4 *>(h + i) = make_float4(v.x * (pn_off + g.x), v.y * (pn_off + g.y), v.z * (pn_off + g.z), v.w * (pn_off + g.w));
+    }
+    ss = wave_sum(ss);
+    if (lane == 0) part[wave] = ss;
+    __syncthreads();
+    float tot = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 16; i++) tot += part[i];
+    const float inv = 1.0f / sqrtf(tot / (float)K + pn_eps);
+    for (int e = wave; e < E; e += 16) {
+        const unsigned short *wr = w + (size_t)e * K;
+        float s = 0.0f;
+#pragma unroll 4
+        for (int i = 8 * lane; i < K; i += 512) {
+            const uint4 q = *reinterpret_cast<const uint4 *>(wr + i);
+            const float4 a = *reinterpret_cast<const float4 *>(h + i), b = *reinterpret_cast<const float4 *>(h + i + 4);
+            s = fmaf(a.x, __uint_as_float(q.x << 16), s); s = fmaf(a.y, __uint_as_float(q.x & 0xffff0000u), s);
+            s = fmaf(a.z, __uint_as_float(q.y << 16), s); s = fmaf(a.w, __uint_as_float(q.y & 0xffff0000u), s);
+            s = fmaf(b.x, __uint_as_float(q.z << 16), s); s = fmaf(b.y, __uint_as_float(q.z & 0xffff0000u), s);
+            s = fmaf(b.z, __uint_as_float(q.w << 16), s); s = fmaf(b.w, __uint_as_float(q.w & 0xffff0000u), s);
+        }
+        s = wave_sum(s) * inv;
+        if (lane == 0) { z[e] = s; c[e] = 1.0f / (1.0f + expf(-s)) + (bias ? bias[e] : 0.0f); }
+    }
+    __syncthreads();
+    if (wave != 0) return;
+    for (int r = 0; r < k; r++) {
+        float bv = -INFINITY; int bi = E;
+        for (int i = lane; i < E; i += 64) if (c[i] > bv) { bv = c[i]; bi = i; }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) {
+            const float ov = __shfl_xor(bv, o, 64); const int oi = __shfl_xor(bi, o, 64);
+            if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+        }
+        if (bi >= E) bi = 0;                                     // (only where every score is -inf or not a number)
+        if (lane == (bi & 63)) c[bi] = -INFINITY;                // (the lane that reads the entry again)
+        if (lane == 0) { ids[(size_t)t * k + r] = bi; wt[(size_t)t * k + r] = 1.0f / (1.0f + expf(-z[bi])); }
+    }
+}
+bool moe_router_rows_ok(int K, int E) { return K % 8 == 0 && (size_t)(K + 2 * E) * sizeof(float) <= 60 * 1024 && (long long)K * E <= 512 * 1024; }
+hipError_t launch_moe_router_rows(const float *x, int ld_x, const float *pn_w, float pn_off, float pn_eps, const unsigned short *w, int K, const float *bias, int T, int E, int k,
+                                  int32_t *ids, float *wt, hipStream_t st) {
+    if (T <= 0) return hipSuccess;
+    const auto al16 = [](const void *p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+    if (!moe_router_rows_ok(K, E) || E < 1 || k < 1 || k > E || (ld_x & 3) != 0 || !al16(x) || !al16(w) || !al16(pn_w)) return hipErrorInvalidValue;
+    hipLaunchKernelGGL(moe_router_rows_kernel, dim3((unsigned)T), dim3(1024), (size_t)(K + 2 * E) * sizeof(float), st, x, ld_x, pn_w, pn_off, pn_eps, w, K, bias, E, k, ids, wt);
+    return hipGetLastError();
+}
+
 // out[t][d] = sum_j w[t][j] * y[row(t, j)][d] (rank order) + sigmoid(sg[t * ld_sg]) * b[t][d]
 __global__ void moe_weighted_combine_kernel(float *out, const float *y, const float *w, const int32_t *slot_of, const float *b, const float *sg, int ld_sg, int T, int E, int k) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;

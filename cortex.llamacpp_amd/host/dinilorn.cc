@@ -311,9 +311,13 @@ hipError_t Context::nvx_routed_feed_forward(const NvxLayer &L, int T, bool *clos
         DNL_TRY(hipEventRecord(nvx_join_ev_[0], nvx_side_[0]));
         stream_ = main_stream;
     }
-    DNL_TRY(nvx_linear(L.route, h, W, T, nvx_a_, L.route.N, MMB_STORE, nullptr, 1.0f, pn));
     bool added = false;
-    DNL_TRY(nvx_routed_experts(L, h, pn, T, nvx_a_, L.route.N, closed ? &added : nullptr));
+    const float *z = nvx_a_;
+    if (pn && L.route_kind == NVX_ROUTE_SIGMOID_BIAS && L.n_group == 1 && !shared && moe_router_rows_ok(W, L.n_expert)) {
+        DNL_TRY(launch_moe_router_rows(h, W, pn, M.norm_off, M.eps, L.route.w, W, L.route_bias, T, L.n_expert, L.top, nvx_ids_, nvx_rw_, stream_));
+        z = nullptr;                                             // (the choice is made)
+    } else DNL_TRY(nvx_linear(L.route, h, W, T, nvx_a_, L.route.N, MMB_STORE, nullptr, 1.0f, pn));
+    DNL_TRY(nvx_routed_experts(L, h, pn, T, z, L.route.N, closed ? &added : nullptr));
     if (fork) DNL_TRY(hipStreamWaitEvent(main_stream, nvx_join_ev_[0], 0));
     else if (shared) DNL_TRY(nvx_shared_expert(L, h, pn, T));
     const int32_t *slot_of = grouped ? nvx_slot_ : nullptr;
