@@ -22,11 +22,6 @@ __device__ __forceinline__ float wave_sum(float v) {
     for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
     return v;
 }
-__device__ __forceinline__ float wave_max(float v) {
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, 64));
-    return v;
-}
 __device__ float block_sum_256(float v, float *sh) {
     v = wave_sum(v);
     __syncthreads();
@@ -267,7 +262,6 @@ constexpr int LT_NW = 8;
 constexpr int lt_pieces(int R, int BC) { return (BC / 16) * R; }
 constexpr int lt_ks(int R, int BC) { return lt_pieces(R, BC) >= LT_NW ? 1 : LT_NW / lt_pieces(R, BC); }
 constexpr size_t lt_lds_floats(int R, int BC, int LQ) { return (size_t)16 * R * (LQ + 4) + (size_t)lt_ks(R, BC) * 16 * R * (BC + 4) + 3 * 16 * R + 4 + 64 * R + 2 * 16 * R; }
-constexpr size_t LT_LDS_MAX = 156 * 1024;
 
 // NT: tasks (64 latent entries x 16 pairs) a wave owns at most
 template <int R, int BC, int NT>
@@ -300,7 +294,7 @@ __global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs 
     // the row's length and for pairs past the end
     {
         const int K4 = KR >> 2, QD = a.dim + RT;
-#pragma unroll 8
+#pragma unroll 4
         for (int i = tid; i < BQ * K4; i += 64 * LT_NW) {
             const int r = i / K4, d = (i - r * K4) * 4;
             f32x4 v = {0.0f, 0.0f, 0.0f, 0.0f};
@@ -308,6 +302,7 @@ __global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs 
             *reinterpret_cast<f32x4 *>(Q + (size_t)r * LDQ + d) = f32x4{v.x * a.scale, v.y * a.scale, v.z * a.scale, v.w * a.scale};
         }
         const int half = a.rot_dims >> 1, rest = LQ - KR - a.rot_dims;
+#pragma unroll 1
         for (int i = tid; i < BQ * half; i += 64 * LT_NW) {
             const int r = i / half, pr = i - r * half, p = p0 + r, iu = a.rot_halves ? pr : 2 * pr, iv = a.rot_halves ? pr + half : 2 * pr + 1;
             float x = 0.0f, y = 0.0f;
@@ -322,6 +317,7 @@ __global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs 
             Q[(size_t)r * LDQ + KR + iu] = x;
             Q[(size_t)r * LDQ + KR + iv] = y;
         }
+#pragma unroll 1
         for (int i = tid; i < BQ * rest; i += 64 * LT_NW) {
             const int r = i / rest, e = a.rot_dims + i - r * rest;
             Q[(size_t)r * LDQ + KR + e] = p0 + r < P && e < RT ? a.q[(size_t)(p0 + r) * QD + a.dim + e] * a.scale : 0.0f;
@@ -384,6 +380,7 @@ __global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs 
         }
         __syncthreads();
         // ---- softmax: 16 lanes per pair
+#pragma unroll 1
         for (int r = tid >> 4; r < BQ; r += 32) {
             const uint64_t seen = vmask[r];
             float x[NS];
@@ -422,20 +419,26 @@ __global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs 
 #pragma unroll
             for (int jj = 0; jj < 4; jj++) { o[i][jj].x *= alpha; o[i][jj].y *= alpha; o[i][jj].z *= alpha; o[i][jj].w *= alpha; }
             const bool in = 64 * J + 4 * l16 < KR;
-            const float *vb = a.cache + 64 * J + 4 * l16;
-#pragma unroll
-            for (int s = 0; s < NS; s++) {
-                const f32x4 p4 = *reinterpret_cast<const f32x4 *>(S + (size_t)(16 * rt + l16) * LDS_S + 16 * s + 4 * lg);
-                f32x4 v[4];
+            const float *vb = a.cache + 64 * J + 4 * l16, *pb = S + (size_t)(16 * rt + l16) * LDS_S + 4 * lg;
+            f32x4 v[4], vn[4];
+            const auto fetch = [&](int s, f32x4 (&dst)[4]) {
 #pragma unroll
                 for (int e = 0; e < 4; e++) {
                     const int c = c0 + 16 * s + 4 * lg + e;      // (cells past the end repeat the last one with weight 0)
-                    v[e] = in ? *reinterpret_cast<const f32x4 *>(vb + (size_t)(c < c_end ? c : c_end - 1) * L) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+                    dst[e] = in ? *reinterpret_cast<const f32x4 *>(vb + (size_t)(c < c_end ? c : c_end - 1) * L) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
                 }
+            };
+            fetch(0, v);
+#pragma unroll 1
+            for (int s = 0; s < NS; s++) {
+                if (s + 1 < NS) fetch(s + 1, vn);
+                const f32x4 p4 = *reinterpret_cast<const f32x4 *>(pb + 16 * s);
 #pragma unroll
                 for (int e = 0; e < 4; e++)
 #pragma unroll
                     for (int jj = 0; jj < 4; jj++) o[i][jj] = __builtin_amdgcn_mfma_f32_16x16x4f32(v[e][jj], p4[e], o[i][jj], 0, 0, 0);
+#pragma unroll
+                for (int e = 0; e < 4; e++) v[e] = vn[e];
             }
         }
         // (no barrier: the next block's scores are written behind the barrier that ends its visibility test)
@@ -448,29 +451,25 @@ __global__ __launch_bounds__(64 * LT_NW) void latent_tile_kernel(LatentAttnArgs 
         const int J = task / R, rt = task - J * R, r = 16 * rt + l16, p = p0 + r;
         if (p >= P) continue;
         const int t = p / H, h = p - t * H;
-        if (gridDim.y > 1) {
-            float *rec = a.part + ((size_t)p * gridDim.y + blockIdx.y) * (size_t)(KR + 2);
-            if (J == 0 && lg == 0) { rec[0] = ms[r]; rec[1] = ls[r]; }
-#pragma unroll
-            for (int rr = 0; rr < 4; rr++)
-#pragma unroll
-                for (int jj = 0; jj < 4; jj++) {
-                    const int col = 64 * J + 16 * lg + 4 * rr + jj;
-                    if (col < KR) rec[2 + col] = o[i][jj][rr];
-                }
-            continue;
+        float *out, inv = 1.0f;
+        if (gridDim.y > 1) {                                    // this run's record (sink and gate enter at the merge)
+            out = a.part + ((size_t)p * gridDim.y + blockIdx.y) * (size_t)(KR + 2);
+            if (J == 0 && lg == 0) *reinterpret_cast<float2 *>(out) = make_float2(ms[r], ls[r]);
+            out += 2;
+        } else {
+            const float MM = a.sink ? fmaxf(ms[r], a.sink[h]) : ms[r];
+            const float sc = ls[r] > 0.0f ? expf(ms[r] - MM) : 0.0f;
+            const float den = ls[r] * sc + (a.sink ? expf(a.sink[h] - MM) : 0.0f);
+            inv = latent_out_factor(a, t, h, den) * sc;
+            out = a.out + (size_t)t * a.ld_out + (size_t)h * KR;
         }
-        const float MM = a.sink ? fmaxf(ms[r], a.sink[h]) : ms[r];
-        const float sc = ls[r] > 0.0f ? expf(ms[r] - MM) : 0.0f;
-        const float den = ls[r] * sc + (a.sink ? expf(a.sink[h] - MM) : 0.0f);
-        const float inv = latent_out_factor(a, t, h, den) * sc;
 #pragma unroll
-        for (int rr = 0; rr < 4; rr++)
-#pragma unroll
-            for (int jj = 0; jj < 4; jj++) {
-                const int col = 64 * J + 16 * lg + 4 * rr + jj;
-                if (col < KR) a.out[(size_t)t * a.ld_out + (size_t)h * KR + col] = o[i][jj][rr] * inv;
-            }
+        for (int rr = 0; rr < 4; rr++) {
+            const int col = 64 * J + 16 * lg + 4 * rr;           // (kv_rank is a multiple of 4: four entries are inside or outside together)
+            if (col >= KR) continue;
+            *reinterpret_cast<float2 *>(out + col) = make_float2(o[i][0][rr] * inv, o[i][1][rr] * inv);
+            *reinterpret_cast<float2 *>(out + col + 2) = make_float2(o[i][2][rr] * inv, o[i][3][rr] * inv);
+        }
     }
 }
 
@@ -514,14 +513,13 @@ hipError_t launch_latent_prep(const LatentPrepArgs &a, hipStream_t st) {
 hipError_t launch_latent_attn(const LatentAttnArgs &a, hipStream_t st) {
     if (a.T <= 0) return hipSuccess;
     if (!latent_attn_shape_ok(a.kv_rank, a.rot) || a.rot_dims > a.rot || (a.rot_dims & 1)) return hipErrorInvalidValue;
-    const int L = a.kv_rank + a.rot, LQ = (L + 15) & ~15;
-    // rows that allow 16-byte loads take the matrix cores: batches in tiles of 64 or 32 (row, head) pairs and blocks of 64 cells, steps of few pairs in
+    const int L = a.kv_rank + a.rot;
+    // rows that allow 16-byte loads take the matrix cores: batches in tiles of 32 (row, head) pairs (64 measured slower: fewer workgroups per CU) and blocks of 64 cells, steps of few pairs in
     // tiles of 16 or 32 pairs and blocks of 32 cells
     if ((L & 3) == 0 && (a.kv_rank & 3) == 0 && a.ld_qa == a.H * a.kv_rank && a.ld_q == a.H * (a.dim + a.rot) && (reinterpret_cast<uintptr_t>(a.qa) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0) {
         const long long P = (long long)a.T * a.H;
         if (P <= 16) return launch_latent_tile_nt<1, 32>(a, st);
         if (P <= LATENT_STEP_MAX_PAIRS) return launch_latent_tile_nt<2, 32>(a, st);
-        if (P >= 1024 && lt_lds_floats(4, 64, LQ) * sizeof(float) <= LT_LDS_MAX) return launch_latent_tile_nt<4, 64>(a, st);
         return launch_latent_tile_nt<2, 64>(a, st);
     }
     if (L <= 128) return launch_latent_attn_nj<2>(a, st);

@@ -43,6 +43,10 @@ __device__ __forceinline__ float epi_apply(int epi, float a, float b, float lim 
     return a;
 }
 
+// the epilogue as a template argument: a workgroup's finished tile runs through its code once, so what is not asked for should not lie in between (EPI_ANY: a.epi)
+constexpr int EPI_ANY = -1;
+template <int EPI> __device__ __forceinline__ float epi_fixed(const MMBArgs &a, float s1, float s2) { return epi_apply(EPI == EPI_ANY ? a.epi : EPI, s1, s2, a.epi_limit); }
+
 // where the rows of outer index z live: first row and row count of X / Y, the weight set
 struct ZView { const float *x; const unsigned short *w, *w2; float *y; const float *resid; int rows, x0, y0; };   // x, y, resid: bases; row t of z: x0 + t, y0 + t
 __device__ __forceinline__ ZView z_view(const MMBArgs &a, int z) {
@@ -63,16 +67,17 @@ __device__ __forceinline__ ZView z_view(const MMBArgs &a, int z) {
 __device__ __forceinline__ const float *x_row(const MMBArgs &a, const ZView &v, int t) { return v.x + (size_t)(a.x_map ? a.x_map[v.x0 + t] : v.x0 + t) * a.ldx; }
 __device__ __forceinline__ size_t y_row(const MMBArgs &a, const ZView &v, int t) { return (size_t)(a.y_map ? a.y_map[v.y0 + t] : v.y0 + t) * a.ldy; }
 // output (t, n) from its finished sums; yr = y_row(t), rs = the row's factor, res = the residual's entry (0: none)
+template <int EPI>
 __device__ __forceinline__ void y_store(const MMBArgs &a, const ZView &v, size_t yr, int n, float s1, float s2, float rs, float res) {
     s1 *= rs; s2 *= rs;
-    v.y[yr + n] = epi_apply(a.epi, a.bias ? s1 + a.bias[n] : s1, s2, a.epi_limit) * a.out_scale + res;
+    v.y[yr + n] = epi_fixed<EPI>(a, a.bias ? s1 + a.bias[n] : s1, s2) * a.out_scale + res;
 }
 
 // ---------------------------------------------------------------- few rows: one wave per output column
 // Few rows against MANY output columns (single-token steps: the head, the feed-forward): a wave owns NR adjacent weight rows and keeps the activations of a
 // 512-wide piece of k in registers for all of them - the activation and norm-weight loads, which every wave repeats out of the caches, are paid once per NR
 // weight rows instead of once per row.  Up to TBR rows of X; 16-byte aligned operands; same arithmetic per output as mmb_vec_kernel.
-template <int NR, int TBR>
+template <int NR, int TBR, int EPI>
 __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = (blockIdx.x * 4 + wave) * NR;
@@ -146,7 +151,7 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) { s1 += __shfl_xor(s1, o, 64); s2 += __shfl_xor(s2, o, 64); }
             if (pn) { s1 *= inv; s2 *= inv; }
-            if (lane == 0 && n0 + r < a.N) y_store(a, v, y_row(a, v, i), n0 + r, s1, s2, rsc[i], res[r][i]);
+            if (lane == 0 && n0 + r < a.N) y_store<EPI>(a, v, y_row(a, v, i), n0 + r, s1, s2, rsc[i], res[r][i]);
         }
     }
 }
@@ -154,7 +159,7 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
 // With the norm prologue the row's sum of squares is gathered in the same pass as the products: y = inv_rms(x) * sum_k w_k (x_k (off + g_k)) - one trip
 // through memory per wave, the scale applied to the finished sum.
 // TB: rows per pass - 1 for single rows (a short program: a step runs it once per launch, its first fetch is part of the time), else 8
-template <bool VEC, int TB>
+template <bool VEC, int TB, int EPI>
 __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n = blockIdx.x * 4 + wave;
@@ -221,7 +226,7 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) { s += __shfl_xor(s, o, 64); s2 += __shfl_xor(s2, o, 64); q += __shfl_xor(q, o, 64); }
             if (pn) { const float inv = 1.0f / sqrtf(q / (float)a.K + a.pn_eps); s *= inv; s2 *= inv; }
-            if (lane == 0) y_store(a, v, y_row(a, v, t0 + i), n, s, s2, rsc[i], res[i]);
+            if (lane == 0) y_store<EPI>(a, v, y_row(a, v, t0 + i), n, s, s2, rsc[i], res[i]);
         }
     }
 }
@@ -284,7 +289,7 @@ __global__ __launch_bounds__(256) void mmb_f32_kernel(MMBArgs a) {
 #pragma unroll
         for (int j = 0; j < 4; j++) {
             const int n = n0 + tx * 4 + j;
-            if (n < a.N) y_store(a, v, yr, n, acc[i][j], acc2[i][j], rs, v.resid ? v.resid[yr + n] : 0.0f);
+            if (n < a.N) y_store<EPI_ANY>(a, v, yr, n, acc[i][j], acc2[i][j], rs, v.resid ? v.resid[yr + n] : 0.0f);
         }
     }
 }
@@ -294,8 +299,9 @@ __global__ __launch_bounds__(256) void mmb_f32_kernel(MMBArgs a) {
 // of 16-byte pieces), X rounded to bf16 once on its way there, the stages after next already on their way from memory in registers.  A wave owns 32 RN x 32 RT
 // outputs (v_mfma_f32_32x32x16_bf16).  The workgroups that read the same weight rows sit on the same XCD, side by side: its L2 fetches them once.
 constexpr int MMT_K = 64, MMT_LD = MMT_K + 8;                   // bf16 per LDS row
-template <int RN, int RT, bool GATED>
+template <int RN, int RT, int EPI>
 __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a, int n_tiles, int t_tiles) {
+    constexpr bool GATED = EPI >= MMB_SILU_MUL;
     constexpr int TN = 64 * RN, TT = 64 * RT, NW = 2 * RN, NX = 4 * RT;   // 16-byte loads per thread and stage
     __shared__ __attribute__((aligned(16))) unsigned short sW[2][TN][MMT_LD], sW2[GATED ? 2 : 1][GATED ? TN : 1][MMT_LD], sX[2][TT][MMT_LD];
     const ZView v = z_view(a, blockIdx.z);
@@ -400,16 +406,36 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a, int n_tiles, i
 #pragma unroll
             for (int r = 0; r < 16; r++) {
                 const int n = n0 + (wave & 1) * 32 * RN + 32 * i + (r & 3) + 8 * (r >> 2) + 4 * kg;
-                if (n < a.N) y_store(a, v, yr, n, acc[i][j][r], GATED ? acc2[i][j][r] : 0.0f, rs, v.resid ? v.resid[yr + n] : 0.0f);
+                if (n < a.N) y_store<EPI>(a, v, yr, n, acc[i][j][r], GATED ? acc2[i][j][r] : 0.0f, rs, v.resid ? v.resid[yr + n] : 0.0f);
             }
     }
 }
 
-template <int RN, int RT, bool GATED>
+template <int RN, int RT, int EPI>
 static hipError_t launch_mmb_mfma(const MMBArgs &a, int rows_max, hipStream_t st) {
     const int nt = (a.N + 64 * RN - 1) / (64 * RN), tt = (rows_max + 64 * RT - 1) / (64 * RT);
-    hipLaunchKernelGGL((mmb_mfma_kernel<RN, RT, GATED>), dim3((unsigned)((nt + 7) / 8 * 8 * tt), 1, (unsigned)a.nz), dim3(256), 0, st, a, nt, tt);
+    hipLaunchKernelGGL((mmb_mfma_kernel<RN, RT, EPI>), dim3((unsigned)((nt + 7) / 8 * 8 * tt), 1, (unsigned)a.nz), dim3(256), 0, st, a, nt, tt);
     return hipGetLastError();
+}
+// the tile by what a stage costs a CU in bytes fetched (KB: weights 8 per 64 rows and set, X 16 per 64 rows) times the rounds of workgroups the device needs; a
+// grouped batch sizes its grid for the most rows ONE expert could hold, what counts is the rows an expert holds on average
+template <int EPI>
+static hipError_t launch_mmb_mfma_tile(const MMBArgs &a, int rows_max, hipStream_t st) {
+    const long long rows = a.meta ? (a.T + a.nz - 1) / a.nz : rows_max;
+    const auto rounds = [&](int rn, int rt, int kb) {
+        const double wg = (double)((a.N + 64 * rn - 1) / (64 * rn)) * (double)((rows + 64 * rt - 1) / (64 * rt)) * a.nz;
+        return (wg > 256.0 ? wg / 256.0 : 1.0) * kb;
+    };
+    if (EPI >= MMB_SILU_MUL) return rounds(1, 2, 48) < rounds(1, 1, 32) ? launch_mmb_mfma<1, 2, EPI>(a, rows_max, st) : launch_mmb_mfma<1, 1, EPI>(a, rows_max, st);
+    const double r11 = rounds(1, 1, 24), r21 = rounds(2, 1, 32), r22 = rounds(2, 2, 48);
+    if (r22 <= r11 && r22 <= r21) return launch_mmb_mfma<(EPI >= MMB_SILU_MUL ? 1 : 2), (EPI >= MMB_SILU_MUL ? 1 : 2), EPI>(a, rows_max, st);
+    return r21 <= r11 ? launch_mmb_mfma<(EPI >= MMB_SILU_MUL ? 1 : 2), 1, EPI>(a, rows_max, st) : launch_mmb_mfma<1, 1, EPI>(a, rows_max, st);
+}
+template <bool VEC, int TB>
+static void launch_mmb_vec(const MMBArgs &a, dim3 grid, hipStream_t st) {
+    if (TB == 1 && a.epi == MMB_STORE) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (TB == 1 ? (int)MMB_STORE : EPI_ANY)>), grid, dim3(256), 0, st, a);
+    else if (TB == 1 && a.epi == MMB_SILU_MUL) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (TB == 1 ? (int)MMB_SILU_MUL : EPI_ANY)>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, EPI_ANY>), grid, dim3(256), 0, st, a);
 }
 
 }  // namespace
@@ -429,27 +455,25 @@ hipError_t launch_mmb(const MMBArgs &a, hipStream_t st) {
         // many columns, a handful of rows: four weight rows per wave (the grid still has thousands of waves)
         if (vec && !a.sel && !a.meta && rows_max <= 4 && (long long)a.N * a.nz >= 4096) {
             const dim3 g4((unsigned)((a.N + 15) / 16), (unsigned)a.nz);
-            if (rows_max == 1) hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 1>), g4, dim3(256), 0, st, a);
-            else hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 4>), g4, dim3(256), 0, st, a);
+            if (rows_max == 1 && a.epi == MMB_STORE) hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 1, MMB_STORE>), g4, dim3(256), 0, st, a);
+            else if (rows_max == 1) hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 1, EPI_ANY>), g4, dim3(256), 0, st, a);
+            else hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 4, EPI_ANY>), g4, dim3(256), 0, st, a);
             return hipGetLastError();
         }
-        if (vec && rows_max == 1) hipLaunchKernelGGL((mmb_vec_kernel<true, 1>), grid, dim3(256), 0, st, a);
-        else if (vec) hipLaunchKernelGGL((mmb_vec_kernel<true, 8>), grid, dim3(256), 0, st, a);
-        else hipLaunchKernelGGL((mmb_vec_kernel<false, 8>), grid, dim3(256), 0, st, a);
+        if (vec && rows_max == 1) launch_mmb_vec<true, 1>(a, grid, st);
+        else if (vec) launch_mmb_vec<true, 8>(a, grid, st);
+        else launch_mmb_vec<false, 8>(a, grid, st);
         return hipGetLastError();
     }
     if (!a.f32 && vec && (a.K % 16) == 0) {
-        // the tile by what a stage costs a CU in bytes fetched (KB: weights 8 RN, X 16 RT) times the rounds of workgroups the device needs; a grouped batch sizes
-        // its grid for the most rows ONE expert could hold, what counts is the rows an expert holds on average
-        const long long rows = a.meta ? (a.T + a.nz - 1) / a.nz : rows_max;
-        const auto rounds = [&](int rn, int rt, int kb) {
-            const double wg = (double)((a.N + 64 * rn - 1) / (64 * rn)) * (double)((rows + 64 * rt - 1) / (64 * rt)) * a.nz;
-            return (wg > 256.0 ? wg / 256.0 : 1.0) * kb;
-        };
-        if (gated) return rounds(1, 2, 48) < rounds(1, 1, 32) ? launch_mmb_mfma<1, 2, true>(a, rows_max, st) : launch_mmb_mfma<1, 1, true>(a, rows_max, st);
-        const double r11 = rounds(1, 1, 24), r21 = rounds(2, 1, 32), r22 = rounds(2, 2, 48);
-        if (r22 <= r11 && r22 <= r21) return launch_mmb_mfma<2, 2, false>(a, rows_max, st);
-        return r21 <= r11 ? launch_mmb_mfma<2, 1, false>(a, rows_max, st) : launch_mmb_mfma<1, 1, false>(a, rows_max, st);
+        switch (a.epi) {
+            case MMB_STORE: return launch_mmb_mfma_tile<MMB_STORE>(a, rows_max, st);
+            case MMB_RELU2: return launch_mmb_mfma_tile<MMB_RELU2>(a, rows_max, st);
+            case MMB_SILU_MUL: return launch_mmb_mfma_tile<MMB_SILU_MUL>(a, rows_max, st);
+            case MMB_GELU_MUL: return launch_mmb_mfma_tile<MMB_GELU_MUL>(a, rows_max, st);
+            case MMB_CLAMP_SWIGLU: return launch_mmb_mfma_tile<MMB_CLAMP_SWIGLU>(a, rows_max, st);
+            default: return hipErrorInvalidValue;
+        }
     }
     const dim3 grid((unsigned)((a.N + 63) / 64), (unsigned)((rows_max + 63) / 64), (unsigned)a.nz);
     if (gated) hipLaunchKernelGGL(mmb_f32_kernel<true>, grid, dim3(256), 0, st, a);

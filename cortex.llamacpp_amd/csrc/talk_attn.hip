@@ -57,9 +57,18 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         c_lo += (int)blockIdx.y * per;
         c_hi = c_lo + per < c_hi ? c_lo + per : c_hi;
     }
-    for (int i = tid; i < H * D; i += TKR_NT) qv[i] = a.q[(size_t)t * a.ld_q + i];
-    if (H <= TKR_TALK_LDS) for (int i = tid; i < H * H; i += TKR_NT) tk[i] = a.talk[i];
+    if (VEC) {
+#pragma unroll 1
+        for (int i = 4 * tid; i < H * D; i += 4 * TKR_NT) *reinterpret_cast<f32x4 *>(qv + i) = *reinterpret_cast<const f32x4 *>(a.q + (size_t)t * a.ld_q + i);
+    } else {
+#pragma unroll 1
+        for (int i = tid; i < H * D; i += TKR_NT) qv[i] = a.q[(size_t)t * a.ld_q + i];
+    }
+#pragma unroll 1
+    for (int i = tid; H <= TKR_TALK_LDS && i < H * H; i += TKR_NT) tk[i] = a.talk[i];
+#pragma unroll 1
     for (int i = tid; i < H * VD; i += TKR_NT) acc[i] = 0.0f;
+#pragma unroll 1
     for (int i = tid; i < H; i += TKR_NT) { ms[i] = -INFINITY; ls[i] = 0.0f; }
     const auto fetch = [&](int c, int kvh, float (&dst)[NJ][4]) {
         const float *kr = a.cache + (size_t)c * L + (size_t)kvh * D;
@@ -89,7 +98,7 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         // ---- raw scores
         for (int kvh = 0; kvh < G; kvh++) {
             if (kvh + 1 < G) fetch(c, kvh + 1, nk);
-#pragma unroll 4
+#pragma unroll 2
             for (int g = kvh * HG; g < (kvh + 1) * HG; g++) {
                 const float *q = qv + (size_t)g * D;
                 float dot = 0.0f;
@@ -118,6 +127,7 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         }
         __syncthreads();
         // ---- mixed scores and the running softmax: lane = cell, 32 lanes per head
+#pragma unroll 1
         for (int idx = tid; idx < ((H * TKR_BC + 63) & ~63); idx += TKR_NT) {      // (whole waves: the shuffles below)
             const int h = idx / TKR_BC < H ? idx / TKR_BC : H - 1, cc = idx & (TKR_BC - 1);
             const float *tr = talk + (size_t)h * H;
@@ -141,6 +151,7 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         const int nc = c_hi - c0 < TKR_BC ? c_hi - c0 : TKR_BC;
         if (VEC) {
             const int V4 = VD >> 2;
+#pragma unroll 1
             for (int idx = tid; idx < H * V4; idx += TKR_NT) {
                 const int h = idx / V4, col = (idx - h * V4) * 4;
                 const float *vr = a.cache + (size_t)c0 * L + voff + (size_t)(h / HG) * VD + col, *p = pw + h * (TKR_BC + 1);
@@ -169,12 +180,14 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
     }
     __syncthreads();
     if (gridDim.y > 1) {                                        // this run's records (sink and gate enter at the merge)
+#pragma unroll 1
         for (int idx = tid; idx < H * (VD + 2); idx += TKR_NT) {
             const int h = idx / (VD + 2), i = idx - h * (VD + 2);
             a.part[(((size_t)t * H + h) * gridDim.y + blockIdx.y) * (size_t)(VD + 2) + i] = i == 0 ? ms[h] : i == 1 ? ls[h] : acc[(size_t)h * VD + i - 2];
         }
         return;
     }
+#pragma unroll 1
     for (int idx = tid; idx < H * VD; idx += TKR_NT) {
         const int h = idx / VD;
         const float MM = a.sink ? fmaxf(ms[h], a.sink[h]) : ms[h];
@@ -192,28 +205,30 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
 //   raw scores:  A = keys (i = cell), B = queries (j = row): a wave takes (head, half of the block's cells) tasks; result -> LDS, 4 cells of a row per write
 //   mix:         A = talk (i = head, k = head), B = raw scores (k = head, j = (row, cell) pair): a wave owns 16 pairs at a time for ALL heads, so the mixed scores
 //                take the raw ones' places without a barrier in between
-//   softmax:     a wave owns heads (and, with few heads, a share of the value columns); lane = (row l & 15, cells 16 s + 4 (l >> 4) + e): the row's statistics
-//                meet over 4 lanes
-//   values:      A = values (i = column), B = weights (k = cell, j = row): the result's column is the lane's row, so the rescale needs no exchange; column i of
+//   softmax:     16 lanes per (head, row); weights back to LDS
+//   values:      a wave owns heads (and, with few heads, a share of the value columns); A = values (i = column), B = weights (k = cell, j = row): the result's column is the lane's row, so the rescale needs no exchange; column i of
 //                tile jj stands for value column 64 J + 4 i + jj, which makes every load 16 bytes and every lane's results 16 neighbouring columns
 constexpr int TKT_NW = 8, TKT_BQ = 16;
 constexpr int tkt_head_stride(int BC) { return TKT_BQ * (BC + 4) + 16; }
-constexpr size_t tkt_lds_floats(int H, int BC) { return (size_t)H * tkt_head_stride(BC) + 2 * TKT_BQ + 4 + 4 * TKT_BQ; }
+constexpr size_t tkt_lds_floats(int H, int BC) { return (size_t)(H + 1) * tkt_head_stride(BC) + 3 * (size_t)H * TKT_BQ + 2 * TKT_BQ + 4 + 4 * TKT_BQ; }   // (one more head: where the mix drops its padding)
 constexpr size_t TKT_LDS_MAX = 156 * 1024;
 
 // HPW: heads a wave finishes; NV = ceil(vdim / 64); the block's heads are [blockIdx.z * 8 * HPW, + 8 * HPW)
 template <int BC, int HPW, int NV>
 __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, int wph) {
-    constexpr int LDR = BC + 4, HS = tkt_head_stride(BC), NS = BC / 16, CT = TKT_BQ * NS / TKT_NW, HT = BC == 64 ? 2 : 4;   // (at most 16 HT heads)
+    constexpr int LDR = BC + 4, HS = tkt_head_stride(BC), NS = BC / 16, HT = BC == 64 ? 2 : 4;   // (at most 16 HT heads)
     extern __shared__ float lds[];
     const int H = a.H, G = a.G, D = a.dim, VD = a.vdim, HG = H / G;
-    float *S = lds;                                             // [H][16][LDR], head stride HS
-    int *rpos = reinterpret_cast<int *>(S + (size_t)H * HS), *rseq = rpos + TKT_BQ, *red = rseq + TKT_BQ;
-    uint64_t *vmask2 = reinterpret_cast<uint64_t *>(red + 4);    // [2][16]: the cells of a block each row sees, two blocks in turn (H * HS + 36 floats in: 8-byte aligned)
+    float *S = lds;                                             // [H + 1][16][LDR], head stride HS
+    float *ms = S + (size_t)(H + 1) * HS, *ls = ms + H * TKT_BQ, *al = ls + H * TKT_BQ;      // [H][16]: running maximum and sum, this block's rescale
+    int *rpos = reinterpret_cast<int *>(al + H * TKT_BQ), *rseq = rpos + TKT_BQ, *red = rseq + TKT_BQ;
+    uint64_t *vmask2 = reinterpret_cast<uint64_t *>(red + 4);    // [2][16]: the cells of a block each row sees, two blocks in turn (an even number of floats in: 8-byte aligned)
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lg = lane >> 4;
     const int row0 = blockIdx.x * TKT_BQ;
     const size_t L = (size_t)G * (D + VD), voff = (size_t)G * D;
     const int n_kv = *a.n_kv_dev;
+#pragma unroll 1
+    for (int i = tid; i < H * TKT_BQ; i += 64 * TKT_NW) { ms[i] = -INFINITY; ls[i] = 0.0f; }
     if (tid < 64) {
         int lo = 0x7fffffff, hi = 0;
         if (tid < TKT_BQ) {
@@ -240,15 +255,12 @@ __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, in
     // what this wave finishes: heads h0 + hh (hh < HPW), value columns of the 64-blocks J with J % wph == sub (wph waves share a head when there are few)
     const int sub = wave % wph, h0 = (int)blockIdx.z * TKT_NW * HPW + (wave / wph) * HPW;
     f32x4 o[HPW][NV][4];
-    float m[HPW], l[HPW];
 #pragma unroll
-    for (int hh = 0; hh < HPW; hh++) {
-        m[hh] = -INFINITY; l[hh] = 0.0f;
+    for (int hh = 0; hh < HPW; hh++)
 #pragma unroll
         for (int J = 0; J < NV; J++)
 #pragma unroll
             for (int jj = 0; jj < 4; jj++) o[hh][J][jj] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-    }
     const float *qrow = a.q + (size_t)(row0 + l16 < a.T ? row0 + l16 : a.T - 1) * a.ld_q;    // (rows past the end repeat the last one and see nothing)
     uint64_t *vmask = vmask2;
     for (int c0 = c_begin; c0 < c_end; c0 += BC) {
@@ -281,7 +293,7 @@ __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, in
                 kr[s] = kb + (size_t)(c < c_end ? c : c_end - 1) * L;
                 acc[s] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
             }
-#pragma unroll 4
+#pragma unroll 2
             for (int d0 = 0; d0 < D; d0 += 16) {                 // (dim is a multiple of 16)
                 const int d = d0 + 4 * lg;
                 const f32x4 q4 = *reinterpret_cast<const f32x4 *>(qb + d);
@@ -297,11 +309,12 @@ __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, in
             for (int s = 0; s < NS / 2; s++) *reinterpret_cast<f32x4 *>(S + (size_t)g * HS + l16 * LDR + 16 * (s0 + s) + 4 * lg) = acc[s];
         }
         __syncthreads();
-        // ---- mix: the wave's column pieces side by side, so that every fragment of talk is fetched once and its trip overlaps their products
-        {
-            f32x4 mx[CT][HT];
+        // ---- mix: four of the wave's column pieces side by side, so that the trip of a fragment of talk overlaps their products
+#pragma unroll 1
+        for (int ct0 = wave; ct0 < TKT_BQ * NS; ct0 += 4 * TKT_NW) {
+            f32x4 mx[4][HT];
 #pragma unroll
-            for (int i = 0; i < CT; i++)
+            for (int i = 0; i < 4; i++)
 #pragma unroll
                 for (int ht = 0; ht < HT; ht++) mx[i][ht] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
             const auto fragment = [&](int g0, float (&w)[HT]) {
@@ -314,8 +327,8 @@ __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, in
                 fragment(g0 + 4, wn);
                 const bool in = g0 + lg < H;
 #pragma unroll
-                for (int i = 0; i < CT; i++) {
-                    const int ct = wave + TKT_NW * i;
+                for (int i = 0; i < 4; i++) {
+                    const int ct = ct0 + TKT_NW * i;
                     const float b = in ? S[(size_t)(g0 + lg) * HS + (ct / NS) * LDR + (ct % NS) * 16 + l16] : 0.0f;
 #pragma unroll
                     for (int ht = 0; ht < HT; ht++) if (16 * ht < H) mx[i][ht] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[ht], b, mx[i][ht], 0, 0, 0);
@@ -324,106 +337,117 @@ __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, in
                 for (int ht = 0; ht < HT; ht++) w[ht] = wn[ht];
             }
 #pragma unroll
-            for (int i = 0; i < CT; i++) {
-                const int ct = wave + TKT_NW * i;
+            for (int i = 0; i < 4; i++) {
+                const int ct = ct0 + TKT_NW * i;
                 float *col = S + (ct / NS) * LDR + (ct % NS) * 16 + l16;
 #pragma unroll
-                for (int ht = 0; ht < HT; ht++)
+                for (int ht = 0; ht < HT; ht++) {
+                    if (16 * ht >= H) continue;
 #pragma unroll
-                    for (int r = 0; r < 4; r++) if (16 * ht + 4 * lg + r < H) col[(size_t)(16 * ht + 4 * lg + r) * HS] = mx[i][ht][r];
+                    for (int r = 0; r < 4; r++) {
+                        const int h = 16 * ht + 4 * lg + r;
+                        col[(size_t)(h < H ? h : H) * HS] = mx[i][ht][r];
+                    }
+                }
             }
         }
         __syncthreads();
-        // ---- softmax and values
-        const uint64_t seen = vmask[l16];
+        // ---- softmax: 16 lanes per (head, row)
+#pragma unroll 1
+        for (int hr = tid >> 4; hr < H * TKT_BQ; hr += 4 * TKT_NW) {
+            const uint64_t seen = vmask[hr & (TKT_BQ - 1)] >> l16;
+            float *row = S + (size_t)(hr >> 4) * HS + (hr & (TKT_BQ - 1)) * LDR + l16;
+            float x[NS], bm = -INFINITY;
+#pragma unroll
+            for (int j = 0; j < NS; j++) {
+                x[j] = (seen >> (16 * j)) & 1 ? row[16 * j] : -INFINITY;
+                bm = fmaxf(bm, x[j]);
+            }
+            bm = fmaxf(bm, dpp_f<DPP_QP_1032>(bm));
+            bm = fmaxf(bm, dpp_f<DPP_QP_2301>(bm));
+            bm = fmaxf(bm, dpp_f<DPP_HALF_MIRROR>(bm));
+            bm = fmaxf(bm, dpp_f<DPP_MIRROR>(bm));
+            const float m0 = ms[hr], mn = fmaxf(m0, bm), mx = mn == -INFINITY ? 0.0f : mn;
+            float ps = 0.0f;
+#pragma unroll
+            for (int j = 0; j < NS; j++) {
+                const float p = expf(x[j] - mx);                 // (an unseen cell: e^-inf)
+                row[16 * j] = p;
+                ps += p;
+            }
+            ps = row_sum16(ps);
+            const float alpha = expf(m0 - mx);                   // (nothing seen so far: e^-inf)
+            if (l16 == 0) { ls[hr] = ls[hr] * alpha + ps; ms[hr] = mn; al[hr] = alpha; }
+        }
+        __syncthreads();
+        // ---- values
 #pragma unroll
         for (int hh = 0; hh < HPW; hh++) {
             const int h = h0 + hh;
             if (h >= H) continue;
-            f32x4 p[NS];
-            float bm = -INFINITY;
-#pragma unroll
-            for (int s = 0; s < NS; s++) {
-                p[s] = *reinterpret_cast<const f32x4 *>(S + (size_t)h * HS + l16 * LDR + 16 * s + 4 * lg);
-#pragma unroll
-                for (int e = 0; e < 4; e++) if ((seen >> (16 * s + 4 * lg + e)) & 1) bm = fmaxf(bm, p[s][e]);
-            }
-            bm = fmaxf(bm, __shfl_xor(bm, 16, 64));
-            bm = fmaxf(bm, __shfl_xor(bm, 32, 64));
-            const float mn = fmaxf(m[hh], bm), alpha = m[hh] == -INFINITY ? 0.0f : expf(m[hh] - mn);
-            float ps = 0.0f;
-#pragma unroll
-            for (int s = 0; s < NS; s++)
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    const float x = (seen >> (16 * s + 4 * lg + e)) & 1 ? expf(p[s][e] - mn) : 0.0f;
-                    p[s][e] = x;
-                    ps += x;
-                }
-            ps += __shfl_xor(ps, 16, 64);
-            ps += __shfl_xor(ps, 32, 64);
-            l[hh] = l[hh] * alpha + ps;
-            m[hh] = mn;
-            const float *vb = a.cache + voff + (size_t)(h / HG) * VD + 4 * l16;
+            const float alpha = al[h * TKT_BQ + l16];
+            const float *vb = a.cache + voff + (size_t)(h / HG) * VD + 4 * l16, *pb = S + (size_t)h * HS + l16 * LDR + 4 * lg;
 #pragma unroll
             for (int J = 0; J < NV; J++) {
                 if (J % wph != sub) continue;
 #pragma unroll
                 for (int jj = 0; jj < 4; jj++) { o[hh][J][jj].x *= alpha; o[hh][J][jj].y *= alpha; o[hh][J][jj].z *= alpha; o[hh][J][jj].w *= alpha; }
                 const bool in = 64 * J + 4 * l16 < VD;
-#pragma unroll
-                for (int s = 0; s < NS; s++) {
-                    f32x4 v[4];
+                f32x4 v[4], vn[4];
+                const auto fetch = [&](int s, f32x4 (&dst)[4]) {
 #pragma unroll
                     for (int e = 0; e < 4; e++) {
                         const int c = c0 + 16 * s + 4 * lg + e;  // (cells past the end repeat the last one with weight 0)
-                        v[e] = in ? *reinterpret_cast<const f32x4 *>(vb + (size_t)(c < c_end ? c : c_end - 1) * L + 64 * J) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+                        dst[e] = in ? *reinterpret_cast<const f32x4 *>(vb + (size_t)(c < c_end ? c : c_end - 1) * L + 64 * J) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
                     }
+                };
+                fetch(0, v);
+#pragma unroll 1
+                for (int s = 0; s < NS; s++) {
+                    if (s + 1 < NS) fetch(s + 1, vn);
+                    const f32x4 p = *reinterpret_cast<const f32x4 *>(pb + 16 * s);
 #pragma unroll
                     for (int e = 0; e < 4; e++)
 #pragma unroll
-                        for (int jj = 0; jj < 4; jj++) o[hh][J][jj] = __builtin_amdgcn_mfma_f32_16x16x4f32(v[e][jj], p[s][e], o[hh][J][jj], 0, 0, 0);
+                        for (int jj = 0; jj < 4; jj++) o[hh][J][jj] = __builtin_amdgcn_mfma_f32_16x16x4f32(v[e][jj], p[e], o[hh][J][jj], 0, 0, 0);
+#pragma unroll
+                    for (int e = 0; e < 4; e++) v[e] = vn[e];
                 }
             }
         }
         // (no barrier: the next block writes scores only behind the barrier that ends its visibility test)
     }
     // lane = (row l16, columns 64 J + 16 lg + 4 r + jj)
+    __syncthreads();                                            // (a run without a visible cell has passed no barrier behind the start values of ms and ls)
     const int r = row0 + l16;
     if (r >= a.T) return;
 #pragma unroll
     for (int hh = 0; hh < HPW; hh++) {
         const int h = h0 + hh;
         if (h >= H) continue;
-        if (gridDim.y > 1) {
-            float *rec = a.part + (((size_t)r * H + h) * gridDim.y + blockIdx.y) * (size_t)(VD + 2);
-            if (lg == 0 && sub == 0) { rec[0] = m[hh]; rec[1] = l[hh]; }
-#pragma unroll
-            for (int J = 0; J < NV; J++) {
-                if (J % wph != sub) continue;
-#pragma unroll
-                for (int rr = 0; rr < 4; rr++)
-#pragma unroll
-                    for (int jj = 0; jj < 4; jj++) {
-                        const int col = 64 * J + 16 * lg + 4 * rr + jj;
-                        if (col < VD) rec[2 + col] = o[hh][J][jj][rr];
-                    }
-            }
-            continue;
+        const float m = ms[h * TKT_BQ + l16], l = ls[h * TKT_BQ + l16];
+        float *out, inv = 1.0f;
+        if (gridDim.y > 1) {                                    // this run's record (sink and gate enter at the merge)
+            out = a.part + (((size_t)r * H + h) * gridDim.y + blockIdx.y) * (size_t)(VD + 2);
+            if (lg == 0 && sub == 0) *reinterpret_cast<float2 *>(out) = make_float2(m, l);
+            out += 2;
+        } else {
+            const float MM = a.sink ? fmaxf(m, a.sink[h]) : m;
+            const float sc = l > 0.0f ? expf(m - MM) : 0.0f;
+            const float den = l * sc + (a.sink ? expf(a.sink[h] - MM) : 0.0f);
+            inv = den > 0.0f ? sc / den : 0.0f;
+            if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)r * a.ld_gate + h]));
+            out = a.out + (size_t)r * a.ld_out + (size_t)h * VD;
         }
-        const float MM = a.sink ? fmaxf(m[hh], a.sink[h]) : m[hh];
-        const float sc = l[hh] > 0.0f ? expf(m[hh] - MM) : 0.0f;
-        const float den = l[hh] * sc + (a.sink ? expf(a.sink[h] - MM) : 0.0f);
-        float inv = den > 0.0f ? sc / den : 0.0f;
-        if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)r * a.ld_gate + h]));
-        float *out = a.out + (size_t)r * a.ld_out + (size_t)h * VD;
 #pragma unroll
         for (int J = 0; J < NV; J++) {
             if (J % wph != sub) continue;
 #pragma unroll
             for (int rr = 0; rr < 4; rr++) {
-                const int col = 64 * J + 16 * lg + 4 * rr;
-                if (col < VD) *reinterpret_cast<f32x4 *>(out + col) = f32x4{o[hh][J][0][rr] * inv, o[hh][J][1][rr] * inv, o[hh][J][2][rr] * inv, o[hh][J][3][rr] * inv};
+                const int col = 64 * J + 16 * lg + 4 * rr;       // (vdim is a multiple of 4: four columns are inside or outside together)
+                if (col >= VD) continue;
+                *reinterpret_cast<float2 *>(out + col) = make_float2(o[hh][J][0][rr] * inv, o[hh][J][1][rr] * inv);
+                *reinterpret_cast<float2 *>(out + col + 2) = make_float2(o[hh][J][2][rr] * inv, o[hh][J][3][rr] * inv);
             }
         }
     }
