@@ -303,6 +303,7 @@ template <int RN, int RT, int EPI>
 __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a, int n_tiles, int t_tiles) {
     constexpr bool GATED = EPI >= MMB_SILU_MUL;
     constexpr int TN = 64 * RN, TT = 64 * RT, NW = 2 * RN, NX = 4 * RT;   // 16-byte loads per thread and stage
+    constexpr int SETS = RN * RT == 1 ? 4 : 2;                  // stages on their way from memory
     __shared__ __attribute__((aligned(16))) unsigned short sW[2][TN][MMT_LD], sW2[GATED ? 2 : 1][GATED ? TN : 1][MMT_LD], sX[2][TT][MMT_LD];
     const ZView v = z_view(a, blockIdx.z);
     // block -> tile: consecutive blocks go to the XCDs in turn; the t tiles of one n tile take consecutive turns of ONE of them
@@ -327,8 +328,8 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a, int n_tiles, i
         for (int j = 0; j < RT; j++)
 #pragma unroll
             for (int r = 0; r < 16; r++) { acc[i][j][r] = 0.0f; if (GATED) acc2[i][j][r] = 0.0f; }
-    u16x8 lw[2][NW], lw2[2][GATED ? NW : 1];
-    f32x4 lx[2][NX];
+    u16x8 lw[SETS][NW], lw2[SETS][GATED ? NW : 1];
+    f32x4 lx[SETS][NX];
     const auto request = [&](auto set, int k0) {                // (K is a multiple of 16: a 16-byte piece is inside a row or behind its end)
         constexpr int b = decltype(set)::value;
 #pragma unroll
@@ -345,20 +346,20 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a, int n_tiles, i
         }
     };
     const auto stage = [&](auto set) {
-        constexpr int b = decltype(set)::value;
+        constexpr int w = decltype(set)::value, b = w & 1;
 #pragma unroll
         for (int i = 0; i < NW; i++) {
-            *reinterpret_cast<u16x8 *>(&sW[b][64 * (i >> 1) + r4][32 * (i & 1) + 8 * q4]) = lw[b][i];
-            if (GATED) *reinterpret_cast<u16x8 *>(&sW2[b][64 * (i >> 1) + r4][32 * (i & 1) + 8 * q4]) = lw2[b][i];
+            *reinterpret_cast<u16x8 *>(&sW[b][64 * (i >> 1) + r4][32 * (i & 1) + 8 * q4]) = lw[w][i];
+            if (GATED) *reinterpret_cast<u16x8 *>(&sW2[b][64 * (i >> 1) + r4][32 * (i & 1) + 8 * q4]) = lw2[w][i];
         }
 #pragma unroll
         for (int i = 0; i < NX; i++) {
-            const f32x4 x = lx[b][i];
+            const f32x4 x = lx[w][i];
             *reinterpret_cast<bf16x4 *>(&sX[b][64 * (i >> 2) + r4][16 * (i & 3) + 4 * q4]) = bf16x4{(__bf16)x.x, (__bf16)x.y, (__bf16)x.z, (__bf16)x.w};   // (round to nearest even)
         }
     };
     const auto multiply = [&](auto set) {
-        constexpr int b = decltype(set)::value;
+        constexpr int b = decltype(set)::value & 1;
 #pragma unroll
         for (int u = 0; u < MMT_K / 16; u++) {
             bf16x8 wa[RN], wb[RN], xb[RT];
@@ -379,20 +380,22 @@ __global__ __launch_bounds__(256) void mmb_mfma_kernel(MMBArgs a, int n_tiles, i
                 }
         }
     };
-    const std::integral_constant<int, 0> s0;
-    const std::integral_constant<int, 1> s1;
-    request(s0, 0);
-    request(s1, MMT_K);                                         // (a stage past K is all zeros)
-    for (int k0 = 0; k0 < a.K; k0 += 2 * MMT_K) {
-        stage(s0);
-        if (k0 + 2 * MMT_K < a.K) request(s0, k0 + 2 * MMT_K);
-        __syncthreads();
-        multiply(s0);
-        if (k0 + MMT_K >= a.K) break;
-        stage(s1);
-        if (k0 + 3 * MMT_K < a.K) request(s1, k0 + 3 * MMT_K);
-        __syncthreads();
-        multiply(s1);
+    const auto each_set = [&](auto f) {                         // f(0), f(1), .. until one says stop
+        if (!f(std::integral_constant<int, 0>()) || !f(std::integral_constant<int, 1>())) return false;
+        if constexpr (SETS == 4) return f(std::integral_constant<int, 2>()) && f(std::integral_constant<int, 3>());
+        return true;
+    };
+    each_set([&](auto set) { request(set, decltype(set)::value * MMT_K); return true; });   // (a stage past K is all zeros)
+    for (int k0 = 0; k0 < a.K; k0 += SETS * MMT_K) {
+        if (!each_set([&](auto set) {
+                const int k = k0 + decltype(set)::value * MMT_K;
+                if (k >= a.K) return false;
+                stage(set);
+                if (k + SETS * MMT_K < a.K) request(set, k + SETS * MMT_K);
+                __syncthreads();
+                multiply(set);
+                return true;
+            })) break;
     }
     // register r of a lane: weight row (r & 3) + 8 (r >> 2) + 4 kg of the tile, token = lane & 31
 #pragma unroll
