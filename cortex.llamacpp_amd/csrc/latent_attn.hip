@@ -8,6 +8,9 @@
 // a learned per-head logit with neither key nor value behind it.  An optional output gate multiplies head h's attended latent by sigmoid(gate[t][h]) (a factor per
 // head: it commutes with W_uv).  Everything here is f32: positions, angles, scores, weights, the running sums.
 //
+// latent_tile (rows that allow 16-byte loads): (row, head) pairs as the columns of products on the f32 matrix cores; latent_attn: one workgroup per pair, any alignment.
+// Scans cut into runs of cells leave records that latent_attn_merge joins.
+//
 // latent_prep: per token, the two RMS norms behind the down-projections (query latent -> cq, key / value latent -> cache row) and the rotation of the
 // shared key part into the cache row.  Interleaved pairs (2i, 2i + 1), or entry i with entry i + half the turning part; the per-pair frequency table (YaRN blend included) comes from the host.
 #include "attn_merge_dev.h"

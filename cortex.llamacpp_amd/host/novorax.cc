@@ -299,7 +299,7 @@ bool Context::init_novorax(std::string &err) {
     nvx_seq_len_.assign(NS, 0);
     nvx_prev_tok_.assign(NS, -1);
     // activations
-    const size_t A = (size_t)std::max(M.max_down, M.max_proj), TOP = (size_t)std::max(M.max_top, 1);
+    const size_t A = (size_t)((std::max(M.max_down, M.max_proj) + 3) & ~3), TOP = (size_t)std::max(M.max_top, 1);
     x_ = (float *)dalloc(T * W * 4);
     xn_ = (float *)dalloc(T * W * 4);
     xo_ = (float *)dalloc(T * W * 4);
@@ -336,7 +336,6 @@ bool Context::init_novorax(std::string &err) {
     }
     if (!x_ || !xn_ || !xo_ || !nvx_x0_ || !nvx_xcat_ || !nvx_y_ || !nvx_a_ || !nvx_cq_ || !nvx_q_ || !nvx_qa_ || !nvx_lat_ || !nvx_att_ || !nvx_o_ || !nvx_ff_) { err = "activation buffer allocation failed"; return false; }
     if (M.max_top > 0) {
-        nvx_xg_ = (float *)dalloc(T * TOP * W * 4);
         nvx_yg_ = (float *)dalloc(T * TOP * W * 4);
         nvx_ids_ = (int32_t *)dalloc(T * TOP * 4);
         nvx_meta_ = (int32_t *)dalloc((size_t)(2 * M.max_expert + 1) * 4);
@@ -344,7 +343,7 @@ bool Context::init_novorax(std::string &err) {
         nvx_tokof_ = (int32_t *)dalloc(T * TOP * 4);
         nvx_rw_ = (float *)dalloc(T * TOP * 4);
         nvx_rwg_ = (float *)dalloc(T * TOP * 4);
-        if (!nvx_xg_ || !nvx_yg_ || !nvx_ids_ || !nvx_meta_ || !nvx_slot_ || !nvx_tokof_ || !nvx_rw_ || !nvx_rwg_) { err = "expert batch buffers allocation failed"; return false; }
+        if (!nvx_yg_ || !nvx_ids_ || !nvx_meta_ || !nvx_slot_ || !nvx_tokof_ || !nvx_rw_ || !nvx_rwg_) { err = "expert batch buffers allocation failed"; return false; }
     }
     if (M.max_mlstm_heads > 0) {
         const size_t TH = T * (size_t)M.max_mlstm_heads;
@@ -599,7 +598,7 @@ hipError_t Context::run_layers_novorax(int T) {
             NVX_TRY(nvx_close_linear(L.o, nvx_att_, H * L.vdim, T, L.norm1b));
             prof_mark("latent_attention");
         } else if (L.type == NVX_MLSTM) {
-            const int LD_P = L.proj.N;
+            const int LD_P = (L.proj.N + 3) & ~3;                // (rows on 16-byte boundaries whatever the head count)
             NVX_TRY(nvx_linear(L.proj, x_, W, T, nvx_a_, LD_P, MMB_STORE, nullptr, 1.0f, L.norm1));
             MlstmArgs ma{};
             ma.p = nvx_a_; ma.ld_p = LD_P; ma.o = nvx_o_; ma.ld_o = H * L.vdim; ma.H = H; ma.D = L.dim; ma.VD = L.vdim; ma.gate_cap = L.gate_cap;

@@ -215,7 +215,7 @@ class Context {
     float *nvx_mw_A_ = nullptr, *nvx_mw_v_ = nullptr; double *nvx_mw_F_ = nullptr;   // the mLSTM's work buffers for long segments (MlstmArgs)
     float *nvx_part_ = nullptr;                             // records of attention scans that were cut into runs (single-token steps; short prompt batches)
     size_t nvx_part_floats_ = 0;
-    float *nvx_att_ = nullptr, *nvx_o_ = nullptr, *nvx_ff_ = nullptr, *nvx_xg_ = nullptr, *nvx_yg_ = nullptr;
+    float *nvx_att_ = nullptr, *nvx_o_ = nullptr, *nvx_ff_ = nullptr, *nvx_yg_ = nullptr;
     int32_t *nvx_ids_ = nullptr, *nvx_meta_ = nullptr, *nvx_slot_ = nullptr, *nvx_tokof_ = nullptr;
     // [7][n_ubatch]: start, length, slot of every segment; upper and lower scan bound of every token; rows of its segment in front of every token; its row of the bigram table
     int32_t *h_seg_ = nullptr, *d_seg_ = nullptr;
