@@ -450,11 +450,12 @@ hipError_t launch_moe_combine(float *x, const float *eo, const float *w, int T, 
 // One workgroup of 16 waves.  The selections are staged in LDS; wave w owns experts w, w + 16, ...: it walks the selections
 // 64 at a time in (token, rank) order, a ballot marks the ones that chose its expert and a prefix count of the ballot
 // gives each its row: stable, deterministic, no atomics.  (Runs once per layer of a prompt batch: a few microseconds.)
-__global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *ids, int n_sel, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, const float *w, float *w_of) {
-    extern __shared__ int32_t sid[];               // [n_sel]
+__global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *ids, int n_sel, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, const float *w, float *w_of, int w_staged) {
+    extern __shared__ int32_t sid[];               // [n_sel], then - w_staged - the weights [n_sel]
+    float *const sw = reinterpret_cast<float *>(sid + n_sel);
     __shared__ int cnt[64], off[65];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    for (int i = tid; i < n_sel; i += 1024) sid[i] = ids[i];
+    for (int i = tid; i < n_sel; i += 1024) { sid[i] = ids[i]; if (w_staged) sw[i] = w[i]; }
     __syncthreads();
     for (int e = wave; e < n_expert; e += 16) {
         int c = 0;
@@ -487,7 +488,7 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *ids, int
                 const int row = r + __popcll(m & ((1ull << lane) - 1ull));
                 slot_of[b + lane] = row;
                 tok_of[row] = (b + lane) / k;
-                if (w_of) w_of[row] = w[b + lane];
+                if (w_of) w_of[row] = w_staged ? sw[b + lane] : w[b + lane];
             }
             r += __popcll(m);
         }
@@ -496,7 +497,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *ids, int
 hipError_t launch_moe_group(const int32_t *ids, int T, int k, int n_expert, int32_t *meta, int32_t *slot_of, int32_t *tok_of, hipStream_t st, const float *w, float *w_of) {
     if (w_of && !w) return hipErrorInvalidValue;
     if (n_expert > 64 || T * k <= 0 || (size_t)T * k * 4 > 60 * 1024) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), (size_t)T * k * 4, st, ids, T * k, k, n_expert, meta, slot_of, tok_of, w, w_of);
+    const int staged = w_of && (size_t)T * k * 8 <= 60 * 1024 ? 1 : 0;
+    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), (size_t)T * k * (staged ? 8 : 4), st, ids, T * k, k, n_expert, meta, slot_of, tok_of, w, w_of, staged);
     return hipGetLastError();
 }
 // one workgroup per grouped row: 16-byte copies of the code plane(s), then the small per-block planes
