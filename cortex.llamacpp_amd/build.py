@@ -17,9 +17,9 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 EXPERIMENTS = os.environ.get("MI355_BUILD_EXPERIMENTS", "0") == "1"
 SRC = [
     "csrc/mmvq.hip", "csrc/mmvq_fast.hip", "csrc/mmvq_stream.hip", "csrc/mmq.hip", "csrc/mmq_q80.hip", "csrc/act.hip", "csrc/misc.hip", "csrc/mmf.hip", "csrc/attn.hip", "csrc/attn_out.hip", "csrc/attn_prefill.hip", "csrc/clip.hip",
-    "csrc/mmb.hip", "csrc/latent_attn.hip", "csrc/mlstm.hip", "csrc/gq_attn.hip", "csrc/talk_attn.hip", "csrc/delta_rule.hip", "csrc/retention.hip", "csrc/routed_ff.hip",
+    "csrc/mmb.hip", "csrc/latent_attn.hip", "csrc/mlstm.hip", "csrc/gq_attn.hip", "csrc/talk_attn.hip", "csrc/delta_rule.hip", "csrc/retention.hip", "csrc/routed_ff.hip", "csrc/gated_scan.hip",
 ] + (["csrc/decode_engine.hip", "csrc/decode_mega.hip"] if EXPERIMENTS else ["csrc/experiments_absent.cc"]) + [
-    "host/gguf.cc", "host/runtime.cc", "host/novorax.cc", "host/fidepel.cc", "host/tuterax.cc", "host/dinilorn.cc", "host/vuzazen.cc", "host/tp_comm.cc", "host/vocab.cc", "host/sampling.cc", "host/grammar.cc", "host/json_schema.cc", "host/log.cc", "host/server_context.cc", "host/engine.cc",
+    "host/gguf.cc", "host/runtime.cc", "host/novorax.cc", "host/fidepel.cc", "host/tuterax.cc", "host/dinilorn.cc", "host/vuzazen.cc", "host/rarutar.cc", "host/tp_comm.cc", "host/vocab.cc", "host/sampling.cc", "host/grammar.cc", "host/json_schema.cc", "host/log.cc", "host/server_context.cc", "host/engine.cc",
     "host/hip_backend.cc", "host/tp_split.cc", "host/clip.cc", "host/image_decode.cc", "csrc/c_api.cc",
 ]
 HDRS = ["csrc/dev_common.h", "csrc/kernels.h", "csrc/attn_merge_dev.h", "csrc/quant_dev.h", "csrc/mmvq_fast_dev.h", "csrc/mmvq_stream_dev.h", "csrc/attn_decode_dev.h", "host/gguf.h", "host/runtime.h", "host/tp_comm.h", "host/json.h", "host/vocab.h",

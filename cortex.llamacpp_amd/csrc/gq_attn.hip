@@ -12,7 +12,8 @@
 //
 // Optional per layer: a query multiplier that grows with the logarithm of the position (in steps of `every` positions); a learned bias per (distance bucket,
 // head) added to the score behind the soft cap (the host hands over the distance -> bucket table); cells at the first `keep_first` positions that stay seen
-// outside the window; the neighbour layout of the rotation (entry 2i with 2i + 1); several score maps per head over the same values - every (head, map) then
+// outside the window; chunks of positions instead of a window (a token sees its own chunk only); values that are the projected keys; queries and keys
+// divided by their root mean square behind the turn; a factor of cos and sin; the neighbour layout of the rotation (entry 2i with 2i + 1); several score maps per head over the same values - every (head, map) then
 // runs as a query head of its own with its own key head, and gq_maps_out joins two maps: a1 - lambda a2, unit RMS, a constant, an elementwise sigmoid gate.
 //
 // Turned values (optional): every value head is stored turned by its own position over all its entries, in the same half-and-half pairing; the weighted sum
@@ -55,11 +56,12 @@ __global__ __launch_bounds__(NT) void gq_prep_kernel(GqPrepArgs a) {
     const int t = blockIdx.x, tid = threadIdx.x;
     const int GK = a.G * (a.maps > 1 ? a.maps : 1);             // key heads: one per (value head, map)
     const int NQ = a.H * a.dim, NK = GK * a.dim, NV = a.G * a.vdim, half = a.rot_dims >> 1;
-    float *const conv_row = gq_lds, *const head_inv = gq_lds + (CONV ? NQ + NK + NV : 0);       // norm per head: [H + GK] inverse root mean squares; v_unit: [G] behind them
+    const int NVP = a.v_is_k ? 0 : NV;                          // value rows of p
+    float *const conv_row = gq_lds, *const head_inv = gq_lds + (CONV ? NQ + NK + NVP : 0);       // norm per head: [H + GK] inverse root mean squares; v_unit: [G] behind them
     float *const v_inv = head_inv + a.H + GK;
     const float *qr = a.p + (size_t)t * a.ld_p;
     if (CONV) {
-        const int C = NQ + NK + NV, back = a.conv_taps - 1, ago = a.tok_ago[t];
+        const int C = NQ + NK + NVP, back = a.conv_taps - 1, ago = a.tok_ago[t];
         float *state = a.conv_state + (size_t)a.tok_slot[t] * back * C;
         const bool vec = ((C | a.ld_p) & 3) == 0 && ((reinterpret_cast<uintptr_t>(a.p) | reinterpret_cast<uintptr_t>(a.conv_wt) | reinterpret_cast<uintptr_t>(a.conv_state)) & 15) == 0;
         if (vec) {                                              // four channels per thread
@@ -94,7 +96,7 @@ __global__ __launch_bounds__(NT) void gq_prep_kernel(GqPrepArgs a) {
         __syncthreads();
         qr = conv_row;
     }
-    const float *kr = qr + NQ, *vr = kr + NK;
+    const float *kr = qr + NQ, *vr = a.v_is_k ? kr : kr + NK;
     float inv_q = 1.0f, inv_k = 1.0f;
     if (a.v_unit) {                                             // sixteen lanes per value head
         for (int g = tid >> 4; g < a.G; g += NT / 16) {
@@ -105,13 +107,15 @@ __global__ __launch_bounds__(NT) void gq_prep_kernel(GqPrepArgs a) {
             if ((tid & 15) == 0) v_inv[g] = 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
         }
     }
-    const bool per_head = a.norm_per_head && a.wq_norm && a.wk_norm;
+    const bool per_head = (a.norm_per_head && a.wq_norm && a.wk_norm) || a.unit_behind;
     if (per_head) {
         // sixteen lanes per head, queries then keys (q | k lie side by side in the row): every lane group's loads are on their way at once
         for (int hh = tid >> 4; hh < a.H + GK; hh += NT / 16) {
             const float *src = qr + (size_t)hh * a.dim;
             float ss = 0.0f;
-            for (int i = tid & 15; i < a.dim; i += 16) { const float v = src[i]; ss = fmaf(v, v, ss); }
+            // (behind the turn: a turn changes no sum of squares, the factor of its cos and sin does)
+            const float turned = a.unit_behind ? a.rot_mscale : 1.0f;
+            for (int i = tid & 15; i < a.dim; i += 16) { const float v = i < a.rot_dims ? src[i] * turned : src[i]; ss = fmaf(v, v, ss); }
 #pragma unroll
             for (int o = 8; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
             if ((tid & 15) == 0) head_inv[hh] = 1.0f / sqrtf(ss / (float)a.dim + a.eps);
@@ -129,7 +133,11 @@ __global__ __launch_bounds__(NT) void gq_prep_kernel(GqPrepArgs a) {
     const float p = (float)a.tok_pos[t];
     // (positions are exact in f32 up to 2^24, and so is the floor of the correctly rounded quotient for a whole-number step)
     const float q_temp = a.q_temp_every > 0.0f ? 1.0f + a.q_temp_coef * logf(floorf((p + 1.0f) / a.q_temp_every) + 1.0f) : 1.0f;
-    if (tid < half) sincosf(p * a.rot_freq[tid], &cs[1][tid], &cs[0][tid]);
+    if (tid < half) {
+        float sn, co;
+        sincosf(p * a.rot_freq[tid], &sn, &co);
+        cs[1][tid] = sn * a.rot_mscale; cs[0][tid] = co * a.rot_mscale;
+    }
     const int vhalf = a.v_rot_freq ? a.vdim >> 1 : 0;
     if (tid >= 128 && tid - 128 < vhalf) {                       // (the upper waves: beside the key / query table of the lower ones)
         const int j = tid - 128;
@@ -214,6 +222,8 @@ __device__ __forceinline__ GqHeads gq_heads(const GqAttnArgs &a, int h) {
     o.voff = (size_t)a.G * maps * a.dim + (size_t)kvh * a.vdim;
     return o;
 }
+// the first position a token at position p sees (keep_first aside)
+__device__ __forceinline__ int gq_first(const GqAttnArgs &a, int p) { return a.window > 0 ? p - a.window + 1 : a.chunk > 0 ? p - p % a.chunk : 0; }
 // the learned bias of head h at distance dist >= 0
 __device__ __forceinline__ float gq_rel_bias(const GqAttnArgs &a, int dist, int h) {
     const int b = dist < a.n_dist ? a.dist_bucket[dist] : a.rel_rows - 1;
@@ -250,7 +260,7 @@ __global__ __launch_bounds__(512) void gq_attn_kernel(GqAttnArgs a) {
     const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, li = lane & 15;
     const GqHeads hd = gq_heads(a, h);
     const size_t L = hd.row, koff = hd.koff, voff = hd.voff;
-    const int tpos = a.tok_pos[t];
+    const int tpos = a.tok_pos[t], first = gq_first(a, tpos);
     const uint64_t sbit = 1ull << (a.tok_seq[t] & 63);
     for (int i = tid; i < LP; i += blockDim.x) qv[i] = i < D ? a.q[(size_t)t * a.ld_q + (size_t)h * D + i] : 0.0f;
     __syncthreads();
@@ -276,7 +286,7 @@ __global__ __launch_bounds__(512) void gq_attn_kernel(GqAttnArgs a) {
         if (c >= c_hi) return false;
         const int cp = a.cell_pos[c];
         dist = tpos - cp;
-        return cp >= 0 && cp <= tpos && (a.cell_seq[c] & sbit) != 0 && !(a.window > 0 && tpos - cp >= a.window && cp >= a.keep_first);
+        return cp >= 0 && cp <= tpos && (a.cell_seq[c] & sbit) != 0 && (cp >= first || cp < a.keep_first);
     };
     const auto fetch = [&](int c, bool vis, float (&dk)[NJ][4], float (&dv)[NJ][4]) {
         const float *kr = a.cache + (size_t)c * L + koff, *vr = a.cache + (size_t)c * L + voff;
@@ -368,6 +378,7 @@ __global__ __launch_bounds__(512) void gq_attn_kernel(GqAttnArgs a) {
     for (int w = 0; w < NW; w++) den += wl[w] > 0.0f ? wl[w] * expf(wm[w] - MM) : 0.0f;
     float inv = den > 0.0f ? 1.0f / den : 0.0f;
     if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)t * a.ld_gate + h]));
+    inv *= a.out_mult;
     if (a.v_cs) {                                               // (vdim is even)
         const int vhalf = VD >> 1;
         const float *cs = a.v_cs + (size_t)t * VD;
@@ -399,6 +410,7 @@ __global__ __launch_bounds__(NT) void gq_attn_merge_kernel(GqAttnArgs a, int spl
     const float den = attn_merge_runs<NT>(a.part + ((size_t)t * a.H + h) * splits * (size_t)(VD + 2), splits, VD, a.sink ? a.sink[h] : -INFINITY, fac, part, sums);
     float inv = den > 0.0f ? 1.0f / den : 0.0f;
     if (a.gate) inv *= 1.0f / (1.0f + expf(-gate));
+    inv *= a.out_mult;
     float *out = a.out + (size_t)t * a.ld_out + (size_t)h * VD;
     if (a.v_cs) {                                               // (vdim is even)
         const int vhalf = VD >> 1;
@@ -442,7 +454,7 @@ static hipError_t launch_gq_attn_nj(const GqAttnArgs &a, hipStream_t st) {
 // owns RPT rows x 4 columns per slice).  NVC = ceil(vdim / 64).  dim and vdim multiples of 4.  RPT = 4 (64-row tiles) where that still gives the device
 // two workgroups per CU, else 2: a short prompt is bound by the chain of blocks one workgroup walks, not by arithmetic.
 constexpr int GQT_B = 64, GQT_DC = 32, GQT_LDQ = GQT_DC + 4, GQT_LDP = GQT_B + 4;
-constexpr size_t gqt_lds_floats(int rows) { return (size_t)(rows + GQT_B) * GQT_LDQ + (size_t)(rows + GQT_B) * GQT_LDP + 2 * rows + 3 * GQT_B; }
+constexpr size_t gqt_lds_floats(int rows) { return (size_t)(rows + GQT_B) * GQT_LDQ + (size_t)(rows + GQT_B) * GQT_LDP + 3 * rows + 3 * GQT_B; }
 
 template <int NVC, int RPT>
 __global__ __launch_bounds__(256) void gq_attn_tile_kernel(GqAttnArgs a) {
@@ -450,22 +462,24 @@ __global__ __launch_bounds__(256) void gq_attn_tile_kernel(GqAttnArgs a) {
     extern __shared__ float lds[];
     float *Qc = lds, *Kc = Qc + BQ * GQT_LDQ, *P = Kc + GQT_B * GQT_LDQ, *Vc = P + BQ * GQT_LDP;
     uint64_t *cseq = reinterpret_cast<uint64_t *>(Vc + GQT_B * GQT_LDP);                     // (an even number of floats in: 8-byte aligned)
-    int *cpos = reinterpret_cast<int *>(cseq + GQT_B), *rpos = cpos + GQT_B, *rseq = rpos + BQ;
+    int *cpos = reinterpret_cast<int *>(cseq + GQT_B), *rpos = cpos + GQT_B, *rseq = rpos + BQ, *rfirst = rseq + BQ;
     __shared__ int red[4];
     const int D = a.dim, VD = a.vdim, tid = threadIdx.x, tq = tid >> 4, tc = tid & 15;
     const int row0 = blockIdx.x * BQ, h = blockIdx.y;
     const GqHeads hd = gq_heads(a, h);
     const size_t L = hd.row, koff = hd.koff, voff = hd.voff;
     const int n_kv = *a.n_kv_dev;
-    // the tile's rows: position and sequence of each; over the tile: first and last position, the union of sequences, the range of cells to walk
+    // the tile's rows: position, first position seen and sequence of each; over the tile: the first position any of them sees, the last position, the union of
+    // sequences, the range of cells to walk
     int my_lo = 0x7fffffff, my_hi = 0, my_pmin = 0x7fffffff, my_pmax = -1;
     if (tid < BQ) {
         const int r = row0 + tid;
         const bool live = r < a.T;
         rpos[tid] = live ? a.tok_pos[r] : -1;
+        rfirst[tid] = live ? gq_first(a, rpos[tid]) : 0;
         rseq[tid] = live ? (a.tok_seq[r] & 63) : -1;
         if (live) {
-            my_pmin = my_pmax = rpos[tid];
+            my_pmin = rfirst[tid]; my_pmax = rpos[tid];
             my_lo = a.tok_lo ? a.tok_lo[r] : 0;
             my_hi = a.tok_hi ? (a.tok_hi[r] < n_kv ? a.tok_hi[r] : n_kv) : n_kv;
         }
@@ -503,7 +517,7 @@ __global__ __launch_bounds__(256) void gq_attn_tile_kernel(GqAttnArgs a) {
             int cp = -1; uint64_t cs = 0;
             if (c < c_end) { cp = a.cell_pos[c]; cs = a.cell_seq[c]; }
             cpos[tid] = cp; cseq[tid] = cs;
-            any = cp >= 0 && cp <= pmax && (cs & seqs) != 0 && !(a.window > 0 && pmin - cp >= a.window && cp >= a.keep_first);
+            any = cp >= 0 && cp <= pmax && (cs & seqs) != 0 && (cp >= pmin || cp < a.keep_first);
         }
         if (!__syncthreads_or(any)) continue;
         // ---- S = Q K^T
@@ -550,14 +564,14 @@ __global__ __launch_bounds__(256) void gq_attn_tile_kernel(GqAttnArgs a) {
         // ---- the running softmax of each row; P to LDS
 #pragma unroll
         for (int i = 0; i < RPT; i++) {
-            const int r = tq * RPT + i, rp = rpos[r];
+            const int r = tq * RPT + i, rp = rpos[r], rf = rfirst[r];
             const uint64_t rbit = rseq[r] >= 0 ? 1ull << rseq[r] : 0ull;
             bool vis[4];
             float bm = -INFINITY;
 #pragma unroll
             for (int j = 0; j < 4; j++) {
                 const int cp = cpos[tc + 16 * j];
-                vis[j] = cp >= 0 && cp <= rp && (cseq[tc + 16 * j] & rbit) != 0 && !(a.window > 0 && rp - cp >= a.window && cp >= a.keep_first);
+                vis[j] = cp >= 0 && cp <= rp && (cseq[tc + 16 * j] & rbit) != 0 && (cp >= rf || cp < a.keep_first);
                 if (vis[j]) {
                     if (a.rel) s[i][j] += gq_rel_bias(a, rp - cp, h);
                     bm = fmaxf(bm, s[i][j]);
@@ -635,7 +649,8 @@ __global__ __launch_bounds__(256) void gq_attn_tile_kernel(GqAttnArgs a) {
             den = l[i] * sc + expf(a.sink[h] - MM);
         }
         float inv = den > 0.0f ? sc / den : 0.0f;
-        if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)r * a.ld_gate + h]));   // (a factor per head: it commutes with the turn back that may follow)
+        if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)r * a.ld_gate + h]));   // (a factor per head, like the one below: it commutes with the turn back that may follow)
+        inv *= a.out_mult;
 #pragma unroll
         for (int vc = 0; vc < NVC; vc++) {
             const int col = vc * 64 + tc * 4;
@@ -687,13 +702,15 @@ hipError_t launch_gq_prep(const GqPrepArgs &a, hipStream_t st) {
     if (a.v_rot_freq && ((a.vdim & 1) || a.vdim > GQ_MAX_D || !a.v_cs)) return hipErrorInvalidValue;
     const int n_heads = a.H + a.G * (a.maps > 1 ? a.maps : 1);
     if (a.maps > 1 && a.H % a.maps != 0) return hipErrorInvalidValue;
-    if (a.norm_per_head && (size_t)n_heads * sizeof(float) > 32 * 1024) return hipErrorInvalidValue;
-    size_t lds = (a.norm_per_head || a.v_unit ? (size_t)n_heads : 0) + (a.v_unit ? (size_t)a.G : 0);
+    if (a.v_is_k && (a.vdim != a.dim || a.maps > 1)) return hipErrorInvalidValue;
+    if (a.unit_behind && (a.wq_norm || a.wk_norm)) return hipErrorInvalidValue;
+    if ((a.norm_per_head || a.unit_behind) && (size_t)n_heads * sizeof(float) > 32 * 1024) return hipErrorInvalidValue;
+    size_t lds = (a.norm_per_head || a.unit_behind || a.v_unit ? (size_t)n_heads : 0) + (a.v_unit ? (size_t)a.G : 0);
     if (!a.conv_wt) {
         hipLaunchKernelGGL((gq_prep_kernel<256, false>), dim3((unsigned)a.T), dim3(256), lds * sizeof(float), st, a);
         return hipGetLastError();
     }
-    const size_t C = (size_t)a.H * a.dim + (size_t)a.G * (a.maps > 1 ? a.maps : 1) * a.dim + (size_t)a.G * a.vdim;
+    const size_t C = (size_t)a.H * a.dim + (size_t)a.G * (a.maps > 1 ? a.maps : 1) * a.dim + (a.v_is_k ? 0 : (size_t)a.G * a.vdim);
     if (a.conv_taps < 1 || !a.tok_ago || !a.tok_slot || (a.conv_taps > 1 && !a.conv_state) || C > (size_t)GQ_CONV_MAX_CHANNELS) return hipErrorInvalidValue;
     lds = (lds + C) * sizeof(float);
     const auto allow = [&](const void *f) { return lds > 60 * 1024 ? hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) : hipSuccess; };
@@ -731,6 +748,7 @@ hipError_t launch_gq_attn(const GqAttnArgs &a, hipStream_t st) {
     if (a.T <= 0) return hipSuccess;
     const int maps = a.maps > 1 ? a.maps : 1;
     if (a.H % maps != 0 || !gq_attn_shape_ok(a.H / maps, a.G, a.dim, a.vdim) || (a.v_cs && (a.vdim & 1))) return hipErrorInvalidValue;
+    if (a.chunk > 0 && (a.window > 0 || a.talk)) return hipErrorInvalidValue;
     if (a.rel && (!a.dist_bucket || a.n_dist < 0 || a.rel_rows < 1)) return hipErrorInvalidValue;
     if (a.talk) return launch_talk_attn(a, st);
     // batches: the tiled pass (16-byte loads everywhere: head sizes, strides and bases must allow them); a few rows: one workgroup per (row, head)

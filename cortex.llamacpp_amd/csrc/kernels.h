@@ -267,8 +267,8 @@ hipError_t launch_moe_scatter_combine(float *x, const float *y, const float *w, 
 // Outer index z < nz, one of: plain strides (x_zs / w_zs / y_zs elements; per-head products); meta != nullptr: z is an expert, its rows of X and Y are
 // [meta[nz + z], + meta[z]) (launch_moe_group's counts | offsets; T = upper bound of any expert's rows); sel != nullptr: z is a (token, rank) pair - weight set
 // sel[z], row z / sel_div of X, row z of Y.
-// y | relu(y)^2 | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = min(W x, epi_limit), u = clamp(W2 x, -epi_limit, epi_limit)
-enum { MMB_STORE = 0, MMB_RELU2 = 1, MMB_SILU_MUL = 2, MMB_GELU_MUL = 3, MMB_CLAMP_SWIGLU = 4 };
+// y | relu(y)^2 | sigmoid(y)^epi_limit | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = min(W x, epi_limit), u = clamp(W2 x, -epi_limit, epi_limit)
+enum { MMB_STORE = 0, MMB_RELU2 = 1, MMB_SIGMOID_POW = 2, MMB_SILU_MUL = 3, MMB_GELU_MUL = 4, MMB_CLAMP_SWIGLU = 5 };   // (from MMB_SILU_MUL on: gated, two weight sets)
 constexpr int MMB_VEC_ROWS = 16;                               // up to this many rows take the one-wave-per-column kernel
 struct MMBArgs {
     const float *x = nullptr; int ldx = 0;
@@ -276,7 +276,7 @@ struct MMBArgs {
     float *y = nullptr; int ldy = 0;
     int T = 0, N = 0, K = 0, epi = MMB_STORE, f32 = 0;
     float out_scale = 1.0f;                                    // multiplies every stored value (a model's logit scale)
-    float epi_limit = 0.0f;                                    // MMB_CLAMP_SWIGLU: the clamp
+    float epi_limit = 0.0f;                                    // MMB_CLAMP_SWIGLU: the clamp; MMB_SIGMOID_POW: the exponent
     const float *bias = nullptr;                               // nullable, [N] f32: added to W x before the epilogue (the same vector for every outer index)
     const float *row_scale = nullptr;                          // nullable, a factor on W x (and W2 x) of every row, by the row's place in Y in front of y_map; in front of the bias
     const float *resid = nullptr;                              // nullable, indexed like Y (and may be Y): added behind the epilogue
@@ -286,6 +286,9 @@ struct MMBArgs {
     const int32_t *sel = nullptr; int sel_div = 1;
     // prologue of the few-rows kernel (T <= MMB_VEC_ROWS): the rows of X are RMS-normed on the fly, x / sqrt(mean(x^2) + pn_eps) * (pn_off + pn_w[k])
     const float *pn_w = nullptr; float pn_off = 0.0f, pn_eps = 0.0f;
+    // ... or layer-normed instead, (x - mean) / sqrt(var + pn_eps) * pn_w[k] + b[k]: ln (and ln2 beside w2) set, [2][N] f32 - what every output column makes of the norm's
+    // weight and of its bias alone: sum_k w[n][k] pn_w[k], then sum_k w[n][k] b[k] (nz = 1, no sel / meta)
+    const float *ln = nullptr, *ln2 = nullptr;
 };
 hipError_t launch_mmb(const MMBArgs &a, hipStream_t st);
 
@@ -329,7 +332,9 @@ struct GqPrepArgs {
     int T, H, G, dim, vdim;
     const float *wq_norm, *wk_norm; float eps;   // nullable: RMS norm over the whole query / key projection (all heads at once), plain weights [H*dim] / [G*dim]
     int norm_per_head;                     // 1: the statistic is taken over each head's dim entries instead, and the weights are [dim], shared by the heads
+    int unit_behind;                       // 1: every query and key head is divided by its root mean square behind the turn, no weights (wq_norm / wk_norm unset)
     int rot_dims; const float *rot_freq;   // the first rot_dims entries of every q / k head turn, entry i with entry i + rot_dims / 2; [rot_dims / 2] radians per position
+    float rot_mscale;                      // multiplies cos and sin
     float q_scale; const float *head_scale;      // the query is multiplied by q_scale * head_scale[h] (nullable): the score's constant factors
     int maps;                              // score maps per head (0 or 1: one)
     int rot_neighbours;                    // 1: entry 2i turns with entry 2i + 1 instead of entry i with entry i + rot_dims / 2
@@ -341,6 +346,7 @@ struct GqPrepArgs {
     // the attention's output is then turned back by the query's position, so that only position differences remain in the sum.  v_cs: [T][vdim] - the token's
     // cos (first vdim / 2) and sin per pair, written here for the attention launch (GqAttnArgs::v_cs)
     const float *v_rot_freq; float *v_cs;
+    int v_is_k;                            // 1: p holds no value rows - a value head is its key head as projected (vdim = dim), in front of norm and turn
     int v_unit;                            // 1: every value head is divided by its root mean square (eps as above, no weight) before it is stored
     // nullable: a short causal convolution over time on every channel of q, k and v, in front of all of the above: u_t = sum_j conv_wt[j][c] p_(t - taps + 1 + j),
     // zeros before the sequence's start.  conv_wt: [taps][C], C = H*dim + G*dim + G*vdim in p's channel order; conv_state: [slot][taps - 1][C], the inputs before
@@ -361,6 +367,8 @@ struct GqAttnArgs {
     const int32_t *cell_pos; const uint64_t *cell_seq; const int32_t *tok_pos, *tok_seq; const int32_t *n_kv_dev;
     int window;                            // cells at distance 0 .. window - 1 are seen; 0 = every earlier cell
     int keep_first;                        // with a window: cells at positions below keep_first stay seen at any distance
+    int chunk;                             // > 0 (no window): cells whose position lies in the token's own chunk of `chunk` positions, counted from position 0
+    float out_mult;                        // multiplies every output behind softmax and gate
     int maps;                              // score maps per head (0 or 1: one); H counts (head, map) pairs, G the value heads
     // nullable: a learned bias per (distance bucket, head) added to the score behind the soft cap: rel[bucket(d) * H + h], bucket(d) = dist_bucket[d]
     // for d < n_dist, else rel_rows - 1
@@ -502,6 +510,46 @@ inline int delta_work_row(int H, int G, int D, int VD, int per_channel) { return
 bool delta_shape_ok(int H, int G, int D, int VD, int taps);
 hipError_t launch_delta_prep(const DeltaArgs &a, hipStream_t st);    // convolution + silu, beta, decays for the segments' rows; moves the convolution state on
 hipError_t launch_delta_scan(const DeltaArgs &a, hipStream_t st);    // unit q / k and the recurrence, from each slot's state and back into it
+
+// ---------------------------------------------------------------- linear recurrences with a learned decay (gated_scan.hip)
+// Per head a state S [D][VD] f32 per sequence slot:  S <- diag(a) S + k v^T;  o = S^T (q_scale q) [+ skip v].  Decay per key channel (dt == nullptr): a = alpha, or from
+// its low-rank form in steps; one decay per head (dt set): d = softplus(dt + dt_bias), a = exp(-exp(A_log) d), and k counts d times.  Head h reads q / k head h / share.
+struct GatedScanArgs {
+    const float *p; int ld_p;              // [T] rows; q / k / v of a row start at columns off_q / off_k / off_v: [H / share][D], [H / share][D], [H][VD]
+    int off_q, off_k, off_v, share;
+    float q_scale;
+    const float *alpha; int ld_alpha;      // [T][H*D] decays per key channel (batches; steps without lr_w)
+    // steps, nullable: a = sigmoid(lr_w z1 + lr_bias)^inv_tau, z1 = the row's `rank` entries at column off_lr of p; lr_w [H*D][rank] bf16, lr_bias [H*D]
+    const unsigned short *lr_w; const float *lr_bias; int rank, off_lr; float inv_tau;
+    const float *dt; int ld_dt; const float *dt_bias, *A_log;   // one decay per head: [T][H] pre-activations, [H], [H]
+    const float *skip;                     // nullable, [H]
+    // steps, nullable: q, k and v are channels of p that go through a short causal convolution with bias and silu first: conv_wt [taps][conv_C], conv_b [conv_C]
+    // (nullable), conv_state [slot][taps - 1][conv_C] oldest first, read only; batches come convolved (launch_conv_silu)
+    const float *conv_wt, *conv_b, *conv_state; int conv_taps, conv_C;
+    float *S;                              // [slot][H][D][VD]
+    float *o; int ld_o;                    // [T][H][VD]
+    int H, D, VD;
+    // steps, nullable (gated_step_closes(VD)): y = o / rms(o over the head) * norm_w [VD] * silu(gate) instead of o
+    float *y; int ld_y; const float *gate; int ld_gate; const float *norm_w; float eps;
+    const int32_t *seg_start, *seg_len, *seg_slot; int n_seg;   // runs of consecutive batch rows of one sequence each, side by side; no slot twice in a launch
+    int row0, max_len;                     // first row of the first segment; rows of the longest one (1: a step)
+    // work buffers of longer segments, by batch row: A [T][H][64]; per channel: scaled q and k [T][H][D]; per head: factors of a row [T][H] each; by chunk
+    // (gated_scan_chunks places): decay of the chunk [H][D] or [H], state in front of it [H][D][VD]
+    float *w_A, *w_q, *w_k, *w_p, *w_s, *w_g, *w_S;
+};
+constexpr int GATED_SCAN_MAX_DIM = 4096;
+inline size_t gated_scan_chunks(size_t rows, size_t segs) { return rows / 64 + segs + 1; }
+bool gated_scan_shape_ok(int H, int share, int D, int VD);
+bool gated_step_closes(int VD);
+hipError_t launch_gated_scan(const GatedScanArgs &a, hipStream_t st);
+// y[t][c] = silu(bias[c] + sum_j wt[j][c] u[t - taps + 1 + j][c]) over rows of p (C channels); tok_ago: rows of the token's own segment in front of it; what lies further back
+// comes from state [slot][taps - 1][C] (launch_conv_state moves it on behind)
+hipError_t launch_conv_silu(const float *p, int ld_p, int C, const float *wt, const float *bias, int taps, const float *state, const int32_t *tok_ago, const int32_t *tok_slot, int T,
+                            float *y, int ld_y, hipStream_t st);
+// y[t] = u * w, u = o silu(z) with each of `parts` parts of n entries over its own root mean square.  mv (state set; every row a segment of its own): the rows' convolution
+// state moves on in the same launch
+struct ConvMove { float *state; const float *p; int ld_p, C, taps; const int32_t *seg_slot; };
+hipError_t launch_gated_norm(const float *o, int ld_o, const float *z, int ld_z, const float *w, int T, int parts, int n, float eps, float *y, int ld_y, const ConvMove &mv, hipStream_t st);
 
 // ---------------------------------------------------------------- attention side (attn.hip)
 // words between two merge-ticket counters / hand-over flags of the decode attention kernels (attn_decode_dev.h, attn_out.hip): one 128-byte line each

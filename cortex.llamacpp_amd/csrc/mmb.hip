@@ -12,7 +12,7 @@
 //   * mmb_mfma  - batches in bf16 mode: LDS-tiled, activations rounded to bf16 on the way in, v_mfma_f32_32x32x16_bf16, f32 accumulation.
 //   * mmb_f32   - batches in f32 mode (and every shape the other two refuse): LDS-tiled, v_fma_f32 only - products of an f32 activation and a bf16 weight
 //                 widened exactly, no reduced-precision matrix mode anywhere.
-// Epilogues: store | relu(y)^2 | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = W x capped from above and u = W2 x clamped
+// Epilogues: store | relu(y)^2 | sigmoid(y)^e | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = W x capped from above and u = W2 x clamped
 // to +- the same limit (the gated ones: two weight sets, one pass over the activations).  Around the epilogue, each optional: a factor per row on W x (and W2 x)
 // - linear layers without a bias: the row of X itself times that number -, an f32 bias per output column in front of it, a residual row added behind it.  A
 // grouped batch may read its rows of X, and write its rows of Y, through maps (no gather in front of the launch, no scatter behind it).
@@ -37,6 +37,7 @@ __device__ __forceinline__ float epi_apply(int epi, float a, float b, float lim 
         const float g = fminf(a, lim), u = fminf(fmaxf(b, -lim), lim);
         return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
     }
+    if (epi == MMB_SIGMOID_POW) return expf(-lim * (fmaxf(-a, 0.0f) + log1pf(expf(-fabsf(a)))));   // (sigmoid = e^-softplus(-a))
     if (epi == MMB_RELU2) { const float r = a > 0.0f ? a : 0.0f; return r * r; }
     if (epi == MMB_SILU_MUL) return a / (1.0f + expf(-a)) * b;
     if (epi == MMB_GELU_MUL) return 0.5f * a * (1.0f + tanhf(0.7978845608028654f * (a + 0.044715f * a * a * a))) * b;   // the tanh form of gelu; sqrt(2 / pi)
@@ -73,11 +74,34 @@ __device__ __forceinline__ void y_store(const MMBArgs &a, const ZView &v, size_t
     v.y[yr + n] = epi_fixed<EPI>(a, a.bias ? s1 + a.bias[n] : s1, s2) * a.out_scale + res;
 }
 
+// ---- the layer norm of a row inside a product (LN): the walk over k sums (x - c) w_k g_k, (x - c) and (x - c)^2 around a value c near the row's mean - the mean of its
+// first entries, so that nothing is lost in the difference of large sums -, and what is left follows from the column's own sums with the norm's weight and bias
+template <bool VEC>
+__device__ __forceinline__ float row_middle(const float *x, int K, int lane) {
+    float s = 0.0f;
+    if (VEC) {
+        if (lane * 8 < K) {
+            const f32x4 u = *reinterpret_cast<const f32x4 *>(x + lane * 8), w = *reinterpret_cast<const f32x4 *>(x + lane * 8 + 4);
+            s = ((u.x + u.y) + (u.z + u.w)) + ((w.x + w.y) + (w.z + w.w));
+        }
+    } else s = lane < K ? x[lane] : 0.0f;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+    const int n = VEC ? 512 : 64;
+    return s / (float)(K < n ? K : n);
+}
+__device__ __forceinline__ float row_offset(float sx, int K) {  // mean - c
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) sx += __shfl_xor(sx, o, 64);
+    return sx / (float)K;
+}
+__device__ __forceinline__ float ln_close(float s, float off, float inv, const float *ln, int n, int N) { return fmaf(s - off * ln[n], inv, ln[N + n]); }
+
 // ---------------------------------------------------------------- few rows: one wave per output column
 // Few rows against MANY output columns (single-token steps: the head, the feed-forward): a wave owns NR adjacent weight rows and keeps the activations of a
 // 512-wide piece of k in registers for all of them - the activation and norm-weight loads, which every wave repeats out of the caches, are paid once per NR
 // weight rows instead of once per row.  Up to TBR rows of X; 16-byte aligned operands; same arithmetic per output as mmb_vec_kernel.
-template <int NR, int TBR, int EPI>
+template <int NR, int TBR, int EPI, bool LN>
 __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = (blockIdx.x * 4 + wave) * NR;
@@ -91,10 +115,11 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
         wr[r] = v.w + (size_t)n * a.ldw;
         wr2[r] = gated ? v.w2 + (size_t)n * a.ldw : wr[r];
     }
-    float acc[NR][TBR], acc2[NR][TBR], ss[TBR];
+    float acc[NR][TBR], acc2[NR][TBR], ss[TBR], sx[LN ? TBR : 1], mid[LN ? TBR : 1];
 #pragma unroll
     for (int i = 0; i < TBR; i++) {
         ss[i] = 0.0f;
+        if (LN) sx[i] = 0.0f;
 #pragma unroll
         for (int r = 0; r < NR; r++) { acc[r][i] = 0.0f; acc2[r][i] = 0.0f; }
     }
@@ -105,6 +130,7 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
         rsc[i] = a.row_scale && i < nt ? a.row_scale[v.y0 + i] : 1.0f;
 #pragma unroll
         for (int r = 0; r < NR; r++) res[r][i] = v.resid && i < nt && n0 + r < a.N ? v.resid[y_row(a, v, i) + n0 + r] : 0.0f;
+        if (LN) mid[i] = i < nt ? row_middle<true>(x_row(a, v, i), a.K, lane) : 0.0f;
     }
     for (int k = lane * 8; k < a.K; k += 512) {
         u16x8 w8[NR], w28[NR];
@@ -125,6 +151,10 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
             const float *xr = x_row(a, v, i) + k;
             const f32x4 x0 = *reinterpret_cast<const f32x4 *>(xr), x1 = *reinterpret_cast<const f32x4 *>(xr + 4);
             float xs[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+            if (LN) {
+#pragma unroll
+                for (int e = 0; e < 8; e++) { xs[e] -= mid[i]; sx[i] += xs[e]; }
+            }
             if (pn) {
 #pragma unroll
                 for (int e = 0; e < 8; e++) { ss[i] = fmaf(xs[e], xs[e], ss[i]); xs[e] = xs[e] * pw[e]; }
@@ -144,13 +174,15 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
         float q = ss[i];
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1) q += __shfl_xor(q, o, 64);
-        const float inv = pn ? 1.0f / sqrtf(q / (float)a.K + a.pn_eps) : 1.0f;
+        const float off = LN ? row_offset(sx[i], a.K) : 0.0f;
+        const float inv = pn ? 1.0f / sqrtf(q / (float)a.K - off * off + a.pn_eps) : 1.0f;
 #pragma unroll
         for (int r = 0; r < NR; r++) {
             float s1 = acc[r][i], s2 = acc2[r][i];
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) { s1 += __shfl_xor(s1, o, 64); s2 += __shfl_xor(s2, o, 64); }
-            if (pn) { s1 *= inv; s2 *= inv; }
+            if (LN) { const int n = n0 + r < a.N ? n0 + r : a.N - 1; s1 = ln_close(s1, off, inv, a.ln, n, a.N); if (gated) s2 = ln_close(s2, off, inv, a.ln2, n, a.N); }
+            else if (pn) { s1 *= inv; s2 *= inv; }
             if (lane == 0 && n0 + r < a.N) y_store<EPI>(a, v, y_row(a, v, i), n0 + r, s1, s2, rsc[i], res[r][i]);
         }
     }
@@ -159,7 +191,7 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
 // With the norm prologue the row's sum of squares is gathered in the same pass as the products: y = inv_rms(x) * sum_k w_k (x_k (off + g_k)) - one trip
 // through memory per wave, the scale applied to the finished sum.
 // TB: rows per pass - 1 for single rows (a short program: a step runs it once per launch, its first fetch is part of the time), else 8
-template <bool VEC, int TB, int EPI>
+template <bool VEC, int TB, int EPI, bool LN>
 __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n = blockIdx.x * 4 + wave;
@@ -168,15 +200,16 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
     const unsigned short *wr = v.w + (size_t)n * a.ldw, *wr2 = v.w2 ? v.w2 + (size_t)n * a.ldw : nullptr;
     const bool pn = a.pn_w != nullptr;
     for (int t0 = 0; t0 < v.rows; t0 += TB) {
-        float acc[TB], acc2[TB], ss[TB];
+        float acc[TB], acc2[TB], ss[TB], sx[LN ? TB : 1], mid[LN ? TB : 1];
 #pragma unroll
-        for (int i = 0; i < TB; i++) { acc[i] = 0.0f; acc2[i] = 0.0f; ss[i] = 0.0f; }
+        for (int i = 0; i < TB; i++) { acc[i] = 0.0f; acc2[i] = 0.0f; ss[i] = 0.0f; if (LN) sx[i] = 0.0f; }
         const int nt = v.rows - t0 < TB ? v.rows - t0 : TB;
         float res[TB], rsc[TB];
 #pragma unroll
         for (int i = 0; i < TB; i++) {
             rsc[i] = a.row_scale && i < nt ? a.row_scale[v.y0 + t0 + i] : 1.0f;
             res[i] = v.resid && i < nt ? v.resid[y_row(a, v, t0 + i) + n] : 0.0f;
+            if (LN) mid[i] = i < nt ? row_middle<VEC>(x_row(a, v, t0 + i), a.K, lane) : 0.0f;
         }
         if (VEC) {
             for (int k = lane * 8; k < a.K; k += 512) {
@@ -195,6 +228,10 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
                     const float *xr = x_row(a, v, t0 + i) + k;
                     const f32x4 x0 = *reinterpret_cast<const f32x4 *>(xr), x1 = *reinterpret_cast<const f32x4 *>(xr + 4);
                     float xs[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+                    if (LN) {
+#pragma unroll
+                        for (int e = 0; e < 8; e++) { xs[e] -= mid[i]; sx[i] += xs[e]; }
+                    }
                     if (pn) {
 #pragma unroll
                         for (int e = 0; e < 8; e++) { ss[i] = fmaf(xs[e], xs[e], ss[i]); xs[e] = xs[e] * pw[e]; }
@@ -213,6 +250,7 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
                 for (int i = 0; i < TB; i++) {
                     if (i >= nt) break;
                     float x = x_row(a, v, t0 + i)[k];
+                    if (LN) { x -= mid[i]; sx[i] += x; }
                     if (pn) { ss[i] = fmaf(x, x, ss[i]); x = x * pw; }
                     acc[i] = fmaf(x, w, acc[i]);
                     acc2[i] = fmaf(x, w2, acc2[i]);
@@ -225,7 +263,11 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
             float s = acc[i], s2 = acc2[i], q = ss[i];
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) { s += __shfl_xor(s, o, 64); s2 += __shfl_xor(s2, o, 64); q += __shfl_xor(q, o, 64); }
-            if (pn) { const float inv = 1.0f / sqrtf(q / (float)a.K + a.pn_eps); s *= inv; s2 *= inv; }
+            if (LN) {
+                const float off = row_offset(sx[i], a.K), inv = 1.0f / sqrtf(q / (float)a.K - off * off + a.pn_eps);
+                s = ln_close(s, off, inv, a.ln, n, a.N);
+                if (wr2) s2 = ln_close(s2, off, inv, a.ln2, n, a.N);
+            } else if (pn) { const float inv = 1.0f / sqrtf(q / (float)a.K + a.pn_eps); s *= inv; s2 *= inv; }
             if (lane == 0) y_store<EPI>(a, v, y_row(a, v, t0 + i), n, s, s2, rsc[i], res[i]);
         }
     }
@@ -436,9 +478,20 @@ static hipError_t launch_mmb_mfma_tile(const MMBArgs &a, int rows_max, hipStream
 }
 template <bool VEC, int TB>
 static void launch_mmb_vec(const MMBArgs &a, dim3 grid, hipStream_t st) {
-    if (TB == 1 && a.epi == MMB_STORE) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (TB == 1 ? (int)MMB_STORE : EPI_ANY)>), grid, dim3(256), 0, st, a);
-    else if (TB == 1 && a.epi == MMB_SILU_MUL) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (TB == 1 ? (int)MMB_SILU_MUL : EPI_ANY)>), grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, EPI_ANY>), grid, dim3(256), 0, st, a);
+    constexpr bool one = TB == 1;                               // (the epilogue as an argument: single rows only)
+    if (a.ln) {
+        if (one && a.epi == MMB_STORE) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (one ? (int)MMB_STORE : EPI_ANY), true>), grid, dim3(256), 0, st, a);
+        else if (one && a.epi == MMB_CLAMP_SWIGLU) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (one ? (int)MMB_CLAMP_SWIGLU : EPI_ANY), true>), grid, dim3(256), 0, st, a);
+        else hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, EPI_ANY, true>), grid, dim3(256), 0, st, a);
+    } else if (one && a.epi == MMB_STORE) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (one ? (int)MMB_STORE : EPI_ANY), false>), grid, dim3(256), 0, st, a);
+    else if (one && a.epi == MMB_SILU_MUL) hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, (one ? (int)MMB_SILU_MUL : EPI_ANY), false>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((mmb_vec_kernel<VEC, TB, EPI_ANY, false>), grid, dim3(256), 0, st, a);
+}
+template <bool LN>
+static void launch_mmb_vec_rows(const MMBArgs &a, int rows_max, dim3 grid, hipStream_t st) {
+    if (rows_max == 1 && a.epi == MMB_STORE) hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 1, MMB_STORE, LN>), grid, dim3(256), 0, st, a);
+    else if (rows_max == 1) hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 1, EPI_ANY, LN>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 4, EPI_ANY, LN>), grid, dim3(256), 0, st, a);
 }
 
 }  // namespace
@@ -453,14 +506,14 @@ hipError_t launch_mmb(const MMBArgs &a, hipStream_t st) {
                      (!a.w2 || al(a.w2, 16)) && (!a.pn_w || al(a.pn_w, 16));
     const int rows_max = a.sel ? 1 : a.T;                        // most rows any outer index can hold
     if (a.pn_w && rows_max > MMB_VEC_ROWS) return hipErrorInvalidValue;   // (the norm prologue lives in the few-rows kernel only)
+    if (a.ln && (!a.pn_w || a.sel || a.meta || a.nz != 1 || (gated && !a.ln2))) return hipErrorInvalidValue;
     if (rows_max <= MMB_VEC_ROWS || a.sel) {
         const dim3 grid((unsigned)((a.N + 3) / 4), (unsigned)a.nz);
         // many columns, a handful of rows: four weight rows per wave (the grid still has thousands of waves)
         if (vec && !a.sel && !a.meta && rows_max <= 4 && (long long)a.N * a.nz >= 4096) {
             const dim3 g4((unsigned)((a.N + 15) / 16), (unsigned)a.nz);
-            if (rows_max == 1 && a.epi == MMB_STORE) hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 1, MMB_STORE>), g4, dim3(256), 0, st, a);
-            else if (rows_max == 1) hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 1, EPI_ANY>), g4, dim3(256), 0, st, a);
-            else hipLaunchKernelGGL((mmb_vec_rows_kernel<4, 4, EPI_ANY>), g4, dim3(256), 0, st, a);
+            if (a.ln) launch_mmb_vec_rows<true>(a, rows_max, g4, st);
+            else launch_mmb_vec_rows<false>(a, rows_max, g4, st);
             return hipGetLastError();
         }
         if (vec && rows_max == 1) launch_mmb_vec<true, 1>(a, grid, st);
@@ -472,6 +525,7 @@ hipError_t launch_mmb(const MMBArgs &a, hipStream_t st) {
         switch (a.epi) {
             case MMB_STORE: return launch_mmb_mfma_tile<MMB_STORE>(a, rows_max, st);
             case MMB_RELU2: return launch_mmb_mfma_tile<MMB_RELU2>(a, rows_max, st);
+            case MMB_SIGMOID_POW: return launch_mmb_mfma_tile<MMB_SIGMOID_POW>(a, rows_max, st);
             case MMB_SILU_MUL: return launch_mmb_mfma_tile<MMB_SILU_MUL>(a, rows_max, st);
             case MMB_GELU_MUL: return launch_mmb_mfma_tile<MMB_GELU_MUL>(a, rows_max, st);
             case MMB_CLAMP_SWIGLU: return launch_mmb_mfma_tile<MMB_CLAMP_SWIGLU>(a, rows_max, st);

@@ -195,6 +195,7 @@ __global__ __launch_bounds__(TKR_NT) void talk_row_kernel(GqAttnArgs a) {
         const float den = ls[h] * sc + (a.sink ? expf(a.sink[h] - MM) : 0.0f);
         float inv = den > 0.0f ? sc / den : 0.0f;
         if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)t * a.ld_gate + h]));
+        inv *= a.out_mult;
         a.out[(size_t)t * a.ld_out + idx] = acc[idx] * inv;
     }
 }
@@ -437,6 +438,7 @@ __global__ __launch_bounds__(64 * TKT_NW) void talk_tile_kernel(GqAttnArgs a, in
             const float den = l * sc + (a.sink ? expf(a.sink[h] - MM) : 0.0f);
             inv = den > 0.0f ? sc / den : 0.0f;
             if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(size_t)r * a.ld_gate + h]));
+            inv *= a.out_mult;
             out = a.out + (size_t)r * a.ld_out + (size_t)h * VD;
         }
 #pragma unroll

@@ -1,9 +1,10 @@
 // config_model.h — what the loaders of the folder models (config.json + model.safetensors, bf16 weights) share: reading the configuration, checking every
 // tensor against it on the way to the device, and laying out the order of layer runs with its looped span.  One loader per design (novorax.cc, fidepel.cc,
-// tuterax.cc, dinilorn.cc, vuzazen.cc); config_model_load picks it by the configuration's "architecture".
+// tuterax.cc, dinilorn.cc, vuzazen.cc, rarutar.cc); config_model_load picks it by the configuration's "architecture".
 #pragma once
 
 #include <algorithm>
+#include <cmath>
 #include <cstring>
 #include <string>
 #include <vector>
@@ -43,11 +44,12 @@ struct Bf16Loader {
         }
         return t;
     }
-    // several [rows_i][K] bf16 tensors under each other as one device matrix
+    // several [rows_i][K] bf16 tensors under each other as one device matrix (an empty name: rows of zeros)
     BfMat rows(const std::vector<std::pair<std::string, int>> &parts, int K) {
         BfMat o;
         std::vector<unsigned short> host;
         for (const auto &pr : parts) {
+            if (pr.first.empty()) { host.insert(host.end(), (size_t)pr.second * K, 0); o.N += pr.second; continue; }
             const SafeTensor *t = need(pr.first, "BF16", {pr.second, K});
             if (!t) return o;
             const unsigned short *s = (const unsigned short *)t->data;
@@ -58,14 +60,91 @@ struct Bf16Loader {
         o.w = (unsigned short *)dev(host.data(), host.size() * 2);
         return o;
     }
+    // several [N][K_i] bf16 tensors side by side as one device matrix
+    BfMat cols(const std::vector<std::pair<std::string, int>> &parts, int N) {
+        BfMat o;
+        int K = 0, at = 0;
+        for (const auto &pr : parts) K += pr.second;
+        std::vector<unsigned short> host((size_t)N * K);
+        for (const auto &pr : parts) {
+            const SafeTensor *t = need(pr.first, "BF16", {N, pr.second});
+            if (!t) return o;
+            const unsigned short *s = (const unsigned short *)t->data;
+            for (int n = 0; n < N; n++) std::copy(s + (size_t)n * pr.second, s + (size_t)(n + 1) * pr.second, host.begin() + (ptrdiff_t)((size_t)n * K + at));
+            at += pr.second;
+        }
+        o.N = N; o.K = K;
+        o.w = (unsigned short *)dev(host.data(), host.size() * 2);
+        return o;
+    }
     static float widen(unsigned short b) { const uint32_t u = (uint32_t)b << 16; float f; memcpy(&f, &u, 4); return f; }
-    float *vec(const std::string &name, int n) {
+    float *vec(const std::string &name, int n, float mult = 1.0f) {
         const SafeTensor *t = need(name, "BF16", {n});
         if (!t) return nullptr;
         std::vector<float> h((size_t)n);
         const unsigned short *s = (const unsigned short *)t->data;
-        for (int i = 0; i < n; i++) h[(size_t)i] = widen(s[i]);
+        for (int i = 0; i < n; i++) h[(size_t)i] = widen(s[i]) * mult;
         return (float *)dev(h.data(), h.size() * 4);
+    }
+    // a layer norm's [n] weight and, behind it, its [n] bias (tensor name + ".b")
+    float *norm_pair(const std::string &name, int n) {
+        const SafeTensor *w = need(name, "BF16", {n}), *b = w ? need(name + ".b", "BF16", {n}) : nullptr;
+        if (!b) return nullptr;
+        std::vector<float> h((size_t)2 * n);
+        for (int i = 0; i < n; i++) { h[(size_t)i] = widen(((const unsigned short *)w->data)[i]); h[(size_t)(n + i)] = widen(((const unsigned short *)b->data)[i]); }
+        return (float *)dev(h.data(), h.size() * 4);
+    }
+    // w reads rows behind this layer norm (norm_pair of w.K entries): its rows' sums with the norm's weight and bias, made on the device in f32
+    void reads_layer_norm(BfMat &w, const float *norm) {
+        if (!err.empty() || !w.w || !norm) return;
+        void *p = nullptr;
+        if (hipMalloc(&p, (size_t)2 * w.N * 4) != hipSuccess) { err = "device allocation of a norm's row sums failed"; return; }
+        m->arenas.push_back((uint8_t *)p);
+        w.ln = (float *)p;
+        MMBArgs a;
+        a.x = norm; a.ldx = w.K; a.w = w.w; a.ldw = w.K; a.y = w.ln; a.ldy = w.N; a.T = 2; a.N = w.N; a.K = w.K; a.f32 = 1;
+        if (launch_mmb(a, nullptr) != hipSuccess) err = "a norm's row sums failed";
+    }
+    // several [rows_i][K] bf16 tensors under each other, widened to f32 and transposed: [K][sum of rows]
+    float *rows_f32_transposed(const std::vector<std::pair<std::string, int>> &parts, int K) {
+        size_t N = 0, at = 0;
+        for (const auto &pr : parts) N += (size_t)pr.second;
+        std::vector<float> h(N * (size_t)K);
+        for (const auto &pr : parts) {
+            const SafeTensor *t = need(pr.first, "BF16", {pr.second, K});
+            if (!t) return nullptr;
+            const unsigned short *s = (const unsigned short *)t->data;
+            for (int r = 0; r < pr.second; r++, at++)
+                for (int k = 0; k < K; k++) h[(size_t)k * N + at] = widen(s[(size_t)r * K + k]);
+        }
+        return (float *)dev(h.data(), h.size() * 4);
+    }
+    // radians per position of pair i of `dims` turning entries: base^(-2i / dims), made in double.  With a scaling object {factor, original, fast, slow} (YaRN):
+    // blended towards 1 / factor of itself where the pair turns too slowly for the original context (ramp 0 below `lo`, 1 above `hi`); *mscale = the factor of cos and
+    // sin, 0.1 ln(factor) + 1 then, else 1
+    float *rot_table(double base, int dims, const Json &scaling, float *mscale) {
+        std::vector<float> fr((size_t)std::max(dims / 2, 1), 0.0f);
+        double factor = 1.0, lo = 0.0, hi = 0.0;
+        const bool yarn = scaling.is_object() && dims > 0;
+        if (mscale) *mscale = 1.0f;
+        if (yarn) {
+            factor = scaling["factor"].as_double(1.0);
+            const double orig = scaling["original"].as_double(1.0), fast = scaling["fast"].as_double(32.0), slow = scaling["slow"].as_double(1.0);
+            if (!(factor > 0.0) || !(orig > 0.0) || !(fast > 0.0) || !(slow > 0.0) || !(base > 1.0)) { if (err.empty()) err = "configuration: rot.scaling values must be positive"; return nullptr; }
+            const auto corr = [&](double turns) { return dims * std::log(orig / (2.0 * M_PI * turns)) / (2.0 * std::log(base)); };
+            lo = std::max(std::floor(corr(fast)), 0.0);
+            hi = std::min(std::ceil(corr(slow)), (double)(dims - 1));
+            if (mscale) *mscale = (float)(0.1 * std::log(factor) + 1.0);
+        }
+        for (int i = 0; i < dims / 2; i++) {
+            double f = std::pow(base, -2.0 * i / dims);
+            if (yarn) {
+                const double ramp = std::min(1.0, std::max(0.0, (i - lo) / std::max(hi - lo, 0.001)));
+                f = f / factor * ramp + f * (1.0 - ramp);
+            }
+            fr[(size_t)i] = (float)f;
+        }
+        return (float *)dev(fr.data(), fr.size() * 4);
     }
     // rows of a [rows][K] tensor whose row count the configuration does not name (a low-rank projection's inner size): -1 (err set) if absent or not 2-d
     int rows_of(const std::string &name, int K) {
@@ -153,5 +232,6 @@ Model *fidepel_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
 Model *tuterax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
 Model *dinilorn_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
 Model *vuzazen_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
+Model *rarutar_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status);
 
 }  // namespace mi355

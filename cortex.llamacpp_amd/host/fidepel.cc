@@ -161,16 +161,25 @@ bool nvx_routed_as_groups(const NvxLayer &L, int T) {
     return L.ff_kind == NVX_FF_ROUTED && T * L.top > 32 && L.n_expert <= 64 && (size_t)T * L.top * 4 <= 60 * 1024;
 }
 
-// behind the block projection (nvx_a_): queries prepared, keys and values stored, attention, output projection (nvx_close_linear).  With several score maps per head
-// every (head, map) pair runs as a query head of its own; launch_gq_maps_out joins the maps in front of the output projection.
+// behind the block projection (nvx_a_): queries prepared, keys and values stored, attention, output projection (nvx_close_linear)
 hipError_t Context::nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T) {
+    FDP_TRY(nvx_gq_heads(L, r, T, nvx_a_, L.proj.N, nvx_att_, L.heads * L.vdim));
+    FDP_TRY(nvx_close_linear(L.o, nvx_att_, L.heads * L.vdim, T, L.norm1b, L.o_bias));
+    prof_mark("gq_attention");
+    return hipSuccess;
+}
+
+// the heads' outputs -> out[t][heads * vdim] from the projection rows p.  With several score maps per head every (head, map) pair runs as a query head of its own;
+// launch_gq_maps_out joins the maps.
+hipError_t Context::nvx_gq_heads(const NvxLayer &L, const NvxRun &r, int T, const float *p, int LD_P, float *out, int ld_out) {
     const NovoraxModel &M = *model->nvx;
-    const int G = L.kv_heads, LD_P = L.proj.N, maps = L.maps > 1 ? L.maps : 1;
+    const int G = L.kv_heads, maps = L.maps > 1 ? L.maps : 1;
     const int H = L.heads * maps;                               // query heads as the kernels count them
     float *cache = nvx_cache_[(size_t)r.plane];
     GqPrepArgs pa{};
-    pa.p = nvx_a_; pa.ld_p = LD_P; pa.T = T; pa.H = H; pa.G = G; pa.dim = L.dim; pa.vdim = L.vdim;
-    pa.wq_norm = L.q_norm; pa.wk_norm = L.k_norm; pa.eps = M.eps; pa.rot_dims = L.rot_dims; pa.rot_freq = L.rot_freq;
+    pa.p = p; pa.ld_p = LD_P; pa.T = T; pa.H = H; pa.G = G; pa.dim = L.dim; pa.vdim = L.vdim;
+    pa.wq_norm = L.q_norm; pa.wk_norm = L.k_norm; pa.eps = M.eps; pa.rot_dims = L.rot_dims; pa.rot_freq = L.rot_freq; pa.rot_mscale = L.rot_mscale;
+    pa.unit_behind = L.qk_unit ? 1 : 0; pa.v_is_k = L.v_is_k ? 1 : 0;
     pa.norm_per_head = L.qk_norm_per_head ? 1 : 0; pa.v_rot_freq = L.v_rot_freq; pa.v_cs = L.v_rot_freq ? nvx_vcs_ : nullptr;
     pa.q_scale = L.scale; pa.head_scale = L.head_scale; pa.tok_pos = d_pos_; pa.tok_cell = d_cell_;
     pa.maps = maps; pa.rot_neighbours = L.rot_neighbours ? 1 : 0; pa.q_temp_coef = L.q_temp_coef; pa.q_temp_every = L.q_temp_every;
@@ -180,7 +189,7 @@ hipError_t Context::nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T) 
         // the convolution reaches back over a segment's start into its slot's last inputs: a launch per set of segments that share no slot, and the slots move on
         // with it (single rows) or behind it
         const size_t TU = cp.n_ubatch;
-        pa.conv_wt = L.conv_wt; pa.conv_taps = L.conv_taps; pa.conv_state = r.conv_state >= 0 ? nvx_n_[(size_t)r.conv_state] : nullptr;
+        pa.conv_wt = L.conv_wt; pa.conv_taps = L.conv_taps; pa.conv_state = r.side_state >= 0 ? nvx_n_[(size_t)r.side_state] : nullptr;
         for (const auto &wv : nvx_waves_) {
             const int *start = h_seg_ + wv.first, *len = h_seg_ + TU + wv.first;
             const int row0 = start[0], rows = start[wv.second - 1] + len[wv.second - 1] - row0;
@@ -190,29 +199,27 @@ hipError_t Context::nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T) 
             if (pw.v_cs) pw.v_cs += (size_t)row0 * L.vdim;
             pw.conv_move = rows == wv.second ? 1 : 0;
             FDP_TRY(launch_gq_prep(pw, stream_));
-            if (!pw.conv_move && r.conv_state >= 0)
-                FDP_TRY(launch_conv_state(nvx_a_, LD_P, L.conv_channels(), L.conv_taps, nvx_n_[(size_t)r.conv_state], d_seg_ + wv.first, d_seg_ + TU + wv.first,
+            if (!pw.conv_move && r.side_state >= 0)
+                FDP_TRY(launch_conv_state(p, LD_P, L.conv_channels(), L.conv_taps, nvx_n_[(size_t)r.side_state], d_seg_ + wv.first, d_seg_ + TU + wv.first,
                                           d_seg_ + 2 * TU + wv.first, wv.second, stream_));
         }
     }
     GqAttnArgs aa{};
-    aa.q = nvx_q_; aa.ld_q = H * L.dim; aa.out = maps > 1 ? nvx_o_ : nvx_att_; aa.ld_out = H * L.vdim; aa.T = T; aa.H = H; aa.G = G; aa.dim = L.dim; aa.vdim = L.vdim;
+    aa.q = nvx_q_; aa.ld_q = H * L.dim; aa.out = maps > 1 ? nvx_o_ : out; aa.ld_out = maps > 1 ? H * L.vdim : ld_out; aa.T = T; aa.H = H; aa.G = G; aa.dim = L.dim; aa.vdim = L.vdim;
     aa.maps = maps; aa.keep_first = L.keep_first; aa.rel = L.rel; aa.dist_bucket = L.dist_bucket; aa.n_dist = L.n_dist; aa.rel_rows = L.rel_rows;
     aa.cache = cache; aa.cell_pos = d_cell_pos_; aa.cell_seq = d_cell_seq_; aa.tok_pos = d_pos_; aa.tok_seq = d_seq_; aa.n_kv_dev = d_nkv_;
-    aa.window = L.window; aa.sink = L.sink; aa.gate = L.off_gate >= 0 && !L.gate_per_entry ? nvx_a_ + L.off_gate : nullptr; aa.ld_gate = LD_P;
+    aa.window = L.window; aa.chunk = L.chunk; aa.out_mult = L.out_mult; aa.sink = L.sink; aa.gate = L.off_gate >= 0 && !L.gate_per_entry ? p + L.off_gate : nullptr; aa.ld_gate = LD_P;
     aa.talk = L.talk;
     aa.softcap = L.softcap; aa.v_cs = L.v_rot_freq ? nvx_vcs_ : nullptr;
     aa.tok_hi = d_seg_ + 3 * (size_t)cp.n_ubatch;
-    aa.tok_lo = M.max_window > 0 && L.window > 0 ? d_seg_ + 4 * (size_t)cp.n_ubatch : nullptr;
+    aa.tok_lo = M.max_window > 0 && (L.window > 0 || L.chunk > 0) ? d_seg_ + 4 * (size_t)cp.n_ubatch : nullptr;
     aa.part = nvx_part_; aa.part_floats = nvx_part_floats_; aa.n_kv_hint = n_kv_;
     aa.splits = (long long)T * H <= LATENT_ATTN_SPLIT_MAX_PAIRS ? LATENT_ATTN_SPLITS : 1;
     FDP_TRY(launch_gq_attn(aa, stream_));
     if (maps == 2)
-        FDP_TRY(launch_gq_maps_out(nvx_o_, H * L.vdim, L.gate_per_entry ? nvx_a_ + L.off_gate : nullptr, LD_P, T, L.heads, L.vdim, L.map_lambda, L.map_mult, M.eps,
-                                   nvx_att_, L.heads * L.vdim, stream_));
+        FDP_TRY(launch_gq_maps_out(nvx_o_, H * L.vdim, L.gate_per_entry ? p + L.off_gate : nullptr, LD_P, T, L.heads, L.vdim, L.map_lambda, L.map_mult, M.eps,
+                                   out, ld_out, stream_));
     else if (maps != 1) return hipErrorInvalidValue;
-    FDP_TRY(nvx_close_linear(L.o, nvx_att_, L.heads * L.vdim, T, L.norm1b, L.o_bias));
-    prof_mark("gq_attention");
     return hipSuccess;
 }
 

@@ -1,7 +1,8 @@
 // novorax.cc — the folder models (config.json + model.safetensors): the registry that picks a design's loader by "architecture", the Novorax loader, and what
 // every such design shares inside Context - buffers, cache planes and state slots, segment lists and scan bounds, the layer-run loop, the output head
 // (novorax.h describes the designs, runtime.h the context; the Fidepel loader and its block are in fidepel.cc, the Tuterax loader and the delta-rule mixer
-// in tuterax.cc, the Dinilorn loader, its retention mixer and its feed-forward in dinilorn.cc, the Vuzazen loader in vuzazen.cc).
+// in tuterax.cc, the Dinilorn loader, its retention mixer and its feed-forward in dinilorn.cc, the Vuzazen loader in vuzazen.cc, the Rarutar loader
+// and its recurrences in rarutar.cc).
 //
 // The context's own machinery carries them: the cell table (find / free / sequence masks) addresses the attention layers' cache planes, the micro-batch staging
 // block brings tokens, positions, cells and sequence ids to the device, the sequence id is the slot of the recurrent state, logits / arg-max / top-k leave
@@ -51,6 +52,7 @@ Model *config_model_load(const std::string &dir, int main_gpu, std::string &err,
         {"Tuterax", tuterax_build},
         {"Dinilorn", dinilorn_build},
         {"Vuzazen", vuzazen_build},
+        {"Rarutar", rarutar_build},
     };
     status = -102;
     std::ifstream cf(dir + "/config.json");
@@ -126,34 +128,7 @@ Model *novorax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
             const Json &rot = mx["rot"];
             L.rot_dims = rot.is_object() ? (int)rot["dims"].as_int(L.rot) : 0;
             if (L.rot_dims > L.rot || (L.rot_dims & 1) || L.rot_dims < 0) { err = "configuration: rot.dims must be even and at most rot_dim"; return nullptr; }
-            {
-                // radians per position of pair i: base^(-2i / dims), blended towards 1 / factor of itself where YaRN says the pair turns too slowly for the
-                // original context (ramp 0 below `lo`, 1 above `hi`); cos and sin carry the attention scale 0.1 ln(factor) + 1
-                const int half = L.rot_dims / 2;
-                const double base = rot["base"].as_double(10000.0);
-                std::vector<float> fr((size_t)std::max(half, 1), 0.0f);
-                const Json &scg = rot["scaling"];
-                double factor = 1.0, lo = 0.0, hi = 0.0;
-                const bool yarn = scg.is_object() && half > 0;
-                if (yarn) {
-                    factor = scg["factor"].as_double(1.0);
-                    const double orig = scg["original"].as_double(1.0), fast = scg["fast"].as_double(32.0), slow = scg["slow"].as_double(1.0);
-                    if (!(factor > 0.0) || !(orig > 0.0) || !(fast > 0.0) || !(slow > 0.0) || !(base > 1.0)) { err = "configuration: rot.scaling values must be positive"; return nullptr; }
-                    const auto corr = [&](double turns) { return L.rot_dims * std::log(orig / (2.0 * M_PI * turns)) / (2.0 * std::log(base)); };
-                    lo = std::max(std::floor(corr(fast)), 0.0);
-                    hi = std::min(std::ceil(corr(slow)), (double)(L.rot_dims - 1));
-                    L.rot_mscale = (float)(0.1 * std::log(factor) + 1.0);
-                }
-                for (int i = 0; i < half; i++) {
-                    double f = std::pow(base, -2.0 * i / L.rot_dims);
-                    if (yarn) {
-                        const double ramp = std::min(1.0, std::max(0.0, (i - lo) / std::max(hi - lo, 0.001)));
-                        f = f / factor * ramp + f * (1.0 - ramp);
-                    }
-                    fr[(size_t)i] = (float)f;
-                }
-                L.rot_freq = (float *)ld.dev(fr.data(), fr.size() * 4);
-            }
+            L.rot_freq = ld.rot_table(rot["base"].as_double(10000.0), L.rot_dims, rot["scaling"], &L.rot_mscale);
             const int QD = L.dim + L.rot;
             L.down = ld.rows({{pm + "dq", L.q_rank}, {pm + "dkv", L.kv_rank + L.rot}}, W);
             L.dq_norm = ld.vec(pm + "dq.norm", L.q_rank);
@@ -250,14 +225,25 @@ Model *novorax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
 // floats one sequence slot holds for a recurrent layer run: the state matrices; the second set (mLSTM: normalisers, delta rule: the convolutions' last
 // taps - 1 inputs); the third (mLSTM: running maxima)
 static void nvx_state_sizes(const NvxLayer &L, size_t &s_sz, size_t &n_sz, size_t &m_sz) {
-    if (L.type == NVX_GQ) { s_sz = m_sz = 0; n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.conv_channels(); return; }   // (attention: the convolution's last inputs)
+    s_sz = n_sz = m_sz = 0;
+    switch (L.type) {
+        case NVX_BESIDE:
+            for (const NvxLayer &x : L.mixers) if (x.type != NVX_GQ) nvx_state_sizes(x, s_sz, n_sz, m_sz);   // (one recurrence beside the attention)
+            return;
+        case NVX_GQ: n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.conv_channels(); return;       // (attention: the convolution's last inputs)
+        case NVX_MLSTM: {
+            const size_t c = (size_t)mlstm_state_copies(L.vdim);
+            n_sz = (size_t)L.heads * L.dim * c; m_sz = (size_t)L.heads * c;
+            break;
+        }
+        case NVX_DELTA: n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.delta_channels(); break;
+        case NVX_SSD: n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.conv_channels(); break;
+        default: break;
+    }
     s_sz = (size_t)L.heads * L.dim * L.vdim;
-    if (L.type == NVX_MLSTM) { const size_t c = (size_t)mlstm_state_copies(L.vdim); n_sz = (size_t)L.heads * L.dim * c; m_sz = (size_t)L.heads * c; }
-    else if (L.type == NVX_RETENTION) { n_sz = 0; m_sz = 0; }
-    else { n_sz = (size_t)std::max(L.conv_taps - 1, 0) * (size_t)L.delta_channels(); m_sz = 0; }
 }
-static bool nvx_recurrent(const NvxLayer &L) { return L.type == NVX_MLSTM || L.type == NVX_DELTA || L.type == NVX_RETENTION; }
-static int nvx_state_set(const NvxLayer &L, const NvxRun &r) { return nvx_recurrent(L) ? r.plane : r.conv_state; }   // index of a run's state set, -1: none
+static bool nvx_recurrent(const NvxLayer &L) { return L.type == NVX_MLSTM || L.type == NVX_DELTA || L.type == NVX_RETENTION || L.type == NVX_GLA || L.type == NVX_SSD; }
+static int nvx_state_set(const NvxLayer &L, const NvxRun &r) { return nvx_recurrent(L) ? r.plane : r.side_state; }   // index of a run's state set, -1: none
 
 bool Context::init_novorax(std::string &err) {
     const NovoraxModel &M = *model->nvx;
@@ -314,13 +300,18 @@ bool Context::init_novorax(std::string &err) {
     nvx_att_ = (float *)dalloc(T * (size_t)std::max(M.max_att, 1) * 4);
     nvx_o_ = (float *)dalloc(T * (size_t)std::max(M.max_att, 1) * 4);
     nvx_ff_ = (float *)dalloc(T * TOP * (size_t)std::max(M.max_ff, 1) * 4);
+    std::vector<const NvxLayer *> mixers;                        // of all layers, those side by side one by one
+    for (const NvxLayer &L : M.layers) {
+        if (L.type == NVX_BESIDE) for (const NvxLayer &x : L.mixers) mixers.push_back(&x);
+        else mixers.push_back(&L);
+    }
     {
         int kr = 1;                                              // widest record of a split attention scan: the latent, or a value head
-        for (const NvxLayer &L : M.layers) kr = std::max(kr, L.type == NVX_LATENT ? L.kv_rank : L.type == NVX_GQ ? L.vdim : 1);
+        for (const NvxLayer *Lp : mixers) { const NvxLayer &L = *Lp; kr = std::max(kr, L.type == NVX_LATENT ? L.kv_rank : L.type == NVX_GQ ? L.vdim : 1); }
         nvx_part_floats_ = (size_t)LATENT_ATTN_SPLIT_MAX_PAIRS * LATENT_ATTN_SPLITS * (size_t)(kr + 2);
         // grouped-query layers also cut the block chains of short prompt batches: records for up to 1024 rows x 4 runs of the widest layer
-        for (const NvxLayer &L : M.layers)
-            if (L.type == NVX_GQ) nvx_part_floats_ = std::max(nvx_part_floats_, std::min<size_t>(T, 1024) * (size_t)L.heads * (size_t)std::max(L.maps, 1) * 4 * (size_t)(L.vdim + 2));
+        for (const NvxLayer *Lp : mixers)
+            if (const NvxLayer &L = *Lp; L.type == NVX_GQ) nvx_part_floats_ = std::max(nvx_part_floats_, std::min<size_t>(T, 1024) * (size_t)L.heads * (size_t)std::max(L.maps, 1) * 4 * (size_t)(L.vdim + 2));
         // latent layers: steps of up to 512 (row, head) pairs hold 512 / tiles runs of 16 or 32 pairs; batches up to 8 runs of up to 1024 rows
         for (const NvxLayer &L : M.layers)
             if (L.type == NVX_LATENT)
@@ -351,6 +342,26 @@ bool Context::init_novorax(std::string &err) {
         nvx_mw_F_ = (double *)dalloc(TH * 8);
         nvx_mw_v_ = (float *)dalloc(3 * TH * 4);
         if (!nvx_mw_A_ || !nvx_mw_F_ || !nvx_mw_v_) { err = "recurrence work buffers allocation failed"; return false; }
+    }
+    {
+        // the gated recurrences' work buffers for segments of several rows (GatedScanArgs)
+        size_t heads = 0, keys = 0, rows_p = 0, dec = 0, mat = 0;
+        for (const NvxLayer *L : mixers) {
+            if (L->type != NVX_GLA && L->type != NVX_SSD) continue;
+            const size_t H = (size_t)L->heads, HD = H * (size_t)L->dim;
+            heads = std::max(heads, H); mat = std::max(mat, HD * (size_t)L->vdim);
+            if (L->type == NVX_GLA) { keys = std::max(keys, HD); dec = std::max(dec, HD); }
+            else { rows_p = std::max(rows_p, H); dec = std::max(dec, H); }
+        }
+        if (heads > 0) {
+            const size_t places = gated_scan_chunks(T, std::min<size_t>(T, NS));
+            nvx_gs_A_ = (float *)dalloc(T * heads * 64 * 4);
+            nvx_gs_q_ = (float *)dalloc(2 * T * std::max<size_t>(keys, 1) * 4);
+            nvx_gs_p_ = (float *)dalloc(2 * T * std::max<size_t>(rows_p, 1) * 4);
+            nvx_gs_g_ = (float *)dalloc(places * dec * 4);
+            nvx_gs_S_ = (float *)dalloc(places * mat * 4);
+            if (!nvx_gs_A_ || !nvx_gs_q_ || !nvx_gs_p_ || !nvx_gs_g_ || !nvx_gs_S_) { err = "recurrence work buffers allocation failed"; return false; }
+        }
     }
     if (M.max_shared_ff > 0) {
         nvx_sh_ = (float *)dalloc(T * (size_t)M.max_shared_ff * 4);
@@ -477,13 +488,19 @@ bool Context::nvx_stage_segments(int n, const int32_t *tokens, const int32_t *se
     return hipMemcpyAsync(d_seg_, h_seg_, 7 * T * 4, hipMemcpyHostToDevice, stream_) == hipSuccess;
 }
 
-// pn != nullptr: the rows of x are RMS-normed with weight (norm_off + pn) on the way in (few rows: inside the launch; batches: a norm launch into xn_ first)
+// pn != nullptr: the rows of x are RMS-normed with weight (norm_off + pn) - or layer-normed, in a design of layer norms - on the way in (few rows: inside the launch; batches: a norm launch into xn_ first)
 hipError_t Context::nvx_linear(const BfMat &w, const float *x, int ldx, int T, float *y, int ldy, int epi, const BfMat *w2, float out_scale, const float *pn,
                                const float *bias, float epi_limit, const float *resid) {
     MMBArgs a;
+    const bool ln = model->nvx->layer_norm && pn;
     if (pn && T > MMB_VEC_ROWS) {
-        NVX_TRY(launch_rmsnorm_f32(x, ldx, pn, model->nvx->norm_off, nullptr, xn_, w.K, w.K, T, model->nvx->eps, stream_));
+        if (!ln) NVX_TRY(launch_rmsnorm_f32(x, ldx, pn, model->nvx->norm_off, nullptr, xn_, w.K, w.K, T, model->nvx->eps, stream_));
+        else if (ldx != w.K) return hipErrorInvalidValue;
+        else NVX_TRY(launch_layer_norm(x, pn, pn + w.K, w.K, T, model->nvx->eps, xn_, stream_));
         x = xn_; ldx = w.K; pn = nullptr;
+    } else if (ln) {
+        if (!w.ln || (w2 && !w2->ln)) return hipErrorInvalidValue;
+        a.ln = w.ln; a.ln2 = w2 ? w2->ln : nullptr;
     }
     a.pn_w = pn; a.pn_off = model->nvx->norm_off; a.pn_eps = model->nvx->eps;
     a.x = x; a.ldx = ldx; a.w = w.w; a.w2 = w2 ? w2->w : nullptr; a.ldw = w.K; a.y = y; a.ldy = ldy;
@@ -503,7 +520,7 @@ hipError_t Context::nvx_feed_forward(const NvxLayer &L, int T, bool *closed) {
     const int W = M.width;
     if (L.ff_kind == NVX_FF_ROUTED) return nvx_routed_feed_forward(L, T, closed);
     if (L.ff_kind == NVX_FF_DENSE) {
-        if (L.gate.w) NVX_TRY(nvx_linear(L.gate, x_, W, T, nvx_ff_, L.ff, L.ff_silu ? MMB_SILU_MUL : MMB_GELU_MUL, &L.up, 1.0f, L.norm2));
+        if (L.gate.w) NVX_TRY(nvx_linear(L.gate, x_, W, T, nvx_ff_, L.ff, L.ff_limit > 0.0f ? MMB_CLAMP_SWIGLU : L.ff_silu ? MMB_SILU_MUL : MMB_GELU_MUL, &L.up, 1.0f, L.norm2, nullptr, L.ff_limit));
         else NVX_TRY(nvx_linear(L.up, x_, W, T, nvx_ff_, L.ff, MMB_RELU2, nullptr, 1.0f, L.norm2));
         if (closed && !L.norm2b) *closed = true;                 // (nothing behind the feed-forward: its last product adds into the stream)
         return nvx_close_linear(L.down_ff, nvx_ff_, L.ff, T, L.norm2b);
@@ -625,6 +642,12 @@ hipError_t Context::run_layers_novorax(int T) {
             NVX_TRY(nvx_delta_mixer(L, r, T));
         } else if (L.type == NVX_RETENTION) {
             NVX_TRY(nvx_retention_mixer(L, r, T));
+        } else if (L.type == NVX_BESIDE) {
+            NVX_TRY(nvx_beside_mixers(L, r, T));
+        } else if (L.type == NVX_GLA) {
+            NVX_TRY(nvx_gla_mixer(L, r, T));
+        } else if (L.type == NVX_SSD) {
+            NVX_TRY(nvx_ssd_mixer(L, r, T));
         } else return hipErrorInvalidValue;
         // norm on the sublayer's output, added to the stream (norm1 / norm2 in front of a sublayer are nullptr in a design whose sublayers read the stream itself; norm1b / norm2b
         // behind it in a design without them - its last product has added into the stream already)

@@ -1,4 +1,4 @@
-// novorax.h — the layer stack of the folder models (config.json + model.safetensors, bf16 weights) as this runtime holds it.  Five designs fill it.
+// novorax.h — the layer stack of the folder models (config.json + model.safetensors, bf16 weights) as this runtime holds it.  Six designs fill it.
 //
 // Novorax: a decoder whose layers each pick a token mixer (latent attention with a sliding window and a
 // softmax sink, or the mLSTM matrix-memory recurrence) and a feed-forward (dense relu^2, or experts chosen by a token-id table), norms on both sides of every
@@ -35,6 +35,12 @@
 // earlier token, halves turning, a sigmoid gate per head); grouped-query attention without positions: short causal convolutions on q / k / v, whole-projection
 // q / k norms, unit values, scores mixed across the heads before the softmax, a sigmoid gate per head.  Feed-forward: silu-gated, dense or experts picked by
 // their sigmoid scores, the score multiplying what the expert reads.
+//
+// Rarutar: layer norms (mean taken off, weight and bias) in front of the sublayers only; the embedding row enters times a constant, the table is the output head.
+// Mixers: two side by side on one input - windowed grouped-query attention (YaRN rotation, a sigmoid gate per head) and gated linear attention (a decay per key
+// channel through a low-rank projection, per-head unit-RMS output times silu(gate)) -, each times a constant; attention inside chunks of positions (values are the
+// projected keys, keys and queries divided by their RMS behind the turn, a softmax sink, a sigmoid gate per head); Mamba-2 (a short convolution with bias and silu, one
+// decay per head, a skip, the gate in front of an RMS norm in equal parts).  Feed-forward: g sigmoid(1.702 g) (u + 1), g and u clamped, or none.
 #pragma once
 
 #include <cstdint>
@@ -46,9 +52,12 @@ namespace mi355 {
 struct BfMat {                      // bf16 rows on the device
     unsigned short *w = nullptr;
     int N = 0, K = 0;               // rows (outputs), row length (inputs)
+    float *ln = nullptr;            // [2][N] f32 for a matrix that reads layer-normed rows: its rows' sums with the norm's weight, then with its bias
 };
 
-enum { NVX_LATENT = 0, NVX_MLSTM = 1, NVX_GQ = 2, NVX_DELTA = 3, NVX_RETENTION = 4 };   // token mixers: latent attention, matrix-memory recurrence, grouped-query attention, gated delta rule, retention
+// token mixers: latent attention, matrix-memory recurrence, grouped-query attention, gated delta rule, retention, gated linear attention, state-space recurrence
+// (Mamba-2), several mixers side by side on one input
+enum { NVX_LATENT = 0, NVX_MLSTM = 1, NVX_GQ = 2, NVX_DELTA = 3, NVX_RETENTION = 4, NVX_GLA = 5, NVX_SSD = 6, NVX_BESIDE = 7 };
 enum { NVX_ROUTE_SOFTMAX_GROUPS = 0, NVX_ROUTE_SIGMOID_BIAS = 1 };   // routers of NVX_FF_ROUTED: softmax scores, groups by their best, normalised weights | sigmoid scores + selection bias, groups by their two best, raw weights
 enum { NVX_FF_NONE = 0, NVX_FF_DENSE = 1, NVX_FF_EXPERTS = 2, NVX_FF_ROUTED = 3 };   // dense; experts by a token-id table; experts by a router
 
@@ -115,7 +124,24 @@ struct NvxLayer {
     // heads, scores mixed across the heads (talk [heads][heads] f32)
     float *conv_wt = nullptr, *talk = nullptr;
     bool v_unit = false;
-    int conv_channels() const { return heads * maps * dim + kv_heads * maps * dim + kv_heads * vdim; }
+    int conv_channels() const { return type == NVX_SSD ? heads * vdim + 2 * kv_heads * dim : heads * maps * dim + kv_heads * maps * dim + kv_heads * vdim; }
+    // ... and: a token sees its own chunk of `chunk` positions only; q and k heads divided by their RMS behind the turn (no weights); value heads are the projected
+    // keys; a constant on the output (folded into the output norm's weight by a recurrence)
+    int chunk = 0;
+    bool qk_unit = false, v_is_k = false;
+    float out_mult = 1.0f;
+    // gated linear attention: proj = [q: heads*dim ; k: heads*dim ; v: heads*vdim ; g: heads*vdim (off_g) ; a1: rank_a (off_a)], decays sigmoid(a2 a1 + a2_bias)^inv_tau
+    float *a2_bias = nullptr;
+    float inv_tau = 1.0f;
+    // state-space recurrence: proj = [z: heads*vdim ; x: heads*vdim ; B: groups*state ; C: groups*state ; dt: heads (off_a)], kv_heads = groups, dim = state; conv_wt over
+    // [x ; B ; C] with conv_b; A_log, dt_bias, skip [heads]; the output norm in norm_parts equal parts (mix_norm)
+    float *conv_b = nullptr, *skip = nullptr;
+    int norm_parts = 1;
+    // mixers side by side: each one's projection starts at column off_p of this layer's fused proj, its output at column off_att of the row that o (their W_o side by
+    // side) closes
+    std::vector<NvxLayer> mixers;
+    int off_p = 0, off_att = 0;
+    float ff_limit = 0.0f;          // > 0: the gated dense feed-forward is g sigmoid(1.702 g) (u + 1) with g, u clamped by it
     // latent attention: entry i of the turning part pairs with entry i + half instead of its neighbour; the gate rows of `down` start at off_gate (-1: no gate)
     bool rot_halves = false;
     // gated feed-forwards (dense, routed): silu; routed: the router's weight multiplies the expert's input instead of its output
@@ -123,14 +149,14 @@ struct NvxLayer {
     float map_lambda = 0.0f, map_mult = 1.0f;
     // retention: proj = [q: heads*dim ; k: heads*dim ; v: heads*vdim ; g: heads*vdim] rows (off_g: the gate's column), decay [heads]; rot_dims / rot_freq as above
     float *decay = nullptr;
-    int cache_row() const { return type == NVX_LATENT ? kv_rank + rot : type == NVX_GQ ? kv_heads * (maps * dim + vdim) : 0; }   // f32 per cell of a run's cache plane
+    int cache_row() const { return type == NVX_LATENT ? kv_rank + rot : type == NVX_GQ ? kv_heads * (maps * dim + vdim) : type == NVX_BESIDE ? mixers[0].cache_row() : 0; }   // f32 per cell of a run's cache plane
 };
 
 struct NvxRun {
     int layer = 0;
     int pass = -1;                  // >= 0: first layer of loop pass `pass` (input projection + step vector come first)
     int plane = -1;                 // attention mixers: index of this run's cache plane; recurrent mixers: of its state set
-    int conv_state = -1;            // attention mixers with a convolution of several taps: index of the state set that keeps its last inputs
+    int side_state = -1;            // attention mixers that keep sequence state too (a convolution's last inputs, the recurrence beside them): index of its state set
 };
 
 struct NovoraxModel {
@@ -146,13 +172,14 @@ struct NovoraxModel {
     int64_t bigram_mul_prev = 0, bigram_mul_cur = 0;
     // what a sequence keeps beside its cache cells: recurrent state, convolution inputs, the previous token - it cannot be cut back to an earlier position
     bool has_sequence_state() const { return n_state_runs > 0 || bigram.w != nullptr; }
-    std::string design;             // "novorax" | "fidepel" | "tuterax" | "dinilorn" | "vuzazen"
+    std::string design;             // "novorax" | "fidepel" | "tuterax" | "dinilorn" | "vuzazen" | "rarutar"
     bool loop_add_embed = false;    // every pass of the looped span but the first opens with x += embedding rows
     int max_keep_first = 0;         // most first positions a windowed layer keeps seen (scan bounds)
     // norm weights: the factor is norm_off + w (1: zero-centred weights, 0: plain ones).  parallel_block: one norm per layer, mixer and feed-forward both read
     // it, x += residual_mult * (their sum); otherwise norms on both sides of each sublayer
     float norm_off = 1.0f, residual_mult = 1.0f;
     bool parallel_block = false;
+    bool layer_norm = false;        // the norms are layer norms: a norm vector holds the weights and, behind them, the biases (norm_off 0)
     int width = 0, n_vocab = 0;
     int n_cache_runs = 0, n_state_runs = 0;   // attention runs (cache planes) and recurrent runs (state sets per sequence slot)
     int max_window = 0;             // largest window of the windowed attention layers, 0 if one of them sees every earlier cell (scan bounds)

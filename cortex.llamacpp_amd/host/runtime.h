@@ -74,7 +74,7 @@ struct Model {
     DevTensor tok_embd, out_norm, output, rope_freqs;
     DevTensor tok_types, tok_norm, tok_norm_b;       // encoder files: token-type table (row 0 is added to every token), LayerNorm of the embeddings
     std::vector<LayerWeights> layers;
-    std::unique_ptr<NovoraxModel> nvx;  // a folder model (config.json + model.safetensors; architectures Novorax, Fidepel, Tuterax, Dinilorn, Vuzazen): its own layer stack, see novorax.h
+    std::unique_ptr<NovoraxModel> nvx;  // a folder model (config.json + model.safetensors; architectures Novorax, Fidepel, Tuterax, Dinilorn, Vuzazen, Rarutar): its own layer stack, see novorax.h
     uint64_t device_bytes = 0, host_bytes = 0, file_tensor_bytes = 0, bytes_per_token = 0, planes_bytes = 0;
     ~Model();
 };
@@ -193,6 +193,13 @@ class Context {
     // fidepel.cc: a block whose mixer and feed-forward read one norm; grouped-query attention on the run's cache plane; experts picked by a router
     hipError_t nvx_parallel_block(const NvxLayer &L, const NvxRun &r, int T);
     hipError_t nvx_gq_attention(const NvxLayer &L, const NvxRun &r, int T);
+    hipError_t nvx_gq_heads(const NvxLayer &L, const NvxRun &r, int T, const float *p, int LD_P, float *out, int ld_out);
+    // rarutar.cc: several mixers on one input behind one projection; gated linear attention; the state-space recurrence
+    hipError_t nvx_beside_mixers(const NvxLayer &L, const NvxRun &r, int T);
+    hipError_t nvx_gla_mixer(const NvxLayer &L, const NvxRun &r, int T);
+    hipError_t nvx_gla_heads(const NvxLayer &L, int state_set, int T, const float *p, int LD_P, float *out, int ld_out);
+    hipError_t nvx_ssd_mixer(const NvxLayer &L, const NvxRun &r, int T);
+    float *nvx_gs_A_ = nullptr, *nvx_gs_q_ = nullptr, *nvx_gs_p_ = nullptr, *nvx_gs_g_ = nullptr, *nvx_gs_S_ = nullptr;   // work buffers of the gated recurrences (GatedScanArgs)
     hipError_t nvx_delta_mixer(const NvxLayer &L, const NvxRun &r, int T);   // tuterax.cc: projections, convolution, recurrence, gated unit-RMS output, W_o -> nvx_y_
     hipError_t nvx_routed_experts(const NvxLayer &L, const float *h, const float *pn, int T, const float *z, int ld_z, bool *closed = nullptr);   // z: the router's logits [T][n_expert], row stride ld_z; closed: see nvx_feed_forward
     hipError_t nvx_shared_expert(const NvxLayer &L, const float *h, const float *pn, int T);

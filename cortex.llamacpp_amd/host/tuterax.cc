@@ -22,13 +22,6 @@ void set_error(const char *fmt, ...);
         }                                                                                          \
     } while (0)
 
-// radians per position of pair i of `dims` turning entries: base^(-2i / dims), made in double
-static float *rot_table(Bf16Loader &ld, double base, int dims) {
-    std::vector<float> fr((size_t)std::max(dims / 2, 1), 0.0f);
-    for (int i = 0; i < dims / 2; i++) fr[(size_t)i] = (float)std::pow(base, -2.0 * i / dims);
-    return (float *)ld.dev(fr.data(), fr.size() * 4);
-}
-
 Model *tuterax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status) {
     (void)dir;
     status = -102;
@@ -75,8 +68,8 @@ Model *tuterax_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
                 const double base = rot["base"].as_double(10000.0);
                 if (!(base > 0.0)) { err = "configuration: rot.base must be positive"; return nullptr; }
                 if (VD & 1) { err = "configuration: mixer.vdim must be even (the value heads turn in pairs)"; return nullptr; }
-                if (L.rot_dims > 0) L.rot_freq = rot_table(ld, base, L.rot_dims);
-                L.v_rot_freq = rot_table(ld, base, VD);           // the values turn over ALL their entries, with the same base
+                if (L.rot_dims > 0) L.rot_freq = ld.rot_table(base, L.rot_dims, Json(), nullptr);
+                L.v_rot_freq = ld.rot_table(base, VD, Json(), nullptr);          // the values turn over ALL their entries, with the same base
             }
             L.qk_norm_per_head = true;
             L.q_norm = ld.vec(pm + "q.norm", D);

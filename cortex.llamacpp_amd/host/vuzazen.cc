@@ -11,27 +11,6 @@
 
 namespace mi355 {
 
-static float *rot_table_plain(Bf16Loader &ld, double base, int dims) {   // radians per position of pair i: base^(-2i / dims), made in double
-    std::vector<float> fr((size_t)std::max(dims / 2, 1), 0.0f);
-    for (int i = 0; i < dims / 2; i++) fr[(size_t)i] = (float)std::pow(base, -2.0 * i / dims);
-    return (float *)ld.dev(fr.data(), fr.size() * 4);
-}
-
-// several [rows_i][K] bf16 tensors under each other, widened to f32 and transposed: [K][sum of rows]
-static float *rows_f32_transposed(Bf16Loader &ld, const std::vector<std::pair<std::string, int>> &parts, int K) {
-    size_t N = 0, at = 0;
-    for (const auto &pr : parts) N += (size_t)pr.second;
-    std::vector<float> h(N * (size_t)K);
-    for (const auto &pr : parts) {
-        const SafeTensor *t = ld.need(pr.first, "BF16", {pr.second, K});
-        if (!t) return nullptr;
-        const unsigned short *s = (const unsigned short *)t->data;
-        for (int r = 0; r < pr.second; r++, at++)
-            for (int k = 0; k < K; k++) h[(size_t)k * N + at] = Bf16Loader::widen(s[(size_t)r * K + k]);
-    }
-    return (float *)ld.dev(h.data(), h.size() * 4);
-}
-
 Model *vuzazen_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, std::string &err, int &status) {
     (void)dir;
     status = -102;
@@ -98,7 +77,7 @@ Model *vuzazen_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
             L.rot_halves = true;
             const double base = mx["rot"]["base"].as_double(10000.0);
             if (!(base > 0.0)) { err = at + "rot.base must be positive"; return nullptr; }
-            L.rot_freq = rot_table_plain(ld, base, L.rot_dims);
+            L.rot_freq = ld.rot_table(base, L.rot_dims, Json(), nullptr);
             const int QD = D + L.rot;
             L.down = ld.rows({{pm + "dq", L.q_rank}, {pm + "dkv", L.kv_rank + L.rot}, {pm + "g", H}}, W);
             L.off_gate = L.q_rank + L.kv_rank + L.rot;
@@ -125,7 +104,7 @@ Model *vuzazen_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
             L.conv_taps = (int)mx["conv"].as_int(1);
             if (!cfg_positive(err, "mixer.conv", L.conv_taps, 64)) return nullptr;
             if (L.off_gate > GQ_CONV_MAX_CHANNELS) { err = at + "q, k and v have more rows than the convolution holds (" + std::to_string(GQ_CONV_MAX_CHANNELS) + ")"; return nullptr; }
-            L.conv_wt = rows_f32_transposed(ld, {{pm + "q.conv", NQ}, {pm + "k.conv", NK}, {pm + "v.conv", NV}}, L.conv_taps);
+            L.conv_wt = ld.rows_f32_transposed({{pm + "q.conv", NQ}, {pm + "k.conv", NK}, {pm + "v.conv", NV}}, L.conv_taps);
             L.q_norm = ld.vec(pm + "q.norm", NQ);
             L.k_norm = ld.vec(pm + "k.norm", NK);
             L.v_unit = true;
@@ -180,7 +159,7 @@ Model *vuzazen_build(const Json &cfg, const std::string &dir, Bf16Loader &ld, st
         const NvxLayer &L = M.layers[(size_t)il];
         NvxRun r; r.layer = il;
         r.plane = L.type == NVX_MLSTM ? M.n_state_runs++ : M.n_cache_runs++;
-        if (L.type == NVX_GQ && L.conv_taps > 1) r.conv_state = M.n_state_runs++;
+        if (L.type == NVX_GQ && L.conv_taps > 1) r.side_state = M.n_state_runs++;
         M.runs.push_back(r);
     }
     HParams &hp = m->hp;
