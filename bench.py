@@ -399,6 +399,19 @@ def vuzazen_section(args) -> int:
     return _time_folder_pair(args, args.vuzazen, "vuzazen_prefill_decode_tok_s_vs_novorax", pair)
 
 
+def rarutar_section(args) -> int:
+    """--rarutar SIZES: prefill and decode throughput of synthetic Rarutar models (bf16 weights, serving precision) beside the closest model this backend
+    already had - the Tuterax folder design of the same name: grouped-query attention on f32 cache rows, gated recurrences with a decay per head or per key
+    channel behind short convolutions, gated dense feed-forwards, a tied head, the same bf16 linear kernels, cell table and step function, equal width, depth,
+    vocabulary and feed-forward - with each side's distance from its roofline: prefill as a fraction of the dense 16-bit matrix-core peak (2 FLOP per active
+    weight and token), decode as a fraction of the HBM peak (weight bytes one token reads).  One JSON line; the default workload of this script is untouched."""
+    def pair(pkg):
+        m, o = pkg.rarutar_synth, pkg.tuterax_synth
+        return (("rarutar", m, m.write_synthetic_rarutar, lambda cfg, s: m.weight_bytes_per_token(cfg, s.rank)),
+                ("tuterax", o, o.write_synthetic_tuterax, lambda cfg, s: o.weight_bytes_per_token(cfg, s.rank_a, s.rank_g)))
+    return _time_folder_pair(args, args.rarutar, "rarutar_prefill_decode_tok_s_vs_tuterax", pair)
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--novorax", default="", help="comma list of synthetic Novorax sizes (w1024, w2048, w4096): time them beside an F16 Llama twin and exit")
@@ -406,6 +419,7 @@ def main() -> int:
     ap.add_argument("--tuterax", default="", help="comma list of synthetic Tuterax sizes (w1024, w2048, w4096): time them beside the Novorax model of that size and exit")
     ap.add_argument("--dinilorn", default="", help="comma list of synthetic Dinilorn sizes (w1024, w2048, w4096): time them beside the Fidepel model of that size and exit")
     ap.add_argument("--vuzazen", default="", help="comma list of synthetic Vuzazen sizes (w1024, w2048, w4096): time them beside the Novorax model of that size and exit")
+    ap.add_argument("--rarutar", default="", help="comma list of synthetic Rarutar sizes (w1024, w2048, w4096): time them beside the Tuterax model of that size and exit")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)
     ap.add_argument("--warmup", type=int, default=16)
@@ -455,6 +469,8 @@ def main() -> int:
         return dinilorn_section(args)
     if args.vuzazen:
         return vuzazen_section(args)
+    if args.rarutar:
+        return rarutar_section(args)
 
     rank = int(os.environ.get("RANK", "0"))
     local_rank = int(os.environ.get("LOCAL_RANK", "0"))
