@@ -12,9 +12,10 @@
 //       o_t = (q_t P_t)^T S_0 + sum_(s <= t) A_ts v_s      P_t = a_1 .. a_t      A_ts = sum_d q_td k_sd (a_(s+1) .. a_t)_d
 //       S   = diag(P_end) S_0 + sum_s (k_s a_(s+1) .. a_end) v_s^T
 //   All factors are PRODUCTS of decays over the tokens between - never a quotient of two prefix products and never an exponent's difference, so a decay that
-//   closes (a = 0) or a long chunk of small ones underflows to the zero it stands for.  Three launches: A with the scaled q and k of every chunk at once
-//   (gated_intra_*), the walk over the chunks with S in registers, which leaves the state in front of every chunk (gated_state), and the outputs of every chunk
-//   at once (gated_out).  The products of the last two, and A of the one-decay form, run on the f32 matrix cores (v_mfma_f32_16x16x4_f32).
+//   closes (a = 0) or a long chunk of small ones underflows to the zero it stands for.  Everything but the walk from
+//   chunk to chunk is made for all chunks at once: A with the scaled q and k (gated_intra_*), what a chunk adds to the state (gated_update), and the outputs
+//   (gated_out); the walk itself touches every entry of the state once per chunk (gated_carry) and leaves the state in front of the chunk in the place of what the
+//   chunk adds.  The products of update and outputs, and A of the one-decay form, run on the f32 matrix cores (v_mfma_f32_16x16x4_f32).
 //
 // conv_silu: the short causal convolution over time with bias and silu in front of a batch (steps do it inside).  gated_norm: y = o silu(z) over its root mean
 // square in equal parts, times a weight.
@@ -58,23 +59,34 @@ __global__ __launch_bounds__(64 * GSS_NW) void gated_step_kernel(GatedScanArgs a
     const int back = a.conv_taps - 1;
     const float *cs = a.conv_wt ? a.conv_state + (size_t)slot * back * a.conv_C : nullptr;
     const auto input = [&](int c) {                             // channel c of the token, convolved where the layer does that
-        if (!a.conv_wt) return p[c];
+        const float x = p[c];
+        if (!a.conv_wt) return x;
+        float w[8], u[8];                                       // (taps on their way together)
+#pragma unroll
+        for (int j = 0; j < 8; j++) { const bool in = j < back; w[j] = in ? a.conv_wt[(size_t)j * a.conv_C + c] : 0.0f; u[j] = in ? cs[(size_t)j * a.conv_C + c] : 0.0f; }
+        const float wl = a.conv_wt[(size_t)back * a.conv_C + c];
         float s = a.conv_b ? a.conv_b[c] : 0.0f;
-        for (int j = 0; j < back; j++) s = fmaf(a.conv_wt[(size_t)j * a.conv_C + c], cs[(size_t)j * a.conv_C + c], s);
-        return gs_silu(fmaf(a.conv_wt[(size_t)back * a.conv_C + c], p[c], s));
+#pragma unroll
+        for (int j = 0; j < 8; j++) s = fmaf(w[j], u[j], s);
+        for (int j = 8; j < back; j++) s = fmaf(a.conv_wt[(size_t)j * a.conv_C + c], cs[(size_t)j * a.conv_C + c], s);
+        return gs_silu(fmaf(wl, x, s));
     };
     float ah = 1.0f, kmul = 1.0f;
     if (a.dt) {                                                 // one decay per head
         kmul = gs_softplus(a.dt[(size_t)row * a.ld_dt + h] + a.dt_bias[h]);
         ah = expf(-expf(a.A_log[h]) * kmul);
     }
-    const int qk = (h / a.share) * D;
-    for (int d = tid; d < D; d += 64 * GSS_NW) {
-        sq[d] = input(a.off_q + qk + d) * a.q_scale;
-        sk[d] = input(a.off_k + qk + d) * kmul;
-        if (a.dt) sa[d] = ah;
-        else if (!a.lr_w) sa[d] = a.alpha[(size_t)row * a.ld_alpha + (size_t)h * D + d];
+    const int qk = (h / a.share) * D, NI = 2 * D + 64 * NCOL;   // query and key entries, value columns: one item per thread at a time
+    for (int i = tid; i < NI; i += 64 * GSS_NW) {
+        const int d = i < D ? i : i - D, c = i - 2 * D;
+        if (c < 0) {
+            const bool isq = i < D;
+            const float u = input((isq ? a.off_q : a.off_k) + qk + d);
+            if (isq) sq[d] = u * a.q_scale; else sk[d] = u * kmul;
+        } else sv[c] = c0 + c < VD ? input(a.off_v + h * VD + c0 + c) : 0.0f;
     }
+    if (a.dt) for (int d = tid; d < D; d += 64 * GSS_NW) sa[d] = ah;
+    else if (!a.lr_w) for (int d = tid; d < D; d += 64 * GSS_NW) sa[d] = a.alpha[(size_t)row * a.ld_alpha + (size_t)h * D + d];
     if (!a.dt && a.lr_w) {                                      // the second half of the low-rank decay: four lanes share a channel's dot product
         const float *z1 = p + a.off_lr;
         for (int d0 = 0; d0 < D; d0 += 16 * GSS_NW) {
@@ -89,7 +101,6 @@ __global__ __launch_bounds__(64 * GSS_NW) void gated_step_kernel(GatedScanArgs a
             if (d < D && (tid & 3) == 0) sa[d] = expf(-gs_softplus(-(z + a.lr_bias[(size_t)h * D + d])) * a.inv_tau);
         }
     }
-    for (int c = tid; c < 64 * NCOL; c += 64 * GSS_NW) sv[c] = c0 + c < VD ? input(a.off_v + h * VD + c0 + c) : 0.0f;
     __syncthreads();
     float v[NCOL], num[NCOL];
 #pragma unroll
@@ -137,6 +148,40 @@ __global__ __launch_bounds__(64 * GSS_NW) void gated_step_kernel(GatedScanArgs a
 }
 
 // ---------------------------------------------------------------- chunks
+// the decays of a batch: alpha[t][n] = sigmoid(sum_r w[n][r] z1[t][r] + bias[n])^inv_tau; thread = channel, eight tokens at a time, the low-rank row in pieces of 32
+constexpr int GSD_T = 8, GSD_R = 32;
+__global__ __launch_bounds__(256) void gated_decay_kernel(const float *z1, int ld_z, int T, int rank, const unsigned short *w, const float *bias, float inv_tau, int N, float *alpha, int ld_a) {
+    __shared__ float sz[GSD_T][GSD_R];
+    const int t0 = blockIdx.x * GSD_T, n = blockIdx.y * 256 + threadIdx.x, tid = threadIdx.x;
+    const unsigned short *wn = w + (size_t)(n < N ? n : N - 1) * rank;
+    float acc[GSD_T];
+#pragma unroll
+    for (int t = 0; t < GSD_T; t++) acc[t] = 0.0f;
+    for (int r0 = 0; r0 < rank; r0 += GSD_R) {
+        const int nr = rank - r0 < GSD_R ? rank - r0 : GSD_R;
+        unsigned short u[GSD_R];
+#pragma unroll
+        for (int r = 0; r < GSD_R; r++) u[r] = r < nr ? wn[r0 + r] : 0;
+        if (r0 > 0) __syncthreads();
+        {
+            const int t = tid >> 5, r = tid & 31;
+            sz[t][r] = t0 + t < T && r < nr ? z1[(size_t)(t0 + t) * ld_z + r0 + r] : 0.0f;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int r = 0; r < GSD_R; r++) {
+            const float wr = __uint_as_float((unsigned)u[r] << 16);
+#pragma unroll
+            for (int t = 0; t < GSD_T; t++) acc[t] = fmaf(wr, sz[t][r], acc[t]);
+        }
+    }
+    if (n >= N) return;
+    const float b = bias[n];
+#pragma unroll
+    for (int t = 0; t < GSD_T; t++)
+        if (t0 + t < T) alpha[(size_t)(t0 + t) * ld_a + n] = expf(-gs_softplus(-(acc[t] + b)) * inv_tau);
+}
+
 // place of a chunk among all chunks of the launch: no two chunks share one, and rows / 64 + segments places hold them all
 __device__ __forceinline__ int gs_chunk_at(const GatedScanArgs &a, int seg, int row0) { return ((row0 - a.row0) >> 6) + seg; }
 
@@ -144,7 +189,7 @@ __device__ __forceinline__ int gs_chunk_at(const GatedScanArgs &a, int seg, int 
 // Lane = key row s, the four waves share the channels of a slice; a key's running product walks down the rows.
 constexpr int GSI_DC = 32, GSI_LD = GSI_DC + 4;
 __global__ __launch_bounds__(256) void gated_intra_channel_kernel(GatedScanArgs a, int chunks) {
-    __shared__ __attribute__((aligned(16))) float sa[GS_T][GSI_LD], sk[GS_T][GSI_LD], skr[GS_T][GSI_LD], sq[16][GSI_LD];
+    __shared__ __attribute__((aligned(16))) float sa[GS_T][GSI_LD], sk[GS_T][GSI_LD], skr[GS_T][GSI_LD], sq[16][GSI_LD], sp[16][GSI_LD];
     __shared__ float G[4][GSI_DC];
     __shared__ float part[4][16][GS_T];
     const int seg = blockIdx.x / chunks, c = blockIdx.x - seg * chunks, h = blockIdx.y, I = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -157,36 +202,51 @@ __global__ __launch_bounds__(256) void gated_intra_channel_kernel(GatedScanArgs 
     float acc[16];
 #pragma unroll
     for (int t = 0; t < 16; t++) acc[t] = 0.0f;
-    for (int dc = 0; dc < D; dc += GSI_DC) {
-        __syncthreads();                                        // (the previous slice has been used up)
+    // a slice's inputs travel memory -> registers -> LDS: the next slice's are on their way while this one is worked on
+    float ra[8], rk[8], rq[2];
+    const auto request = [&](int dc) {
 #pragma unroll
         for (int i = 0; i < 8; i++) {
             const int idx = tid + 256 * i, t = idx >> 5, d = idx & 31;
             const bool in = t < nc && dc + d < D;
-            sa[t][d] = in ? al[(size_t)(row0 + t) * a.ld_alpha + dc + d] : 1.0f;     // (rows past the end: nothing fades, nothing is written)
-            sk[t][d] = in ? k[(size_t)(row0 + t) * a.ld_p + dc + d] : 0.0f;
+            ra[i] = in ? al[(size_t)(row0 + t) * a.ld_alpha + dc + d] : 1.0f;        // (rows past the end: nothing fades, nothing is written)
+            rk[i] = in ? k[(size_t)(row0 + t) * a.ld_p + dc + d] : 0.0f;
         }
 #pragma unroll
         for (int i = 0; i < 2; i++) {
             const int idx = tid + 256 * i, t = idx >> 5, d = idx & 31;
-            sq[t][d] = 16 * I + t < nc && dc + d < D ? q[(size_t)(row0 + 16 * I + t) * a.ld_p + dc + d] * a.q_scale : 0.0f;
+            rq[i] = 16 * I + t < nc && dc + d < D ? q[(size_t)(row0 + 16 * I + t) * a.ld_p + dc + d] * a.q_scale : 0.0f;
         }
+    };
+    request(0);
+    for (int dc = 0; dc < D; dc += GSI_DC) {
+        __syncthreads();                                        // (the previous slice has been used up)
+#pragma unroll
+        for (int i = 0; i < 8; i++) { const int idx = tid + 256 * i; sa[idx >> 5][idx & 31] = ra[i]; sk[idx >> 5][idx & 31] = rk[i]; }
+#pragma unroll
+        for (int i = 0; i < 2; i++) { const int idx = tid + 256 * i; sq[idx >> 5][idx & 31] = rq[i]; }
         __syncthreads();
+        if (dc + GSI_DC < D) request(dc + GSI_DC);
         if (tid < 128) {                                        // keys times the decays behind them inside their block; a block's whole product
             const int d = tid & 31, b = tid >> 5;
             float r = 1.0f;
 #pragma unroll
             for (int t = 15; t >= 0; t--) { skr[16 * b + t][d] = sk[16 * b + t][d] * r; r *= sa[16 * b + t][d]; }
             G[b][d] = r;
+        } else if (tid < 160) {                                 // beside them: the decays up to every row of this workgroup's block
+            const int d = tid & 31;
+            float r = 1.0f;
+#pragma unroll
+            for (int t = 0; t < 16; t++) { r *= sa[16 * I + t][d]; sp[t][d] = r; }
         }
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < 2; i++) {
             const int d = tid & 31, t = (tid >> 5) + 8 * i, row = 16 * I + t;
             if (row < nc && dc + d < D) {
-                float pf = 1.0f, sf = 1.0f;
-                for (int b = 0; b < 4; b++) { if (b < I) pf *= G[b][d]; else if (b > I) sf *= G[b][d]; }
-                for (int u = 0; u <= t; u++) pf *= sa[16 * I + u][d];
+                float pf = sp[t][d], sf = 1.0f;
+#pragma unroll
+                for (int b = 0; b < 4; b++) { const float g = G[b][d]; if (b < I) pf *= g; else if (b > I) sf *= g; }
                 qh[(size_t)(row0 + row) * ((size_t)H * D) + dc + d] = sq[t][d] * pf;
                 kh[(size_t)(row0 + row) * ((size_t)H * D) + dc + d] = skr[row][d] * sf;
             }
@@ -278,15 +338,25 @@ __global__ __launch_bounds__(256) void gated_intra_head_kernel(GatedScanArgs a, 
     {
         // lane = key row: its factor walks down the rows, each wave keeps its own 16; the last wave's final product is what the key still counts at the chunk's end
         float w = 0.0f;
-        const int hi = 16 * wave + 15;
-        for (int u = 0; u <= hi; u++) {
-            w = u == lane ? 1.0f : w * sa[u];
-            if (u >= 16 * wave) wt[u][lane] = w * sdt[lane] * a.q_scale;
+        const float by = sdt[lane] * a.q_scale;
+#pragma unroll 4
+        for (int u4 = 0; u4 < 4 * wave + 4; u4++) {
+            const f32x4 a4 = *reinterpret_cast<const f32x4 *>(&sa[4 * u4]);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                w = 4 * u4 + e == lane ? 1.0f : w * a4[e];
+                if (u4 >= 4 * wave) wt[4 * u4 + e][lane] = w * by;
+            }
         }
         if (wave == 3 && lane < nc) a.w_s[(size_t)(row0 + lane) * H + h] = w * sdt[lane];
         if (wave == 0) {
             float p = 1.0f;
-            for (int u = 0; u < GS_T; u++) p *= u <= lane ? sa[u] : 1.0f;
+#pragma unroll 4
+            for (int u4 = 0; u4 < GS_T / 4; u4++) {
+                const f32x4 a4 = *reinterpret_cast<const f32x4 *>(&sa[4 * u4]);
+#pragma unroll
+                for (int e = 0; e < 4; e++) p *= 4 * u4 + e <= lane ? a4[e] : 1.0f;
+            }
             if (lane < nc) a.w_p[(size_t)(row0 + lane) * H + h] = p * a.q_scale;
             if (lane == GS_T - 1) a.w_g[(size_t)gs_chunk_at(a, seg, row0) * H + h] = p;
         }
@@ -304,68 +374,62 @@ __global__ __launch_bounds__(256) void gated_intra_head_kernel(GatedScanArgs a, 
     }
 }
 
-// the walk over a segment's chunks: a wave owns 32 rows x 16 columns of S in the matrix cores' result layout (lane = column l & 15, register r of tile i = row 16 i +
-// 4 (l >> 4) + r), writes the state in front of every chunk for gated_out, and takes the next chunk's operands while a chunk is multiplied.  No wave waits for another.
+// what one chunk adds to the state: sum_s (k_s a_(s+1) .. a_end) v_s^T; a wave makes 32 rows x 16 columns of it (lane = column l & 15, register r of tile i = row
+// 16 i + 4 (l >> 4) + r).  No wave waits for another.
 template <bool PERCH>
-__global__ __launch_bounds__(256) void gated_state_kernel(GatedScanArgs a, int CB) {
-    const int seg = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, lg = lane >> 4;
+__global__ __launch_bounds__(256) void gated_update_kernel(GatedScanArgs a, int chunks, int CB) {
+    const int seg = blockIdx.x / chunks, c = blockIdx.x - seg * chunks, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, lg = lane >> 4;
     const int H = a.H, D = a.D, VD = a.VD, d0 = ((int)blockIdx.z / CB) * 32, col = ((int)blockIdx.z % CB) * 64 + 16 * wave + l16;
-    const int start = a.seg_start[seg], len = a.seg_len[seg], slot = a.seg_slot[seg];
+    const int len = a.seg_len[seg] - c * GS_T, row0 = a.seg_start[seg] + c * GS_T;
+    if (len <= 0) return;
+    const int nc = len < GS_T ? len : GS_T;
     const bool cin = col < VD;
-    float *Sg = a.S + ((size_t)slot * H + h) * (size_t)D * VD + col;
     const float *kb = PERCH ? a.w_k + (size_t)h * D : a.p + a.off_k + (size_t)(h / a.share) * D;
-    const size_t ld_k = PERCH ? (size_t)H * D : (size_t)a.ld_p;
+    const int ld_k = PERCH ? H * D : a.ld_p;
     const float *vb = a.p + a.off_v + (size_t)h * VD + col;
-    f32x4 S[2], ng[2];
-    float nk[2][16], nv[16];
+    float k[2][16], v[16];
 #pragma unroll
-    for (int i = 0; i < 2; i++)
+    for (int j = 0; j < 16; j++) {
+        const int s = 16 * (j >> 2) + 4 * lg + (j & 3), row = row0 + (s < nc ? s : nc - 1);
 #pragma unroll
-        for (int r = 0; r < 4; r++) { const int d = d0 + 16 * i + 4 * lg + r; S[i][r] = cin && d < D ? Sg[(size_t)d * VD] : 0.0f; }
-    const auto request = [&](int t0) {
-        const int nc = len - t0 < GS_T ? len - t0 : GS_T, row0 = start + t0;
-        const int at = gs_chunk_at(a, seg, row0) * H + h;
-#pragma unroll
-        for (int j = 0; j < 16; j++) {
-            const int s = 16 * (j >> 2) + 4 * lg + (j & 3);
-            const size_t row = (size_t)(row0 + (s < nc ? s : nc - 1));
-#pragma unroll
-            for (int i = 0; i < 2; i++) { const int d = d0 + 16 * i + l16; nk[i][j] = d < D ? kb[row * ld_k + d] : 0.0f; }
-            nv[j] = s < nc && cin ? vb[row * a.ld_p] : 0.0f;
-            if (!PERCH) nv[j] *= a.w_s[row * H + h];
-        }
-#pragma unroll
-        for (int i = 0; i < 2; i++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) {
-                const int d = d0 + 16 * i + 4 * lg + r;
-                ng[i][r] = PERCH ? (d < D ? a.w_g[(size_t)at * D + d] : 0.0f) : a.w_g[at];
-            }
-    };
-    request(0);
-    for (int t0 = 0; t0 < len; t0 += GS_T) {
-        float k[2][16], v[16];
-        f32x4 g[2];
-#pragma unroll
-        for (int j = 0; j < 16; j++) { k[0][j] = nk[0][j]; k[1][j] = nk[1][j]; v[j] = nv[j]; }
-        g[0] = ng[0]; g[1] = ng[1];
-        float *Sc = a.w_S + ((size_t)gs_chunk_at(a, seg, start + t0) * H + h) * (size_t)D * VD + col;
-#pragma unroll
-        for (int i = 0; i < 2; i++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) { const int d = d0 + 16 * i + 4 * lg + r; if (cin && d < D) Sc[(size_t)d * VD] = S[i][r]; }
-        if (t0 + GS_T < len) request(t0 + GS_T);
-#pragma unroll
-        for (int i = 0; i < 2; i++) {
-            S[i] *= g[i];
-#pragma unroll
-            for (int j = 0; j < 16; j++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(k[i][j], v[j], S[i], 0, 0, 0);
-        }
+        for (int i = 0; i < 2; i++) { const int d = d0 + 16 * i + l16; k[i][j] = d < D ? kb[(size_t)row * ld_k + d] : 0.0f; }
+        v[j] = s < nc && cin ? vb[(size_t)row * a.ld_p] : 0.0f;
+        if (!PERCH) v[j] *= a.w_s[(size_t)row * H + h];
     }
+    f32x4 U[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
+#pragma unroll
+    for (int j = 0; j < 16; j++)
+#pragma unroll
+        for (int i = 0; i < 2; i++) U[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(k[i][j], v[j], U[i], 0, 0, 0);
+    float *Uc = a.w_S + ((size_t)gs_chunk_at(a, seg, row0) * H + h) * (size_t)D * VD + col;
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int r = 0; r < 4; r++) { const int d = d0 + 16 * i + 4 * lg + r; if (cin && d < D) Sg[(size_t)d * VD] = S[i][r]; }
+        for (int r = 0; r < 4; r++) { const int d = d0 + 16 * i + 4 * lg + r; if (cin && d < D) Uc[(size_t)d * VD] = U[i][r]; }
+}
+
+// the walk over a segment's chunks, one entry of the state per thread: S <- g S + (what the chunk adds), the state in front of the chunk takes the addition's place
+constexpr int GSC_AHEAD = 8;
+template <bool PERCH>
+__global__ __launch_bounds__(256) void gated_carry_kernel(GatedScanArgs a) {
+    const int seg = blockIdx.x, h = blockIdx.y, e = (int)blockIdx.z * 256 + (int)threadIdx.x, H = a.H, D = a.D, VD = a.VD;
+    if (e >= D * VD) return;
+    const int start = a.seg_start[seg], len = a.seg_len[seg], n = (len + GS_T - 1) / GS_T, at0 = gs_chunk_at(a, seg, start);   // (a segment's chunks lie side by side)
+    float *Sg = a.S + ((size_t)a.seg_slot[seg] * H + h) * (size_t)D * VD + e;
+    float *U = a.w_S + ((size_t)at0 * H + h) * (size_t)D * VD + e;
+    const float *g = PERCH ? a.w_g + ((size_t)at0 * H + h) * D + e / VD : a.w_g + (size_t)at0 * H + h;
+    const size_t us = (size_t)H * D * VD, gs = PERCH ? (size_t)H * D : (size_t)H;
+    float S = *Sg;
+    for (int c0 = 0; c0 < n; c0 += GSC_AHEAD) {
+        float u[GSC_AHEAD], f[GSC_AHEAD];
+#pragma unroll
+        for (int i = 0; i < GSC_AHEAD; i++)
+            if (c0 + i < n) { u[i] = U[(size_t)(c0 + i) * us]; f[i] = g[(size_t)(c0 + i) * gs]; }
+#pragma unroll
+        for (int i = 0; i < GSC_AHEAD; i++)
+            if (c0 + i < n) { U[(size_t)(c0 + i) * us] = S; S = fmaf(f[i], S, u[i]); }
+    }
+    *Sg = S;
 }
 
 // the outputs of 64 columns of one chunk of one head: (q P) S_0 + A V (+ skip v); a wave per 16 tokens, S_0 and V through LDS
@@ -381,34 +445,39 @@ __global__ __launch_bounds__(256) void gated_out_kernel(GatedScanArgs a, int chu
     const int t = 16 * wave + l16, tr = row0 + (t < nc ? t : nc - 1);
     const float *q = PERCH ? a.w_q + ((size_t)tr * H + h) * D : a.p + (size_t)tr * a.ld_p + a.off_q + (size_t)(h / a.share) * D;
     const float *A = a.w_A + ((size_t)tr * H + h) * GS_T;
+    float nv[16], ns[16];
+    f32x4 A4[4], acc[4], q4[4];
+    const auto request = [&](int ds) {
 #pragma unroll
-    for (int i = 0; i < 16; i++) {
-        const int s = wave + 4 * i;
-        sV[s][lane] = s < nc && col < VD ? a.p[(size_t)(row0 + s) * a.ld_p + a.off_v + (size_t)h * VD + col] : 0.0f;
-    }
-    f32x4 A4[4], acc[4];
+        for (int u = 0; u < 4; u++) q4[u] = gs_load4<VEC>(q, ds + 16 * u + 4 * lg, D);
+#pragma unroll
+        for (int i = 0; i < 16; i++) { const int d = ds + wave + 4 * i; ns[i] = d < D && col < VD ? Sc[(size_t)d * VD + col] : 0.0f; }
+    };
+    request(0);                                                 // (everything the first products need is on its way before any of it is waited for)
+#pragma unroll
+    for (int i = 0; i < 16; i++) { const int s = wave + 4 * i; nv[i] = s < nc && col < VD ? a.p[(size_t)(row0 + s) * a.ld_p + a.off_v + (size_t)h * VD + col] : 0.0f; }
 #pragma unroll
     for (int u = 0; u < 4; u++) {
         A4[u] = u <= wave ? *reinterpret_cast<const f32x4 *>(A + 16 * u + 4 * lg) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
         acc[u] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     }
+#pragma unroll
+    for (int i = 0; i < 16; i++) sV[wave + 4 * i][lane] = nv[i];
     for (int ds = 0; ds < D; ds += GS_T) {
-        f32x4 q4[4];
-#pragma unroll
-        for (int u = 0; u < 4; u++) q4[u] = gs_load4<VEC>(q, ds + 16 * u + 4 * lg, D);
         if (ds > 0) __syncthreads();                            // (the previous slice has been used up)
+        f32x4 qs[4];
 #pragma unroll
-        for (int i = 0; i < 16; i++) {
-            const int d = wave + 4 * i;
-            sS[d][lane] = ds + d < D && col < VD ? Sc[(size_t)(ds + d) * VD + col] : 0.0f;
-        }
+        for (int u = 0; u < 4; u++) qs[u] = q4[u];
+#pragma unroll
+        for (int i = 0; i < 16; i++) sS[wave + 4 * i][lane] = ns[i];
         __syncthreads();
+        if (ds + GS_T < D) request(ds + GS_T);
 #pragma unroll
         for (int u = 0; u < 4; u++)
 #pragma unroll
             for (int e = 0; e < 4; e++)
 #pragma unroll
-                for (int ct = 0; ct < 4; ct++) acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[u][e], sS[16 * u + 4 * lg + e][16 * ct + l16], acc[ct], 0, 0, 0);
+                for (int ct = 0; ct < 4; ct++) acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(qs[u][e], sS[16 * u + 4 * lg + e][16 * ct + l16], acc[ct], 0, 0, 0);
     }
     if (!PERCH) {
         f32x4 w;
@@ -530,13 +599,14 @@ hipError_t launch_gated_scan(const GatedScanArgs &a, hipStream_t st) {
         return launch_gated_step<1>(a, (a.VD + 63) / 64, st);
     }
     if ((perch && (!a.alpha || !a.w_q || !a.w_k)) || (!perch && (!a.w_p || !a.w_s)) || !a.w_A || !a.w_g || !a.w_S || !a.o) return hipErrorInvalidValue;
-    const int chunks = (a.max_len + GS_T - 1) / GS_T, CB = (a.VD + 63) / 64, DB = (a.D + 31) / 32;
+    const int chunks = (a.max_len + GS_T - 1) / GS_T, CB = (a.VD + 63) / 64, DB = (a.D + 31) / 32, EB = (int)(((long long)a.D * a.VD + 255) / 256);
     const auto al16 = [](const void *p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
-    const dim3 ic((unsigned)(a.n_seg * chunks), (unsigned)a.H), sg((unsigned)a.n_seg, (unsigned)a.H, (unsigned)(DB * CB)), og((unsigned)(a.n_seg * chunks), (unsigned)a.H, (unsigned)CB);
+    const dim3 ic((unsigned)(a.n_seg * chunks), (unsigned)a.H), ug(ic.x, ic.y, (unsigned)(DB * CB)), cg((unsigned)a.n_seg, (unsigned)a.H, (unsigned)EB), og((unsigned)(a.n_seg * chunks), (unsigned)a.H, (unsigned)CB);
     if (perch) {
         const bool vec = (a.D & 3) == 0 && al16(a.w_q);
         hipLaunchKernelGGL(gated_intra_channel_kernel, dim3(ic.x, ic.y, 4), dim3(256), 0, st, a, chunks);
-        hipLaunchKernelGGL(gated_state_kernel<true>, sg, dim3(256), 0, st, a, CB);
+        hipLaunchKernelGGL(gated_update_kernel<true>, ug, dim3(256), 0, st, a, chunks, CB);
+        hipLaunchKernelGGL(gated_carry_kernel<true>, cg, dim3(256), 0, st, a);
         if (vec) hipLaunchKernelGGL((gated_out_kernel<true, true>), og, dim3(256), 0, st, a, chunks);
         else hipLaunchKernelGGL((gated_out_kernel<true, false>), og, dim3(256), 0, st, a, chunks);
         return hipGetLastError();
@@ -544,9 +614,17 @@ hipError_t launch_gated_scan(const GatedScanArgs &a, hipStream_t st) {
     const bool vec = ((a.D | a.ld_p | a.off_q | a.off_k) & 3) == 0 && al16(a.p);
     if (vec) hipLaunchKernelGGL(gated_intra_head_kernel<true>, ic, dim3(256), 0, st, a, chunks);
     else hipLaunchKernelGGL(gated_intra_head_kernel<false>, ic, dim3(256), 0, st, a, chunks);
-    hipLaunchKernelGGL(gated_state_kernel<false>, sg, dim3(256), 0, st, a, CB);
+    hipLaunchKernelGGL(gated_update_kernel<false>, ug, dim3(256), 0, st, a, chunks, CB);
+    hipLaunchKernelGGL(gated_carry_kernel<false>, cg, dim3(256), 0, st, a);
     if (vec) hipLaunchKernelGGL((gated_out_kernel<false, true>), og, dim3(256), 0, st, a, chunks);
     else hipLaunchKernelGGL((gated_out_kernel<false, false>), og, dim3(256), 0, st, a, chunks);
+    return hipGetLastError();
+}
+
+hipError_t launch_gated_decay(const float *z1, int ld_z, int T, int rank, const unsigned short *w, const float *bias, float inv_tau, int N, float *alpha, int ld_a, hipStream_t st) {
+    if (T <= 0 || N <= 0) return hipSuccess;
+    if (rank < 1 || !z1 || !w || !bias || !alpha) return hipErrorInvalidValue;
+    hipLaunchKernelGGL(gated_decay_kernel, dim3((unsigned)((T + GSD_T - 1) / GSD_T), (unsigned)((N + 255) / 256)), dim3(256), 0, st, z1, ld_z, T, rank, w, bias, inv_tau, N, alpha, ld_a);
     return hipGetLastError();
 }
 

@@ -267,8 +267,8 @@ hipError_t launch_moe_scatter_combine(float *x, const float *y, const float *w, 
 // Outer index z < nz, one of: plain strides (x_zs / w_zs / y_zs elements; per-head products); meta != nullptr: z is an expert, its rows of X and Y are
 // [meta[nz + z], + meta[z]) (launch_moe_group's counts | offsets; T = upper bound of any expert's rows); sel != nullptr: z is a (token, rank) pair - weight set
 // sel[z], row z / sel_div of X, row z of Y.
-// y | relu(y)^2 | sigmoid(y)^epi_limit | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = min(W x, epi_limit), u = clamp(W2 x, -epi_limit, epi_limit)
-enum { MMB_STORE = 0, MMB_RELU2 = 1, MMB_SIGMOID_POW = 2, MMB_SILU_MUL = 3, MMB_GELU_MUL = 4, MMB_CLAMP_SWIGLU = 5 };   // (from MMB_SILU_MUL on: gated, two weight sets)
+// y | relu(y)^2 | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = min(W x, epi_limit), u = clamp(W2 x, -epi_limit, epi_limit)
+enum { MMB_STORE = 0, MMB_RELU2 = 1, MMB_SILU_MUL = 2, MMB_GELU_MUL = 3, MMB_CLAMP_SWIGLU = 4 };   // (from MMB_SILU_MUL on: gated, two weight sets)
 constexpr int MMB_VEC_ROWS = 16;                               // up to this many rows take the one-wave-per-column kernel
 struct MMBArgs {
     const float *x = nullptr; int ldx = 0;
@@ -276,7 +276,7 @@ struct MMBArgs {
     float *y = nullptr; int ldy = 0;
     int T = 0, N = 0, K = 0, epi = MMB_STORE, f32 = 0;
     float out_scale = 1.0f;                                    // multiplies every stored value (a model's logit scale)
-    float epi_limit = 0.0f;                                    // MMB_CLAMP_SWIGLU: the clamp; MMB_SIGMOID_POW: the exponent
+    float epi_limit = 0.0f;                                    // MMB_CLAMP_SWIGLU: the clamp
     const float *bias = nullptr;                               // nullable, [N] f32: added to W x before the epilogue (the same vector for every outer index)
     const float *row_scale = nullptr;                          // nullable, a factor on W x (and W2 x) of every row, by the row's place in Y in front of y_map; in front of the bias
     const float *resid = nullptr;                              // nullable, indexed like Y (and may be Y): added behind the epilogue
@@ -542,6 +542,8 @@ inline size_t gated_scan_chunks(size_t rows, size_t segs) { return rows / 64 + s
 bool gated_scan_shape_ok(int H, int share, int D, int VD);
 bool gated_step_closes(int VD);
 hipError_t launch_gated_scan(const GatedScanArgs &a, hipStream_t st);
+// a batch's decays per key channel: alpha[t][n] = sigmoid(sum_r w[n][r] z1[t][r] + bias[n])^inv_tau (f32 throughout)
+hipError_t launch_gated_decay(const float *z1, int ld_z, int T, int rank, const unsigned short *w, const float *bias, float inv_tau, int N, float *alpha, int ld_a, hipStream_t st);
 // y[t][c] = silu(bias[c] + sum_j wt[j][c] u[t - taps + 1 + j][c]) over rows of p (C channels); tok_ago: rows of the token's own segment in front of it; what lies further back
 // comes from state [slot][taps - 1][C] (launch_conv_state moves it on behind)
 hipError_t launch_conv_silu(const float *p, int ld_p, int C, const float *wt, const float *bias, int taps, const float *state, const int32_t *tok_ago, const int32_t *tok_slot, int T,

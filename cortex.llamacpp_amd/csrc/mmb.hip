@@ -12,7 +12,7 @@
 //   * mmb_mfma  - batches in bf16 mode: LDS-tiled, activations rounded to bf16 on the way in, v_mfma_f32_32x32x16_bf16, f32 accumulation.
 //   * mmb_f32   - batches in f32 mode (and every shape the other two refuse): LDS-tiled, v_fma_f32 only - products of an f32 activation and a bf16 weight
 //                 widened exactly, no reduced-precision matrix mode anywhere.
-// Epilogues: store | relu(y)^2 | sigmoid(y)^e | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = W x capped from above and u = W2 x clamped
+// Epilogues: store | relu(y)^2 | silu(W x) * (W2 x) | gelu_tanh(W x) * (W2 x) | g sigmoid(1.702 g) (u + 1) with g = W x capped from above and u = W2 x clamped
 // to +- the same limit (the gated ones: two weight sets, one pass over the activations).  Around the epilogue, each optional: a factor per row on W x (and W2 x)
 // - linear layers without a bias: the row of X itself times that number -, an f32 bias per output column in front of it, a residual row added behind it.  A
 // grouped batch may read its rows of X, and write its rows of Y, through maps (no gather in front of the launch, no scatter behind it).
@@ -37,7 +37,6 @@ __device__ __forceinline__ float epi_apply(int epi, float a, float b, float lim 
         const float g = fminf(a, lim), u = fminf(fmaxf(b, -lim), lim);
         return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
     }
-    if (epi == MMB_SIGMOID_POW) return expf(-lim * (fmaxf(-a, 0.0f) + log1pf(expf(-fabsf(a)))));   // (sigmoid = e^-softplus(-a))
     if (epi == MMB_RELU2) { const float r = a > 0.0f ? a : 0.0f; return r * r; }
     if (epi == MMB_SILU_MUL) return a / (1.0f + expf(-a)) * b;
     if (epi == MMB_GELU_MUL) return 0.5f * a * (1.0f + tanhf(0.7978845608028654f * (a + 0.044715f * a * a * a))) * b;   // the tanh form of gelu; sqrt(2 / pi)
@@ -209,13 +208,23 @@ __global__ __launch_bounds__(256) void mmb_vec_kernel(MMBArgs a) {
         for (int i = 0; i < TB; i++) {
             rsc[i] = a.row_scale && i < nt ? a.row_scale[v.y0 + t0 + i] : 1.0f;
             res[i] = v.resid && i < nt ? v.resid[y_row(a, v, t0 + i) + n] : 0.0f;
-            if (LN) mid[i] = i < nt ? row_middle<VEC>(x_row(a, v, t0 + i), a.K, lane) : 0.0f;
+        }
+        u16x8 w8n = {0, 0, 0, 0, 0, 0, 0, 0}, w28n = w8n;           // (LN: a piece's weights are on their way while the row's middle value, or the piece before, is worked on)
+        const auto ahead = [&](int k) {
+            if (k >= a.K) return;
+            w8n = *reinterpret_cast<const u16x8 *>(wr + k);
+            if (wr2) w28n = *reinterpret_cast<const u16x8 *>(wr2 + k);
+        };
+        if (LN) {
+            if (VEC) ahead(lane * 8);
+#pragma unroll
+            for (int i = 0; i < TB; i++) mid[i] = i < nt ? row_middle<VEC>(x_row(a, v, t0 + i), a.K, lane) : 0.0f;
         }
         if (VEC) {
             for (int k = lane * 8; k < a.K; k += 512) {
-                const u16x8 w8 = *reinterpret_cast<const u16x8 *>(wr + k);
-                u16x8 w28 = w8;
-                if (wr2) w28 = *reinterpret_cast<const u16x8 *>(wr2 + k);
+                if (!LN) ahead(k);
+                const u16x8 w8 = w8n, w28 = w28n;
+                if (LN) ahead(k + 512);
                 float pw[8];
                 if (pn) {
                     const f32x4 g0 = *reinterpret_cast<const f32x4 *>(a.pn_w + k), g1 = *reinterpret_cast<const f32x4 *>(a.pn_w + k + 4);
@@ -525,7 +534,6 @@ hipError_t launch_mmb(const MMBArgs &a, hipStream_t st) {
         switch (a.epi) {
             case MMB_STORE: return launch_mmb_mfma_tile<MMB_STORE>(a, rows_max, st);
             case MMB_RELU2: return launch_mmb_mfma_tile<MMB_RELU2>(a, rows_max, st);
-            case MMB_SIGMOID_POW: return launch_mmb_mfma_tile<MMB_SIGMOID_POW>(a, rows_max, st);
             case MMB_SILU_MUL: return launch_mmb_mfma_tile<MMB_SILU_MUL>(a, rows_max, st);
             case MMB_GELU_MUL: return launch_mmb_mfma_tile<MMB_GELU_MUL>(a, rows_max, st);
             case MMB_CLAMP_SWIGLU: return launch_mmb_mfma_tile<MMB_CLAMP_SWIGLU>(a, rows_max, st);

@@ -244,9 +244,9 @@ hipError_t Context::nvx_gla_heads(const NvxLayer &L, int state_set, int T, const
     const NovoraxModel &M = *model->nvx;
     const int H = L.heads, D = L.dim, VD = L.vdim;
     const size_t TU = cp.n_ubatch;
-    bool batch = false;                                         // some segment holds several rows: its decays are made by a product over all rows
+    bool batch = false;                                         // some segment holds several rows: its decays are made for all rows at once
     for (const auto &wv : nvx_waves_) for (int s = 0; s < wv.second; s++) batch = batch || h_seg_[TU + (size_t)(wv.first + s)] > 1;
-    if (batch) RRT_TRY(nvx_linear(L.a2, p + L.off_a, LD_P, T, nvx_qa_, H * D, MMB_SIGMOID_POW, nullptr, 1.0f, nullptr, L.a2_bias, L.inv_tau));
+    if (batch) RRT_TRY(launch_gated_decay(p + L.off_a, LD_P, T, L.rank_a, L.a2.w, L.a2_bias, L.inv_tau, H * D, nvx_qa_, H * D, stream_));
     GatedScanArgs ga{};
     ga.p = p; ga.ld_p = LD_P; ga.off_q = 0; ga.off_k = H * D; ga.off_v = 2 * H * D; ga.share = 1; ga.q_scale = L.scale;
     ga.alpha = nvx_qa_; ga.ld_alpha = H * D; ga.lr_bias = L.a2_bias; ga.rank = L.rank_a; ga.off_lr = L.off_a; ga.inv_tau = L.inv_tau;
