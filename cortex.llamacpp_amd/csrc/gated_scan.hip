@@ -38,12 +38,12 @@ __device__ __forceinline__ float gs_wave_sum(float v) {
 constexpr int GS_T = 64;                                        // tokens per chunk
 
 // ---------------------------------------------------------------- single rows
-// A workgroup owns 64 NCOL columns of one head of one segment: lane = column (NCOL of them, 64 apart), the eight waves share the rows.  The first 128 rows of the
+// A workgroup owns 64 NCOL columns of one head of one segment: lane = column (NCOL of them, 64 apart), the NW waves share the rows.  The first 128 rows of the
 // state are on their way from memory while q, k and the decays are made.
-constexpr int GSS_NW = 8, GSS_PRE = 16;
-template <int NCOL>
+template <int NCOL, int GSS_NW>
 __global__ __launch_bounds__(64 * GSS_NW) void gated_step_kernel(GatedScanArgs a) {
     extern __shared__ float gs_lds[];
+    constexpr int GSS_PRE = 128 / GSS_NW;
     const int D = a.D, VD = a.VD, H = a.H, tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     float *sq = gs_lds, *sk = sq + D, *sa = sk + D, *sv = sa + D, *red = sv + 64 * NCOL;        // [D], [D], [D], [64 NCOL], [NW][64 NCOL]
     const int seg = blockIdx.x, h = blockIdx.y, row = a.row0 + seg, slot = a.seg_slot[seg], c0 = blockIdx.z * 64 * NCOL;
@@ -540,9 +540,24 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const float *p, int ld_p
 
 // y = o silu(z), every one of `parts` equal parts of the row over its root mean square, times w.  mv.state set (every row is a segment of its own): the launch also
 // moves the convolution inputs on - nobody reads them any more
-__global__ __launch_bounds__(256) void gated_norm_kernel(const float *o, int ld_o, const float *z, int ld_z, const float *w, int n, float eps, float *y, int ld_y, ConvMove mv) {
+__global__ __launch_bounds__(256) void gated_norm_kernel(const float *o, int ld_o, const float *z, int ld_z, const float *w, int parts, int n, float eps, float *y, int ld_y,
+                                                         ConvMove mv) {
     __shared__ float sh[4];
     const int t = blockIdx.x, part = blockIdx.y, tid = threadIdx.x;
+    if (part >= parts) {                                        // (the launch's further workgroups: a channel per thread)
+        const int c = (part - parts) * 256 + tid, back = mv.taps - 1;
+        if (c >= mv.C) return;
+        float *st = mv.state + (size_t)mv.seg_slot[t] * back * mv.C + c;
+        const float u = mv.p[(size_t)t * mv.ld_p + c];
+        float keep[8];
+#pragma unroll
+        for (int j = 0; j < 8; j++) keep[j] = j + 1 < back ? st[(size_t)(j + 1) * mv.C] : 0.0f;
+#pragma unroll
+        for (int j = 0; j < 8; j++) if (j + 1 < back) st[(size_t)j * mv.C] = keep[j];
+        for (int j = 8; j + 1 < back; j++) st[(size_t)j * mv.C] = st[(size_t)(j + 1) * mv.C];
+        st[(size_t)(back - 1) * mv.C] = u;
+        return;
+    }
     const float *orow = o + (size_t)t * ld_o + (size_t)part * n, *zr = z + (size_t)t * ld_z + (size_t)part * n;
     float keep[8], ss = 0.0f;
 #pragma unroll
@@ -561,21 +576,15 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const float *o, int ld_
 #pragma unroll
     for (int i = 0; i < 8; i++) { const int c = tid + 256 * i; if (c < n) yr[c] = keep[i] * inv * wr[c]; }
     for (int c = tid + 2048; c < n; c += 256) yr[c] = orow[c] * gs_silu(zr[c]) * inv * wr[c];
-    if (mv.state) {
-        const int back = mv.taps - 1;
-        float *st = mv.state + (size_t)mv.seg_slot[t] * back * mv.C;
-        const float *u = mv.p + (size_t)t * mv.ld_p;
-        for (int c = part * 256 + tid; c < mv.C; c += 256 * gridDim.y) {
-            for (int j = 0; j + 1 < back; j++) st[(size_t)j * mv.C + c] = st[(size_t)(j + 1) * mv.C + c];
-            st[(size_t)(back - 1) * mv.C + c] = u[c];
-        }
-    }
 }
 
 template <int NCOL>
 static hipError_t launch_gated_step(const GatedScanArgs &a, int nz, hipStream_t st) {
-    const size_t lds = ((size_t)3 * a.D + 64 * NCOL + (size_t)GSS_NW * 64 * NCOL) * sizeof(float);
-    hipLaunchKernelGGL(gated_step_kernel<NCOL>, dim3((unsigned)a.n_seg, (unsigned)a.H, (unsigned)nz), dim3(64 * GSS_NW), lds, st, a);
+    const int nw = a.D >= 64 ? 16 : 8;                          // (a head's state is read by one workgroup: the more waves, the more of it is on its way)
+    const size_t lds = ((size_t)3 * a.D + 64 * NCOL + (size_t)nw * 64 * NCOL) * sizeof(float);
+    const dim3 grid((unsigned)a.n_seg, (unsigned)a.H, (unsigned)nz);
+    if (nw == 16) hipLaunchKernelGGL((gated_step_kernel<NCOL, 16>), grid, dim3(1024), lds, st, a);
+    else hipLaunchKernelGGL((gated_step_kernel<NCOL, 8>), grid, dim3(512), lds, st, a);
     return hipGetLastError();
 }
 
@@ -642,7 +651,8 @@ hipError_t launch_conv_silu(const float *p, int ld_p, int C, const float *wt, co
 hipError_t launch_gated_norm(const float *o, int ld_o, const float *z, int ld_z, const float *w, int T, int parts, int n, float eps, float *y, int ld_y, const ConvMove &mv, hipStream_t st) {
     if (T <= 0) return hipSuccess;
     if (parts < 1 || n < 1 || !o || !z || !w || !y || (mv.state && (mv.taps < 2 || mv.C < 1 || !mv.p || !mv.seg_slot))) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(gated_norm_kernel, dim3((unsigned)T, (unsigned)parts), dim3(256), 0, st, o, ld_o, z, ld_z, w, n, eps, y, ld_y, mv);
+    const unsigned movers = mv.state ? (unsigned)((mv.C + 255) / 256) : 0;
+    hipLaunchKernelGGL(gated_norm_kernel, dim3((unsigned)T, (unsigned)parts + movers), dim3(256), 0, st, o, ld_o, z, ld_z, w, parts, n, eps, y, ld_y, mv);
     return hipGetLastError();
 }
 

@@ -707,7 +707,8 @@ hipError_t launch_gq_prep(const GqPrepArgs &a, hipStream_t st) {
     if ((a.norm_per_head || a.unit_behind) && (size_t)n_heads * sizeof(float) > 32 * 1024) return hipErrorInvalidValue;
     size_t lds = (a.norm_per_head || a.unit_behind || a.v_unit ? (size_t)n_heads : 0) + (a.v_unit ? (size_t)a.G : 0);
     if (!a.conv_wt) {
-        hipLaunchKernelGGL((gq_prep_kernel<256, false>), dim3((unsigned)a.T), dim3(256), lds * sizeof(float), st, a);
+        if (a.T < 64) hipLaunchKernelGGL((gq_prep_kernel<1024, false>), dim3((unsigned)a.T), dim3(1024), lds * sizeof(float), st, a);   // (few rows: a token's trips to memory are the time)
+        else hipLaunchKernelGGL((gq_prep_kernel<256, false>), dim3((unsigned)a.T), dim3(256), lds * sizeof(float), st, a);
         return hipGetLastError();
     }
     const size_t C = (size_t)a.H * a.dim + (size_t)a.G * (a.maps > 1 ? a.maps : 1) * a.dim + (a.v_is_k ? 0 : (size_t)a.G * a.vdim);

@@ -129,15 +129,29 @@ __global__ __launch_bounds__(256) void mmb_vec_rows_kernel(MMBArgs a) {
         rsc[i] = a.row_scale && i < nt ? a.row_scale[v.y0 + i] : 1.0f;
 #pragma unroll
         for (int r = 0; r < NR; r++) res[r][i] = v.resid && i < nt && n0 + r < a.N ? v.resid[y_row(a, v, i) + n0 + r] : 0.0f;
-        if (LN) mid[i] = i < nt ? row_middle<true>(x_row(a, v, i), a.K, lane) : 0.0f;
     }
-    for (int k = lane * 8; k < a.K; k += 512) {
-        u16x8 w8[NR], w28[NR];
+    u16x8 w8n[NR], w28n[NR];                                    // (LN: a piece's weights are on their way while the rows' middle values, or the piece before, are worked on)
+#pragma unroll
+    for (int r = 0; r < NR; r++) w8n[r] = w28n[r] = u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    const auto ahead = [&](int k) {
+        if (k >= a.K) return;
 #pragma unroll
         for (int r = 0; r < NR; r++) {
-            w8[r] = *reinterpret_cast<const u16x8 *>(wr[r] + k);
-            if (gated) w28[r] = *reinterpret_cast<const u16x8 *>(wr2[r] + k);
+            w8n[r] = *reinterpret_cast<const u16x8 *>(wr[r] + k);
+            if (gated) w28n[r] = *reinterpret_cast<const u16x8 *>(wr2[r] + k);
         }
+    };
+    if (LN) {
+        ahead(lane * 8);
+#pragma unroll
+        for (int i = 0; i < TBR; i++) mid[i] = i < nt ? row_middle<true>(x_row(a, v, i), a.K, lane) : 0.0f;
+    }
+    for (int k = lane * 8; k < a.K; k += 512) {
+        if (!LN) ahead(k);
+        u16x8 w8[NR], w28[NR];
+#pragma unroll
+        for (int r = 0; r < NR; r++) { w8[r] = w8n[r]; w28[r] = w28n[r]; }
+        if (LN) ahead(k + 512);
         float pw[8];
         if (pn) {
             const f32x4 g0 = *reinterpret_cast<const f32x4 *>(a.pn_w + k), g1 = *reinterpret_cast<const f32x4 *>(a.pn_w + k + 4);
