@@ -338,6 +338,16 @@ def test_a_recurrent_sequence_cannot_be_cut_back_but_can_be_copied(full):
     assert close(got2, full.ref(t[:25] + tail)[25:])
 
 
+def test_attention_layers_alone_can_be_cut_back(pkg, tmp_path):
+    """No recurrence anywhere: a sequence's tail can be removed and fed again."""
+    rig = Rig(pkg, tmp_path / "cut", S.config([S.attention(mlp=S.dense()), S.attention(size=9)]), seed=27)
+    t, tail = toks(40, rig.cfg["vocab"], 28), toks(20, rig.cfg["vocab"], 29)
+    c = rig.ctx()
+    feed(c, t)
+    assert c.kv_seq_rm(0, 17, -1)
+    assert close(feed(c, tail, 17), rig.ref(t[:17] + tail)[17:])
+
+
 # ------------------------------------------------------------------------------------------ keys and memories made loud
 D0 = 9                                                          # the loud coordinate (of the first head): one that does not turn
 
